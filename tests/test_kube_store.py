@@ -115,8 +115,11 @@ def test_reference_samples_validate(apiserver, kube):
     import glob
     import os
 
+    paths = sorted(glob.glob(os.path.join(REF_SAMPLES, "*.yaml")))
+    if not paths:
+        pytest.skip("reference samples are not mounted")
     applied = 0
-    for path in sorted(glob.glob(os.path.join(REF_SAMPLES, "*.yaml"))):
+    for path in paths:
         if path.endswith("kustomization.yaml"):
             continue
         with open(path) as f:
