@@ -20,6 +20,9 @@ from conftest import wait_for
 from mock_apiserver import MockAPIServer
 
 REF_SAMPLES = "/root/reference/acp/config/samples"
+requires_samples = pytest.mark.skipif(
+    not os.path.isdir(REF_SAMPLES), reason="reference samples are not mounted"
+)
 
 
 @pytest.fixture()
@@ -110,14 +113,13 @@ def test_lease_semantics(kube):
     assert kube.acquire_lease("task-llm-x", "pod-b", 30) is True
 
 
+@requires_samples
 def test_reference_samples_validate(apiserver, kube):
     """Reference sample manifests apply byte-for-byte against our CRDs."""
     import glob
     import os
 
     paths = sorted(glob.glob(os.path.join(REF_SAMPLES, "*.yaml")))
-    if not paths:
-        pytest.skip("reference samples are not mounted")
     applied = 0
     for path in paths:
         if path.endswith("kustomization.yaml"):
@@ -171,6 +173,7 @@ class _MockOpenAI(BaseHTTPRequestHandler):
         pass
 
 
+@requires_samples
 def test_kubectl_apply_e2e(apiserver):
     """Reference Agent + Task sample YAML applied unchanged through the
     Kubernetes wire reach FinalAnswer (VERDICT item 2's done-criterion,
