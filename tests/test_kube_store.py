@@ -7,6 +7,7 @@ validated against this repo's generated CRDs (config/crd/bases/)."""
 from __future__ import annotations
 
 import json
+import os
 import threading
 from http.server import BaseHTTPRequestHandler, ThreadingHTTPServer
 
