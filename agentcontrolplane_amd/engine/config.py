@@ -2,12 +2,56 @@
 
 Model presets are the architectures BASELINE.json names (Llama-3 8B/70B,
 Mixtral 8x7B) plus tiny test configs; weights are random-init (no network),
-shapes and dtypes are the real ones.
+shapes and dtypes are the real ones.  A checkpoint directory whose
+config.json names a registered architecture needs no preset: model="auto"
+reads it (models/configs.py).
 """
 from __future__ import annotations
 
 import dataclasses
-from typing import Optional
+from typing import Optional, Tuple
+
+
+@dataclasses.dataclass(frozen=True)
+class LatentAttentionSpec:
+    """Attention over one cached low-rank latent per token plus one rotated
+    key part shared by all heads (models/latent_attention.py)."""
+
+    heads: int
+    dim: int                      # unrotated query/key dims per head
+    rot_dim: int                  # rotated query/key dims per head
+    vdim: int                     # value dims per head
+    kv_rank: int                  # latent size
+    scale: float                  # on the scores
+    rope_base: float
+    q_rank: Optional[int] = None  # low-rank query; None = direct projection
+    window: Optional[int] = None  # keys visible, self included; None = all
+    head_gate: bool = True        # sigmoid gate per head on the output
+
+
+@dataclasses.dataclass(frozen=True)
+class ClampedGluSpec:
+    """min(gate, limit) * sigmoid(alpha * .) * (clamp(up, +-limit) + offset)."""
+
+    width: int
+    limit: float
+    alpha: float = 1.702
+    offset: float = 1.0
+
+
+@dataclasses.dataclass(frozen=True)
+class LayerSpec:
+    mixer: LatentAttentionSpec
+    mlp: Optional[ClampedGluSpec] = None
+
+
+@dataclasses.dataclass(frozen=True)
+class LoopSpec:
+    """Layers [start, stop) run ``times`` times in a row on the same weights."""
+
+    start: int
+    stop: int
+    times: int
 
 
 @dataclasses.dataclass
@@ -30,12 +74,35 @@ class ModelConfig:
     num_experts: int = 0
     num_experts_per_tok: int = 2
     dtype: str = "bfloat16"
+    # models/registry key; "" picks llama or mixtral by num_experts
+    architecture: str = ""
+    # designs whose layers differ from each other list them; the head/MLP
+    # sizes above are then unused
+    layers: Tuple[LayerSpec, ...] = ()
+    loop: Optional[LoopSpec] = None
+    # per-layer token embedding: dims per layer, 0 = none
+    token_side_dim: int = 0
+
+    @property
+    def layer_runs(self) -> Tuple[Tuple[int, bool], ...]:
+        """(layer, enters a loop pass) in execution order: one entry, and
+        one cache, per layer and pass."""
+        n = len(self.layers) or self.num_layers
+        if self.loop is None:
+            return tuple((i, False) for i in range(n))
+        lo, hi = self.loop.start, self.loop.stop
+        runs = [(i, False) for i in range(lo)]
+        for _ in range(self.loop.times):
+            runs += [(i, i == lo) for i in range(lo, hi)]
+        return tuple(runs + [(i, False) for i in range(hi, n)])
 
     @property
     def is_moe(self) -> bool:
         return self.num_experts > 0
 
     def params_bytes(self, dtype_bytes: int = 2) -> int:
+        if self.layers:
+            return self._listed_layer_params() * dtype_bytes
         h, i, v, L = self.hidden_size, self.intermediate_size, self.vocab_size, self.num_layers
         kvh = self.num_kv_heads * self.head_dim
         qh = self.num_heads * self.head_dim
@@ -46,6 +113,48 @@ class ModelConfig:
         per_layer = attn + mlp + 2 * h
         total = L * per_layer + 2 * v * h + h
         return total * dtype_bytes
+
+    def _listed_layer_params(self) -> int:
+        w, v = self.hidden_size, self.vocab_size
+        total = v * w + w
+        for layer in self.layers:
+            m = layer.mixer
+            qdim = m.heads * (m.dim + m.rot_dim)
+            total += w
+            total += m.q_rank * (w + 1 + qdim) if m.q_rank else w * qdim
+            total += w * (m.kv_rank + m.rot_dim) + m.kv_rank
+            total += m.kv_rank * m.heads * (m.dim + m.vdim) + m.heads * m.vdim * w
+            total += w * m.heads if m.head_gate else 0
+            total += 3 * w * layer.mlp.width if layer.mlp else 0
+            if self.token_side_dim:
+                total += 2 * w * self.token_side_dim + w + v * self.token_side_dim
+        return total + (2 * w * w if self.loop else 0)
+
+
+def _fetolix(name: str, *, width: int, heads: int, layers: int, ff: int,
+             kv_rank: int, q_rank: int, dim: int, rot_dim: int, vdim: int,
+             window: int, vocab: int, side: int, limit: float = 7.0,
+             loop: Optional[LoopSpec] = None, full_every: int = 4,
+             **kw) -> ModelConfig:
+    """Every ``full_every``-th layer sees all keys with a direct query; the
+    others see a window with a low-rank query."""
+    def mixer(i: int) -> LatentAttentionSpec:
+        full = i % full_every == full_every - 1
+        return LatentAttentionSpec(
+            heads=heads, dim=dim, rot_dim=rot_dim, vdim=vdim, kv_rank=kv_rank,
+            scale=(dim + rot_dim) ** -0.5, rope_base=1e6 if full else 1e4,
+            q_rank=None if full else q_rank, window=None if full else window,
+        )
+
+    return ModelConfig(
+        name=name, architecture="Fetolix", vocab_size=vocab, hidden_size=width,
+        intermediate_size=ff, num_layers=layers, num_heads=heads,
+        num_kv_heads=1, head_dim=dim + rot_dim, tie_embeddings=True,
+        layers=tuple(
+            LayerSpec(mixer(i), ClampedGluSpec(ff, limit)) for i in range(layers)
+        ),
+        loop=loop, token_side_dim=side, **kw,
+    )
 
 
 PRESETS = {
@@ -87,6 +196,25 @@ PRESETS = {
         rope_theta=1000000.0,
         num_experts=8,
         num_experts_per_tok=2,
+    ),
+    # Fetolix at the layer sizes of an 8B-class dense model (random weights):
+    # width and head count of llama3-8b, a 512-wide latent
+    "fetolix-8b": _fetolix(
+        "fetolix-8b", width=4096, heads=32, layers=24, ff=14336, kv_rank=512,
+        q_rank=1536, dim=128, rot_dim=64, vdim=128, window=4096, vocab=128256,
+        side=64, loop=LoopSpec(4, 12, 2),
+    ),
+    # half the width, 16 heads
+    "fetolix-2b": _fetolix(
+        "fetolix-2b", width=2048, heads=16, layers=16, ff=8192, kv_rank=512,
+        q_rank=768, dim=128, rot_dim=64, vdim=128, window=1024, vocab=32000,
+        side=64, loop=LoopSpec(4, 8, 2),
+    ),
+    "tiny-fetolix": _fetolix(
+        "tiny-fetolix", width=48, heads=3, layers=4, ff=72, kv_rank=24,
+        q_rank=20, dim=12, rot_dim=8, vdim=10, window=19, vocab=300, side=6,
+        limit=1.5, loop=LoopSpec(1, 3, 2), full_every=2, max_position=4096,
+        dtype="float32",
     ),
     # tiny GPU config: real head_dim/GQA shape for the CDNA4 kernels at
     # test scale (kernels require head_dim 128)
@@ -162,7 +290,10 @@ PRESETS = {
 
 @dataclasses.dataclass
 class EngineConfig:
+    # a PRESETS name, or "auto": the checkpoint's own config.json
     model: str = "llama3-8b"
+    # overrides the model's dtype ("bfloat16" | "float32")
+    dtype: Optional[str] = None
     device: str = "cuda"                 # "cuda" (ROCm) or "cpu"
     kv_block_size: int = 16
     # KV pool: fraction of free HBM to claim (288 GB/GPU on MI355X), or an
@@ -195,6 +326,14 @@ class EngineConfig:
     tokenizer_path: Optional[str] = None
 
     def model_config(self) -> ModelConfig:
-        if self.model not in PRESETS:
+        if self.model == "auto":
+            from ..models.configs import read_model_config
+
+            if self.checkpoint_path is None:
+                raise ValueError('model="auto" needs checkpoint_path')
+            cfg = read_model_config(self.checkpoint_path)
+        elif self.model in PRESETS:
+            cfg = PRESETS[self.model]
+        else:
             raise KeyError(f"unknown model preset {self.model!r}; have {sorted(PRESETS)}")
-        return PRESETS[self.model]
+        return dataclasses.replace(cfg, dtype=self.dtype) if self.dtype else cfg

@@ -30,7 +30,7 @@ from .config import EngineConfig
 from .kv import make_block_manager
 from .request import ChatResult, InferenceRequest, SamplingParams
 from .scheduler import Scheduler, Sequence
-from .tokenizer import N_SPECIAL, ByteTokenizer
+from .tokenizer import N_SPECIAL, ByteTokenizer, IdTokenizer
 
 
 class InferenceEngine:
@@ -51,6 +51,8 @@ class InferenceEngine:
             from .tokenizer import HFTokenizer
 
             self.tokenizer = HFTokenizer(tok_path, self.mcfg.vocab_size)
+        elif self.mcfg.vocab_size < N_SPECIAL:
+            self.tokenizer = IdTokenizer(self.mcfg.vocab_size)
         else:
             self.tokenizer = ByteTokenizer(self.mcfg.vocab_size)
         self._eot = self.tokenizer.eot
@@ -523,13 +525,7 @@ class InferenceEngine:
             from ..parallel.tp import broadcast_step
 
             broadcast_step(batch_to_wire(batch))
-        logits = None
-        if self.graph_runner is not None and not batch.prefills:
-            logits = self.graph_runner.run(batch)
-            if logits is not None:
-                self._m["graph_steps"] = self._m.get("graph_steps", 0) + 1
-        if logits is None:
-            logits = self.model.forward(batch)
+        logits = self.forward_batch(batch)
         self._m["compute_time_s"] += time.monotonic() - t1
         self._m["steps"] += 1
         self._m["prompt_tokens"] += batch.num_prefill_tokens
@@ -548,6 +544,16 @@ class InferenceEngine:
             self._m.get("sample_launch_time_s", 0.0) + time.monotonic() - t2
         )
         return pending
+
+    def forward_batch(self, batch) -> torch.Tensor:
+        """Logits of one scheduled batch: the captured graph of a decode-only
+        step, else the model's forward."""
+        logits = None
+        if self.graph_runner is not None and not batch.prefills:
+            logits = self.graph_runner.run(batch)
+            if logits is not None:
+                self._m["graph_steps"] = self._m.get("graph_steps", 0) + 1
+        return self.model.forward(batch) if logits is None else logits
 
     def step(self) -> bool:
         """One serial scheduler round + forward + sampling (tests and the

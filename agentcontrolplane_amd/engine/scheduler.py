@@ -301,7 +301,57 @@ class Scheduler:
                     preempted.append(victim)
             return SchedulerOutput(batch=None, preempted=preempted)
 
-        # 3) materialize the flat batch
+        batch = self._build_batch(
+            prefills, decode_seqs, spec_src if spec_after is not None else None
+        )
+        return SchedulerOutput(batch=batch, preempted=preempted)
+
+    def schedule_portions(
+        self, portions: List[Tuple[Sequence, int, List[int]]]
+    ) -> Tuple[FlatBatch, List[Tuple[int, int]]]:
+        """Build the batch of an externally chosen schedule (trace replay):
+        each sequence's next ``count`` tokens, already appended to its
+        prompt, and the offsets among them whose logits are wanted.  One
+        token after cached ones runs as a decode row, anything else as a
+        prefill chunk.  Returns the batch and, per logit row, the portion and
+        offset it belongs to."""
+        self.stager.step()
+        prefills, decode_seqs = [], []
+        wanted: Dict[int, List[int]] = {}
+        index: Dict[int, int] = {}
+        for n, (s, count, want) in enumerate(portions):
+            if s in self.waiting:
+                if len(self.running) >= self.cfg.max_batch_size:
+                    raise RuntimeError("more live sequences than max_batch_size")
+                self.waiting.remove(s)
+                self.running.append(s)
+                self.bm.add_seq(s.seq_id)
+            index[s.seq_id] = n
+            wanted[s.seq_id] = want
+            if count == 1 and s.num_processed > 0:
+                s.num_processed += 1
+                s.state = DECODE
+                decode_seqs.append(s)
+            else:
+                s.state = PREFILL
+                prefills.append((s, count))
+        batch = self._build_batch(prefills, decode_seqs, None, wanted)
+        places = [
+            (index[s.seq_id], k) for s, _ in prefills for k in wanted[s.seq_id]
+        ] + [(index[s.seq_id], 0) for s in decode_seqs]
+        return batch, places
+
+    def _build_batch(
+        self,
+        prefills: List[Tuple[Sequence, int]],
+        decode_seqs: List[Sequence],
+        spec_src: Optional[Dict[int, int]],
+        wanted: Optional[Dict[int, List[int]]] = None,
+    ) -> FlatBatch:
+        """Reserve KV slots and lay the step's rows out as one FlatBatch:
+        prefill chunks, then one row per decode sequence.  ``spec_src`` marks
+        a speculative step (seq_id -> sample row of the step in flight);
+        ``wanted`` replaces the rows that get logits in prefill chunks."""
         token_ids: List[int] = []
         positions: List[int] = []
         slot_mapping: List[int] = []
@@ -328,9 +378,10 @@ class Scheduler:
                     needs_logits=done,
                 )
             )
+            rows = wanted[s.seq_id] if wanted is not None else [chunk - 1] if done else []
+            logit_rows.extend(row + k for k in rows)
+            sample_seq_ids.extend([s.seq_id] * len(rows))
             if done:
-                logit_rows.append(row + chunk - 1)
-                sample_seq_ids.append(s.seq_id)
                 s.state = DECODE
             row += chunk
         num_prefill_tokens = row
@@ -343,7 +394,7 @@ class Scheduler:
         if decode_seqs:
             lens = []
             for s in decode_seqs:
-                if spec_after is not None:
+                if spec_src is not None:
                     tok = 0  # filled on device from the previous step's samples
                     pos = s.total_len  # the in-flight token occupies total_len
                     spec_rows.append(spec_src[s.seq_id])
@@ -403,9 +454,9 @@ class Scheduler:
         }
         if decode_tables_i32 is not None:
             batch._decode_tables_i32 = decode_tables_i32
-        if spec_after is not None and spec_rows:
+        if spec_rows:
             batch.spec_src_rows = self.stager.tensor("spec", spec_rows, "int64")
-        return SchedulerOutput(batch=batch, preempted=preempted)
+        return batch
 
     # ------------------------------------------------------------ commit
 

@@ -82,6 +82,28 @@ class ByteTokenizer:
         return ids
 
 
+class IdTokenizer:
+    """No text: requests bring token ids and get token ids (a model without a
+    tokenizer whose vocabulary is too small for bytes).  Every id is live and
+    none ends a turn."""
+
+    def __init__(self, vocab_size: int):
+        self.vocab_size = self.live_vocab = vocab_size
+        self.eot = self.bos = -1
+
+    def token_bytes(self, tid: int):
+        return None
+
+    def decode(self, ids: Sequence[int]) -> str:
+        return " ".join(str(i) for i in ids)
+
+    def encode_text(self, text: str) -> List[int]:
+        raise ValueError("this model has no tokenizer: send token ids")
+
+    def render_chat(self, messages, tools=None) -> List[int]:
+        return self.encode_text("")
+
+
 # --------------------------------------------------------------- BPE (HF)
 
 

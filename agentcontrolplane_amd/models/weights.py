@@ -71,7 +71,9 @@ def save_checkpoint(model, path: str, max_shard_bytes: int = 4 << 30) -> None:
             "save_checkpoint requires tp_world == 1 (gather shards first)"
         )
     os.makedirs(path, exist_ok=True)
-    tensors = _llama_name_map(model)
+    # designs with their own tensor names export them; the rest use HF names
+    named = getattr(model, "named_tensors", None)
+    tensors = named() if named is not None else _llama_name_map(model)
     shards, cur, cur_bytes = [], {}, 0
     for name, t in tensors.items():
         tb = t.numel() * t.element_size()
@@ -92,9 +94,7 @@ def save_checkpoint(model, path: str, max_shard_bytes: int = 4 << 30) -> None:
         json.dump(index, f)
 
 
-def load_checkpoint(model, path: str) -> None:
-    """Load HF-named safetensors into the model, fusing QKV/gate_up and
-    taking this rank's TP slice."""
+def _read_tensors(path: str) -> Dict[str, torch.Tensor]:
     from safetensors.torch import load_file
 
     idx_path = os.path.join(path, "model.safetensors.index.json")
@@ -109,6 +109,23 @@ def load_checkpoint(model, path: str) -> None:
     tensors: Dict[str, torch.Tensor] = {}
     for fname in files:
         tensors.update(load_file(os.path.join(path, fname)))
+    return tensors
+
+
+def load_checkpoint(model, path: str) -> None:
+    """Load a safetensors directory into the model, taking this rank's TP
+    slice.  Models with their own tensor names fetch them by name; for the
+    others the names are HF's, and QKV and gate_up are fused here."""
+    tensors = _read_tensors(path)
+
+    def get(name):
+        if name not in tensors:
+            raise KeyError(f"checkpoint missing {name}")
+        return tensors[name]
+
+    if hasattr(model, "load_tensors"):
+        model.load_tensors(get)
+        return
 
     cfg = model.cfg
     r, w = model.tp_rank, model.tp_world
@@ -116,11 +133,6 @@ def load_checkpoint(model, path: str) -> None:
     q_per, kv_per = cfg.num_heads // w, cfg.num_kv_heads // w
     inter_per = cfg.intermediate_size // w
     dev, dt = model.device, model.dtype
-
-    def get(name):
-        if name not in tensors:
-            raise KeyError(f"checkpoint missing {name}")
-        return tensors[name]
 
     model.embed = get("model.embed_tokens.weight").to(dev, dt)
     model.final_norm = get("model.norm.weight").to(dev, dt)

@@ -106,6 +106,85 @@ def swiglu(gate_up):
     return _impl(gate_up).swiglu(gate_up)
 
 
+# ------------------------------------------------ fp32-residual norms, GLU, gates
+
+
+def rmsnorm_rows(x, weight, eps: float, n: int):
+    """RMS norm of row-strided [N, K] over the first n columns (the rest are
+    padding: zero in, zero weight, zero out)."""
+    return _impl(x).rmsnorm_rows(x, weight, eps, n)
+
+
+def layernorm(x, weight, eps: float, dtype):
+    """Layer norm without bias of an fp32 residual [N, K] -> dtype."""
+    return _impl(x).layernorm(x, weight, eps, dtype)
+
+
+def add_to_residual(x, y, dtype):
+    """x += y in the fp32 residual x; returns the new x in dtype."""
+    return _impl(x).add_to_residual(x, y, dtype)
+
+
+def residual_norm(x, y, eps: float, y_norm=None, x_norm=None, out=None):
+    """x += y, or x += rmsnorm(y) * y_norm, in the fp32 residual x; then
+    out = layernorm(x) * x_norm, or x itself without x_norm."""
+    return _impl(x).residual_norm(x, y, eps, y_norm, x_norm, out)
+
+
+def clamped_glu(gate_up, limit: float, alpha: float, offset: float, out):
+    """gate_up [N, 2I] (row-strided halves) -> out [N, I] (row-strided):
+    g * sigmoid(alpha g) * (u + offset), g capped at limit, u at +-limit."""
+    return _impl(gate_up).clamped_glu(gate_up, limit, alpha, offset, out)
+
+
+def gelu_gate_(s, token_ids, table, offset: int):
+    """s [N, D] <- gelu_tanh(s) * table[token, offset : offset + D]."""
+    return _impl(s).gelu_gate_(s, token_ids, table, offset)
+
+
+# ------------------------------------------------------------ latent attention
+
+#: latent sizes the MFMA kernels are built for; larger ones run the plain kernel
+LATENT_RANKS = (64, 128, 256, 384, 512)
+
+
+def latent_rank(kv_rank: int) -> int:
+    """The padded latent size kernels and caches use for kv_rank."""
+    for r in LATENT_RANKS:
+        if kv_rank <= r:
+            return r
+    return -(-kv_rank // 64) * 64
+
+
+def latent_cache_write(kv, norm_w, eps: float, kv_rank: int, rot_dim: int, rank: int,
+                       positions, slot_mapping, cos_sin, cache):
+    """kv [N, kv_rank + rot_dim] (row-strided): RMS-norm the latent, rotate the
+    key part (interleaved pairs), scatter [latent -> rank | rotated] rows into
+    cache [blocks, block, row]."""
+    return _impl(kv).latent_cache_write(
+        kv, norm_w, eps, kv_rank, rot_dim, rank, positions, slot_mapping, cos_sin, cache
+    )
+
+
+def head_linear(x, w, out, gate=None):
+    """out[n, h] = w[h] @ x[n, h], times sigmoid(gate[n, h]) if given.
+    x [N, H, K], w [H, O, K], out [N, H, O]; x, out, gate row-strided."""
+    return _impl(x).head_linear(x, w, out, gate)
+
+
+def absorb_query(q, w_uk, positions, cos_sin, d: int, rot_dim: int):
+    """q [N, H, d + rot] (row-strided) -> [N, H, rank + rot]: w_uk[h] @ q[:d],
+    then the rotated rest."""
+    return _impl(q).absorb_query(q, w_uk, positions, cos_sin, d, rot_dim)
+
+
+def latent_attention(q, cache, batch, rank: int, scale: float, window):
+    """Softmax attention of absorbed queries [N, H, row] (all of a FlatBatch)
+    over cached rows; values are a row's first ``rank`` dims: [N, H, rank].
+    window = visible keys per query, None = all."""
+    return _impl(q).latent_attention(q, cache, batch, rank, scale, window)
+
+
 def softmax_sample(logits, temperatures, top_ks, top_ps, gen, mask=None,
                    uniforms=None, mask_map=None):
     """Batch sampling: temperature/top-k/top-p with optional boolean vocab

@@ -21,12 +21,15 @@ def fused_add_rmsnorm(x, residual, weight, eps: float = 1e-5):
     return rmsnorm(new_residual, weight, eps), new_residual
 
 
-def build_cos_sin(max_position: int, head_dim: int, theta: float, device, dtype=torch.float32):
-    """[max_position, head_dim/2] cos and sin tables (rotate-half RoPE)."""
+def build_cos_sin(max_position: int, head_dim: int, theta: float, device, dtype=torch.float32,
+                  exact: bool = False):
+    """[2, max_position, head_dim/2] cos and sin tables of position times
+    theta^(-2i/head_dim).  ``exact`` takes the angles in double precision."""
+    at = torch.float64 if exact else torch.float32
     inv_freq = 1.0 / (
-        theta ** (torch.arange(0, head_dim, 2, device=device, dtype=torch.float32) / head_dim)
+        theta ** (torch.arange(0, head_dim, 2, device=device, dtype=at) / head_dim)
     )
-    t = torch.arange(max_position, device=device, dtype=torch.float32)
+    t = torch.arange(max_position, device=device, dtype=at)
     freqs = torch.outer(t, inv_freq)
     return torch.stack([freqs.cos(), freqs.sin()], dim=0).to(dtype)  # [2, P, D/2]
 
@@ -148,6 +151,121 @@ def _block_size_of(cache):
 def swiglu(gate_up: torch.Tensor) -> torch.Tensor:
     gate, up = gate_up.float().chunk(2, dim=-1)
     return (torch.nn.functional.silu(gate) * up).to(gate_up.dtype)
+
+
+# ------------------------------------------------ fp32-residual norms, GLU, gates
+
+
+def rmsnorm_rows(x, weight, eps: float, n: int):
+    xf = x.float()
+    inv = torch.rsqrt(xf[:, :n].pow(2).mean(-1, keepdim=True) + eps)
+    return (xf * inv * weight.float()).to(x.dtype)
+
+
+def layernorm(x, weight, eps: float, dtype):
+    xc = x - x.mean(-1, keepdim=True)
+    var = xc.pow(2).mean(-1, keepdim=True)
+    return (xc * torch.rsqrt(var + eps) * weight.float()).to(dtype)
+
+
+def add_to_residual(x, y, dtype):
+    x += y.float()
+    return x.to(dtype)
+
+
+def residual_norm(x, y, eps: float, y_norm=None, x_norm=None, out=None):
+    yf = y.float()
+    if y_norm is not None:
+        yf = yf * torch.rsqrt(yf.pow(2).mean(-1, keepdim=True) + eps) * y_norm.float()
+    x += yf
+    if out is not None:
+        out.copy_(layernorm(x, x_norm, eps, out.dtype) if x_norm is not None else x)
+
+
+def clamped_glu(gate_up, limit: float, alpha: float, offset: float, out):
+    g, u = gate_up.float().chunk(2, dim=-1)
+    g = g.clamp(max=limit)
+    out.copy_(g * torch.sigmoid(alpha * g) * (u.clamp(-limit, limit) + offset))
+
+
+def gelu_gate_(s, token_ids, table, offset: int):
+    e = table[token_ids, offset : offset + s.shape[1]].float()
+    s.copy_(torch.nn.functional.gelu(s.float(), approximate="tanh") * e)
+    return s
+
+
+# ------------------------------------------------------------ latent attention
+
+
+def _rotate_interleaved(x, cos, sin):
+    """Rotate the pairs (x[..., 2i], x[..., 2i+1]); cos/sin broadcast over
+    x's pairs."""
+    u, v = x[..., 0::2].float(), x[..., 1::2].float()
+    return torch.stack([u * cos - v * sin, v * cos + u * sin], dim=-1).flatten(-2)
+
+
+def latent_cache_write(kv, norm_w, eps: float, kv_rank: int, rot_dim: int, rank: int,
+                       positions, slot_mapping, cos_sin, cache):
+    c = rmsnorm_rows(kv[:, :kv_rank], norm_w, eps, kv_rank)
+    k_rot = _rotate_interleaved(
+        kv[:, kv_rank : kv_rank + rot_dim], cos_sin[0][positions], cos_sin[1][positions]
+    )
+    row = torch.zeros(kv.shape[0], cache.shape[-1], dtype=cache.dtype, device=cache.device)
+    row[:, :kv_rank] = c.to(cache.dtype)
+    row[:, rank : rank + rot_dim] = k_rot.to(cache.dtype)
+    cache.view(-1, cache.shape[-1])[slot_mapping] = row
+
+
+def head_linear(x, w, out, gate=None):
+    y = torch.matmul(x.float().transpose(0, 1), w.float().transpose(1, 2)).transpose(0, 1)
+    if gate is not None:
+        y = y * torch.sigmoid(gate.float()).unsqueeze(-1)
+    out.copy_(y)
+    return out
+
+
+def absorb_query(q, w_uk, positions, cos_sin, d: int, rot_dim: int):
+    N, H, qk = q.shape
+    rank = w_uk.shape[1]
+    out = torch.zeros(N, H, rank + qk - d, dtype=q.dtype, device=q.device)
+    head_linear(q[:, :, :d], w_uk, out[:, :, :rank])
+    out[:, :, rank : rank + rot_dim] = _rotate_interleaved(
+        q[:, :, d : d + rot_dim],
+        cos_sin[0][positions].unsqueeze(1), cos_sin[1][positions].unsqueeze(1),
+    ).to(q.dtype)
+    return out
+
+
+def _latent_attention_seq(q, cache, block_table, ctx_len: int, rank: int, scale: float, window):
+    """One sequence's rows at positions ctx_len..; q [L, H, row] -> [L, H, rank]."""
+    L, bs = q.shape[0], cache.shape[1]
+    j = torch.arange(ctx_len + L, device=q.device)
+    table = torch.as_tensor(block_table, device=q.device)
+    rows = cache.view(-1, cache.shape[-1])[table[j // bs] * bs + j % bs].float()
+    i = torch.arange(ctx_len, ctx_len + L, device=q.device).view(-1, 1)
+    hidden = j > i
+    if window is not None:
+        hidden |= (i - j) >= window
+    scores = torch.matmul(q.float(), rows.t()) * scale        # [L, H, S]
+    probs = torch.softmax(scores.masked_fill(hidden.unsqueeze(1), float("-inf")), dim=-1)
+    return torch.matmul(probs, rows[:, :rank]).to(q.dtype)
+
+
+def latent_attention(q, cache, batch, rank: int, scale: float, window):
+    out = torch.empty(*q.shape[:2], rank, dtype=q.dtype, device=q.device)
+    row = 0
+    for m in batch.prefills:
+        out[row : row + m.query_len] = _latent_attention_seq(
+            q[row : row + m.query_len], cache, m.block_table, m.ctx_len, rank, scale, window
+        )
+        row += m.query_len
+    for b in range(batch.num_decode):
+        out[row : row + 1] = _latent_attention_seq(
+            q[row : row + 1], cache, batch.decode_block_tables[b],
+            int(batch.decode_seq_lens[b]) - 1, rank, scale, window,
+        )
+        row += 1
+    return out
 
 
 def softmax_sample(logits, temperatures, top_ks, top_ps, gen, mask=None,
