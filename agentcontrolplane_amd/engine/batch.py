@@ -67,14 +67,17 @@ class FlatBatch:
     def num_decode(self) -> int:
         return len(self.decode_seq_ids)
 
-    def prefill_meta(self, tile_q: int = 64) -> "PrefillMeta":
+    def prefill_meta(self, tile_q: int = 64, rows_per_token: int = 1) -> "PrefillMeta":
+        """Tiles of ``tile_q`` query rows; a token is ``rows_per_token`` rows
+        (its heads, for kernels that tile over both)."""
         if self._prefill_meta is None:
             self._prefill_meta = {}
-        if tile_q not in self._prefill_meta:
-            self._prefill_meta[tile_q] = PrefillMeta.build(
-                self.prefills, self.token_ids.device, tile_q, self._stager
+        key = (tile_q, rows_per_token)
+        if key not in self._prefill_meta:
+            self._prefill_meta[key] = PrefillMeta.build(
+                self.prefills, self.token_ids.device, tile_q, self._stager, rows_per_token
             )
-        return self._prefill_meta[tile_q]
+        return self._prefill_meta[key]
 
     def decode_tables_i32(self) -> torch.Tensor:
         if self._decode_tables_i32 is None:
@@ -154,7 +157,7 @@ class PrefillMeta:
 
     @staticmethod
     def build(prefills: List[SeqMeta], device, tile_q: int = 64,
-              stager=None) -> "PrefillMeta":
+              stager=None, rows_per_token: int = 1) -> "PrefillMeta":
         max_blocks = max((len(m.block_table) for m in prefills), default=1)
         tables, seq_lens, ctx_lens, row_starts = [], [], [], []
         tile_seq, tile_q0 = [], []
@@ -164,12 +167,14 @@ class PrefillMeta:
             seq_lens.append(m.seq_len)
             ctx_lens.append(m.ctx_len)
             row_starts.append(row)
-            for q0 in range(0, m.query_len, tile_q):
+            for q0 in range(0, m.query_len * rows_per_token, tile_q):
                 tile_seq.append(i)
                 tile_q0.append(q0)
             row += m.query_len
         if stager is not None:
-            t = lambda n, x: stager.tensor(f"pm{tile_q}_{n}", x, "int32")  # noqa: E731
+            t = lambda n, x: stager.tensor(
+                f"pm{tile_q}x{rows_per_token}_{n}", x, "int32"
+            )  # noqa: E731
         else:
             t = lambda n, x: torch.tensor(x, device=device, dtype=torch.int32)  # noqa: E731
         return PrefillMeta(

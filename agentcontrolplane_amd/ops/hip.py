@@ -108,6 +108,121 @@ def swiglu(gate_up):
     return out
 
 
+# ------------------------------------------------ fp32-residual norms, GLU, gates
+
+
+def rmsnorm_rows(x, weight, eps: float, n: int):
+    out = torch.empty(x.shape, dtype=x.dtype, device=x.device)
+    _C.rmsnorm_rows(out, x, weight, eps, n)
+    return out
+
+
+def layernorm(x, weight, eps: float, dtype):
+    out = torch.empty(x.shape, dtype=dtype, device=x.device)
+    _C.residual_norm(x, None, None, weight, out, eps)
+    return out
+
+
+def add_to_residual(x, y, dtype):
+    if dtype == torch.float32:
+        _C.add_to_residual(x, y, None)
+        return x
+    out = torch.empty(x.shape, dtype=dtype, device=x.device)
+    _C.add_to_residual(x, y, out)
+    return out
+
+
+def residual_norm(x, y, eps: float, y_norm=None, x_norm=None, out=None):
+    _C.residual_norm(x, y, y_norm, x_norm, out, eps)
+
+
+def clamped_glu(gate_up, limit: float, alpha: float, offset: float, out):
+    _C.clamped_glu(out, gate_up, limit, alpha, offset)
+
+
+def gelu_gate_(s, token_ids, table, offset: int):
+    _C.gelu_gate(s, token_ids, table, offset)
+    return s
+
+
+# ------------------------------------------------------------ latent attention
+
+_NO_WINDOW = 1 << 30
+#: workgroups that fill the chip at the MFMA kernel's LDS footprint
+_FILL = 512
+_MAX_SPLIT = 32
+
+
+def latent_cache_write(kv, norm_w, eps: float, kv_rank: int, rot_dim: int, rank: int,
+                       positions, slot_mapping, cos_sin, cache):
+    _C.latent_cache_write(
+        cache, kv, norm_w, positions, slot_mapping, cos_sin, eps, kv_rank, rot_dim, rank
+    )
+
+
+def head_linear(x, w, out, gate=None):
+    _C.head_linear(out, x, w, gate)
+    return out
+
+
+def absorb_query(q, w_uk, positions, cos_sin, d: int, rot_dim: int):
+    N, H, qk = q.shape
+    rank = w_uk.shape[1]
+    out = torch.empty(N, H, rank + qk - d, dtype=q.dtype, device=q.device)
+    _C.head_linear(out[:, :, :rank], q[:, :, :d], w_uk, None)
+    _C.rotate_interleaved(out[:, :, rank:], q[:, :, d:], positions, cos_sin, rot_dim)
+    return out
+
+
+def _latent_attn(out, q, cache, tables, seq_lens, prefill, tiles, mg, max_keys,
+                 scale, window, mfma):
+    """One launch over prefill tiles (prefill = their metadata) or decode
+    rows.  Few tiles split their keys over several workgroups."""
+    n_split = 1
+    if mfma:
+        keys = min(max_keys, window)
+        n_split = max(1, min(_MAX_SPLIT, _FILL // tiles, -(-keys // 128)))
+    part = ml = None
+    if n_split > 1:
+        rows = q.shape[0] * q.shape[1]
+        part = torch.empty(n_split * rows * out.shape[2], dtype=torch.float32, device=q.device)
+        ml = torch.empty(2 * n_split * rows, dtype=torch.float32, device=q.device)
+    m = prefill
+    _C.latent_attn(
+        out, q, cache, tables, seq_lens,
+        *((m.ctx_lens, m.row_starts, m.tile_seq, m.tile_q0) if m else (None,) * 4),
+        part, ml, scale, window, mg, n_split, mfma,
+    )
+
+
+def latent_attention(q, cache, batch, rank: int, scale: float, window):
+    from . import LATENT_RANKS
+
+    N, H, row = q.shape
+    out = torch.empty(N, H, rank, dtype=q.dtype, device=q.device)
+    window = window or _NO_WINDOW
+    mfma = q.dtype == torch.bfloat16 and rank in LATENT_RANKS and row - rank == 64
+    most = 4 if rank <= 256 else 2
+    P = batch.num_prefill_tokens
+    if batch.prefills:
+        mg = most
+        meta = batch.prefill_meta(16 * mg if mfma else 1, H)
+        _latent_attn(
+            out[:P], q[:P], cache, meta.block_tables, meta.seq_lens, meta,
+            meta.tile_seq.numel(), mg, max(m.seq_len for m in batch.prefills),
+            scale, window, mfma,
+        )
+    if batch.num_decode:
+        mg = 1 if H <= 16 else 2 if H <= 32 else most
+        tables = batch.decode_tables_i32()
+        _latent_attn(
+            out[P:], q[P:], cache, tables, batch.decode_lens_i32(), None,
+            batch.num_decode * -(-H // (16 * mg)), mg,
+            tables.shape[1] * cache.shape[1], scale, window, mfma,
+        )
+    return out
+
+
 def softmax_sample(logits, temperatures, top_ks, top_ps, gen, mask=None,
                    uniforms=None, mask_map=None):
     B, V = logits.shape

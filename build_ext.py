@@ -31,6 +31,10 @@ def build(verbose: bool = False) -> str:
         os.path.join(CSRC, "prefill_attn_mfma.hip"),
         os.path.join(CSRC, "mfma_probe.hip"),
         os.path.join(CSRC, "gemm_bf16.hip"),
+        os.path.join(CSRC, "residual_norm.hip"),
+        os.path.join(CSRC, "gated_act.hip"),
+        os.path.join(CSRC, "latent_proj.hip"),
+        os.path.join(CSRC, "latent_attn.hip"),
         os.path.join(CSRC, "sampling.hip"),
         os.path.join(CSRC, "sampling_fullvocab.hip"),
     ]

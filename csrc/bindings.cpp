@@ -6,6 +6,8 @@
 #include <c10/hip/HIPStream.h>
 #include <hip/hip_runtime.h>
 
+#include "latent_attn.h"
+
 namespace py = pybind11;
 
 void register_block_manager(py::module_& m);
@@ -32,6 +34,24 @@ void launch_sample(int64_t*, const float*, const float*, const int64_t*, const f
 void launch_prefill_attn_mfma(void*, const void*, const void*, const void*, const int*,
                               const int*, const int*, const int*, const int*, const int*,
                               float, int, int, int, int, int, int, int64_t, hipStream_t);
+void launch_residual_norm(bool, float*, const void*, const void*, const void*, void*, float,
+                          int, int, int64_t, hipStream_t);
+void launch_rmsnorm_rows(bool, void*, const void*, const void*, float, int, int, int,
+                         int64_t, hipStream_t);
+void launch_add_to_residual(bool, float*, const void*, void*, int64_t, hipStream_t);
+void launch_clamped_glu(bool, void*, const void*, float, float, float, int, int, int64_t,
+                        int64_t, hipStream_t);
+void launch_gelu_gate(bool, void*, const int64_t*, const void*, int, int, int64_t,
+                      hipStream_t);
+void launch_latent_cache_write(bool, void*, const void*, const void*, const int64_t*,
+                               const int64_t*, const float*, float, int, int, int, int,
+                               int, int64_t, int64_t, hipStream_t);
+void launch_rotate_interleaved(bool, void*, const void*, const int64_t*, const float*, int,
+                               int, int, int, int64_t, int64_t, int, int, int64_t,
+                               hipStream_t);
+void launch_head_linear(bool, void*, const void*, const void*, const void*, int, int, int,
+                        int, int64_t, int, int64_t, int, int64_t, hipStream_t);
+bool launch_latent_attn(bool, bool, const LatentArgs*, int, int, int, int, hipStream_t);
 void launch_mfma_probe(float*, const void*, const void*, hipStream_t);
 void launch_gemm_bf16(void*, const void*, const void*, int, int, int, hipStream_t);
 }
@@ -231,6 +251,241 @@ static void sample_fullvocab(torch::Tensor out, torch::Tensor logits,
                           mptr, mapptr, B, V, cur_stream());
 }
 
+// ---- fp32-residual norms, gated activations, latent attention: bf16 or fp32
+
+using OptTensor = c10::optional<torch::Tensor>;
+
+static bool is_bf16(const torch::Tensor& t) {
+  TORCH_CHECK(t.scalar_type() == at::kBFloat16 || t.scalar_type() == at::kFloat,
+              "want bf16 or fp32");
+  return t.scalar_type() == at::kBFloat16;
+}
+
+// [rows, k] with dense rows, any row stride
+static void check_rows(const torch::Tensor& t, at::ScalarType dtype, int64_t rows,
+                       int64_t k) {
+  CHECK_CUDA(t);
+  TORCH_CHECK(t.dim() == 2 && t.size(0) == rows && t.size(1) == k, "row shape mismatch");
+  TORCH_CHECK(t.scalar_type() == dtype, "dtype mismatch");
+  TORCH_CHECK(t.size(1) == 1 || t.stride(1) == 1, "rows must be dense");
+}
+
+static void check_vec(const torch::Tensor& t, at::ScalarType dtype, int64_t k) {
+  CHECK_CUDA(t); CHECK_CONT(t);
+  TORCH_CHECK(t.numel() == k && t.scalar_type() == dtype, "vector mismatch");
+}
+
+static void check_aligned(const torch::Tensor& t) {
+  TORCH_CHECK((uintptr_t)t.data_ptr() % 16 == 0 &&
+                  t.stride(0) * t.element_size() % 16 == 0,
+              "rows must be 16-byte aligned");
+}
+
+static void residual_norm(torch::Tensor x, OptTensor y, OptTensor y_norm, OptTensor x_norm,
+                          OptTensor out, double eps) {
+  CHECK_CUDA(x); CHECK_CONT(x);
+  TORCH_CHECK(x.scalar_type() == at::kFloat && x.dim() == 2);
+  TORCH_CHECK(y || out, "nothing to do");
+  const int n = x.size(0), w = x.size(1);
+  TORCH_CHECK(w <= 16000, "residual width");  // the row is held in LDS
+  const auto dt = y ? y->scalar_type() : out->scalar_type();
+  if (y) { check_rows(*y, dt, n, w); CHECK_CONT((*y)); }
+  if (y_norm) check_vec(*y_norm, dt, w);
+  if (x_norm) check_vec(*x_norm, dt, w);
+  if (out) check_rows(*out, dt, n, w);
+  if (n == 0) return;
+  launch_residual_norm(is_bf16(y ? *y : *out), x.data_ptr<float>(),
+                       y ? y->data_ptr() : nullptr, y_norm ? y_norm->data_ptr() : nullptr,
+                       x_norm ? x_norm->data_ptr() : nullptr,
+                       out ? out->data_ptr() : nullptr, (float)eps, n, w,
+                       out ? out->stride(0) : w, cur_stream());
+}
+
+static void rmsnorm_rows(torch::Tensor out, torch::Tensor x, torch::Tensor weight,
+                         double eps, int64_t n) {
+  const int rows = x.size(0), k = x.size(1);
+  check_rows(x, x.scalar_type(), rows, k);
+  check_rows(out, x.scalar_type(), rows, k); CHECK_CONT(out);
+  check_vec(weight, x.scalar_type(), k);
+  check_aligned(x);
+  TORCH_CHECK(k % 8 == 0 && n <= k);
+  if (rows == 0) return;
+  launch_rmsnorm_rows(is_bf16(x), out.data_ptr(), x.data_ptr(), weight.data_ptr(),
+                      (float)eps, rows, k, n, x.stride(0), cur_stream());
+}
+
+static void add_to_residual(torch::Tensor x, torch::Tensor y, OptTensor out) {
+  CHECK_CUDA(x); CHECK_CONT(x); CHECK_CUDA(y); CHECK_CONT(y);
+  TORCH_CHECK(x.scalar_type() == at::kFloat && x.numel() == y.numel());
+  if (out) {
+    CHECK_CUDA((*out)); CHECK_CONT((*out));
+    TORCH_CHECK(out->scalar_type() == y.scalar_type() && out->numel() == x.numel());
+  }
+  if (x.numel() == 0) return;
+  launch_add_to_residual(is_bf16(y), x.data_ptr<float>(), y.data_ptr(),
+                         out ? out->data_ptr() : nullptr, x.numel(), cur_stream());
+}
+
+static void clamped_glu(torch::Tensor out, torch::Tensor gate_up, double limit,
+                        double alpha, double offset) {
+  const int rows = out.size(0), inter = out.size(1);
+  check_rows(out, gate_up.scalar_type(), rows, inter);
+  check_rows(gate_up, gate_up.scalar_type(), rows, 2 * (int64_t)inter);
+  check_aligned(out); check_aligned(gate_up);
+  TORCH_CHECK(inter % 8 == 0, "padded width must be a multiple of 8");
+  if (rows == 0) return;
+  launch_clamped_glu(is_bf16(out), out.data_ptr(), gate_up.data_ptr(), (float)limit,
+                     (float)alpha, (float)offset, rows, inter, gate_up.stride(0),
+                     out.stride(0), cur_stream());
+}
+
+static void gelu_gate(torch::Tensor s, torch::Tensor token_ids, torch::Tensor table,
+                      int64_t offset) {
+  const int rows = s.size(0), dim = s.size(1);
+  check_rows(s, s.scalar_type(), rows, dim); CHECK_CONT(s);
+  check_rows(table, s.scalar_type(), table.size(0), table.size(1));
+  CHECK_CUDA(token_ids); CHECK_CONT(token_ids);
+  TORCH_CHECK(token_ids.scalar_type() == at::kLong && token_ids.numel() == rows);
+  TORCH_CHECK(offset >= 0 && offset + dim <= table.size(1), "table columns");
+  if (rows == 0) return;
+  launch_gelu_gate(is_bf16(s), s.data_ptr(), token_ids.data_ptr<int64_t>(),
+                   (const char*)table.data_ptr() + offset * table.element_size(), rows, dim,
+                   table.stride(0), cur_stream());
+}
+
+static void check_rotation(const torch::Tensor& cos_sin, const torch::Tensor& positions,
+                           int64_t n, int64_t rot_dim) {
+  CHECK_CUDA(cos_sin); CHECK_CONT(cos_sin); CHECK_CUDA(positions); CHECK_CONT(positions);
+  TORCH_CHECK(cos_sin.scalar_type() == at::kFloat && cos_sin.dim() == 3 &&
+              cos_sin.size(0) == 2 && cos_sin.size(2) * 2 == rot_dim, "rotation table");
+  TORCH_CHECK(positions.scalar_type() == at::kLong && positions.numel() == n);
+}
+
+static void latent_cache_write(torch::Tensor cache, torch::Tensor kv, torch::Tensor norm_w,
+                               torch::Tensor positions, torch::Tensor slots,
+                               torch::Tensor cos_sin, double eps, int64_t kv_rank,
+                               int64_t rot_dim, int64_t rank) {
+  const int n = kv.size(0);
+  check_rows(kv, kv.scalar_type(), n, kv_rank + rot_dim);
+  check_vec(norm_w, kv.scalar_type(), kv_rank);
+  check_rotation(cos_sin, positions, n, rot_dim);
+  CHECK_CUDA(slots); CHECK_CONT(slots); CHECK_CUDA(cache); CHECK_CONT(cache);
+  TORCH_CHECK(slots.scalar_type() == at::kLong && slots.numel() == n);
+  TORCH_CHECK(cache.scalar_type() == kv.scalar_type());
+  const int row = cache.size(-1);
+  TORCH_CHECK(kv_rank <= rank && rank + rot_dim <= row && (row - rank) % 2 == 0);
+  if (n == 0) return;
+  launch_latent_cache_write(is_bf16(kv), cache.data_ptr(), kv.data_ptr(), norm_w.data_ptr(),
+                            positions.data_ptr<int64_t>(), slots.data_ptr<int64_t>(),
+                            cos_sin.data_ptr<float>(), (float)eps, n, kv_rank, rot_dim, rank,
+                            row, kv.stride(0), cos_sin.size(1), cur_stream());
+}
+
+// [N, H, K] with dense vectors, any token and head stride
+static void check_heads(const torch::Tensor& t, at::ScalarType dtype, int64_t n, int64_t h) {
+  CHECK_CUDA(t);
+  TORCH_CHECK(t.dim() == 3 && t.size(0) == n && t.size(1) == h && t.stride(2) == 1,
+              "head shape mismatch");
+  TORCH_CHECK(t.scalar_type() == dtype, "dtype mismatch");
+  check_aligned(t);
+  TORCH_CHECK(t.stride(1) * t.element_size() % 16 == 0, "heads must be 16-byte aligned");
+}
+
+static void rotate_interleaved(torch::Tensor dst, torch::Tensor src, torch::Tensor positions,
+                               torch::Tensor cos_sin, int64_t rot_dim) {
+  const int n = src.size(0), h = src.size(1), rot = dst.size(2);
+  check_heads(src, src.scalar_type(), n, h);
+  check_heads(dst, src.scalar_type(), n, h);
+  check_rotation(cos_sin, positions, n, rot_dim);
+  TORCH_CHECK(rot % 2 == 0 && rot_dim <= rot && src.size(2) == rot);
+  if (n == 0) return;
+  launch_rotate_interleaved(is_bf16(src), dst.data_ptr(), src.data_ptr(),
+                            positions.data_ptr<int64_t>(), cos_sin.data_ptr<float>(), n, h,
+                            rot_dim, rot, dst.stride(0), src.stride(0), src.stride(1),
+                            dst.stride(1), cos_sin.size(1), cur_stream());
+}
+
+static void head_linear(torch::Tensor out, torch::Tensor x, torch::Tensor w,
+                        OptTensor gate) {
+  const int n = x.size(0), h = x.size(1), k = x.size(2), o = out.size(2);
+  check_heads(x, w.scalar_type(), n, h);
+  check_heads(out, w.scalar_type(), n, h);
+  CHECK_CUDA(w); CHECK_CONT(w);
+  TORCH_CHECK(w.dim() == 3 && w.size(0) == h && w.size(1) == o && w.size(2) == k);
+  TORCH_CHECK(k % 32 == 0 && o % 32 == 0, "head_linear wants multiples of 32");
+  if (gate) check_rows(*gate, w.scalar_type(), n, h);
+  if (n == 0) return;
+  launch_head_linear(is_bf16(w), out.data_ptr(), x.data_ptr(), w.data_ptr(),
+                     gate ? gate->data_ptr() : nullptr, n, h, o, k, x.stride(0), x.stride(1),
+                     out.stride(0), out.stride(1), gate ? gate->stride(0) : 0, cur_stream());
+}
+
+static const int* opt_int(const OptTensor& t, int64_t n) {
+  if (!t) return nullptr;
+  CHECK_CUDA((*t)); CHECK_CONT((*t));
+  TORCH_CHECK(t->scalar_type() == at::kInt && t->numel() == n);
+  return t->data_ptr<int>();
+}
+
+// q [tokens, H, row] -> out [tokens, H, rank].  Prefill chunks bring ctx_lens,
+// row_starts and tiles; decode (one token per table row) brings none of them.
+static void latent_attn(torch::Tensor out, torch::Tensor q, torch::Tensor cache,
+                        torch::Tensor tables, torch::Tensor seq_lens, OptTensor ctx_lens,
+                        OptTensor row_starts, OptTensor tile_seq, OptTensor tile_r0,
+                        OptTensor part, OptTensor part_ml, double scale, int64_t window,
+                        int64_t mg, int64_t n_split, bool mfma) {
+  CHECK_CUDA(q); CHECK_CONT(q); CHECK_CONT(out); CHECK_CUDA(cache); CHECK_CONT(cache);
+  CHECK_CUDA(tables); CHECK_CONT(tables); CHECK_CUDA(seq_lens); CHECK_CONT(seq_lens);
+  const bool bf16 = is_bf16(q);
+  const int tokens = q.size(0), H = q.size(1), row = q.size(2), rank = out.size(2);
+  TORCH_CHECK(out.size(0) == tokens && out.size(1) == H && rank <= row);
+  TORCH_CHECK(cache.dim() == 3 && cache.size(2) == row);
+  TORCH_CHECK(cache.scalar_type() == q.scalar_type() && out.scalar_type() == q.scalar_type());
+  TORCH_CHECK(tables.scalar_type() == at::kInt && seq_lens.scalar_type() == at::kInt);
+  const int seqs = tables.size(0);
+  TORCH_CHECK(seq_lens.numel() == seqs);
+  TORCH_CHECK(!mfma || (bf16 && row - rank == 64), "no MFMA kernel for this row");
+  TORCH_CHECK(window > 0 && n_split >= 1 && (mfma || n_split == 1));
+  TORCH_CHECK(mg == 1 || mg == 2 || (mg == 4 && rank <= 256) || !mfma, "row tile");
+  const int per_tile = mfma ? 16 * (int)mg : 1;
+  int tiles;
+  if (tile_seq) {
+    TORCH_CHECK(tile_r0 && ctx_lens && row_starts, "prefill metadata");
+    tiles = tile_seq->numel();
+  } else {
+    TORCH_CHECK(tokens == seqs, "decode has one token per sequence");
+    tiles = seqs * ((H + per_tile - 1) / per_tile);
+  }
+  if (tiles == 0) return;
+  LatentArgs a{};
+  a.out = out.data_ptr();
+  if (n_split > 1) {
+    TORCH_CHECK(part && part_ml && part->is_contiguous() && part_ml->is_contiguous());
+    TORCH_CHECK(part->scalar_type() == at::kFloat && part_ml->scalar_type() == at::kFloat);
+    TORCH_CHECK(part->numel() >= n_split * tokens * H * rank &&
+                part_ml->numel() >= 2 * n_split * tokens * H, "split workspace");
+    a.part = part->data_ptr<float>();
+    a.part_ml = (float2*)part_ml->data_ptr<float>();
+  }
+  a.q = q.data_ptr();
+  a.cache = cache.data_ptr();
+  a.tables = tables.data_ptr<int>();
+  a.seq_lens = seq_lens.data_ptr<int>();
+  a.ctx_lens = opt_int(ctx_lens, seqs);
+  a.row_starts = opt_int(row_starts, seqs);
+  a.tile_seq = opt_int(tile_seq, tiles);
+  a.tile_r0 = opt_int(tile_r0, tiles);
+  a.H = H;
+  a.max_blocks = tables.size(1);
+  a.kv_block = cache.size(1);
+  a.window = (int)window;
+  a.n_split = (int)n_split;
+  a.rows = tokens * H;
+  a.scale = (float)scale;
+  TORCH_CHECK(launch_latent_attn(bf16, mfma, &a, rank, row, (int)mg, tiles, cur_stream()),
+              "latent attention: unsupported sizes rank ", rank, " row ", row);
+}
+
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.doc() = "MI355X-native runtime: paged-KV block manager + CDNA4 kernels";
   register_block_manager(m);
@@ -243,6 +498,15 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("prefill_attn_mfma", &prefill_attn_mfma);
   m.def("mfma_probe", &mfma_probe);
   m.def("gemm_bf16", &gemm_bf16);
+  m.def("residual_norm", &residual_norm);
+  m.def("rmsnorm_rows", &rmsnorm_rows);
+  m.def("add_to_residual", &add_to_residual);
+  m.def("clamped_glu", &clamped_glu);
+  m.def("gelu_gate", &gelu_gate);
+  m.def("latent_cache_write", &latent_cache_write);
+  m.def("rotate_interleaved", &rotate_interleaved);
+  m.def("head_linear", &head_linear);
+  m.def("latent_attn", &latent_attn);
   m.def("sample", &sample);
   m.def("sample_fullvocab", &sample_fullvocab);
 }

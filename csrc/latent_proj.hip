@@ -1,0 +1,211 @@
+// Per-token kernels around latent attention (gfx950): the cache-row write, the
+// per-head products that absorb the key and value up-projections, and the
+// rotation of the query's rotated part.
+//
+// Rotations here pair dimension 2i with 2i+1; cos_sin is [2, P, rot_dim/2] fp32.
+#include "common_t.h"
+
+typedef __bf16 bf16x8_v __attribute__((ext_vector_type(8)));
+typedef float f32x4_v __attribute__((ext_vector_type(4)));
+
+// One wave per token: RMS-norm kv[:kv_rank], rotate kv[kv_rank:+rot_dim], write
+// the padded cache row [kv_rank -> rank | rot_dim -> row - rank] at its slot.
+template <typename T>
+__global__ __launch_bounds__(256) void latent_cache_write_kernel(
+    T* __restrict__ cache, const T* __restrict__ kv, const T* __restrict__ norm_w,
+    const int64_t* __restrict__ positions, const int64_t* __restrict__ slots,
+    const float* __restrict__ cos_sin, const float eps, const int N,
+    const int kv_rank, const int rot_dim, const int rank, const int row,
+    const int64_t kv_stride, const int64_t P) {
+  const int n = blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (n >= N) return;
+  const int lane = threadIdx.x & 63;
+  const T* src = kv + n * kv_stride;
+  T* dst = cache + slots[n] * row;
+  float ss = 0.f;
+  for (int i = lane; i < kv_rank; i += 64) {
+    const float f = to_f(src[i]);
+    ss += f * f;
+  }
+  const float inv = rsqrtf(wave_sum(ss) / kv_rank + eps);
+  for (int i = lane; i < rank; i += 64)
+    dst[i] = from_f<T>(i < kv_rank ? to_f(src[i]) * inv * to_f(norm_w[i]) : 0.f);
+  const int half = rot_dim >> 1;
+  const float* ct = cos_sin + positions[n] * half;
+  const float* st = ct + P * half;
+  for (int i = lane; 2 * i < row - rank; i += 64) {
+    float u = 0.f, v = 0.f;
+    if (i < half) {
+      const float a = to_f(src[kv_rank + 2 * i]), b = to_f(src[kv_rank + 2 * i + 1]);
+      u = a * ct[i] - b * st[i];
+      v = b * ct[i] + a * st[i];
+    }
+    dst[rank + 2 * i] = from_f<T>(u);
+    dst[rank + 2 * i + 1] = from_f<T>(v);
+  }
+}
+
+// dst[n, h, 0:rot] = rotate(src[n, h, 0:rot_dim]) then zeros; one thread a pair.
+template <typename T>
+__global__ __launch_bounds__(256) void rotate_interleaved_kernel(
+    T* __restrict__ dst, const T* __restrict__ src,
+    const int64_t* __restrict__ positions, const float* __restrict__ cos_sin,
+    const int64_t total, const int H, const int rot_dim, const int rot,
+    const int64_t dst_row, const int64_t src_row, const int src_head,
+    const int dst_head, const int64_t P) {
+  const int64_t t = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
+  if (t >= total) return;
+  const int pairs = rot >> 1, half = rot_dim >> 1;
+  const int i = (int)(t % pairs);
+  const int h = (int)(t / pairs % H);
+  const int64_t n = t / ((int64_t)pairs * H);
+  float u = 0.f, v = 0.f;
+  if (i < half) {
+    const T* s = src + n * src_row + (int64_t)h * src_head + 2 * i;
+    const float a = to_f(s[0]), b = to_f(s[1]);
+    const float c = cos_sin[positions[n] * half + i];
+    const float sn = cos_sin[(P + positions[n]) * half + i];
+    u = a * c - b * sn;
+    v = b * c + a * sn;
+  }
+  const float uv[2] = {u, v};
+  store_f<2>(dst + n * dst_row + (int64_t)h * dst_head + 2 * i, uv);
+}
+
+// out[n, h, :O] = W[h] x[n, h, :K] (* sigmoid(gate[n, h])) on the matrix cores.
+// A wave owns 64 outputs x 16*TT tokens; both operands are K-contiguous, so the
+// fragments load straight from global memory (weights are small enough to stay
+// in L2, tokens of one head in L1).  A = weights, B = tokens: a lane ends up
+// with 4 consecutive outputs of one token.
+template <int TT>
+__global__ __launch_bounds__(256) void head_linear_mfma_kernel(
+    bf16_t* __restrict__ out, const bf16_t* __restrict__ x,
+    const bf16_t* __restrict__ w, const bf16_t* __restrict__ gate, const int N,
+    const int O, const int K, const int64_t x_row, const int x_head,
+    const int64_t out_row, const int out_head, const int64_t gate_row) {
+  const int h = blockIdx.z;
+  const int lane = threadIdx.x & 63;
+  const int c = lane & 15, g = lane >> 4;
+  const int o0 = (blockIdx.y * (blockDim.x >> 6) + (threadIdx.x >> 6)) * 64;
+  if (o0 >= O) return;
+  const int n0 = blockIdx.x * (16 * TT);
+  const bf16_t* wp[4];
+  const bf16_t* xp[TT];
+#pragma unroll
+  for (int i = 0; i < 4; ++i)
+    wp[i] = w + ((int64_t)h * O + min(o0 + i * 16 + c, O - 1)) * K + g * 8;
+#pragma unroll
+  for (int t = 0; t < TT; ++t)
+    xp[t] = x + (int64_t)min(n0 + t * 16 + c, N - 1) * x_row + (int64_t)h * x_head + g * 8;
+  f32x4_v acc[4][TT] = {};
+  for (int k = 0; k < K; k += 32) {
+    bf16x8_v a[4], b[TT];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) a[i] = *(const bf16x8_v*)(wp[i] + k);
+#pragma unroll
+    for (int t = 0; t < TT; ++t) b[t] = *(const bf16x8_v*)(xp[t] + k);
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+#pragma unroll
+      for (int t = 0; t < TT; ++t)
+        acc[i][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a[i], b[t], acc[i][t], 0, 0, 0);
+  }
+#pragma unroll
+  for (int t = 0; t < TT; ++t) {
+    const int n = n0 + t * 16 + c;
+    if (n >= N) continue;
+    const float s = gate ? sigmoid_f(bf2f(gate[n * gate_row + h])) : 1.f;
+    bf16_t* dst = out + n * out_row + (int64_t)h * out_head;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int o = o0 + i * 16 + g * 4;  // O is a multiple of 32
+      if (o >= O) continue;
+      const float v[4] = {acc[i][t][0] * s, acc[i][t][1] * s, acc[i][t][2] * s,
+                          acc[i][t][3] * s};
+      store_f<4>(dst + o, v);
+    }
+  }
+}
+
+// fp32 twin: a thread per output, 4 tokens per block in flight.
+__global__ __launch_bounds__(256) void head_linear_f32_kernel(
+    float* __restrict__ out, const float* __restrict__ x, const float* __restrict__ w,
+    const float* __restrict__ gate, const int N, const int O, const int K,
+    const int64_t x_row, const int x_head, const int64_t out_row,
+    const int out_head, const int64_t gate_row) {
+  const int h = blockIdx.z;
+  const int o = blockIdx.y * 64 + (threadIdx.x & 63);
+  const int n = blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (o >= O || n >= N) return;
+  const float* wr = w + ((int64_t)h * O + o) * K;
+  const float* xr = x + n * x_row + (int64_t)h * x_head;
+  float acc = 0.f;
+  for (int k = 0; k < K; k += 4) {
+    float a[4], b[4];
+    load_f<4>(a, wr + k);
+    load_f<4>(b, xr + k);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) acc += a[j] * b[j];
+  }
+  if (gate) acc *= sigmoid_f(gate[n * gate_row + h]);
+  out[n * out_row + (int64_t)h * out_head + o] = acc;
+}
+
+extern "C" {
+
+void launch_latent_cache_write(bool bf16, void* cache, const void* kv, const void* norm_w,
+                               const int64_t* positions, const int64_t* slots,
+                               const float* cos_sin, float eps, int N, int kv_rank,
+                               int rot_dim, int rank, int row, int64_t kv_stride,
+                               int64_t P, hipStream_t stream) {
+  const int grid = (N + 3) / 4;
+  if (bf16)
+    latent_cache_write_kernel<bf16_t><<<grid, 256, 0, stream>>>(
+        (bf16_t*)cache, (const bf16_t*)kv, (const bf16_t*)norm_w, positions, slots,
+        cos_sin, eps, N, kv_rank, rot_dim, rank, row, kv_stride, P);
+  else
+    latent_cache_write_kernel<float><<<grid, 256, 0, stream>>>(
+        (float*)cache, (const float*)kv, (const float*)norm_w, positions, slots,
+        cos_sin, eps, N, kv_rank, rot_dim, rank, row, kv_stride, P);
+}
+
+void launch_rotate_interleaved(bool bf16, void* dst, const void* src,
+                               const int64_t* positions, const float* cos_sin, int N,
+                               int H, int rot_dim, int rot, int64_t dst_row,
+                               int64_t src_row, int src_head, int dst_head, int64_t P,
+                               hipStream_t stream) {
+  const int64_t total = (int64_t)N * H * (rot / 2);
+  const int grid = (int)((total + 255) / 256);
+  if (bf16)
+    rotate_interleaved_kernel<bf16_t><<<grid, 256, 0, stream>>>(
+        (bf16_t*)dst, (const bf16_t*)src, positions, cos_sin, total, H, rot_dim, rot,
+        dst_row, src_row, src_head, dst_head, P);
+  else
+    rotate_interleaved_kernel<float><<<grid, 256, 0, stream>>>(
+        (float*)dst, (const float*)src, positions, cos_sin, total, H, rot_dim, rot,
+        dst_row, src_row, src_head, dst_head, P);
+}
+
+void launch_head_linear(bool bf16, void* out, const void* x, const void* w,
+                        const void* gate, int N, int H, int O, int K, int64_t x_row,
+                        int x_head, int64_t out_row, int out_head, int64_t gate_row,
+                        hipStream_t stream) {
+  if (!bf16) {
+    dim3 grid((N + 3) / 4, (O + 63) / 64, H);
+    head_linear_f32_kernel<<<grid, 256, 0, stream>>>(
+        (float*)out, (const float*)x, (const float*)w, (const float*)gate, N, O, K,
+        x_row, x_head, out_row, out_head, gate_row);
+    return;
+  }
+  const int tiles = (O + 63) / 64;
+  const int waves = tiles < 4 ? tiles : 4;
+  const int tt = N > 2048 ? 4 : N > 16 ? 2 : 1;
+  dim3 grid((N + 16 * tt - 1) / (16 * tt), (tiles + waves - 1) / waves, H);
+  auto k = tt == 4 ? head_linear_mfma_kernel<4>
+                   : tt == 2 ? head_linear_mfma_kernel<2> : head_linear_mfma_kernel<1>;
+  k<<<grid, 64 * waves, 0, stream>>>(
+      (bf16_t*)out, (const bf16_t*)x, (const bf16_t*)w, (const bf16_t*)gate, N, O, K,
+      x_row, x_head, out_row, out_head, gate_row);
+}
+
+}  // extern "C"

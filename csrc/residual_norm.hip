@@ -1,0 +1,180 @@
+// Norms around an fp32 residual stream (gfx950).
+//
+// residual_norm is one pass over a row: optionally add y, or rmsnorm(y) * w_y,
+// to the residual, then emit layernorm(x) * w_x or x itself for the next GEMM.
+// The row lives in LDS between the reductions (each thread re-reads only what
+// it wrote, so the row itself needs no barrier).  Mean first, then the squared
+// deviations: no cancellation.
+#include "common_t.h"
+
+template <typename T, int V>
+__global__ __launch_bounds__(256) void residual_norm_kernel(
+    float* __restrict__ x,            // [n, w], updated if y
+    const T* __restrict__ y,          // [n, w] or null
+    const T* __restrict__ y_norm,     // [w] or null: plain add
+    const T* __restrict__ x_norm,     // [w] or null: out = x
+    T* __restrict__ out,              // [n, w] rows out_stride apart, or null
+    const float eps, const int w, const int64_t out_stride) {
+  extern __shared__ float row[];
+  __shared__ float scratch[3][4];
+  float* xr = x + (int64_t)blockIdx.x * w;
+  const int step = blockDim.x * V;
+  const int i0 = threadIdx.x * V;
+
+  float y_scale = 1.f;
+  if (y && y_norm) {
+    const T* yr = y + (int64_t)blockIdx.x * w;
+    float ss = 0.f;
+    for (int i = i0; i < w; i += step) {
+      float t[V];
+      load_f<V>(t, yr + i);
+#pragma unroll
+      for (int k = 0; k < V; ++k) {
+        ss += t[k] * t[k];
+        row[i + k] = t[k];
+      }
+    }
+    y_scale = rsqrtf(block_sum(ss, scratch[0]) / w + eps);
+  }
+  float sum = 0.f;
+  for (int i = i0; i < w; i += step) {
+    float t[V];
+    load_f<V>(t, xr + i);
+    if (y) {
+      float d[V];
+      if (y_norm) {
+        load_f<V>(d, y_norm + i);
+#pragma unroll
+        for (int k = 0; k < V; ++k) d[k] *= row[i + k] * y_scale;
+      } else {
+        load_f<V>(d, y + (int64_t)blockIdx.x * w + i);
+      }
+#pragma unroll
+      for (int k = 0; k < V; ++k) t[k] += d[k];
+      store_f<V>(xr + i, t);
+    }
+#pragma unroll
+    for (int k = 0; k < V; ++k) {
+      sum += t[k];
+      row[i + k] = t[k];
+    }
+  }
+  if (!out) return;
+  T* orow = out + (int64_t)blockIdx.x * out_stride;
+  float mean = 0.f, inv = 1.f;
+  if (x_norm) {
+    mean = block_sum(sum, scratch[1]) / w;
+    float ss = 0.f;
+    for (int i = i0; i < w; i += step)
+#pragma unroll
+      for (int k = 0; k < V; ++k) {
+        const float c = row[i + k] - mean;
+        ss += c * c;
+      }
+    inv = rsqrtf(block_sum(ss, scratch[2]) / w + eps);
+  }
+  for (int i = i0; i < w; i += step) {
+    float t[V];
+#pragma unroll
+    for (int k = 0; k < V; ++k) t[k] = (row[i + k] - mean) * inv;
+    if (x_norm) {
+      float g[V];
+      load_f<V>(g, x_norm + i);
+#pragma unroll
+      for (int k = 0; k < V; ++k) t[k] *= g[k];
+    }
+    store_f<V>(orow + i, t);
+  }
+}
+
+// RMS norm over the first n of k columns of strided rows; one wave per row.
+template <typename T, int V>
+__global__ __launch_bounds__(256) void rmsnorm_rows_kernel(
+    T* __restrict__ out, const T* __restrict__ x, const T* __restrict__ weight,
+    const float eps, const int rows, const int k, const int n,
+    const int64_t x_stride) {
+  const int r = blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (r >= rows) return;
+  const T* xr = x + r * x_stride;
+  const int lane = threadIdx.x & 63;
+  float ss = 0.f;
+  for (int i = lane * V; i < k; i += 64 * V) {
+    float t[V];
+    load_f<V>(t, xr + i);  // columns n.. are zero
+#pragma unroll
+    for (int j = 0; j < V; ++j) ss += t[j] * t[j];
+  }
+  const float inv = rsqrtf(wave_sum(ss) / n + eps);
+  for (int i = lane * V; i < k; i += 64 * V) {
+    float t[V], g[V];
+    load_f<V>(t, xr + i);
+    load_f<V>(g, weight + i);
+#pragma unroll
+    for (int j = 0; j < V; ++j) t[j] *= inv * g[j];
+    store_f<V>(out + (int64_t)r * k + i, t);
+  }
+}
+
+template <typename T, int V>
+__global__ __launch_bounds__(256) void add_to_residual_kernel(
+    float* __restrict__ x, const T* __restrict__ y, T* __restrict__ out,
+    const int64_t n) {
+  const int64_t step = (int64_t)gridDim.x * blockDim.x * V;
+  for (int64_t i = ((int64_t)blockIdx.x * blockDim.x + threadIdx.x) * V; i < n; i += step) {
+    float a[V], b[V];
+    load_f<V>(a, x + i);
+    load_f<V>(b, y + i);
+#pragma unroll
+    for (int k = 0; k < V; ++k) a[k] += b[k];
+    store_f<V>(x + i, a);
+    if (out) store_f<V>(out + i, a);
+  }
+}
+
+template <typename T>
+static void residual_norm_t(float* x, const void* y, const void* y_norm,
+                            const void* x_norm, void* out, float eps, int n,
+                            int w, int64_t out_stride, hipStream_t stream) {
+  const bool vec = w % 4 == 0 && out_stride % 4 == 0;
+  const int threads = w >= 1024 ? 256 : w >= 512 ? 128 : 64;
+  auto k = vec ? residual_norm_kernel<T, 4> : residual_norm_kernel<T, 1>;
+  k<<<n, threads, w * sizeof(float), stream>>>(
+      x, (const T*)y, (const T*)y_norm, (const T*)x_norm, (T*)out, eps, w, out_stride);
+}
+
+extern "C" {
+
+void launch_residual_norm(bool bf16, float* x, const void* y, const void* y_norm,
+                          const void* x_norm, void* out, float eps, int n, int w,
+                          int64_t out_stride, hipStream_t stream) {
+  (bf16 ? residual_norm_t<bf16_t> : residual_norm_t<float>)(
+      x, y, y_norm, x_norm, out, eps, n, w, out_stride, stream);
+}
+
+void launch_rmsnorm_rows(bool bf16, void* out, const void* x, const void* weight,
+                         float eps, int rows, int k, int n, int64_t x_stride,
+                         hipStream_t stream) {
+  const int grid = (rows + 3) / 4;
+  if (bf16)
+    rmsnorm_rows_kernel<bf16_t, 8><<<grid, 256, 0, stream>>>(
+        (bf16_t*)out, (const bf16_t*)x, (const bf16_t*)weight, eps, rows, k, n, x_stride);
+  else
+    rmsnorm_rows_kernel<float, 4><<<grid, 256, 0, stream>>>(
+        (float*)out, (const float*)x, (const float*)weight, eps, rows, k, n, x_stride);
+}
+
+void launch_add_to_residual(bool bf16, float* x, const void* y, void* out,
+                            int64_t n, hipStream_t stream) {
+  const int v = n % 4 == 0 ? 4 : 1;
+  const int64_t want = (n / v + 255) / 256;
+  const int grid = (int)(want < 4096 ? want : 4096);
+  if (bf16) {
+    auto k = v == 4 ? add_to_residual_kernel<bf16_t, 4> : add_to_residual_kernel<bf16_t, 1>;
+    k<<<grid, 256, 0, stream>>>(x, (const bf16_t*)y, (bf16_t*)out, n);
+  } else {
+    auto k = v == 4 ? add_to_residual_kernel<float, 4> : add_to_residual_kernel<float, 1>;
+    k<<<grid, 256, 0, stream>>>(x, (const float*)y, (float*)out, n);
+  }
+}
+
+}  // extern "C"

@@ -1,0 +1,289 @@
+"""Mechanism ops against their equations in double precision: fp32-residual
+norms, gated activations, interleaved rotation, the latent cache row and
+attention over it.  Runs on the CPU ops and, marked gpu, on the HIP kernels."""
+import pytest
+import torch
+
+import fetolix_oracle as oracle
+from agentcontrolplane_amd import ops
+from agentcontrolplane_amd.engine.batch import FlatBatch, SeqMeta
+from agentcontrolplane_amd.ops.reference import build_cos_sin
+
+GPU = pytest.param("cuda", marks=pytest.mark.gpu)
+BF16, F32 = torch.bfloat16, torch.float32
+
+
+@pytest.fixture(params=["cpu", GPU])
+def device(request):
+    if request.param == "cuda" and not torch.cuda.is_available():
+        pytest.skip("needs a GPU")
+    return request.param
+
+
+@pytest.fixture(params=[BF16, F32], ids=["bf16", "f32"])
+def dtype(request):
+    return request.param
+
+
+def close(got, want, dtype, scale=1.0):
+    tol = (2e-2 if dtype == BF16 else 3e-5) * scale
+    err = (got.double().cpu() - want.double().cpu()).abs().max().item()
+    assert err <= tol * max(1.0, want.abs().max().item()), err
+
+
+def rand(*shape, dtype, device, seed=0, scale=1.0):
+    g = torch.Generator().manual_seed(seed)
+    return (torch.randn(*shape, generator=g) * scale).to(dtype).to(device)
+
+
+# ------------------------------------------------------------------- norms
+
+
+@pytest.mark.parametrize("n,w", [(1, 48), (5, 250), (3, 1027), (9, 4096)])
+def test_layernorm(device, dtype, n, w):
+    x = rand(n, w, dtype=F32, device=device) + 3.0
+    wt = rand(w, dtype=dtype, device=device, seed=1)
+    got = ops.layernorm(x, wt, 1e-3, dtype)
+    assert got.dtype == dtype
+    close(got, oracle.layer_norm(x.double().cpu(), wt.double().cpu(), 1e-3), dtype)
+
+
+@pytest.mark.parametrize("n,w", [(1, 48), (7, 251), (4, 2048)])
+@pytest.mark.parametrize("y_norm,x_norm", [(0, 0), (1, 0), (0, 1), (1, 1)])
+def test_residual_norm(device, dtype, n, w, y_norm, x_norm):
+    """x += y or rms(y) * wy; then layernorm(x) * wx, or x, into a strided view."""
+    x = rand(n, w, dtype=F32, device=device)
+    y = rand(n, w, dtype=dtype, device=device, seed=1, scale=0.01)
+    wy = rand(w, dtype=dtype, device=device, seed=2) if y_norm else None
+    wx = rand(w, dtype=dtype, device=device, seed=3) if x_norm else None
+    eps = 1e-4  # the size of mean(y^2): eps inside the root shows
+    xd, yd = x.double().cpu(), y.double().cpu()
+    want = xd + (oracle.rms(yd, eps) * wy.double().cpu() if y_norm else yd)
+    wide = torch.zeros(n, 2 * w, dtype=dtype, device=device)
+    ops.residual_norm(x, y, eps, wy, wx, wide[:, w:])
+    close(x, want, F32)
+    out = oracle.layer_norm(want, wx.double().cpu(), eps) if x_norm else want
+    close(wide[:, w:], out, dtype)
+    assert not wide[:, :w].any()
+    before = x.clone()
+    ops.residual_norm(x, y, eps)  # no output: the residual only
+    close(x, before.double().cpu() + yd, F32)
+
+
+def test_add_to_residual_and_rmsnorm_rows(device, dtype):
+    x, y = rand(6, 131, dtype=F32, device=device), rand(6, 131, dtype=dtype, device=device, seed=1)
+    want = x.double().cpu() + y.double().cpu()
+    close(ops.add_to_residual(x, y, dtype), want, dtype)
+    close(x, want, F32)
+    # 20 columns padded to 32, read out of a wider buffer
+    wide = rand(6, 64, dtype=dtype, device=device, seed=2, scale=0.02)
+    wide[:, 20:32] = 0
+    w = rand(32, dtype=dtype, device=device, seed=3)
+    w[20:] = 0
+    got = ops.rmsnorm_rows(wide[:, :32], w, 1e-4, 20)
+    want = oracle.rms(wide[:, :20].double().cpu(), 1e-4) * w[:20].double().cpu()
+    close(got[:, :20], want, dtype)
+    assert not got[:, 20:].any()
+
+
+# ------------------------------------------------------- gated activations
+
+
+def test_clamped_glu(device, dtype):
+    """Values inside and outside the limits; gate is capped above only."""
+    inter, limit = 24, 1.25
+    wide = rand(33, 3 * inter, dtype=dtype, device=device, scale=2.0)
+    out = torch.empty(33, 2 * inter, dtype=dtype, device=device)
+    ops.clamped_glu(wide[:, inter:], limit, 1.702, 1.0, out[:, inter:])
+    W = {"gate": torch.eye(2 * inter).double()[:inter],
+         "up": torch.eye(2 * inter).double()[inter:], "down": torch.eye(inter).double()}
+    want = oracle.clamped_glu(wide[:, inter:].double().cpu(), W, "", limit)
+    close(out[:, inter:], want, dtype)
+    ops.clamped_glu(wide[:, inter:], limit, 0.5, 0.0, out[:, inter:])  # other constants
+    g = wide[:, inter : 2 * inter].double().cpu().clamp(max=limit)
+    u = wide[:, 2 * inter :].double().cpu().clamp(-limit, limit)
+    close(out[:, inter:], g * torch.sigmoid(0.5 * g) * u, dtype)
+
+
+def test_gelu_gate(device, dtype):
+    s = rand(19, 7, dtype=dtype, device=device, scale=2.0)
+    table = rand(30, 21, dtype=dtype, device=device, seed=1)
+    tok = torch.arange(19, device=device) * 3 % 30
+    want = oracle.gelu_tanh(s.double().cpu()) * table[tok][:, 7:14].double().cpu()
+    close(ops.gelu_gate_(s, tok, table, 7), want, dtype)
+
+
+# -------------------------------------------------------------- per token
+
+
+@pytest.mark.parametrize("kv_rank,rot_dim", [(24, 8), (100, 34), (512, 64)])
+def test_latent_cache_write(device, dtype, kv_rank, rot_dim):
+    n, base, eps = 11, 3e4, 1e-2
+    rank = ops.latent_rank(kv_rank)
+    row = rank + 64
+    wide = rand(n, kv_rank + rot_dim + 3, dtype=dtype, device=device, scale=0.1)
+    kv = wide[:, 3:]
+    w = rand(kv_rank, dtype=dtype, device=device, seed=1)
+    pos = torch.tensor([0, 1, 2, 7, 300, 301, 999, 5, 64, 63, 65], device=device)
+    slots = torch.randperm(32, generator=torch.Generator().manual_seed(1))[:n].to(device)
+    cache = torch.full((8, 4, row), 7.0, dtype=dtype, device=device)
+    cos_sin = build_cos_sin(1000, rot_dim, base, device, exact=True)
+    ops.latent_cache_write(kv, w, eps, kv_rank, rot_dim, rank, pos, slots, cos_sin, cache)
+    got = cache.view(32, row)[slots].cpu()
+    kd = kv.double().cpu()
+    close(got[:, :kv_rank], oracle.rms(kd[:, :kv_rank], eps) * w.double().cpu(), dtype)
+    close(got[:, rank : rank + rot_dim],
+          oracle.rotate_pairs(kd[:, kv_rank:], pos.cpu(), base), dtype)
+    assert not got[:, kv_rank:rank].any() and not got[:, rank + rot_dim :].any()
+    rest = torch.ones(32, dtype=torch.bool)
+    rest[slots.cpu()] = False
+    assert (cache.view(32, row).cpu()[rest] == 7.0).all()
+
+
+@pytest.mark.parametrize("n", [1, 17, 70, 2100])
+@pytest.mark.parametrize("O,K", [(32, 32), (96, 64), (512, 128), (128, 512)])
+def test_head_linear(device, dtype, n, O, K):
+    if n > 100 and (device == "cpu" or dtype == F32):
+        n = 100
+    H = 3
+    x = rand(n, H, K + 32, dtype=dtype, device=device)[:, :, 32:]
+    w = rand(H, O, K, dtype=dtype, device=device, seed=1, scale=K ** -0.5)
+    gate = rand(n, H + 2, dtype=dtype, device=device, seed=2)[:, 1 : H + 1]
+    out = torch.zeros(n, H, O + 32, dtype=dtype, device=device)
+    want = torch.stack(
+        [x[:, h].double().cpu() @ w[h].double().cpu().T for h in range(H)], 1
+    )
+    ops.head_linear(x, w, out[:, :, 32:])
+    close(out[:, :, 32:], want, dtype)
+    ops.head_linear(x, w, out[:, :, 32:], gate)
+    close(out[:, :, 32:], want * torch.sigmoid(gate.double().cpu()).unsqueeze(-1), dtype)
+    assert not out[:, :, :32].any()
+
+
+def test_absorb_query(device, dtype):
+    n, H, d, rot_dim, base = 9, 5, 32, 12, 1e4
+    q = rand(n, H, d + 64, dtype=dtype, device=device)
+    q[:, :, d + rot_dim :] = 0
+    w = rand(H, 128, d, dtype=dtype, device=device, seed=1, scale=d ** -0.5)
+    pos = torch.arange(n, device=device) * 37
+    got = ops.absorb_query(q, w, pos, build_cos_sin(400, rot_dim, base, device, exact=True),
+                           d, rot_dim)
+    want = torch.stack([q[:, h, :d].double().cpu() @ w[h].double().cpu().T for h in range(H)], 1)
+    close(got[:, :, :128], want, dtype)
+    close(got[:, :, 128 : 128 + rot_dim],
+          oracle.rotate_pairs(q[:, :, d : d + rot_dim].double().cpu(), pos.cpu(), base), dtype)
+    assert not got[:, :, 128 + rot_dim :].any()
+
+
+# -------------------------------------------------------------- attention
+
+
+def make_batch(chunks, block, device, seed=0, spare=3):
+    """chunks: [(ctx, new)].  Chunks of one token after cached ones are decode
+    rows, as in the engine.  Pages are handed out in random order."""
+    chunks = [c for c in chunks if c[1] > 1 or c[0] == 0] + [
+        c for c in chunks if c[1] == 1 and c[0] > 0
+    ]
+    need = [-(-(ctx + new) // block) for ctx, new in chunks]
+    order = torch.randperm(
+        sum(need) + spare, generator=torch.Generator().manual_seed(seed)
+    ).tolist()
+    prefills, tables, lens = [], [], []
+    for i, ((ctx, new), k) in enumerate(zip(chunks, need)):
+        pages, order = order[:k], order[k:]
+        if new == 1 and ctx > 0:
+            tables.append(pages)
+            lens.append(ctx + 1)
+        else:
+            prefills.append(SeqMeta(i, new, ctx + new, ctx, pages, True))
+    width = max(map(len, tables), default=0)
+    t = lambda x: torch.tensor(x, device=device)  # noqa: E731
+    batch = FlatBatch(
+        token_ids=torch.zeros(sum(n for _, n in chunks), dtype=torch.long, device=device),
+        positions=t([ctx + k for ctx, new in chunks for k in range(new)]),
+        slot_mapping=t([0]), prefills=prefills,
+        num_prefill_tokens=sum(m.query_len for m in prefills),
+        decode_seq_ids=list(range(len(tables))),
+        decode_block_tables=t([p + [0] * (width - len(p)) for p in tables]) if tables else None,
+        decode_seq_lens=t(lens) if lens else None,
+        logit_rows=t([0]), sample_seq_ids=[],
+    )
+    return batch, chunks, [m.block_table for m in prefills] + tables, sum(need) + spare
+
+
+def attend(q, rows, ctx, rank, scale, window):
+    """q [L, H, row], rows [S, row] in double -> [L, H, rank]."""
+    L, S = q.shape[0], rows.shape[0]
+    ok = oracle.visible(S, window)[ctx : ctx + L]
+    s = torch.einsum("lhd,sd->lhs", q, rows) * scale
+    p = torch.softmax(s.masked_fill(~ok.unsqueeze(1), float("-inf")), -1)
+    return torch.einsum("lhs,sr->lhr", p, rows[:, :rank])
+
+
+SHAPES = [
+    # heads, kv_rank, window, block, chunks
+    (3, 24, None, 4, [(0, 5), (0, 1), (9, 2), (130, 1), (63, 1)]),
+    (4, 64, 19, 16, [(0, 40), (200, 2), (17, 3), (18, 1), (19, 1), (500, 1), (1, 1)]),
+    (16, 128, None, 16, [(0, 70), (300, 33), (64, 1), (1000, 1)]),
+    (20, 200, 64, 16, [(0, 130), (63, 1), (64, 1), (65, 1), (700, 5)]),
+    (33, 350, 100, 16, [(0, 9), (350, 1), (99, 1), (100, 1)]),
+    (32, 512, None, 16, [(0, 150), (90, 1), (2000, 1), (777, 2)]),
+    (128, 512, 300, 16, [(0, 3), (900, 1), (1200, 1)]),
+    (2, 600, 50, 16, [(0, 60), (70, 1), (70, 2)]),
+]
+
+
+@pytest.mark.parametrize("H,kv_rank,window,block,chunks", SHAPES)
+def test_latent_attention(device, dtype, H, kv_rank, window, block, chunks):
+    rank = ops.latent_rank(kv_rank)
+    row = rank + 64
+    batch, chunks, tables, pages = make_batch(chunks, block, device)
+    # pages outside a sequence hold NaN: reading one shows
+    cache = torch.full((pages, block, row), float("nan"), dtype=dtype)
+    kv = []
+    for i, ((ctx, new), table) in enumerate(zip(chunks, tables)):
+        r = rand(ctx + new, row, dtype=dtype, device="cpu", seed=10 + i)
+        r[:, kv_rank:rank] = 0
+        r[:, rank + 8 :] = 0
+        kv.append(r.double())
+        for p, page in enumerate(table):
+            part = r[p * block : (p + 1) * block]
+            cache[page, : len(part)] = part
+    cache = cache.to(device)
+    q = rand(batch.num_tokens, H, row, dtype=dtype, device=device, seed=5)
+    scale = 0.3 * kv_rank ** -0.5
+    got = ops.latent_attention(q, cache, batch, rank, scale, window).cpu()
+    at = 0
+    for (ctx, new), rows in zip(chunks, kv):
+        want = attend(q[at : at + new].double().cpu(), rows, ctx, rank, scale, window)
+        close(got[at : at + new], want, dtype)
+        at += new
+
+
+@pytest.mark.parametrize("where", ["first", "far", "oldest_visible", "just_hidden", "self"])
+@pytest.mark.parametrize("decode", [True, False])
+def test_standout_key(device, dtype, where, decode):
+    """One key scores far above the rest: attention must return its latent
+    when it is visible, and never when it has just left the window."""
+    H, rank, window, S, block = 4, 64, 40, 171, 16
+    row = rank + 64
+    i = S - 1
+    hit = {"first": 0, "far": 77, "oldest_visible": i - window + 1,
+           "just_hidden": i - window, "self": i}[where]
+    win = None if where in ("first", "far") else window
+    batch, chunks, tables, pages = make_batch([(i, 1)] if decode else [(i - 2, 3)], block, device)
+    rows = rand(S, row, dtype=dtype, device="cpu", seed=3, scale=0.05)
+    rows[:, rank:] = 0
+    rows[hit, rank] = 8.0
+    cache = torch.zeros(pages, block, row, dtype=dtype)
+    for p, page in enumerate(tables[0]):
+        cache[page, : len(rows[p * block : (p + 1) * block])] = rows[p * block : (p + 1) * block]
+    q = torch.zeros(batch.num_tokens, H, row, dtype=dtype)
+    q[:, :, rank] = 8.0
+    got = ops.latent_attention(q.to(device), cache.to(device), batch, rank, 1.0, win)[-1]
+    if where == "just_hidden":
+        want = rows[i - window + 1 :, :rank].double().mean(0)
+        assert (rows[hit, :rank].double() - want).abs().max() > 0.05
+    else:
+        want = rows[hit, :rank].double()
+    close(got, want.expand(H, rank), dtype, scale=0.2)
