@@ -8,7 +8,7 @@ tokens (one per running sequence) — continuous batching.  Rows are ordered
 from __future__ import annotations
 
 import dataclasses
-from typing import List, Optional
+from typing import Callable, List, Optional, Sequence
 
 import torch
 
@@ -49,7 +49,7 @@ class FlatBatch:
     _tokens_gpu: Optional[torch.Tensor] = None
 
     # lazily-built device metadata, shared by every layer's kernels
-    _prefill_meta: Optional["PrefillMeta"] = None
+    _memo: Optional[dict] = None
     #: pinned-staging helper (engine/stage.py); set by the scheduler so the
     #: per-step metadata uploads are async instead of blocking hipMemcpys
     _stager: Optional[object] = None
@@ -67,17 +67,23 @@ class FlatBatch:
     def num_decode(self) -> int:
         return len(self.decode_seq_ids)
 
-    def prefill_meta(self, tile_q: int = 64, rows_per_token: int = 1) -> "PrefillMeta":
-        """Tiles of ``tile_q`` query rows; a token is ``rows_per_token`` rows
-        (its heads, for kernels that tile over both)."""
-        if self._prefill_meta is None:
-            self._prefill_meta = {}
-        key = (tile_q, rows_per_token)
-        if key not in self._prefill_meta:
-            self._prefill_meta[key] = PrefillMeta.build(
-                self.prefills, self.token_ids.device, tile_q, self._stager, rows_per_token
-            )
-        return self._prefill_meta[key]
+    def prefill_meta(self, tile_q: int = 64, **kw) -> "PrefillMeta":
+        """Metadata of the prefill kernels (options: PrefillMeta.build), built
+        once per step and combination."""
+        return self.memo(
+            ("prefill_meta", tile_q, *sorted(kw.items())),
+            lambda: PrefillMeta.build(
+                self.prefills, self.token_ids.device, tile_q, self._stager, **kw
+            ),
+        )
+
+    def memo(self, key, build: Callable):
+        """A per-step value shared by the layers."""
+        if self._memo is None:
+            self._memo = {}
+        if key not in self._memo:
+            self._memo[key] = build()
+        return self._memo[key]
 
     def decode_tables_i32(self) -> torch.Tensor:
         if self._decode_tables_i32 is None:
@@ -154,27 +160,48 @@ class PrefillMeta:
     tile_seq: torch.Tensor      # [num_tiles] int32
     tile_q0: torch.Tensor       # [num_tiles] int32
     tile_q: int
+    # keys gathered into one buffer (window given): the position of a
+    # sequence's first gathered key, its row in the buffer
+    key_first: Optional[torch.Tensor] = None
+    key_starts: Optional[torch.Tensor] = None
+    num_keys: int = 0
+    max_keys: int = 0            # of one sequence
 
     @staticmethod
     def build(prefills: List[SeqMeta], device, tile_q: int = 64,
-              stager=None, rows_per_token: int = 1) -> "PrefillMeta":
-        max_blocks = max((len(m.block_table) for m in prefills), default=1)
+              stager=None, rows_per_token: int = 1,
+              only: Optional[Sequence[int]] = None, row_base: int = 0,
+              window: Optional[int] = None) -> "PrefillMeta":
+        """Tiles of ``tile_q`` query rows; a token is ``rows_per_token`` rows
+        (its heads, for kernels that tile over both).  ``only`` picks chunks;
+        rows count from ``row_base``.  ``window`` lays out the keys the chunks
+        see one after the other."""
+        picked = [
+            (i, m) for i, m in enumerate(prefills) if only is None or i in set(only)
+        ]
+        starts = [0]
+        for m in prefills:
+            starts.append(starts[-1] + m.query_len)
+        max_blocks = max((len(m.block_table) for _, m in picked), default=1)
         tables, seq_lens, ctx_lens, row_starts = [], [], [], []
         tile_seq, tile_q0 = [], []
-        row = 0
-        for i, m in enumerate(prefills):
+        key_first, key_starts, num_keys, max_keys = [], [], 0, 0
+        for n, (i, m) in enumerate(picked):
             tables.append(m.block_table + [0] * (max_blocks - len(m.block_table)))
             seq_lens.append(m.seq_len)
             ctx_lens.append(m.ctx_len)
-            row_starts.append(row)
+            row_starts.append(starts[i] - row_base)
             for q0 in range(0, m.query_len * rows_per_token, tile_q):
-                tile_seq.append(i)
+                tile_seq.append(n)
                 tile_q0.append(q0)
-            row += m.query_len
+            if window is not None:
+                key_first.append(max(0, m.ctx_len - window + 1))
+                key_starts.append(num_keys)
+                num_keys += m.seq_len - key_first[-1]
+                max_keys = max(max_keys, m.seq_len - key_first[-1])
         if stager is not None:
-            t = lambda n, x: stager.tensor(
-                f"pm{tile_q}x{rows_per_token}_{n}", x, "int32"
-            )  # noqa: E731
+            tag = f"pm{tile_q}x{rows_per_token}o{only}b{row_base}w{window}"
+            t = lambda n, x: stager.tensor(f"{tag}_{n}", x, "int32")  # noqa: E731
         else:
             t = lambda n, x: torch.tensor(x, device=device, dtype=torch.int32)  # noqa: E731
         return PrefillMeta(
@@ -185,4 +212,8 @@ class PrefillMeta:
             tile_seq=t("ts", tile_seq),
             tile_q0=t("tq", tile_q0),
             tile_q=tile_q,
+            key_first=t("kf", key_first) if window is not None else None,
+            key_starts=t("ks", key_starts) if window is not None else None,
+            num_keys=num_keys,
+            max_keys=max_keys,
         )

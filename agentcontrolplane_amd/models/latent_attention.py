@@ -57,9 +57,9 @@ class LatentAttention:
         self.spec, self.width, self.eps = spec, width, eps
         self.heads = spec.heads // tp_world
         self.head0 = tp_rank * self.heads
-        self.d = round_up(spec.dim, 32)
+        self.d = ops.latent_head(spec.dim)
         self.rot = round_up(spec.rot_dim, 64)
-        self.v = round_up(spec.vdim, 32)
+        self.v = ops.latent_head(spec.vdim)
         self.rank = ops.latent_rank(spec.kv_rank)
         self.row = self.rank + self.rot          # cache row
         self.q_dim = self.heads * (self.d + self.rot)
@@ -181,8 +181,41 @@ class LatentAttention:
         )
         q = q.as_strided((N, H, self.d + self.rot), (q.stride(0), self.d + self.rot, 1))
         out = out.as_strided((N, H, self.v), (out.stride(0), self.v, 1))
-        qa = ops.absorb_query(
-            q, self.w_uk, batch.positions, self.cos_sin, self.d, s.rot_dim
+        expanded, row0 = batch.memo(
+            ("latent_split", s.window, self.rank, self.d, self.v), lambda: self._split(q, batch)
         )
-        latent = ops.latent_attention(qa, cache, batch, self.rank, s.scale, s.window)
-        ops.head_linear(latent, self.w_uv, out, gate)
+        if row0 < N:
+            qa = torch.empty(N - row0, H, self.rank, dtype=q.dtype, device=q.device)
+            ops.head_linear(q[row0:, :, : self.d], self.w_uk, qa)
+            latent = ops.latent_attention(
+                qa, q[row0:, :, self.d :], self.cos_sin, s.rot_dim, cache, batch, s.scale,
+                s.window, row0, expanded,
+            )
+            ops.head_linear(latent, self.w_uv, out[row0:], None if gate is None else gate[row0:])
+        if expanded:  # after: the rows above may include expanded chunks'
+            ops.latent_expanded_prefill(
+                q, self.w_ukv, gate, self.cos_sin, s.rot_dim, cache, batch, expanded,
+                self.rank, s.scale, s.window, out,
+            )
+
+    def _split(self, q: torch.Tensor, batch: FlatBatch) -> Tuple[Tuple[int, ...], int]:
+        """The prefill chunks to run expanded, by products per head and chunk,
+        and the first row that is not in one of the leading ones."""
+        if not batch.prefills or not ops.can_expand(q, self.d, self.v, self.rot):
+            return (), 0
+        window = self.spec.window or 1 << 30
+        per_expansion = self.rank * (self.d + self.v)
+        chunks = []
+        for i, m in enumerate(batch.prefills):
+            seen = m.query_len * min(window, m.ctx_len + (m.query_len + 1) // 2)
+            keys = m.seq_len - max(0, m.ctx_len - window + 1)
+            expanded = keys * per_expansion + seen * (self.d + self.rot + self.v)
+            absorbed = m.query_len * per_expansion + seen * (2 * self.rank + self.rot)
+            if expanded <= absorbed:
+                chunks.append(i)
+        row0 = 0
+        for i, m in enumerate(batch.prefills):
+            if i not in chunks:
+                break
+            row0 += m.query_len
+        return tuple(chunks), row0

@@ -156,6 +156,18 @@ def latent_rank(kv_rank: int) -> int:
     return -(-kv_rank // 64) * 64
 
 
+#: query/key and value head sizes of the expanded prefill kernel
+LATENT_HEADS = (64, 128, 256)
+
+
+def latent_head(dim: int) -> int:
+    """The padded per-head size for dim."""
+    for n in LATENT_HEADS:
+        if dim <= n:
+            return n
+    return -(-dim // 64) * 64
+
+
 def latent_cache_write(kv, norm_w, eps: float, kv_rank: int, rot_dim: int, rank: int,
                        positions, slot_mapping, cos_sin, cache):
     """kv [N, kv_rank + rot_dim] (row-strided): RMS-norm the latent, rotate the
@@ -172,17 +184,31 @@ def head_linear(x, w, out, gate=None):
     return _impl(x).head_linear(x, w, out, gate)
 
 
-def absorb_query(q, w_uk, positions, cos_sin, d: int, rot_dim: int):
-    """q [N, H, d + rot] (row-strided) -> [N, H, rank + rot]: w_uk[h] @ q[:d],
-    then the rotated rest."""
-    return _impl(q).absorb_query(q, w_uk, positions, cos_sin, d, rot_dim)
+def latent_attention(q, q_rot, cos_sin, rot_dim: int, cache, batch, scale: float, window,
+                     row0: int = 0, skip=()):
+    """Softmax attention of absorbed queries over cached rows, for a FlatBatch's
+    token rows row0.. except the prefill chunks in ``skip`` (left undefined).
+    q [N, H, rank] and its part q_rot [N, H, rot] still to be rotated by the
+    row's position; values are a cache row's first ``rank`` dims.
+    window = visible keys per query, None = all.  Returns [N, H, rank]."""
+    return _impl(q).latent_attention(
+        q, q_rot, cos_sin, rot_dim, cache, batch, scale, window, row0, skip
+    )
 
 
-def latent_attention(q, cache, batch, rank: int, scale: float, window):
-    """Softmax attention of absorbed queries [N, H, row] (all of a FlatBatch)
-    over cached rows; values are a row's first ``rank`` dims: [N, H, rank].
-    window = visible keys per query, None = all."""
-    return _impl(q).latent_attention(q, cache, batch, rank, scale, window)
+def can_expand(t, d: int, v: int, rot: int) -> bool:
+    """Is there a kernel for expanded keys and values of these padded sizes?"""
+    return t.is_cuda and _hip().can_expand(t.dtype, d, v, rot)
+
+
+def latent_expanded_prefill(q, w_ukv, gate, cos_sin, rot_dim: int, cache, batch, chunks,
+                            rank: int, scale: float, window, out):
+    """The prefill chunks ``chunks`` with keys and values expanded from their
+    cached latents by w_ukv [H*d + H*v, rank]; q [N, H, d + rot] not rotated.
+    Writes the chunks' rows of out [N, H, v], gated."""
+    _hip().latent_expanded_prefill(
+        q, w_ukv, gate, cos_sin, rot_dim, cache, batch, chunks, rank, scale, window, out
+    )
 
 
 def softmax_sample(logits, temperatures, top_ks, top_ps, gen, mask=None,

@@ -165,17 +165,8 @@ def head_linear(x, w, out, gate=None):
     return out
 
 
-def absorb_query(q, w_uk, positions, cos_sin, d: int, rot_dim: int):
-    N, H, qk = q.shape
-    rank = w_uk.shape[1]
-    out = torch.empty(N, H, rank + qk - d, dtype=q.dtype, device=q.device)
-    _C.head_linear(out[:, :, :rank], q[:, :, :d], w_uk, None)
-    _C.rotate_interleaved(out[:, :, rank:], q[:, :, d:], positions, cos_sin, rot_dim)
-    return out
-
-
-def _latent_attn(out, q, cache, tables, seq_lens, prefill, tiles, mg, max_keys,
-                 scale, window, mfma):
+def _latent_attn(out, q, q_rot, cos_sin, rot_dim, cache, tables, seq_lens, prefill, tiles,
+                 mg, max_keys, scale, window, mfma):
     """One launch over prefill tiles (prefill = their metadata) or decode
     rows.  Few tiles split their keys over several workgroups."""
     n_split = 1
@@ -185,42 +176,95 @@ def _latent_attn(out, q, cache, tables, seq_lens, prefill, tiles, mg, max_keys,
     part = ml = None
     if n_split > 1:
         rows = q.shape[0] * q.shape[1]
-        part = torch.empty(n_split * rows * out.shape[2], dtype=torch.float32, device=q.device)
-        ml = torch.empty(2 * n_split * rows, dtype=torch.float32, device=q.device)
+        part = torch.empty(n_split * rows * q.shape[2], dtype=torch.float32, device=q.device)
+        # rows no tile covers (skipped chunks) must merge to nothing
+        new = torch.empty if prefill is None else torch.zeros
+        ml = new(2 * n_split * rows, dtype=torch.float32, device=q.device)
     m = prefill
     _C.latent_attn(
-        out, q, cache, tables, seq_lens,
+        out, q, q_rot, cos_sin, rot_dim, cache, tables, seq_lens,
         *((m.ctx_lens, m.row_starts, m.tile_seq, m.tile_q0) if m else (None,) * 4),
         part, ml, scale, window, mg, n_split, mfma,
     )
 
 
-def latent_attention(q, cache, batch, rank: int, scale: float, window):
+def latent_attention(q, q_rot, cos_sin, rot_dim: int, cache, batch, scale: float, window,
+                     row0: int = 0, skip=()):
     from . import LATENT_RANKS
 
-    N, H, row = q.shape
+    N, H, rank = q.shape
     out = torch.empty(N, H, rank, dtype=q.dtype, device=q.device)
     window = window or _NO_WINDOW
-    mfma = q.dtype == torch.bfloat16 and rank in LATENT_RANKS and row - rank == 64
+    mfma = q.dtype == torch.bfloat16 and rank in LATENT_RANKS and q_rot.shape[2] == 64
     most = 4 if rank <= 256 else 2
-    P = batch.num_prefill_tokens
-    if batch.prefills:
-        mg = most
-        meta = batch.prefill_meta(16 * mg if mfma else 1, H)
+    P = batch.num_prefill_tokens - row0
+    common = (cos_sin, rot_dim, cache)
+    chunks = tuple(i for i in range(len(batch.prefills)) if i not in skip)
+    if chunks:
+        meta = batch.prefill_meta(
+            16 * most if mfma else 1, rows_per_token=H, only=chunks, row_base=row0
+        )
         _latent_attn(
-            out[:P], q[:P], cache, meta.block_tables, meta.seq_lens, meta,
-            meta.tile_seq.numel(), mg, max(m.seq_len for m in batch.prefills),
+            out[:P], q[:P], q_rot[:P], *common, meta.block_tables, meta.seq_lens, meta,
+            meta.tile_seq.numel(), most, max(batch.prefills[i].seq_len for i in chunks),
             scale, window, mfma,
         )
     if batch.num_decode:
         mg = 1 if H <= 16 else 2 if H <= 32 else most
         tables = batch.decode_tables_i32()
         _latent_attn(
-            out[P:], q[P:], cache, tables, batch.decode_lens_i32(), None,
+            out[P:], q[P:], q_rot[P:], *common, tables, batch.decode_lens_i32(), None,
             batch.num_decode * -(-H // (16 * mg)), mg,
             tables.shape[1] * cache.shape[1], scale, window, mfma,
         )
     return out
+
+
+#: expanded keys and values built at a time
+_EXPAND_BYTES = 2 << 30
+
+
+def can_expand(dtype, d: int, v: int, rot: int) -> bool:
+    from . import LATENT_HEADS
+
+    return dtype == torch.bfloat16 and rot == 64 and d in LATENT_HEADS and v in LATENT_HEADS
+
+
+def _expansion_groups(batch, chunks, window: int, bytes_per_key: int):
+    groups, at = [], 0
+    for i in chunks:
+        m = batch.prefills[i]
+        keys = (m.seq_len - max(0, m.ctx_len - window + 1)) * bytes_per_key
+        if not groups or at + keys > _EXPAND_BYTES:
+            groups.append([])
+            at = 0
+        groups[-1].append(i)
+        at += keys
+    return [tuple(g) for g in groups]
+
+
+def latent_expanded_prefill(q, w_ukv, gate, cos_sin, rot_dim: int, cache, batch, chunks,
+                            rank: int, scale: float, window, out):
+    from . import linear
+
+    window = window or _NO_WINDOW
+    row = cache.shape[2]
+    groups = batch.memo(
+        ("expansion_groups", chunks, window, w_ukv.shape[0]),
+        lambda: _expansion_groups(batch, chunks, window, 2 * w_ukv.shape[0]),
+    )
+    for group in groups:
+        meta = batch.prefill_meta(128, only=group, window=window)
+        rows = torch.empty(meta.num_keys, row, dtype=q.dtype, device=q.device)
+        _C.latent_gather(
+            rows, cache, meta.block_tables, meta.seq_lens, meta.key_first, meta.key_starts,
+            meta.max_keys,
+        )
+        _C.latent_prefill(
+            out, q, linear(rows[:, :rank], w_ukv), rows[:, rank:], gate, cos_sin, rot_dim,
+            meta.seq_lens, meta.ctx_lens, meta.row_starts, meta.tile_seq, meta.tile_q0,
+            meta.key_first, meta.key_starts, scale, window,
+        )
 
 
 def softmax_sample(logits, temperatures, top_ks, top_ps, gen, mask=None,

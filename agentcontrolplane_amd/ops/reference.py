@@ -224,18 +224,6 @@ def head_linear(x, w, out, gate=None):
     return out
 
 
-def absorb_query(q, w_uk, positions, cos_sin, d: int, rot_dim: int):
-    N, H, qk = q.shape
-    rank = w_uk.shape[1]
-    out = torch.zeros(N, H, rank + qk - d, dtype=q.dtype, device=q.device)
-    head_linear(q[:, :, :d], w_uk, out[:, :, :rank])
-    out[:, :, rank : rank + rot_dim] = _rotate_interleaved(
-        q[:, :, d : d + rot_dim],
-        cos_sin[0][positions].unsqueeze(1), cos_sin[1][positions].unsqueeze(1),
-    ).to(q.dtype)
-    return out
-
-
 def _latent_attention_seq(q, cache, block_table, ctx_len: int, rank: int, scale: float, window):
     """One sequence's rows at positions ctx_len..; q [L, H, row] -> [L, H, rank]."""
     L, bs = q.shape[0], cache.shape[1]
@@ -251,13 +239,22 @@ def _latent_attention_seq(q, cache, block_table, ctx_len: int, rank: int, scale:
     return torch.matmul(probs, rows[:, :rank]).to(q.dtype)
 
 
-def latent_attention(q, cache, batch, rank: int, scale: float, window):
-    out = torch.empty(*q.shape[:2], rank, dtype=q.dtype, device=q.device)
-    row = 0
-    for m in batch.prefills:
-        out[row : row + m.query_len] = _latent_attention_seq(
-            q[row : row + m.query_len], cache, m.block_table, m.ctx_len, rank, scale, window
-        )
+def latent_attention(q, q_rot, cos_sin, rot_dim: int, cache, batch, scale: float, window,
+                     row0: int = 0, skip=()):
+    N, H, rank = q.shape
+    pos = batch.positions[row0:]
+    rot = torch.zeros(N, H, cache.shape[-1] - rank, dtype=q.dtype, device=q.device)
+    rot[:, :, :rot_dim] = _rotate_interleaved(
+        q_rot[:, :, :rot_dim], cos_sin[0][pos].unsqueeze(1), cos_sin[1][pos].unsqueeze(1)
+    ).to(q.dtype)
+    q = torch.cat([q, rot], -1)
+    out = torch.empty(N, H, rank, dtype=q.dtype, device=q.device)
+    row = -row0
+    for n, m in enumerate(batch.prefills):
+        if row >= 0 and n not in skip:
+            out[row : row + m.query_len] = _latent_attention_seq(
+                q[row : row + m.query_len], cache, m.block_table, m.ctx_len, rank, scale, window
+            )
         row += m.query_len
     for b in range(batch.num_decode):
         out[row : row + 1] = _latent_attention_seq(

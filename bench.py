@@ -168,9 +168,23 @@ def main() -> None:
         help="disable the durable WAL (default on: the reference checkpoints "
         "every transition to etcd, so the measured loop includes durability)",
     )
+    p.add_argument(
+        "--design", default=None, metavar="PRESET",
+        help="instead of the agent loop: prefill and decode throughput of this "
+        "preset beside the Llama model of equal size (utils/design_bench.py)",
+    )
     args = p.parse_args()
 
     import torch
+
+    if args.design:
+        from agentcontrolplane_amd.utils import design_bench
+
+        dev = args.device or ("cuda" if torch.cuda.is_available() else "cpu")
+        kw = {} if dev != "cpu" else {
+            "prefill": [(1, 64)], "decode": [(2, 64)], "iters": 1, "rounds": 1}
+        print(json.dumps(design_bench.run(args.design, dev, **kw)))
+        return
 
     from agentcontrolplane_amd.api.types import AGENT, LLM, MCP_SERVER, make_resource
     from agentcontrolplane_amd.engine.config import EngineConfig

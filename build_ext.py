@@ -35,6 +35,7 @@ def build(verbose: bool = False) -> str:
         os.path.join(CSRC, "gated_act.hip"),
         os.path.join(CSRC, "latent_proj.hip"),
         os.path.join(CSRC, "latent_attn.hip"),
+        os.path.join(CSRC, "latent_prefill.hip"),
         os.path.join(CSRC, "sampling.hip"),
         os.path.join(CSRC, "sampling_fullvocab.hip"),
     ]

@@ -46,11 +46,11 @@ void launch_gelu_gate(bool, void*, const int64_t*, const void*, int, int, int64_
 void launch_latent_cache_write(bool, void*, const void*, const void*, const int64_t*,
                                const int64_t*, const float*, float, int, int, int, int,
                                int, int64_t, int64_t, hipStream_t);
-void launch_rotate_interleaved(bool, void*, const void*, const int64_t*, const float*, int,
-                               int, int, int, int64_t, int64_t, int, int, int64_t,
-                               hipStream_t);
 void launch_head_linear(bool, void*, const void*, const void*, const void*, int, int, int,
                         int, int64_t, int, int64_t, int, int64_t, hipStream_t);
+bool launch_latent_prefill(const LatentPrefillArgs*, int, int, hipStream_t);
+void launch_latent_gather(void*, const void*, const int*, const int*, const int*, const int*,
+                          int, int, int, int, int, hipStream_t);
 bool launch_latent_attn(bool, bool, const LatentArgs*, int, int, int, int, hipStream_t);
 void launch_mfma_probe(float*, const void*, const void*, hipStream_t);
 void launch_gemm_bf16(void*, const void*, const void*, int, int, int, hipStream_t);
@@ -391,20 +391,6 @@ static void check_heads(const torch::Tensor& t, at::ScalarType dtype, int64_t n,
   TORCH_CHECK(t.stride(1) * t.element_size() % 16 == 0, "heads must be 16-byte aligned");
 }
 
-static void rotate_interleaved(torch::Tensor dst, torch::Tensor src, torch::Tensor positions,
-                               torch::Tensor cos_sin, int64_t rot_dim) {
-  const int n = src.size(0), h = src.size(1), rot = dst.size(2);
-  check_heads(src, src.scalar_type(), n, h);
-  check_heads(dst, src.scalar_type(), n, h);
-  check_rotation(cos_sin, positions, n, rot_dim);
-  TORCH_CHECK(rot % 2 == 0 && rot_dim <= rot && src.size(2) == rot);
-  if (n == 0) return;
-  launch_rotate_interleaved(is_bf16(src), dst.data_ptr(), src.data_ptr(),
-                            positions.data_ptr<int64_t>(), cos_sin.data_ptr<float>(), n, h,
-                            rot_dim, rot, dst.stride(0), src.stride(0), src.stride(1),
-                            dst.stride(1), cos_sin.size(1), cur_stream());
-}
-
 static void head_linear(torch::Tensor out, torch::Tensor x, torch::Tensor w,
                         OptTensor gate) {
   const int n = x.size(0), h = x.size(1), k = x.size(2), o = out.size(2);
@@ -427,9 +413,10 @@ static const int* opt_int(const OptTensor& t, int64_t n) {
   return t->data_ptr<int>();
 }
 
-// q [tokens, H, row] -> out [tokens, H, rank].  Prefill chunks bring ctx_lens,
+// q [tokens, H, rank] absorbed, q_rot [tokens, H, rot] -> out [tokens, H, rank].  Prefill chunks bring ctx_lens,
 // row_starts and tiles; decode (one token per table row) brings none of them.
-static void latent_attn(torch::Tensor out, torch::Tensor q, torch::Tensor cache,
+static void latent_attn(torch::Tensor out, torch::Tensor q, torch::Tensor q_rot,
+                        torch::Tensor cos_sin, int64_t rot_dim, torch::Tensor cache,
                         torch::Tensor tables, torch::Tensor seq_lens, OptTensor ctx_lens,
                         OptTensor row_starts, OptTensor tile_seq, OptTensor tile_r0,
                         OptTensor part, OptTensor part_ml, double scale, int64_t window,
@@ -437,8 +424,14 @@ static void latent_attn(torch::Tensor out, torch::Tensor q, torch::Tensor cache,
   CHECK_CUDA(q); CHECK_CONT(q); CHECK_CONT(out); CHECK_CUDA(cache); CHECK_CONT(cache);
   CHECK_CUDA(tables); CHECK_CONT(tables); CHECK_CUDA(seq_lens); CHECK_CONT(seq_lens);
   const bool bf16 = is_bf16(q);
-  const int tokens = q.size(0), H = q.size(1), row = q.size(2), rank = out.size(2);
-  TORCH_CHECK(out.size(0) == tokens && out.size(1) == H && rank <= row);
+  const int tokens = q.size(0), H = q.size(1), rank = q.size(2);
+  const int row = rank + q_rot.size(2);
+  TORCH_CHECK(out.sizes() == q.sizes());
+  check_heads(q_rot, q.scalar_type(), tokens, H);
+  CHECK_CUDA(cos_sin); CHECK_CONT(cos_sin);
+  TORCH_CHECK(cos_sin.scalar_type() == at::kFloat && cos_sin.dim() == 3 &&
+              cos_sin.size(0) == 2 && cos_sin.size(2) * 2 == rot_dim &&
+              rot_dim <= q_rot.size(2), "rotation table");
   TORCH_CHECK(cache.dim() == 3 && cache.size(2) == row);
   TORCH_CHECK(cache.scalar_type() == q.scalar_type() && out.scalar_type() == q.scalar_type());
   TORCH_CHECK(tables.scalar_type() == at::kInt && seq_lens.scalar_type() == at::kInt);
@@ -468,6 +461,12 @@ static void latent_attn(torch::Tensor out, torch::Tensor q, torch::Tensor cache,
     a.part_ml = (float2*)part_ml->data_ptr<float>();
   }
   a.q = q.data_ptr();
+  a.q_rot = q_rot.data_ptr();
+  a.rot_token = q_rot.stride(0);
+  a.rot_head = q_rot.stride(1);
+  a.rot_dim = (int)rot_dim;
+  a.cos_sin = cos_sin.data_ptr<float>();
+  a.positions = cos_sin.size(1);
   a.cache = cache.data_ptr();
   a.tables = tables.data_ptr<int>();
   a.seq_lens = seq_lens.data_ptr<int>();
@@ -484,6 +483,74 @@ static void latent_attn(torch::Tensor out, torch::Tensor q, torch::Tensor cache,
   a.scale = (float)scale;
   TORCH_CHECK(launch_latent_attn(bf16, mfma, &a, rank, row, (int)mg, tiles, cur_stream()),
               "latent attention: unsupported sizes rank ", rank, " row ", row);
+}
+
+// rows of out: sequence s's cached rows from position first[s] on, at starts[s]
+static void latent_gather(torch::Tensor out, torch::Tensor cache, torch::Tensor tables,
+                          torch::Tensor seq_lens, torch::Tensor first, torch::Tensor starts,
+                          int64_t max_keys) {
+  CHECK_CUDA(out); CHECK_CONT(out); CHECK_BF16(out);
+  CHECK_CUDA(cache); CHECK_CONT(cache); CHECK_BF16(cache);
+  CHECK_CUDA(tables); CHECK_CONT(tables);
+  TORCH_CHECK(tables.scalar_type() == at::kInt);
+  const int seqs = tables.size(0), row = cache.size(2);
+  TORCH_CHECK(out.size(1) == row && row % 8 == 0);
+  if (seqs == 0 || max_keys == 0) return;
+  launch_latent_gather(out.data_ptr(), cache.data_ptr(), tables.data_ptr<int>(),
+                       opt_int(seq_lens, seqs), opt_int(first, seqs), opt_int(starts, seqs),
+                       seqs, max_keys, row, tables.size(1), cache.size(1), cur_stream());
+}
+
+// q [tokens, H, d + 64], kv [keys, H * (d + v)], k_rot [keys, 64], gate [tokens, H]
+// -> out [tokens, H, v]; rows of sequences without tiles are left alone.
+static void latent_prefill(torch::Tensor out, torch::Tensor q, torch::Tensor kv,
+                           torch::Tensor k_rot, OptTensor gate, torch::Tensor cos_sin,
+                           int64_t rot_dim, torch::Tensor seq_lens, torch::Tensor ctx_lens,
+                           torch::Tensor row_starts, torch::Tensor tile_seq,
+                           torch::Tensor tile_q0, torch::Tensor key_first,
+                           torch::Tensor key_starts, double scale, int64_t window) {
+  const int tokens = q.size(0), H = q.size(1), d = q.size(2) - 64, v = out.size(2);
+  check_heads(q, at::kBFloat16, tokens, H);
+  check_heads(out, at::kBFloat16, tokens, H);
+  TORCH_CHECK(q.stride(1) == d + 64 && out.stride(1) == v, "heads must be dense");
+  const int64_t keys = kv.size(0);
+  check_rows(kv, at::kBFloat16, keys, (int64_t)H * (d + v)); check_aligned(kv);
+  check_rows(k_rot, at::kBFloat16, keys, 64); check_aligned(k_rot);
+  if (gate) check_rows(*gate, at::kBFloat16, tokens, H);
+  CHECK_CUDA(cos_sin); CHECK_CONT(cos_sin);
+  TORCH_CHECK(cos_sin.scalar_type() == at::kFloat && cos_sin.dim() == 3 &&
+              cos_sin.size(0) == 2 && cos_sin.size(2) * 2 == rot_dim && rot_dim <= 64,
+              "rotation table");
+  TORCH_CHECK(window > 0);
+  const int seqs = seq_lens.numel();
+  LatentPrefillArgs a{};
+  a.out = out.data_ptr();
+  a.q = q.data_ptr();
+  a.kv = kv.data_ptr();
+  a.k_rot = k_rot.data_ptr();
+  a.gate = gate ? gate->data_ptr() : nullptr;
+  a.cos_sin = cos_sin.data_ptr<float>();
+  a.n_tiles = tile_seq.numel();
+  a.seq_lens = opt_int(seq_lens, seqs);
+  a.ctx_lens = opt_int(ctx_lens, seqs);
+  a.row_starts = opt_int(row_starts, seqs);
+  a.tile_seq = opt_int(tile_seq, a.n_tiles);
+  a.tile_q0 = opt_int(tile_q0, a.n_tiles);
+  a.key_first = opt_int(key_first, seqs);
+  a.key_starts = opt_int(key_starts, seqs);
+  a.out_stride = out.stride(0);
+  a.q_stride = q.stride(0);
+  a.kv_stride = kv.stride(0);
+  a.rot_stride = k_rot.stride(0);
+  a.gate_stride = gate ? gate->stride(0) : 0;
+  a.positions = cos_sin.size(1);
+  a.H = H;
+  a.rot_dim = (int)rot_dim;
+  a.window = (int)window;
+  a.scale = (float)scale;
+  if (a.n_tiles == 0) return;
+  TORCH_CHECK(launch_latent_prefill(&a, d, v, cur_stream()),
+              "latent prefill: unsupported sizes d ", d, " v ", v);
 }
 
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
@@ -504,9 +571,10 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("clamped_glu", &clamped_glu);
   m.def("gelu_gate", &gelu_gate);
   m.def("latent_cache_write", &latent_cache_write);
-  m.def("rotate_interleaved", &rotate_interleaved);
   m.def("head_linear", &head_linear);
   m.def("latent_attn", &latent_attn);
+  m.def("latent_gather", &latent_gather);
+  m.def("latent_prefill", &latent_prefill);
   m.def("sample", &sample);
   m.def("sample_fullvocab", &sample_fullvocab);
 }

@@ -6,7 +6,9 @@
 DEV float to_f(bf16_t v) { return bf2f(v); }
 DEV float to_f(float v) { return v; }
 template <typename T> DEV T from_f(float v);
-template <> DEV bf16_t from_f<bf16_t>(float v) { return f2bf(v); }
+template <> DEV bf16_t from_f<bf16_t>(float v) {
+  return __builtin_bit_cast(bf16_t, (__bf16)v);  // v_cvt_pk_bf16_f32
+}
 template <> DEV float from_f<float>(float v) { return v; }
 
 // N consecutive elements <-> fp32; N * sizeof(T) is the access width and p is

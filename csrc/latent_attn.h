@@ -1,4 +1,5 @@
-// Launch arguments of the latent attention kernels (latent_attn.hip).
+// Launch arguments of the latent attention kernels: absorbed (latent_attn.hip)
+// and expanded (latent_prefill.hip).
 #pragma once
 #include <hip/hip_runtime.h>
 
@@ -6,7 +7,9 @@ struct LatentArgs {
   void* out;              // [rows, rank] when n_split == 1
   float* part;            // [n_split, rows, rank]
   float2* part_ml;        // [n_split, rows]
-  const void* q;          // [rows, row]
+  const void* q;          // [rows, rank] absorbed queries
+  const void* q_rot;      // [tokens, H, rot] not yet rotated, strides below
+  const float* cos_sin;   // [2, positions, rot_dim / 2]
   const void* cache;      // [slots, row]
   const int* tables;      // [seqs, max_blocks]
   const int* seq_lens;    // [seqs] cached tokens, this step's included
@@ -14,6 +17,23 @@ struct LatentArgs {
   const int* row_starts;  // [seqs] first token row; null: seq
   const int* tile_seq;    // [tiles]; null: decode, tile -> (seq, part of heads)
   const int* tile_r0;     // [tiles] first flattened row within the sequence
+  int64_t rot_token, rot_head, positions;
+  int rot_dim;
   int H, max_blocks, kv_block, window, n_split, rows;
+  float scale;
+};
+
+struct LatentPrefillArgs {
+  void* out;              // [tokens, H * v], rows out_stride apart
+  const void* q;          // [tokens, H, d + rot], rows q_stride apart, not rotated
+  const void* kv;         // [keys, H * d | H * v], rows kv_stride apart
+  const void* k_rot;      // [keys, rot], rows rot_stride apart
+  const void* gate;       // [tokens, H], rows gate_stride apart, or null
+  const float* cos_sin;   // [2, positions, rot_dim / 2]
+  const int *seq_lens, *ctx_lens, *row_starts, *tile_seq, *tile_q0;
+  const int* key_first;   // [seqs] position of a sequence's first key row
+  const int* key_starts;  // [seqs] that row
+  int64_t out_stride, q_stride, kv_stride, rot_stride, gate_stride, positions;
+  int H, n_tiles, rot_dim, window;
   float scale;
 };

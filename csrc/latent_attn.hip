@@ -105,9 +105,28 @@ __global__ __launch_bounds__(256) void latent_attn_kernel(const LatentArgs a) {
     const int r = m * 16 + c;
     const bool live = r < tl.count;
     qpos[m] = live ? tl.ctx + (tl.r0 + r) / a.H : -1;  // -1 sees no key
-    const bf16_t* qr = (const bf16_t*)a.q + (row0 + (live ? r : 0)) * ROW + g * 8;
+    const int64_t row = row0 + (live ? r : 0);
+    const bf16_t* qr = (const bf16_t*)a.q + row * RANK + g * 8;
 #pragma unroll
-    for (int s = 0; s < STEPS; ++s) qf[m][s] = *(const bf16x8_v*)(qr + s * 32);
+    for (int s = 0; s < RANK / 32; ++s) qf[m][s] = *(const bf16x8_v*)(qr + s * 32);
+    // the rest is rotated on the way in: 4 pairs a lane and step
+    const bf16_t* rr = (const bf16_t*)a.q_rot + row / a.H * a.rot_token +
+                       row % a.H * a.rot_head + g * 8;
+    const int pairs = a.rot_dim >> 1;
+    const float* ct = a.cos_sin + (int64_t)max(qpos[m], 0) * pairs;
+    const float* st = ct + a.positions * pairs;
+#pragma unroll
+    for (int s = 0; s < ROT / 32; ++s) {
+      bf16x8_v q8 = *(const bf16x8_v*)(rr + s * 32);
+#pragma unroll
+      for (int p = 0; p < 4; ++p) {
+        const int i = min(s * 16 + g * 4 + p, pairs - 1);  // padding is zero: any angle
+        const float x = (float)q8[2 * p], y = (float)q8[2 * p + 1];
+        q8[2 * p] = (__bf16)(x * ct[i] - y * st[i]);
+        q8[2 * p + 1] = (__bf16)(y * ct[i] + x * st[i]);
+      }
+      qf[m][RANK / 32 + s] = q8;
+    }
   }
 
   auto find_slots = [&](int t) {
@@ -185,12 +204,12 @@ __global__ __launch_bounds__(256) void latent_attn_kernel(const LatentArgs a) {
     for (int m = 0; m < MG; ++m) {
       const float4 w4 = *(const float4*)(red + (m * 16 + c) * 4);
       const float m_new = fmaxf(m_run[m], fmaxf(fmaxf(w4.x, w4.y), fmaxf(w4.z, w4.w)));
-      const float alpha = exp2f(m_run[m] - m_new);
+      const float alpha = __builtin_amdgcn_exp2f(m_run[m] - m_new);
       m_run[m] = m_new;
       float p[4], sum = 0.f;
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
-        p[r] = exp2f(s[m][r] - m_new);
+        p[r] = __builtin_amdgcn_exp2f(s[m][r] - m_new);
         sum += p[r];
       }
       l_run[m] = l_run[m] * alpha + sum;
@@ -276,7 +295,7 @@ __global__ __launch_bounds__(128) void latent_combine_kernel(
     for (int s = 0; s < n_split; ++s) {
       const float2 ml = part_ml[(int64_t)s * rows + row];
       if (ml.y == 0.f) continue;  // its partial was never written
-      const float w = exp2f(ml.x - m);
+      const float w = __builtin_amdgcn_exp2f(ml.x - m);
       l += w * ml.y;
       float v[4];
       load_f<4>(v, part + ((int64_t)s * rows + row) * rank + i);
@@ -304,7 +323,19 @@ __global__ __launch_bounds__(256) void latent_attn_plain_kernel(
 #pragma unroll
   for (int e = 0; e < NE; ++e) {
     const int d = e * 64 + lane;
-    q[e] = d < row ? to_f(((const T*)a.q)[qrow * row + d]) * a.scale : 0.f;
+    q[e] = 0.f;
+    if (d < rank) {
+      q[e] = to_f(((const T*)a.q)[qrow * rank + d]) * a.scale;
+    } else if (d < rank + a.rot_dim) {
+      const int i = (d - rank) >> 1;
+      const T* pair = (const T*)a.q_rot + qrow / a.H * a.rot_token +
+                      qrow % a.H * a.rot_head + 2 * i;
+      const int64_t at = (int64_t)pos * (a.rot_dim >> 1) + i;
+      const float co = a.cos_sin[at];
+      const float si = a.cos_sin[a.positions * (a.rot_dim >> 1) + at];
+      const float u = to_f(pair[0]), v = to_f(pair[1]);
+      q[e] = (d & 1 ? v * co + u * si : u * co - v * si) * a.scale;
+    }
   }
   float m = NEG, l = 0.f;
   for (int k = max(0, pos - a.window + 1) + wid; k <= pos; k += 4) {

@@ -1,6 +1,5 @@
-// Per-token kernels around latent attention (gfx950): the cache-row write, the
-// per-head products that absorb the key and value up-projections, and the
-// rotation of the query's rotated part.
+// Per-token kernels around latent attention (gfx950): the cache-row write and the
+// per-head products that absorb the key and value up-projections.
 //
 // Rotations here pair dimension 2i with 2i+1; cos_sin is [2, P, rot_dim/2] fp32.
 #include "common_t.h"
@@ -43,33 +42,6 @@ __global__ __launch_bounds__(256) void latent_cache_write_kernel(
     dst[rank + 2 * i] = from_f<T>(u);
     dst[rank + 2 * i + 1] = from_f<T>(v);
   }
-}
-
-// dst[n, h, 0:rot] = rotate(src[n, h, 0:rot_dim]) then zeros; one thread a pair.
-template <typename T>
-__global__ __launch_bounds__(256) void rotate_interleaved_kernel(
-    T* __restrict__ dst, const T* __restrict__ src,
-    const int64_t* __restrict__ positions, const float* __restrict__ cos_sin,
-    const int64_t total, const int H, const int rot_dim, const int rot,
-    const int64_t dst_row, const int64_t src_row, const int src_head,
-    const int dst_head, const int64_t P) {
-  const int64_t t = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
-  if (t >= total) return;
-  const int pairs = rot >> 1, half = rot_dim >> 1;
-  const int i = (int)(t % pairs);
-  const int h = (int)(t / pairs % H);
-  const int64_t n = t / ((int64_t)pairs * H);
-  float u = 0.f, v = 0.f;
-  if (i < half) {
-    const T* s = src + n * src_row + (int64_t)h * src_head + 2 * i;
-    const float a = to_f(s[0]), b = to_f(s[1]);
-    const float c = cos_sin[positions[n] * half + i];
-    const float sn = cos_sin[(P + positions[n]) * half + i];
-    u = a * c - b * sn;
-    v = b * c + a * sn;
-  }
-  const float uv[2] = {u, v};
-  store_f<2>(dst + n * dst_row + (int64_t)h * dst_head + 2 * i, uv);
 }
 
 // out[n, h, :O] = W[h] x[n, h, :K] (* sigmoid(gate[n, h])) on the matrix cores.
@@ -167,23 +139,6 @@ void launch_latent_cache_write(bool bf16, void* cache, const void* kv, const voi
     latent_cache_write_kernel<float><<<grid, 256, 0, stream>>>(
         (float*)cache, (const float*)kv, (const float*)norm_w, positions, slots,
         cos_sin, eps, N, kv_rank, rot_dim, rank, row, kv_stride, P);
-}
-
-void launch_rotate_interleaved(bool bf16, void* dst, const void* src,
-                               const int64_t* positions, const float* cos_sin, int N,
-                               int H, int rot_dim, int rot, int64_t dst_row,
-                               int64_t src_row, int src_head, int dst_head, int64_t P,
-                               hipStream_t stream) {
-  const int64_t total = (int64_t)N * H * (rot / 2);
-  const int grid = (int)((total + 255) / 256);
-  if (bf16)
-    rotate_interleaved_kernel<bf16_t><<<grid, 256, 0, stream>>>(
-        (bf16_t*)dst, (const bf16_t*)src, positions, cos_sin, total, H, rot_dim, rot,
-        dst_row, src_row, src_head, dst_head, P);
-  else
-    rotate_interleaved_kernel<float><<<grid, 256, 0, stream>>>(
-        (float*)dst, (const float*)src, positions, cos_sin, total, H, rot_dim, rot,
-        dst_row, src_row, src_head, dst_head, P);
 }
 
 void launch_head_linear(bool bf16, void* out, const void* x, const void* w,

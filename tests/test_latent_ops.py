@@ -160,21 +160,6 @@ def test_head_linear(device, dtype, n, O, K):
     assert not out[:, :, :32].any()
 
 
-def test_absorb_query(device, dtype):
-    n, H, d, rot_dim, base = 9, 5, 32, 12, 1e4
-    q = rand(n, H, d + 64, dtype=dtype, device=device)
-    q[:, :, d + rot_dim :] = 0
-    w = rand(H, 128, d, dtype=dtype, device=device, seed=1, scale=d ** -0.5)
-    pos = torch.arange(n, device=device) * 37
-    got = ops.absorb_query(q, w, pos, build_cos_sin(400, rot_dim, base, device, exact=True),
-                           d, rot_dim)
-    want = torch.stack([q[:, h, :d].double().cpu() @ w[h].double().cpu().T for h in range(H)], 1)
-    close(got[:, :, :128], want, dtype)
-    close(got[:, :, 128 : 128 + rot_dim],
-          oracle.rotate_pairs(q[:, :, d : d + rot_dim].double().cpu(), pos.cpu(), base), dtype)
-    assert not got[:, :, 128 + rot_dim :].any()
-
-
 # -------------------------------------------------------------- attention
 
 
@@ -220,6 +205,7 @@ def attend(q, rows, ctx, rank, scale, window):
     return torch.einsum("lhs,sr->lhr", p, rows[:, :rank])
 
 
+ROT, BASE = 8, 2e3
 SHAPES = [
     # heads, kv_rank, window, block, chunks
     (3, 24, None, 4, [(0, 5), (0, 1), (9, 2), (130, 1), (63, 1)]),
@@ -244,19 +230,31 @@ def test_latent_attention(device, dtype, H, kv_rank, window, block, chunks):
     for i, ((ctx, new), table) in enumerate(zip(chunks, tables)):
         r = rand(ctx + new, row, dtype=dtype, device="cpu", seed=10 + i)
         r[:, kv_rank:rank] = 0
-        r[:, rank + 8 :] = 0
+        r[:, rank + ROT :] = 0
         kv.append(r.double())
         for p, page in enumerate(table):
             part = r[p * block : (p + 1) * block]
             cache[page, : len(part)] = part
     cache = cache.to(device)
-    q = rand(batch.num_tokens, H, row, dtype=dtype, device=device, seed=5)
+    q = rand(batch.num_tokens, H, rank, dtype=dtype, device=device, seed=5)
+    wide = rand(batch.num_tokens, H, 128, dtype=dtype, device=device, seed=6)
+    wide[:, :, 64 + ROT :] = 0
     scale = 0.3 * kv_rank ** -0.5
-    got = ops.latent_attention(q, cache, batch, rank, scale, window).cpu()
+    cos_sin = build_cos_sin(2100, ROT, BASE, device, exact=True)
+    args = (cos_sin, ROT, cache, batch, scale, window)
+    got = ops.latent_attention(q, wide[:, :, 64:], *args).cpu()
+    part = batch.prefills[0].query_len  # rows from the second chunk on
+    tail = ops.latent_attention(q[part:].clone(), wide[part:, :, 64:], *args, part, (0,)).cpu()
+    rot = oracle.rotate_pairs(wide[:, :, 64 : 64 + ROT].double().cpu(), batch.positions.cpu(), BASE)
+    full = torch.zeros(batch.num_tokens, H, row, dtype=torch.float64)
+    full[:, :, :rank] = q.double().cpu()
+    full[:, :, rank : rank + ROT] = rot.to(dtype)
     at = 0
     for (ctx, new), rows in zip(chunks, kv):
-        want = attend(q[at : at + new].double().cpu(), rows, ctx, rank, scale, window)
+        want = attend(full[at : at + new], rows, ctx, rank, scale, window)
         close(got[at : at + new], want, dtype)
+        if at:
+            close(tail[at - part : at - part + new], want, dtype)
         at += new
 
 
@@ -278,12 +276,83 @@ def test_standout_key(device, dtype, where, decode):
     cache = torch.zeros(pages, block, row, dtype=dtype)
     for p, page in enumerate(tables[0]):
         cache[page, : len(rows[p * block : (p + 1) * block])] = rows[p * block : (p + 1) * block]
-    q = torch.zeros(batch.num_tokens, H, row, dtype=dtype)
-    q[:, :, rank] = 8.0
-    got = ops.latent_attention(q.to(device), cache.to(device), batch, rank, 1.0, win)[-1]
+    q = torch.zeros(batch.num_tokens, H, rank, dtype=dtype)
+    q_rot = torch.zeros(batch.num_tokens, H, 64, dtype=dtype)
+    q_rot[:, :, 0] = 8.0
+    still = torch.zeros(2, S, 1, device=device)
+    still[0] = 1.0  # no rotation
+    got = ops.latent_attention(
+        q.to(device), q_rot.to(device), still, 2, cache.to(device), batch, 1.0, win
+    )[-1]
     if where == "just_hidden":
         want = rows[i - window + 1 :, :rank].double().mean(0)
         assert (rows[hit, :rank].double() - want).abs().max() > 0.05
     else:
         want = rows[hit, :rank].double()
     close(got, want.expand(H, rank), dtype, scale=0.2)
+
+
+EXPANDED = [
+    # heads, dim, vdim, kv_rank, window, chunks
+    (3, 64, 64, 64, None, [(0, 5), (0, 200), (100, 130)]),
+    (8, 128, 128, 512, None, [(0, 300), (33, 1), (0, 129), (64, 65)]),
+    (16, 128, 64, 128, 70, [(0, 333), (500, 40), (69, 2), (70, 2)]),
+    (2, 256, 128, 256, 129, [(0, 257), (128, 128), (1000, 128)]),
+    (5, 64, 256, 384, 64, [(0, 64), (64, 64), (63, 66)]),
+    (1, 256, 256, 64, 1, [(0, 130), (77, 3)]),
+]
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("H,d,v,rank,window,chunks", EXPANDED)
+@pytest.mark.parametrize("budget", [1 << 40, 1])
+def test_expanded_prefill(H, d, v, rank, window, chunks, budget, monkeypatch):
+    """Keys and values expanded from latents in one group or one per chunk;
+    chunks left out and decode rows stay untouched."""
+    from agentcontrolplane_amd.ops import hip
+
+    monkeypatch.setattr(hip, "_EXPAND_BYTES", budget)
+    device, dtype, row = "cuda", BF16, rank + 64
+    batch, chunks, tables, pages = make_batch(chunks, 16, device)
+    cache = torch.full((pages, 16, row), float("nan"), dtype=dtype)
+    kv = []
+    for i, ((ctx, new), table) in enumerate(zip(chunks, tables)):
+        r = rand(ctx + new, row, dtype=dtype, device="cpu", seed=10 + i)
+        r[:, rank + ROT :] = 0
+        kv.append(r)
+        for p, page in enumerate(table):
+            part = r[p * 16 : (p + 1) * 16]
+            cache[page, : len(part)] = part
+    N = batch.num_tokens
+    q = rand(N, H, d + 64, dtype=dtype, device=device, seed=5)
+    q[:, :, d + ROT :] = 0
+    w = rand(H * (d + v), rank, dtype=dtype, device=device, seed=6, scale=rank ** -0.5)
+    gate = rand(N, H, dtype=dtype, device=device, seed=7)
+    out = torch.full((N, H, v), 9.0, dtype=dtype, device=device)
+    scale, skip = 0.5 * d ** -0.5, 1
+    pick = tuple(i for i in range(len(batch.prefills)) if i != skip)
+    ops.latent_expanded_prefill(
+        q, w, gate, build_cos_sin(2100, ROT, BASE, device, exact=True), ROT,
+        cache.to(device), batch, pick, rank, scale, window, out,
+    )
+    rot = oracle.rotate_pairs(q[:, :, d : d + ROT].double().cpu(), batch.positions.cpu(), BASE)
+    wk = w[: H * d].double().cpu().view(H, d, rank)
+    wv = w[H * d :].double().cpu().view(H, v, rank)
+    at = 0
+    for i, ((ctx, new), rows) in enumerate(zip(chunks, kv)):
+        got = out[at : at + new].cpu()
+        if i not in pick:
+            assert (got == 9.0).all()
+        else:
+            c = rows[:, :rank].double()
+            k = torch.einsum("sr,hdr->shd", c, wk).to(dtype).double()
+            val = torch.einsum("sr,hvr->shv", c, wv).to(dtype).double()
+            s = torch.einsum("lhd,shd->lhs", q[at : at + new, :, :d].double().cpu(), k)
+            s += torch.einsum("lhd,sd->lhs", rot[at : at + new].to(dtype).double(),
+                              rows[:, rank : rank + ROT].double())
+            ok = oracle.visible(ctx + new, window)[ctx:]
+            p = torch.softmax((s * scale).masked_fill(~ok.unsqueeze(1), float("-inf")), -1)
+            want = torch.einsum("lhs,shv->lhv", p, val)
+            want = want * torch.sigmoid(gate[at : at + new].double().cpu()).unsqueeze(-1)
+            close(got, want, dtype)
+        at += new
