@@ -9,8 +9,8 @@ per-layer token input.
     logits = embed . layernorm(x)
 
 Execution.  The residual is fp32.  Both sublayers read h and are summed, so a
-layer is two large GEMMs: one over [query | latent | head gates | glu gate | glu
-up] and one over [attention heads | glu], whose fp32 accumulation does the sum.
+layer's large GEMMs are one over [query | latent | head gates | glu gate | glu up]
+and one over [attention heads | glu], whose fp32 accumulation does the sum.
 The kernels between them work on slices of those buffers in place.  The residual
 updates, the side norm and the next layer's input norm are one pass over x.
 
@@ -35,6 +35,9 @@ from .latent_attention import Get, LatentAttention, pad_to, round_up
 from .llama import _dtype_of
 
 _ALIGN = 16  # rows between sections of the fused input projection
+#: the longest inner dimension of a fused output projection: beyond it the library's
+#: small-batch kernels slow down more than a second GEMM costs
+_FUSED_OUT = 16384
 
 
 class FetolixLayer:
@@ -68,7 +71,8 @@ class FetolixLayer:
         self.in_rows = at
         self.norm: torch.Tensor = None
         self.w_in: torch.Tensor = None    # [in_rows, width]
-        self.w_out: torch.Tensor = None   # [width, out_dim + ff_pad]
+        # output projections over column ranges of [attention | glu], summed
+        self.w_out: List[torch.Tensor] = []
         self.side_gate = self.side_proj = self.side_norm = None
 
     def load(self, get: Get, p: str, side_dim: int) -> None:
@@ -88,7 +92,9 @@ class FetolixLayer:
             w_in[at + self.ff_pad : at + self.ff_pad + self.ff] = get(p + "mlp.up")[mine]
             outs.append(pad_to(get(p + "mlp.down")[:, mine], self.width, self.ff_pad))
         self.w_in = w_in
-        self.w_out = torch.cat(outs, 1).contiguous()
+        if m.out_dim + self.ff_pad <= _FUSED_OUT:
+            outs = [torch.cat(outs, 1)]
+        self.w_out = [o.contiguous() for o in outs]
         if side_dim:
             self.side_gate = get(p + "side.gate")
             self.side_proj = get(p + "side.proj")
@@ -99,12 +105,13 @@ class FetolixLayer:
         sec = {
             n: self.w_in[at : at + rows] for n, (at, rows) in self.sections.items() if rows
         }
-        sec["o"] = self.w_out[:, : m.out_dim].contiguous()
+        w_out = torch.cat(self.w_out, 1)
+        sec["o"] = w_out[:, : m.out_dim].contiguous()
         out = {p + "norm1": self.norm, **m.export(sec, p + "mix.")}
         if self.mlp:
             out[p + "mlp.gate"] = sec["glu"][: self.ff]
             out[p + "mlp.up"] = sec["glu"][self.ff_pad : self.ff_pad + self.ff]
-            out[p + "mlp.down"] = self.w_out[:, m.out_dim : m.out_dim + self.ff]
+            out[p + "mlp.down"] = w_out[:, m.out_dim : m.out_dim + self.ff]
         if self.side_gate is not None:
             out[p + "side.gate"] = self.side_gate
             out[p + "side.proj"] = self.side_proj
@@ -132,7 +139,11 @@ class FetolixLayer:
             section("q"), section("kv"), section("gate"), batch, cache,
             mixed[:, : m.out_dim],
         )
-        return ops.linear(mixed, self.w_out)
+        at = self.w_out[0].shape[1]
+        y = ops.linear(mixed[:, :at], self.w_out[0])
+        if len(self.w_out) > 1:
+            ops.linear_add_(y, mixed[:, at:], self.w_out[1])
+        return y
 
 
 class FetolixForCausalLM:
@@ -287,8 +298,9 @@ class FetolixForCausalLM:
                 norm, out = self.layers[nxt[0]].norm, torch.empty_like(h)
             if cfg.token_side_dim:
                 d = cfg.token_side_dim
-                s = ops.linear(ops.add_to_residual(x, y, self.dtype), layer.side_gate)
-                ops.gelu_gate_(s, batch.token_ids, self.side_embed, i * d)
+                x, s = ops.side_gate(
+                    x, y, layer.side_gate, batch.token_ids, self.side_embed, i * d
+                )
                 ops.residual_norm(
                     x, ops.linear(s, layer.side_proj), eps, layer.side_norm, norm, out
                 )

@@ -173,12 +173,13 @@ class LatentAttention:
         """q, kv, gate: the sections of the fused projection (row-strided
         views); writes out [N, out_dim] (row-strided view)."""
         s, H, N = self.spec, self.heads, q.shape[0]
-        if s.q_rank:
-            q = ops.linear(ops.rmsnorm_rows(q, self.q_norm, self.eps, s.q_rank), self.uq)
-        ops.latent_cache_write(
+        low_rank = (q, self.q_norm, s.q_rank) if s.q_rank else ()
+        cq = ops.latent_inputs(
             kv, self.kv_norm, self.eps, s.kv_rank, s.rot_dim, self.rank,
-            batch.positions, batch.slot_mapping, self.cos_sin, cache,
+            batch.positions, batch.slot_mapping, self.cos_sin, cache, *low_rank,
         )
+        if s.q_rank:
+            q = ops.linear(cq, self.uq)
         q = q.as_strided((N, H, self.d + self.rot), (q.stride(0), self.d + self.rot, 1))
         out = out.as_strided((N, H, self.v), (out.stride(0), self.v, 1))
         expanded, row0 = batch.memo(

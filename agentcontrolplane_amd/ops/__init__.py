@@ -68,6 +68,11 @@ def linear(x, w):
     return torch.nn.functional.linear(x, w)
 
 
+def linear_add_(y, x, w):
+    """y += x @ w^T in one GEMM."""
+    return y.addmm_(x, w.t())
+
+
 def rmsnorm(x, weight, eps: float = 1e-5):
     return _impl(x).rmsnorm(x, weight, eps)
 
@@ -109,20 +114,9 @@ def swiglu(gate_up):
 # ------------------------------------------------ fp32-residual norms, GLU, gates
 
 
-def rmsnorm_rows(x, weight, eps: float, n: int):
-    """RMS norm of row-strided [N, K] over the first n columns (the rest are
-    padding: zero in, zero weight, zero out)."""
-    return _impl(x).rmsnorm_rows(x, weight, eps, n)
-
-
 def layernorm(x, weight, eps: float, dtype):
     """Layer norm without bias of an fp32 residual [N, K] -> dtype."""
     return _impl(x).layernorm(x, weight, eps, dtype)
-
-
-def add_to_residual(x, y, dtype):
-    """x += y in the fp32 residual x; returns the new x in dtype."""
-    return _impl(x).add_to_residual(x, y, dtype)
 
 
 def residual_norm(x, y, eps: float, y_norm=None, x_norm=None, out=None):
@@ -137,9 +131,10 @@ def clamped_glu(gate_up, limit: float, alpha: float, offset: float, out):
     return _impl(gate_up).clamped_glu(gate_up, limit, alpha, offset, out)
 
 
-def gelu_gate_(s, token_ids, table, offset: int):
-    """s [N, D] <- gelu_tanh(s) * table[token, offset : offset + D]."""
-    return _impl(s).gelu_gate_(s, token_ids, table, offset)
+def side_gate(x, y, gate, token_ids, table, offset: int):
+    """The fp32 residual x + y (x itself may be reused for it) and
+    gelu_tanh(gate (x + y)) * table[token, offset : offset + D]: [N, D]."""
+    return _impl(x).side_gate(x, y, gate, token_ids, table, offset)
 
 
 # ------------------------------------------------------------ latent attention
@@ -168,13 +163,15 @@ def latent_head(dim: int) -> int:
     return -(-dim // 64) * 64
 
 
-def latent_cache_write(kv, norm_w, eps: float, kv_rank: int, rot_dim: int, rank: int,
-                       positions, slot_mapping, cos_sin, cache):
+def latent_inputs(kv, norm_w, eps: float, kv_rank: int, rot_dim: int, rank: int,
+                  positions, slot_mapping, cos_sin, cache, q=None, q_norm=None, q_rank=0):
     """kv [N, kv_rank + rot_dim] (row-strided): RMS-norm the latent, rotate the
     key part (interleaved pairs), scatter [latent -> rank | rotated] rows into
-    cache [blocks, block, row]."""
-    return _impl(kv).latent_cache_write(
-        kv, norm_w, eps, kv_rank, rot_dim, rank, positions, slot_mapping, cos_sin, cache
+    cache [blocks, block, row].  With q [N, K] (low-rank query, row-strided; its
+    columns past q_rank are zero padding) returns rmsnorm(q) * q_norm."""
+    return _impl(kv).latent_inputs(
+        kv, norm_w, eps, kv_rank, rot_dim, rank, positions, slot_mapping, cos_sin, cache,
+        q, q_norm, q_rank,
     )
 
 

@@ -111,24 +111,9 @@ def swiglu(gate_up):
 # ------------------------------------------------ fp32-residual norms, GLU, gates
 
 
-def rmsnorm_rows(x, weight, eps: float, n: int):
-    out = torch.empty(x.shape, dtype=x.dtype, device=x.device)
-    _C.rmsnorm_rows(out, x, weight, eps, n)
-    return out
-
-
 def layernorm(x, weight, eps: float, dtype):
     out = torch.empty(x.shape, dtype=dtype, device=x.device)
     _C.residual_norm(x, None, None, weight, out, eps)
-    return out
-
-
-def add_to_residual(x, y, dtype):
-    if dtype == torch.float32:
-        _C.add_to_residual(x, y, None)
-        return x
-    out = torch.empty(x.shape, dtype=dtype, device=x.device)
-    _C.add_to_residual(x, y, out)
     return out
 
 
@@ -140,24 +125,39 @@ def clamped_glu(gate_up, limit: float, alpha: float, offset: float, out):
     _C.clamped_glu(out, gate_up, limit, alpha, offset)
 
 
-def gelu_gate_(s, token_ids, table, offset: int):
+#: up to this many tokens the fused side_gate kernel beats the GEMM route
+_SIDE_GATE_TOKENS = 256
+
+
+def side_gate(x, y, gate, token_ids, table, offset: int):
+    from . import linear
+
+    if x.shape[0] <= _SIDE_GATE_TOKENS and x.shape[1] % 8 == 0:
+        s = torch.empty(x.shape[0], gate.shape[0], dtype=gate.dtype, device=x.device)
+        x_new = torch.empty_like(x)
+        _C.side_gate(s, x_new, x, y, gate, token_ids, table, offset)
+        return x_new, s
+    xt = None if gate.dtype == torch.float32 else torch.empty_like(y)
+    _C.add_to_residual(x, y, xt)
+    s = linear(x if xt is None else xt, gate)
     _C.gelu_gate(s, token_ids, table, offset)
-    return s
+    return x, s
 
 
 # ------------------------------------------------------------ latent attention
 
 _NO_WINDOW = 1 << 30
-#: workgroups that fill the chip at the MFMA kernel's LDS footprint
-_FILL = 512
 _MAX_SPLIT = 32
 
 
-def latent_cache_write(kv, norm_w, eps: float, kv_rank: int, rot_dim: int, rank: int,
-                       positions, slot_mapping, cos_sin, cache):
-    _C.latent_cache_write(
-        cache, kv, norm_w, positions, slot_mapping, cos_sin, eps, kv_rank, rot_dim, rank
+def latent_inputs(kv, norm_w, eps: float, kv_rank: int, rot_dim: int, rank: int,
+                  positions, slot_mapping, cos_sin, cache, q=None, q_norm=None, q_rank=0):
+    cq = None if q is None else torch.empty(q.shape, dtype=q.dtype, device=q.device)
+    _C.latent_inputs(
+        cache, kv, norm_w, positions, slot_mapping, cos_sin, eps, kv_rank, rot_dim, rank,
+        cq, q, q_norm, q_rank,
     )
+    return cq
 
 
 def head_linear(x, w, out, gate=None):
@@ -172,7 +172,9 @@ def _latent_attn(out, q, q_rot, cos_sin, rot_dim, cache, tables, seq_lens, prefi
     n_split = 1
     if mfma:
         keys = min(max_keys, window)
-        n_split = max(1, min(_MAX_SPLIT, _FILL // tiles, -(-keys // 128)))
+        # workgroups that fill the chip: the tiles of a wide latent take a CU's LDS
+        fill = 256 if q.shape[2] >= 256 else 512
+        n_split = max(1, min(_MAX_SPLIT, fill // tiles, -(-keys // 128)))
     part = ml = None
     if n_split > 1:
         rows = q.shape[0] * q.shape[1]

@@ -168,11 +168,6 @@ def layernorm(x, weight, eps: float, dtype):
     return (xc * torch.rsqrt(var + eps) * weight.float()).to(dtype)
 
 
-def add_to_residual(x, y, dtype):
-    x += y.float()
-    return x.to(dtype)
-
-
 def residual_norm(x, y, eps: float, y_norm=None, x_norm=None, out=None):
     yf = y.float()
     if y_norm is not None:
@@ -188,10 +183,11 @@ def clamped_glu(gate_up, limit: float, alpha: float, offset: float, out):
     out.copy_(g * torch.sigmoid(alpha * g) * (u.clamp(-limit, limit) + offset))
 
 
-def gelu_gate_(s, token_ids, table, offset: int):
-    e = table[token_ids, offset : offset + s.shape[1]].float()
-    s.copy_(torch.nn.functional.gelu(s.float(), approximate="tanh") * e)
-    return s
+def side_gate(x, y, gate, token_ids, table, offset: int):
+    x = x + y.float()
+    s = torch.nn.functional.linear(x.to(gate.dtype), gate).float()
+    e = table[token_ids, offset : offset + gate.shape[0]].float()
+    return x, (torch.nn.functional.gelu(s, approximate="tanh") * e).to(gate.dtype)
 
 
 # ------------------------------------------------------------ latent attention
@@ -204,8 +200,8 @@ def _rotate_interleaved(x, cos, sin):
     return torch.stack([u * cos - v * sin, v * cos + u * sin], dim=-1).flatten(-2)
 
 
-def latent_cache_write(kv, norm_w, eps: float, kv_rank: int, rot_dim: int, rank: int,
-                       positions, slot_mapping, cos_sin, cache):
+def latent_inputs(kv, norm_w, eps: float, kv_rank: int, rot_dim: int, rank: int,
+                  positions, slot_mapping, cos_sin, cache, q=None, q_norm=None, q_rank=0):
     c = rmsnorm_rows(kv[:, :kv_rank], norm_w, eps, kv_rank)
     k_rot = _rotate_interleaved(
         kv[:, kv_rank : kv_rank + rot_dim], cos_sin[0][positions], cos_sin[1][positions]
@@ -214,6 +210,7 @@ def latent_cache_write(kv, norm_w, eps: float, kv_rank: int, rot_dim: int, rank:
     row[:, :kv_rank] = c.to(cache.dtype)
     row[:, rank : rank + rot_dim] = k_rot.to(cache.dtype)
     cache.view(-1, cache.shape[-1])[slot_mapping] = row
+    return None if q is None else rmsnorm_rows(q, q_norm, eps, q_rank)
 
 
 def head_linear(x, w, out, gate=None):

@@ -36,16 +36,17 @@ void launch_prefill_attn_mfma(void*, const void*, const void*, const void*, cons
                               float, int, int, int, int, int, int, int64_t, hipStream_t);
 void launch_residual_norm(bool, float*, const void*, const void*, const void*, void*, float,
                           int, int, int64_t, hipStream_t);
-void launch_rmsnorm_rows(bool, void*, const void*, const void*, float, int, int, int,
-                         int64_t, hipStream_t);
+void launch_side_gate(bool, float*, const float*, const void*, const void*, const int64_t*, const void*,
+                      void*, int, int, int, int64_t, hipStream_t);
 void launch_add_to_residual(bool, float*, const void*, void*, int64_t, hipStream_t);
 void launch_clamped_glu(bool, void*, const void*, float, float, float, int, int, int64_t,
                         int64_t, hipStream_t);
 void launch_gelu_gate(bool, void*, const int64_t*, const void*, int, int, int64_t,
                       hipStream_t);
-void launch_latent_cache_write(bool, void*, const void*, const void*, const int64_t*,
-                               const int64_t*, const float*, float, int, int, int, int,
-                               int, int64_t, int64_t, hipStream_t);
+void launch_latent_inputs(bool, void*, const void*, const void*, const int64_t*,
+                          const int64_t*, const float*, float, int, int, int, int, int,
+                          int64_t, int64_t, void*, const void*, const void*, int, int,
+                          int64_t, hipStream_t);
 void launch_head_linear(bool, void*, const void*, const void*, const void*, int, int, int,
                         int, int64_t, int, int64_t, int, int64_t, hipStream_t);
 bool launch_latent_prefill(const LatentPrefillArgs*, int, int, hipStream_t);
@@ -301,17 +302,27 @@ static void residual_norm(torch::Tensor x, OptTensor y, OptTensor y_norm, OptTen
                        out ? out->stride(0) : w, cur_stream());
 }
 
-static void rmsnorm_rows(torch::Tensor out, torch::Tensor x, torch::Tensor weight,
-                         double eps, int64_t n) {
-  const int rows = x.size(0), k = x.size(1);
-  check_rows(x, x.scalar_type(), rows, k);
-  check_rows(out, x.scalar_type(), rows, k); CHECK_CONT(out);
-  check_vec(weight, x.scalar_type(), k);
-  check_aligned(x);
-  TORCH_CHECK(k % 8 == 0 && n <= k);
-  if (rows == 0) return;
-  launch_rmsnorm_rows(is_bf16(x), out.data_ptr(), x.data_ptr(), weight.data_ptr(),
-                      (float)eps, rows, k, n, x.stride(0), cur_stream());
+// x_out = x + y; s = gelu_tanh(gate x_out) * table[token, offset:]
+static void side_gate(torch::Tensor s, torch::Tensor x_out, torch::Tensor x, torch::Tensor y, torch::Tensor gate,
+                      torch::Tensor token_ids, torch::Tensor table, int64_t offset) {
+  const int n = x.size(0), w = x.size(1), dim = s.size(1);
+  CHECK_CUDA(x); CHECK_CONT(x); CHECK_CUDA(x_out); CHECK_CONT(x_out);
+  TORCH_CHECK(x.scalar_type() == at::kFloat && x_out.scalar_type() == at::kFloat &&
+              x_out.sizes() == x.sizes() && x_out.data_ptr() != x.data_ptr());
+  const auto dt = y.scalar_type();
+  check_rows(y, dt, n, w); CHECK_CONT(y);
+  check_rows(s, dt, n, dim); CHECK_CONT(s);
+  check_rows(gate, dt, dim, w); CHECK_CONT(gate);
+  check_rows(table, dt, table.size(0), table.size(1));
+  CHECK_CUDA(token_ids); CHECK_CONT(token_ids);
+  TORCH_CHECK(token_ids.scalar_type() == at::kLong && token_ids.numel() == n);
+  TORCH_CHECK(offset >= 0 && offset + dim <= table.size(1), "table columns");
+  TORCH_CHECK(w % 8 == 0 && w <= 16000, "residual width");
+  if (n == 0) return;
+  launch_side_gate(is_bf16(y), x_out.data_ptr<float>(), x.data_ptr<float>(), y.data_ptr(), gate.data_ptr(),
+                   token_ids.data_ptr<int64_t>(),
+                   (const char*)table.data_ptr() + offset * table.element_size(),
+                   s.data_ptr(), n, w, dim, table.stride(0), cur_stream());
 }
 
 static void add_to_residual(torch::Tensor x, torch::Tensor y, OptTensor out) {
@@ -361,10 +372,13 @@ static void check_rotation(const torch::Tensor& cos_sin, const torch::Tensor& po
   TORCH_CHECK(positions.scalar_type() == at::kLong && positions.numel() == n);
 }
 
-static void latent_cache_write(torch::Tensor cache, torch::Tensor kv, torch::Tensor norm_w,
-                               torch::Tensor positions, torch::Tensor slots,
-                               torch::Tensor cos_sin, double eps, int64_t kv_rank,
-                               int64_t rot_dim, int64_t rank) {
+// Cache rows of kv, and cq = rmsnorm(q) over q's first q_rank columns (low-rank
+// queries; q, q_norm and cq come together).
+static void latent_inputs(torch::Tensor cache, torch::Tensor kv, torch::Tensor norm_w,
+                          torch::Tensor positions, torch::Tensor slots,
+                          torch::Tensor cos_sin, double eps, int64_t kv_rank,
+                          int64_t rot_dim, int64_t rank, OptTensor cq, OptTensor q,
+                          OptTensor q_norm, int64_t q_rank) {
   const int n = kv.size(0);
   check_rows(kv, kv.scalar_type(), n, kv_rank + rot_dim);
   check_vec(norm_w, kv.scalar_type(), kv_rank);
@@ -374,11 +388,22 @@ static void latent_cache_write(torch::Tensor cache, torch::Tensor kv, torch::Ten
   TORCH_CHECK(cache.scalar_type() == kv.scalar_type());
   const int row = cache.size(-1);
   TORCH_CHECK(kv_rank <= rank && rank + rot_dim <= row && (row - rank) % 2 == 0);
+  int k = 0;
+  if (q) {
+    TORCH_CHECK(cq && q_norm, "low-rank query");
+    k = q->size(1);
+    check_rows(*q, kv.scalar_type(), n, k); check_aligned(*q);
+    check_rows(*cq, kv.scalar_type(), n, k); CHECK_CONT((*cq));
+    check_vec(*q_norm, kv.scalar_type(), k);
+    TORCH_CHECK(k % 8 == 0 && q_rank > 0 && q_rank <= k);
+  }
   if (n == 0) return;
-  launch_latent_cache_write(is_bf16(kv), cache.data_ptr(), kv.data_ptr(), norm_w.data_ptr(),
-                            positions.data_ptr<int64_t>(), slots.data_ptr<int64_t>(),
-                            cos_sin.data_ptr<float>(), (float)eps, n, kv_rank, rot_dim, rank,
-                            row, kv.stride(0), cos_sin.size(1), cur_stream());
+  launch_latent_inputs(is_bf16(kv), cache.data_ptr(), kv.data_ptr(), norm_w.data_ptr(),
+                       positions.data_ptr<int64_t>(), slots.data_ptr<int64_t>(),
+                       cos_sin.data_ptr<float>(), (float)eps, n, kv_rank, rot_dim, rank, row,
+                       kv.stride(0), cos_sin.size(1), q ? cq->data_ptr() : nullptr,
+                       q ? q->data_ptr() : nullptr, q ? q_norm->data_ptr() : nullptr, k,
+                       (int)q_rank, q ? q->stride(0) : 0, cur_stream());
 }
 
 // [N, H, K] with dense vectors, any token and head stride
@@ -438,7 +463,7 @@ static void latent_attn(torch::Tensor out, torch::Tensor q, torch::Tensor q_rot,
   const int seqs = tables.size(0);
   TORCH_CHECK(seq_lens.numel() == seqs);
   TORCH_CHECK(!mfma || (bf16 && row - rank == 64), "no MFMA kernel for this row");
-  TORCH_CHECK(window > 0 && n_split >= 1 && (mfma || n_split == 1));
+  TORCH_CHECK(window > 0 && n_split >= 1 && n_split <= 64 && (mfma || n_split == 1));
   TORCH_CHECK(mg == 1 || mg == 2 || (mg == 4 && rank <= 256) || !mfma, "row tile");
   const int per_tile = mfma ? 16 * (int)mg : 1;
   int tiles;
@@ -566,11 +591,11 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("mfma_probe", &mfma_probe);
   m.def("gemm_bf16", &gemm_bf16);
   m.def("residual_norm", &residual_norm);
-  m.def("rmsnorm_rows", &rmsnorm_rows);
+  m.def("side_gate", &side_gate);
   m.def("add_to_residual", &add_to_residual);
   m.def("clamped_glu", &clamped_glu);
   m.def("gelu_gate", &gelu_gate);
-  m.def("latent_cache_write", &latent_cache_write);
+  m.def("latent_inputs", &latent_inputs);
   m.def("head_linear", &head_linear);
   m.def("latent_attn", &latent_attn);
   m.def("latent_gather", &latent_gather);

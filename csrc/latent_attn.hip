@@ -91,9 +91,9 @@ __global__ __launch_bounds__(256) void latent_attn_kernel(const LatentArgs a) {
   const int t_end = min(n_tiles, t_begin + per_split);
 
   const int64_t row0 = (int64_t)tl.token0 * a.H + tl.r0;
-  if (t_begin >= t_end) {  // an empty split leaves weight zero
+  if (t_begin >= t_end) {  // an empty split; those are a row's last ones
     for (int i = threadIdx.x; i < tl.count; i += 256)
-      a.part_ml[(int64_t)blockIdx.y * a.rows + row0 + i] = float2{NEG, 0.f};
+      a.part_ml[(int64_t)blockIdx.y * a.rows + row0 + i] = float2{NEG, -1.f};
     return;
   }
 
@@ -282,29 +282,30 @@ __global__ __launch_bounds__(256) void latent_attn_kernel(const LatentArgs a) {
   }
 }
 
-// Merge the splits of one row: 128 threads, 4 columns each per pass.
+// Merge the splits (at most 64) of one row.
 __global__ __launch_bounds__(128) void latent_combine_kernel(
     bf16_t* __restrict__ out, const float* __restrict__ part,
     const float2* __restrict__ part_ml, const int rows, const int rank,
     const int n_split) {
-  const int row = blockIdx.x;
-  float m = NEG;
-  for (int s = 0; s < n_split; ++s) m = fmaxf(m, part_ml[(int64_t)s * rows + row].x);
+  __shared__ float weight[64];
+  const int row = blockIdx.x, lane = threadIdx.x & 63;
+  const float2 ml = lane < n_split ? part_ml[(int64_t)lane * rows + row] : float2{NEG, -1.f};
+  const int live = __popcll(__ballot(ml.y >= 0.f));
+  const float m = wave_max(ml.x);
+  const float w = ml.y > 0.f ? __builtin_amdgcn_exp2f(ml.x - m) : 0.f;
+  const float l = wave_sum(w * fmaxf(ml.y, 0.f));
+  if (threadIdx.x < 64) weight[lane] = l > 0.f ? w / l : 0.f;
+  __syncthreads();
   for (int i = threadIdx.x * 4; i < rank; i += 512) {
-    float acc[4] = {}, l = 0.f;
-    for (int s = 0; s < n_split; ++s) {
-      const float2 ml = part_ml[(int64_t)s * rows + row];
-      if (ml.y == 0.f) continue;  // its partial was never written
-      const float w = __builtin_amdgcn_exp2f(ml.x - m);
-      l += w * ml.y;
+    float acc[4] = {};
+    const float* src = part + (int64_t)row * rank + i;
+#pragma unroll 8
+    for (int s = 0; s < live; ++s) {
       float v[4];
-      load_f<4>(v, part + ((int64_t)s * rows + row) * rank + i);
+      load_f<4>(v, src + (int64_t)s * rows * rank);
 #pragma unroll
-      for (int k = 0; k < 4; ++k) acc[k] += w * v[k];
+      for (int k = 0; k < 4; ++k) acc[k] += weight[s] * v[k];
     }
-    const float inv = l > 0.f ? 1.f / l : 0.f;
-#pragma unroll
-    for (int k = 0; k < 4; ++k) acc[k] *= inv;
     store_f<4>(out + (int64_t)row * rank + i, acc);
   }
 }

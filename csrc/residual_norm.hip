@@ -8,7 +8,7 @@
 #include "common_t.h"
 
 template <typename T, int V>
-__global__ __launch_bounds__(256) void residual_norm_kernel(
+__global__ __launch_bounds__(1024) void residual_norm_kernel(
     float* __restrict__ x,            // [n, w], updated if y
     const T* __restrict__ y,          // [n, w] or null
     const T* __restrict__ y_norm,     // [w] or null: plain add
@@ -16,7 +16,7 @@ __global__ __launch_bounds__(256) void residual_norm_kernel(
     T* __restrict__ out,              // [n, w] rows out_stride apart, or null
     const float eps, const int w, const int64_t out_stride) {
   extern __shared__ float row[];
-  __shared__ float scratch[3][4];
+  __shared__ float scratch[3][16];
   float* xr = x + (int64_t)blockIdx.x * w;
   const int step = blockDim.x * V;
   const int i0 = threadIdx.x * V;
@@ -87,34 +87,6 @@ __global__ __launch_bounds__(256) void residual_norm_kernel(
   }
 }
 
-// RMS norm over the first n of k columns of strided rows; one wave per row.
-template <typename T, int V>
-__global__ __launch_bounds__(256) void rmsnorm_rows_kernel(
-    T* __restrict__ out, const T* __restrict__ x, const T* __restrict__ weight,
-    const float eps, const int rows, const int k, const int n,
-    const int64_t x_stride) {
-  const int r = blockIdx.x * 4 + (threadIdx.x >> 6);
-  if (r >= rows) return;
-  const T* xr = x + r * x_stride;
-  const int lane = threadIdx.x & 63;
-  float ss = 0.f;
-  for (int i = lane * V; i < k; i += 64 * V) {
-    float t[V];
-    load_f<V>(t, xr + i);  // columns n.. are zero
-#pragma unroll
-    for (int j = 0; j < V; ++j) ss += t[j] * t[j];
-  }
-  const float inv = rsqrtf(wave_sum(ss) / n + eps);
-  for (int i = lane * V; i < k; i += 64 * V) {
-    float t[V], g[V];
-    load_f<V>(t, xr + i);
-    load_f<V>(g, weight + i);
-#pragma unroll
-    for (int j = 0; j < V; ++j) t[j] *= inv * g[j];
-    store_f<V>(out + (int64_t)r * k + i, t);
-  }
-}
-
 template <typename T, int V>
 __global__ __launch_bounds__(256) void add_to_residual_kernel(
     float* __restrict__ x, const T* __restrict__ y, T* __restrict__ out,
@@ -136,7 +108,9 @@ static void residual_norm_t(float* x, const void* y, const void* y_norm,
                             const void* x_norm, void* out, float eps, int n,
                             int w, int64_t out_stride, hipStream_t stream) {
   const bool vec = w % 4 == 0 && out_stride % 4 == 0;
-  const int threads = w >= 1024 ? 256 : w >= 512 ? 128 : 64;
+  int threads = w >= 1024 ? 256 : w >= 512 ? 128 : 64;
+  // few rows: the latency of one counts
+  while (n <= 512 && threads < 1024 && threads * 4 < w) threads *= 2;
   auto k = vec ? residual_norm_kernel<T, 4> : residual_norm_kernel<T, 1>;
   k<<<n, threads, w * sizeof(float), stream>>>(
       x, (const T*)y, (const T*)y_norm, (const T*)x_norm, (T*)out, eps, w, out_stride);
@@ -149,18 +123,6 @@ void launch_residual_norm(bool bf16, float* x, const void* y, const void* y_norm
                           int64_t out_stride, hipStream_t stream) {
   (bf16 ? residual_norm_t<bf16_t> : residual_norm_t<float>)(
       x, y, y_norm, x_norm, out, eps, n, w, out_stride, stream);
-}
-
-void launch_rmsnorm_rows(bool bf16, void* out, const void* x, const void* weight,
-                         float eps, int rows, int k, int n, int64_t x_stride,
-                         hipStream_t stream) {
-  const int grid = (rows + 3) / 4;
-  if (bf16)
-    rmsnorm_rows_kernel<bf16_t, 8><<<grid, 256, 0, stream>>>(
-        (bf16_t*)out, (const bf16_t*)x, (const bf16_t*)weight, eps, rows, k, n, x_stride);
-  else
-    rmsnorm_rows_kernel<float, 4><<<grid, 256, 0, stream>>>(
-        (float*)out, (const float*)x, (const float*)weight, eps, rows, k, n, x_stride);
 }
 
 void launch_add_to_residual(bool bf16, float* x, const void* y, void* out,

@@ -70,22 +70,6 @@ def test_residual_norm(device, dtype, n, w, y_norm, x_norm):
     close(x, before.double().cpu() + yd, F32)
 
 
-def test_add_to_residual_and_rmsnorm_rows(device, dtype):
-    x, y = rand(6, 131, dtype=F32, device=device), rand(6, 131, dtype=dtype, device=device, seed=1)
-    want = x.double().cpu() + y.double().cpu()
-    close(ops.add_to_residual(x, y, dtype), want, dtype)
-    close(x, want, F32)
-    # 20 columns padded to 32, read out of a wider buffer
-    wide = rand(6, 64, dtype=dtype, device=device, seed=2, scale=0.02)
-    wide[:, 20:32] = 0
-    w = rand(32, dtype=dtype, device=device, seed=3)
-    w[20:] = 0
-    got = ops.rmsnorm_rows(wide[:, :32], w, 1e-4, 20)
-    want = oracle.rms(wide[:, :20].double().cpu(), 1e-4) * w[:20].double().cpu()
-    close(got[:, :20], want, dtype)
-    assert not got[:, 20:].any()
-
-
 # ------------------------------------------------------- gated activations
 
 
@@ -105,19 +89,25 @@ def test_clamped_glu(device, dtype):
     close(out[:, inter:], g * torch.sigmoid(0.5 * g) * u, dtype)
 
 
-def test_gelu_gate(device, dtype):
-    s = rand(19, 7, dtype=dtype, device=device, scale=2.0)
-    table = rand(30, 21, dtype=dtype, device=device, seed=1)
-    tok = torch.arange(19, device=device) * 3 % 30
-    want = oracle.gelu_tanh(s.double().cpu()) * table[tok][:, 7:14].double().cpu()
-    close(ops.gelu_gate_(s, tok, table, 7), want, dtype)
+@pytest.mark.parametrize("n,w,dim", [(3, 40, 7), (19, 250, 5), (300, 64, 16), (2, 4096, 64)])
+def test_side_gate(device, dtype, n, w, dim):
+    """x + y, then the gated gelu of its projection; few and many tokens."""
+    x, y = rand(n, w, dtype=F32, device=device), rand(n, w, dtype=dtype, device=device, seed=1)
+    gate = rand(dim, w, dtype=dtype, device=device, seed=2, scale=w ** -0.5)
+    table = rand(30, 3 * dim, dtype=dtype, device=device, seed=3)
+    tok = torch.arange(n, device=device) * 3 % 30
+    want_x = x.double().cpu() + y.double().cpu()
+    x, got = ops.side_gate(x, y, gate, tok, table, dim)
+    close(x, want_x, F32)
+    want = oracle.gelu_tanh(want_x @ gate.double().cpu().T)
+    close(got, want * table[tok][:, dim : 2 * dim].double().cpu(), dtype)
 
 
 # -------------------------------------------------------------- per token
 
 
 @pytest.mark.parametrize("kv_rank,rot_dim", [(24, 8), (100, 34), (512, 64)])
-def test_latent_cache_write(device, dtype, kv_rank, rot_dim):
+def test_latent_inputs(device, dtype, kv_rank, rot_dim):
     n, base, eps = 11, 3e4, 1e-2
     rank = ops.latent_rank(kv_rank)
     row = rank + 64
@@ -128,7 +118,16 @@ def test_latent_cache_write(device, dtype, kv_rank, rot_dim):
     slots = torch.randperm(32, generator=torch.Generator().manual_seed(1))[:n].to(device)
     cache = torch.full((8, 4, row), 7.0, dtype=dtype, device=device)
     cos_sin = build_cos_sin(1000, rot_dim, base, device, exact=True)
-    ops.latent_cache_write(kv, w, eps, kv_rank, rot_dim, rank, pos, slots, cos_sin, cache)
+    args = (kv, w, eps, kv_rank, rot_dim, rank, pos, slots, cos_sin, cache)
+    assert ops.latent_inputs(*args) is None
+    # a low-rank query: 20 columns padded to 32, read out of a wider buffer
+    buf = rand(n, 64, dtype=dtype, device=device, seed=2, scale=0.1)
+    buf[:, 36:48] = 0
+    qw = rand(32, dtype=dtype, device=device, seed=3)
+    qw[20:] = 0
+    cq = ops.latent_inputs(*args, buf[:, 16:48], qw, 20)
+    close(cq[:, :20], oracle.rms(buf[:, 16:36].double().cpu(), eps) * qw[:20].double().cpu(), dtype)
+    assert not cq[:, 20:].any()
     got = cache.view(32, row)[slots].cpu()
     kd = kv.double().cpu()
     close(got[:, :kv_rank], oracle.rms(kd[:, :kv_rank], eps) * w.double().cpu(), dtype)
