@@ -1,6 +1,6 @@
 """CLI — the cmd/main.go equivalent.
 
-    python -m agentcontrolplane_amd serve [--wal PATH] [--model llama3-8b]
+    python -m agentcontrolplane_amd serve [--wal PATH] [--model llama3-8b | --checkpoint DIR]
         [--device cuda|cpu|none] [--port 8082] [--auto-approve]
     python -m agentcontrolplane_amd apply -f manifest.yaml [-f more.yaml]
         [--server http://127.0.0.1:8082]
@@ -20,10 +20,30 @@ import json
 import sys
 
 
+def _engine_config(args, device: str):
+    """serve's engine: --model names a preset; without it a checkpoint whose
+    config.json names a known architecture brings its own configuration."""
+    from .engine.config import EngineConfig
+    from .models.configs import read_architecture
+
+    if args.model:
+        model = args.model if device == "cuda" else "tiny"
+    elif args.checkpoint and read_architecture(args.checkpoint):
+        model = "auto"
+    else:
+        model = "llama3-8b" if device == "cuda" else "tiny"
+    return EngineConfig(
+        model=model,
+        dtype=args.dtype,
+        device=device,
+        checkpoint_path=args.checkpoint,
+        num_kv_blocks=args.kv_blocks,
+    )
+
+
 def cmd_serve(args) -> None:
     import uvicorn
 
-    from .engine.config import EngineConfig
     from .runtime import ControlPlane
 
     engine = None
@@ -31,13 +51,7 @@ def cmd_serve(args) -> None:
         import torch
 
         device = args.device or ("cuda" if torch.cuda.is_available() else "cpu")
-        model = args.model if device == "cuda" else "tiny"
-        ecfg = EngineConfig(
-            model=model,
-            device=device,
-            checkpoint_path=args.checkpoint,
-            num_kv_blocks=args.kv_blocks,
-        )
+        ecfg = _engine_config(args, device)
         n_gpus = getattr(args, "gpus", 1) or 1
         if device.startswith("cuda") and n_gpus > 1:
             # DP request routing across this node's GPUs (parallel/router)
@@ -200,7 +214,11 @@ def main() -> None:
     s.add_argument("--host", default="127.0.0.1")
     s.add_argument("--port", type=int, default=8082)
     s.add_argument("--wal", default=None, help="WAL path for durable state")
-    s.add_argument("--model", default="llama3-8b")
+    s.add_argument("--model", default=None,
+                   help="preset name; default: the checkpoint's config.json if it "
+                   "names a known architecture, else llama3-8b")
+    s.add_argument("--dtype", default=None, choices=["bfloat16", "float32"],
+                   help="override the model's dtype")
     s.add_argument("--checkpoint", default=None, help="safetensors checkpoint dir")
     s.add_argument("--device", default=None, help="cuda | cpu | none (no engine)")
     s.add_argument("--kv-blocks", type=int, default=None)

@@ -158,8 +158,9 @@ class FetolixForCausalLM:
         self.layers: List[FetolixLayer] = [
             FetolixLayer(s, cfg, tp_rank, tp_world) for s in cfg.layers
         ]
-        # one rotation table per distinct rotation
-        positions = min(ecfg.max_model_len, cfg.max_position)
+        # one rotation table per distinct rotation; a speculative step may run
+        # one position past the limit
+        positions = min(ecfg.max_model_len, cfg.max_position) + 1
         tables: Dict[Tuple[float, int], torch.Tensor] = {}
         for layer in self.layers:
             key = (layer.mixer.spec.rope_base, layer.mixer.spec.rot_dim)
