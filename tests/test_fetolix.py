@@ -68,6 +68,16 @@ CONFIGS = {
         ],
         "loop": {"start": 0, "stop": 2, "times": 2}, "token_side": {"dim": 16},
     },
+    # beyond the matrix-core kernels' sizes
+    "large": {
+        "architecture": "Fetolix", "vocab": 290, "width": 64, "norm": {"eps": 1e-3},
+        "layers": [
+            full(heads=2, dim=130, rot=80, vdim=20, rank=40, base=1e4, scale=0.1, ff=64),
+            win(heads=3, dim=24, rot=16, vdim=260, rank=530, base=1e5, q_rank=24, window=40,
+                scale=0.2, ff=16),
+        ],
+        "loop": {"start": 0, "stop": 1, "times": 2}, "token_side": {"dim": 3},
+    },
     # nothing repeated: a loop of one pass, a window of one token, one head
     "ones": {
         "architecture": "Fetolix", "vocab": 270, "width": 16, "norm": {"eps": 0.5},
