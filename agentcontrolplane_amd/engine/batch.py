@@ -21,6 +21,7 @@ class SeqMeta:
     ctx_len: int          # cached length before this step (causal offset)
     block_table: List[int]
     needs_logits: bool    # prompt fully processed after this chunk
+    state_slot: int = 0   # recurrent state (models that have one)
 
 
 @dataclasses.dataclass
@@ -38,6 +39,8 @@ class FlatBatch:
     # decode rows), aligned with sample_seq_ids
     logit_rows: torch.Tensor
     sample_seq_ids: List[int]
+    # [Bd] int32 — recurrent state per decode row (models that have one)
+    decode_state_slots: Optional[torch.Tensor] = None
 
     # speculative step: decode-row tokens come from the PREVIOUS step's
     # GPU-resident sampled tokens (gathered by these row indices) instead of
@@ -107,7 +110,7 @@ def batch_to_wire(batch: FlatBatch) -> dict:
         v = h.get(name)
         return v if v is not None else (tensor.tolist() if tensor is not None else None)
 
-    return {
+    wire = {
         "token_ids": of("token_ids", batch.token_ids),
         "positions": of("positions", batch.positions),
         "slot_mapping": of("slot_mapping", batch.slot_mapping),
@@ -122,18 +125,23 @@ def batch_to_wire(batch: FlatBatch) -> dict:
         "logit_rows": of("logit_rows", batch.logit_rows),
         "sample_seq_ids": batch.sample_seq_ids,
     }
+    if "state_slots" in h:  # models with recurrent state: chunks', then decode rows'
+        wire["state_slots"] = h["state_slots"]
+    return wire
 
 
 def batch_from_wire(d: dict, device) -> FlatBatch:
     t = lambda x: torch.tensor(x, device=device, dtype=torch.long)  # noqa: E731
+    n = len(d["prefills"])
+    slots = d.get("state_slots")
     return FlatBatch(
         token_ids=t(d["token_ids"]),
         positions=t(d["positions"]),
         slot_mapping=t(d["slot_mapping"]),
         prefills=[
             SeqMeta(seq_id=s, query_len=q, seq_len=sl, ctx_len=c, block_table=bt,
-                    needs_logits=nl)
-            for (s, q, sl, c, bt, nl) in d["prefills"]
+                    needs_logits=nl, state_slot=slots[i] if slots else 0)
+            for i, (s, q, sl, c, bt, nl) in enumerate(d["prefills"])
         ],
         num_prefill_tokens=d["num_prefill_tokens"],
         decode_seq_ids=d["decode_seq_ids"],
@@ -145,6 +153,7 @@ def batch_from_wire(d: dict, device) -> FlatBatch:
         ),
         logit_rows=t(d["logit_rows"]),
         sample_seq_ids=d["sample_seq_ids"],
+        decode_state_slots=t(slots[n:]).int() if slots and d["decode_seq_ids"] else None,
     )
 
 
@@ -160,6 +169,7 @@ class PrefillMeta:
     tile_seq: torch.Tensor      # [num_tiles] int32
     tile_q0: torch.Tensor       # [num_tiles] int32
     tile_q: int
+    state_slots: torch.Tensor   # [num_seqs] int32
     # keys gathered into one buffer (window given): the position of a
     # sequence's first gathered key, its row in the buffer
     key_first: Optional[torch.Tensor] = None
@@ -183,7 +193,7 @@ class PrefillMeta:
         for m in prefills:
             starts.append(starts[-1] + m.query_len)
         max_blocks = max((len(m.block_table) for _, m in picked), default=1)
-        tables, seq_lens, ctx_lens, row_starts = [], [], [], []
+        tables, seq_lens, ctx_lens, row_starts, slots = [], [], [], [], []
         tile_seq, tile_q0 = [], []
         key_first, key_starts, num_keys, max_keys = [], [], 0, 0
         for n, (i, m) in enumerate(picked):
@@ -191,6 +201,7 @@ class PrefillMeta:
             seq_lens.append(m.seq_len)
             ctx_lens.append(m.ctx_len)
             row_starts.append(starts[i] - row_base)
+            slots.append(m.state_slot)
             for q0 in range(0, m.query_len * rows_per_token, tile_q):
                 tile_seq.append(n)
                 tile_q0.append(q0)
@@ -212,6 +223,7 @@ class PrefillMeta:
             tile_seq=t("ts", tile_seq),
             tile_q0=t("tq", tile_q0),
             tile_q=tile_q,
+            state_slots=t("st", slots),
             key_first=t("kf", key_first) if window is not None else None,
             key_starts=t("ks", key_starts) if window is not None else None,
             num_keys=num_keys,

@@ -9,7 +9,8 @@ reads it (models/configs.py).
 from __future__ import annotations
 
 import dataclasses
-from typing import Optional, Tuple
+import math
+from typing import Optional, Tuple, Union
 
 
 @dataclasses.dataclass(frozen=True)
@@ -28,6 +29,57 @@ class LatentAttentionSpec:
     window: Optional[int] = None  # keys visible, self included; None = all
     head_gate: bool = True        # sigmoid gate per head on the output
 
+    def params(self, w: int) -> int:
+        qdim = self.heads * (self.dim + self.rot_dim)
+        n = self.q_rank * (w + 1 + qdim) if self.q_rank else w * qdim
+        n += w * (self.kv_rank + self.rot_dim) + self.kv_rank
+        n += self.kv_rank * self.heads * (self.dim + self.vdim) + self.heads * self.vdim * w
+        return n + (w * self.heads if self.head_gate else 0)
+
+
+@dataclasses.dataclass(frozen=True)
+class GroupedAttentionSpec:
+    """Attention without rotation over cached keys and values shared by groups of
+    query heads (models/grouped_attention.py)."""
+
+    heads: int
+    kv_heads: int
+    dim: int                        # query/key size per head
+    vdim: int                       # value size per head
+    scale: float                    # on the scores
+    softcap: Optional[float] = None  # scores -> softcap * tanh(score / softcap)
+    window: Optional[int] = None    # keys visible, self included; None = all
+    keep_first: int = 0             # first tokens that stay visible beyond the window
+    bias: bool = True               # on the query, key and value projections
+    sink: bool = True               # learned logit per head in the denominator
+    kv_from: Optional[int] = None   # the layer whose keys and values are used
+
+    def params(self, w: int) -> int:
+        q, o = self.heads * self.dim, self.heads * self.vdim
+        kv = 0 if self.kv_from is not None else self.kv_heads * (self.dim + self.vdim)
+        return (q + kv) * (w + self.bias) + o * w + (self.heads if self.sink else 0)
+
+
+@dataclasses.dataclass(frozen=True)
+class ChannelDeltaSpec:
+    """Gated delta rule with one decay per head and key channel
+    (models/channel_delta.py)."""
+
+    heads: int                      # value heads, one state each
+    kv_heads: int                   # query/key heads
+    dim: int                        # query/key size per head
+    vdim: int                       # value size per head
+    conv: int                       # taps of the short convolutions
+    decay_rank: int                 # inner size of the decay projection
+    gate_rank: int                  # inner size of the output gate's projection
+    unit_eps: float = 1e-6          # in the unit vectors' sum of squares
+
+    def params(self, w: int) -> int:
+        qk, v = 2 * self.kv_heads * self.dim, self.heads * self.vdim
+        n = (qk + v) * (w + self.conv) + self.heads * (w + 1) + self.vdim + v * w
+        n += self.decay_rank * (w + self.heads * self.dim) + self.heads * self.dim
+        return n + self.gate_rank * (w + v)
+
 
 @dataclasses.dataclass(frozen=True)
 class ClampedGluSpec:
@@ -39,10 +91,16 @@ class ClampedGluSpec:
     offset: float = 1.0
 
 
+def silu_glu(width: int) -> ClampedGluSpec:
+    """silu(gate) * up."""
+    return ClampedGluSpec(width, limit=math.inf, alpha=1.0, offset=0.0)
+
+
 @dataclasses.dataclass(frozen=True)
 class LayerSpec:
-    mixer: LatentAttentionSpec
+    mixer: Union[LatentAttentionSpec, GroupedAttentionSpec, ChannelDeltaSpec]
     mlp: Optional[ClampedGluSpec] = None
+    sandwich: bool = False  # mixer, then mlp, each normed on its way in and out
 
 
 @dataclasses.dataclass(frozen=True)
@@ -82,6 +140,14 @@ class ModelConfig:
     loop: Optional[LoopSpec] = None
     # per-layer token embedding: dims per layer, 0 = none
     token_side_dim: int = 0
+    # on every sublayer's output
+    residual_mult: float = 1.0
+    # what a layer hands on is a learned mix of all layers' results so far
+    depth_average: bool = False
+    # sinusoidal positions added to the embedding: the base, None = none
+    position_base: Optional[float] = None
+    # logits -> cap * tanh(logits / cap)
+    logit_softcap: Optional[float] = None
 
     @property
     def layer_runs(self) -> Tuple[Tuple[int, bool], ...]:
@@ -117,15 +183,13 @@ class ModelConfig:
     def _listed_layer_params(self) -> int:
         w, v = self.hidden_size, self.vocab_size
         total = v * w + w
-        for layer in self.layers:
-            m = layer.mixer
-            qdim = m.heads * (m.dim + m.rot_dim)
-            total += w
-            total += m.q_rank * (w + 1 + qdim) if m.q_rank else w * qdim
-            total += w * (m.kv_rank + m.rot_dim) + m.kv_rank
-            total += m.kv_rank * m.heads * (m.dim + m.vdim) + m.heads * m.vdim * w
-            total += w * m.heads if m.head_gate else 0
+        for i, layer in enumerate(self.layers):
+            total += w + layer.mixer.params(w)
             total += 3 * w * layer.mlp.width if layer.mlp else 0
+            if layer.sandwich:
+                total += w + (2 * w if layer.mlp else 0)
+            if self.depth_average:
+                total += i + 2
             if self.token_side_dim:
                 total += 2 * w * self.token_side_dim + w + v * self.token_side_dim
         return total + (2 * w * w if self.loop else 0)
@@ -154,6 +218,35 @@ def _fetolix(name: str, *, width: int, heads: int, layers: int, ff: int,
             LayerSpec(mixer(i), ClampedGluSpec(ff, limit)) for i in range(layers)
         ),
         loop=loop, token_side_dim=side, **kw,
+    )
+
+
+def _tezinex(name: str, *, width: int, layers: int, ff: int, heads: int, kv_heads: int,
+             dim: int, vdim: int, window: int, keep_first: int, d_heads: int, d_kv_heads: int,
+             d_dim: int, d_vdim: int, rank: int, vocab: int, conv: int = 4,
+             attn_every: int = 4, share: int = 2, **kw) -> ModelConfig:
+    """Every ``attn_every``-th layer is windowed attention, the others delta
+    layers; of ``share`` consecutive attention layers all use the first one's keys."""
+    delta = ChannelDeltaSpec(d_heads, d_kv_heads, d_dim, d_vdim, conv, rank, rank)
+
+    def mixer(i: int):
+        nth, at = divmod(i, attn_every)
+        if at != attn_every - 1:
+            return delta
+        owner = (nth - nth % share) * attn_every + attn_every - 1
+        return GroupedAttentionSpec(
+            heads=heads, kv_heads=kv_heads, dim=dim, vdim=vdim, scale=dim ** -0.5,
+            softcap=50.0, window=window, keep_first=keep_first,
+            kv_from=None if owner == i else owner,
+        )
+
+    return ModelConfig(
+        name=name, architecture="Tezinex", vocab_size=vocab, hidden_size=width,
+        intermediate_size=ff, num_layers=layers, num_heads=heads, num_kv_heads=kv_heads,
+        head_dim=dim, tie_embeddings=True, residual_mult=0.5, depth_average=True,
+        position_base=10000.0, logit_softcap=30.0,
+        layers=tuple(LayerSpec(mixer(i), silu_glu(ff), sandwich=True) for i in range(layers)),
+        **kw,
     )
 
 
@@ -215,6 +308,24 @@ PRESETS = {
         q_rank=20, dim=12, rot_dim=8, vdim=10, window=19, vocab=300, side=6,
         limit=1.5, loop=LoopSpec(1, 3, 2), full_every=2, max_position=4096,
         dtype="float32",
+    ),
+    # Tezinex at the layer sizes of an 8B-class dense model (random weights):
+    # width, heads and feed-forward of llama3-8b
+    "tezinex-8b": _tezinex(
+        "tezinex-8b", width=4096, layers=32, ff=14336, heads=32, kv_heads=8, dim=128,
+        vdim=128, window=4096, keep_first=16, d_heads=32, d_kv_heads=32, d_dim=128,
+        d_vdim=128, rank=128, vocab=128256,
+    ),
+    # half the width, 16 heads
+    "tezinex-2b": _tezinex(
+        "tezinex-2b", width=2048, layers=20, ff=8192, heads=16, kv_heads=8, dim=128,
+        vdim=128, window=1024, keep_first=4, d_heads=16, d_kv_heads=16, d_dim=128,
+        d_vdim=128, rank=64, vocab=32000,
+    ),
+    "tiny-tezinex": _tezinex(
+        "tiny-tezinex", width=44, layers=6, ff=60, heads=6, kv_heads=3, dim=10, vdim=14,
+        window=21, keep_first=3, d_heads=4, d_kv_heads=2, d_dim=12, d_vdim=18, rank=7,
+        vocab=300, conv=3, attn_every=2, max_position=4096, dtype="float32",
     ),
     # tiny GPU config: real head_dim/GQA shape for the CDNA4 kernels at
     # test scale (kernels require head_dim 128)
@@ -300,6 +411,9 @@ class EngineConfig:
     # explicit block count for tests
     gpu_memory_utilization: float = 0.85
     num_kv_blocks: Optional[int] = None
+    # models with recurrent state: sequences that hold a state at a time (None:
+    # max_batch_size, less if they would take over half of the memory budget)
+    num_state_slots: Optional[int] = None
     max_batch_size: int = 2048
     # chunked-prefill token budget per step: 16384 measured ~7% faster
     # wave p50 than 8192 at 1k concurrency (r02 A/B, gpurun_out/bench3b) —

@@ -30,6 +30,7 @@ from .config import EngineConfig
 from .kv import make_block_manager
 from .request import ChatResult, InferenceRequest, SamplingParams
 from .scheduler import Scheduler, Sequence
+from .state import StateSlots
 from .tokenizer import N_SPECIAL, ByteTokenizer, IdTokenizer
 
 
@@ -78,13 +79,18 @@ class InferenceEngine:
             else:
                 self.model = create_model(self.mcfg, config, config.device)
                 self._init_weights()
+        self.states = None
+        if getattr(self.model, "state_slot_bytes", 0):
+            self.states = StateSlots(self._size_state_pool())
+            # +1 scratch slot: hipGraph decode padding rows
+            self.model.allocate_state(self.states.num_slots + 1)
         num_blocks = self._size_kv_pool()
         # +1 scratch block: hipGraph decode padding rows write their KV there
         self.model.allocate_kv_cache(num_blocks + 1, config.kv_block_size)
         self.bm = make_block_manager(
             num_blocks, config.kv_block_size, prefer_native=True
         )
-        self.scheduler = Scheduler(config, self.bm, self.device)
+        self.scheduler = Scheduler(config, self.bm, self.device, self.states)
         if getattr(self.tokenizer, "token_bytes", None) and self._live > N_SPECIAL:
             # BPE tokenizer: token-trie constrained decoding (token_grammar)
             from .token_grammar import TokenGrammar, TokenTrie
@@ -134,6 +140,7 @@ class InferenceEngine:
                 max_blocks_per_seq=max_blocks_per_seq,
                 scratch_block=num_blocks,
                 kv_block_size=config.kv_block_size,
+                scratch_state=self.states.num_slots if self.states else None,
             )
         self._ctx_limit = min(config.max_model_len, self.mcfg.max_position)
         self._gen = torch.Generator(device=self.device.type)
@@ -215,18 +222,30 @@ class InferenceEngine:
 
     # ------------------------------------------------------------- sizing
 
+    def _memory_budget(self) -> int:
+        """Bytes the caches may take on the GPU."""
+        free, total = torch.cuda.mem_get_info(self.device)
+        budget = int(total * self.cfg.gpu_memory_utilization) - (total - free)
+        # keep headroom for activations: 4 GB or 5% of total
+        return budget - max(4 << 30, int(0.05 * total))
+
+    def _size_state_pool(self) -> int:
+        if self.cfg.num_state_slots is not None:
+            return self.cfg.num_state_slots
+        n = self.cfg.max_batch_size
+        if self.device.type != "cuda":
+            return n
+        return int(max(1, min(n, self._memory_budget() // 2 // self.model.state_slot_bytes)))
+
     def _size_kv_pool(self) -> int:
         if self.cfg.num_kv_blocks is not None:
             return self.cfg.num_kv_blocks
         if self.device.type != "cuda":
             return 1024
-        free, total = torch.cuda.mem_get_info(self.device)
-        budget = int(total * self.cfg.gpu_memory_utilization) - (total - free)
-        block_bytes = self.model.kv_block_bytes(self.cfg.kv_block_size)
-        # keep headroom for activations: 4 GB or 5% of total
-        headroom = max(4 << 30, int(0.05 * total))
-        n = max(64, (budget - headroom) // block_bytes)
-        return int(n)
+        block_bytes = max(1, self.model.kv_block_bytes(self.cfg.kv_block_size))
+        # block and slot numbers are 32-bit in the kernels' metadata
+        most = (1 << 31) // self.cfg.kv_block_size - 2
+        return int(min(most, max(64, self._memory_budget() // block_bytes)))
 
     # ----------------------------------------------------------- lifecycle
 
@@ -754,6 +773,7 @@ class InferenceEngine:
                     s.grammar.advance(self._eot)
                     s.request.output_ids.pop()  # EOT is not part of the JSON
                     s.output_ids.pop()
+                    s.end_token = tok
                     self._m["requests_completed"] += 1
                     self.scheduler.finish_seq(s, "tool_calls")
                     continue
@@ -786,6 +806,7 @@ class InferenceEngine:
             if tok == self._eot:
                 s.request.output_ids.pop()
                 s.output_ids.pop()
+                s.end_token = tok
                 self._m["requests_completed"] += 1
                 self.scheduler.finish_seq(s, "stop")
                 continue
@@ -831,6 +852,8 @@ class InferenceEngine:
         m["uptime_s"] = elapsed
         m["tokens_per_s"] = self._m["generated_tokens"] / max(1e-9, elapsed)
         m["kv_occupancy"] = self.bm.used_blocks / max(1, self.bm.num_blocks)
+        if self.states is not None:
+            m["state_slots_free"] = self.states.free
         m["running_seqs"] = len(self.scheduler.running)
         m["waiting_seqs"] = len(self.scheduler.waiting)
         m["retired_seqs"] = len(self.scheduler.retired)

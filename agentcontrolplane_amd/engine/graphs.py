@@ -9,7 +9,8 @@ inputs — one launch instead of ~400.
 
 Buckets pad the decode batch up to {4, 8, …, max}; padding rows point at a
 dedicated scratch KV block (beyond the allocator's range) so their cache
-writes land nowhere meaningful, and their logits are never sampled.
+writes land nowhere meaningful, and their logits are never sampled.  Models
+with recurrent state have a scratch slot for them likewise.
 """
 from __future__ import annotations
 
@@ -24,11 +25,14 @@ BUCKETS = [4, 8, 16, 32, 64, 96, 128, 192, 256, 384, 512, 768, 1024]
 
 class DecodeGraphRunner:
     def __init__(self, model, max_batch: int, max_blocks_per_seq: int,
-                 scratch_block: int, kv_block_size: int):
+                 scratch_block: int, kv_block_size: int,
+                 scratch_state: Optional[int] = None):
         self.model = model
         self.device = model.device
         self.max_blocks = max_blocks_per_seq
         self.scratch_slot = scratch_block * kv_block_size
+        # state slot of padding rows; None: the model keeps no state
+        self.scratch_state = scratch_state
         self.buckets = [b for b in BUCKETS if b <= max_batch]
         if not self.buckets or self.buckets[-1] < max_batch:
             self.buckets.append(max_batch)
@@ -51,6 +55,10 @@ class DecodeGraphRunner:
             "seq_lens": torch.ones(b, dtype=torch.int32, device=dev),
             "logit_rows": torch.arange(b, dtype=torch.long, device=dev),
         }
+        if self.scratch_state is not None:
+            static["state_slots"] = torch.full(
+                (b,), self.scratch_state, dtype=torch.int32, device=dev
+            )
         batch = FlatBatch(
             token_ids=static["token_ids"],
             positions=static["positions"],
@@ -62,6 +70,7 @@ class DecodeGraphRunner:
             decode_seq_lens=None,
             logit_rows=static["logit_rows"],
             sample_seq_ids=list(range(b)),
+            decode_state_slots=static.get("state_slots"),
         )
         # the attention op reads the int32 views; install the static ones
         batch._decode_tables_i32 = static["block_tables"]
@@ -102,6 +111,10 @@ class DecodeGraphRunner:
         if n < b:
             st["slot_mapping"][n:].fill_(self.scratch_slot)
             st["seq_lens"][n:].fill_(1)
+            if self.scratch_state is not None:
+                st["state_slots"][n:].fill_(self.scratch_state)
+        if self.scratch_state is not None:
+            st["state_slots"][:n].copy_(batch.decode_state_slots, non_blocking=True)
         tables = batch.decode_tables_i32()
         w = tables.shape[1]
         st["block_tables"][:n, :w].copy_(tables, non_blocking=True)

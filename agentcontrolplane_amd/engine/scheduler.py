@@ -25,6 +25,7 @@ from .batch import FlatBatch, SeqMeta
 from .config import EngineConfig
 from .grammar import ToolCallGrammar
 from .request import InferenceRequest
+from .state import StateSlots
 
 WAITING, PREFILL, DECODE, FINISHED = "waiting", "prefill", "decode", "finished"
 
@@ -53,7 +54,7 @@ def worst_case_output_tokens(request: InferenceRequest) -> int:
 class Sequence:
     __slots__ = (
         "seq_id", "request", "prompt_ids", "output_ids", "num_processed",
-        "state", "grammar", "arrival",
+        "state", "grammar", "arrival", "end_token",
     )
 
     def __init__(self, seq_id: int, request: InferenceRequest, grammar_factory=None):
@@ -64,6 +65,9 @@ class Sequence:
         self.num_processed = 0      # prompt tokens already in the KV cache
         self.state = WAITING
         self.grammar: Optional[ToolCallGrammar] = None
+        # a sampled end token: not part of the output, yet a speculative step
+        # may have run it through the model
+        self.end_token: Optional[int] = None
         self.arrival = request.submit_time
         if request.constrained:
             if grammar_factory is not None:
@@ -95,11 +99,14 @@ class SchedulerOutput:
 
 
 class Scheduler:
-    def __init__(self, config: EngineConfig, block_manager, device):
+    def __init__(self, config: EngineConfig, block_manager, device,
+                 states: Optional[StateSlots] = None):
         from .stage import HostStager
 
         self.cfg = config
         self.bm = block_manager
+        # slots of recurrent state; None: the model keeps none
+        self.states = states
         self.device = torch.device(device)
         self.stager = HostStager(device)
         # set by the engine for BPE tokenizers (token-trie constrained
@@ -259,11 +266,18 @@ class Scheduler:
                 avail += self.bm.free_blocks - before
             if fit_chunk(0, 0, 1) <= 0:
                 break
-            self.waiting.pop(0)
             adopted = self._try_adopt(s)
             if not adopted:
-                self.bm.add_seq(s.seq_id)
+                if self.states is not None:
+                    before = self.bm.free_blocks
+                    while not self.states.free and self._evict_one_retired():
+                        pass
+                    avail += self.bm.free_blocks - before
+                    if not self.states.free:
+                        break
+                self._add_seq(s)
                 s.num_processed = 0
+            self.waiting.pop(0)
             cur = self.bm.seq_len(s.seq_id)
             have = len(self.bm.block_table(s.seq_id))
             want = min(len(s.prompt_ids) - s.num_processed, budget)
@@ -325,7 +339,7 @@ class Scheduler:
                     raise RuntimeError("more live sequences than max_batch_size")
                 self.waiting.remove(s)
                 self.running.append(s)
-                self.bm.add_seq(s.seq_id)
+                self._add_seq(s)
             index[s.seq_id] = n
             wanted[s.seq_id] = want
             if count == 1 and s.num_processed > 0:
@@ -362,10 +376,9 @@ class Scheduler:
         for s, chunk in prefills:
             start = s.num_processed
             toks = s.prompt_ids[start : start + chunk]
-            slots = self.bm.append_tokens(s.seq_id, chunk)
             token_ids.extend(toks)
             positions.extend(range(start, start + chunk))
-            slot_mapping.extend(slots)
+            slot_mapping.extend(self.bm.append_tokens(s.seq_id, chunk))
             s.num_processed += chunk
             done = s.num_processed == len(s.prompt_ids)
             prefill_metas.append(
@@ -376,6 +389,7 @@ class Scheduler:
                     ctx_len=start,
                     block_table=list(self.bm.block_table(s.seq_id)),
                     needs_logits=done,
+                    state_slot=self.states.slot(s.seq_id) if self.states else 0,
                 )
             )
             rows = wanted[s.seq_id] if wanted is not None else [chunk - 1] if done else []
@@ -388,6 +402,8 @@ class Scheduler:
 
         decode_block_tables = None
         decode_seq_lens = None
+        decode_state_slots = None
+        decode_slots: List[int] = []
         decode_tables_i32 = None
         decode_ids: List[int] = []
         spec_rows: List[int] = []
@@ -401,10 +417,9 @@ class Scheduler:
                 else:
                     tok = s.output_ids[-1] if s.output_ids else s.prompt_ids[-1]
                     pos = s.total_len - 1
-                slots = self.bm.append_tokens(s.seq_id, 1)
                 token_ids.append(tok)
                 positions.append(pos)
-                slot_mapping.extend(slots)
+                slot_mapping.extend(self.bm.append_tokens(s.seq_id, 1))
                 lens.append(pos + 1)
                 logit_rows.append(row)
                 sample_seq_ids.append(s.seq_id)
@@ -427,6 +442,9 @@ class Scheduler:
                 self._decode_cache = (decode_block_tables, decode_tables_i32)
                 self._decode_cache_host = padded
             decode_seq_lens = self.stager.tensor("dlens", lens, "int64")
+            if self.states is not None:
+                decode_slots = [self.states.slot(i) for i in decode_ids]
+                decode_state_slots = self.stager.tensor("dstate", decode_slots, "int32")
 
         batch = FlatBatch(
             token_ids=self.stager.tensor("tok", token_ids, "int64"),
@@ -439,6 +457,7 @@ class Scheduler:
             decode_seq_lens=decode_seq_lens,
             logit_rows=self.stager.tensor("lrow", logit_rows, "int64"),
             sample_seq_ids=sample_seq_ids,
+            decode_state_slots=decode_state_slots,
         )
         batch._stager = self.stager
         # host-side copies for the TP wire broadcast (batch_to_wire):
@@ -452,11 +471,26 @@ class Scheduler:
             if decode_block_tables is not None else None,
             "decode_seq_lens": lens if decode_seqs else None,
         }
+        if self.states is not None:
+            batch._host["state_slots"] = [m.state_slot for m in prefill_metas] + decode_slots
         if decode_tables_i32 is not None:
             batch._decode_tables_i32 = decode_tables_i32
         if spec_rows:
             batch.spec_src_rows = self.stager.tensor("spec", spec_rows, "int64")
         return batch
+
+    # ------------------------------------------------------------ storage
+
+    def _add_seq(self, seq: Sequence) -> None:
+        """Pages, and a state slot if the model keeps state."""
+        if self.states is not None:
+            self.states.acquire(seq.seq_id)
+        self.bm.add_seq(seq.seq_id)
+
+    def _free_seq(self, seq_id: int) -> None:
+        self.bm.free_seq(seq_id)
+        if self.states is not None:
+            self.states.release(seq_id)
 
     # ------------------------------------------------------------ commit
 
@@ -475,7 +509,7 @@ class Scheduler:
             if self.continuation_cache and self.bm.seq_len(seq.seq_id) >= self.cfg.kv_block_size:
                 self._retire(seq)
             else:
-                self.bm.free_seq(seq.seq_id)
+                self._free_seq(seq.seq_id)
         self._by_id.pop(seq.seq_id, None)
         seq.request.finish(reason)
 
@@ -497,10 +531,13 @@ class Scheduler:
     def _retire(self, seq: Sequence) -> None:
         tokens = tuple(seq.prompt_ids + seq.output_ids)
         cached = self.bm.seq_len(seq.seq_id)
+        if self.states is not None and seq.end_token is not None:
+            tokens += (seq.end_token,)
         tokens = tokens[:cached]
         hashes = self._prefix_hashes(tokens)
-        if not hashes:
-            self.bm.free_seq(seq.seq_id)
+        # a state serves only the continuation of exactly the tokens it covers
+        if not hashes or (self.states is not None and len(tokens) < cached):
+            self._free_seq(seq.seq_id)
             return
         self.retired[seq.seq_id] = tokens
         self._retired_hashes[seq.seq_id] = hashes
@@ -526,7 +563,7 @@ class Scheduler:
         old_id = next(iter(self.retired))
         self.retired.pop(old_id)
         self._unindex(old_id)
-        self.bm.free_seq(old_id)
+        self._free_seq(old_id)
         return True
 
     def _reclaim(self, need_blocks: int) -> None:
@@ -538,7 +575,11 @@ class Scheduler:
         prefix (refcounted, full blocks only); returns True if the sequence
         was registered with the block manager.  Retirees stay cached so any
         number of requests reuse them — the same task's next turn (long
-        match) or sibling tasks sharing a system prompt (short match)."""
+        match) or sibling tasks sharing a system prompt (short match).
+
+        A recurrent state cannot be cut back to a shared prefix: with states,
+        only a retiree whose every token begins the prompt is taken, pages and
+        state, and is a retiree no longer."""
         bs = self.cfg.kv_block_size
         if not self.continuation_cache or len(seq.prompt_ids) <= bs:
             return False
@@ -550,6 +591,14 @@ class Scheduler:
             for cand in self._prefix_index.get(hashes[b], ()):  # longest first
                 toks = self.retired[cand]
                 want = (b + 1) * bs
+                if self.states is not None:
+                    n = len(toks)
+                    if n // bs != b + 1 or n >= len(seq.prompt_ids):
+                        continue
+                    if toks != tuple(seq.prompt_ids[:n]):
+                        continue
+                    self._take_over(seq, cand)
+                    return True
                 if len(toks) >= want and toks[:want] == tuple(seq.prompt_ids[:want]):
                     best_id, n_blocks = cand, b + 1
                     break
@@ -563,11 +612,21 @@ class Scheduler:
         self.continuation_tokens_saved += n_blocks * bs
         return True
 
+    def _take_over(self, seq: Sequence, old_id: int) -> None:
+        """seq goes on from everything a retired sequence has cached."""
+        n = len(self.retired.pop(old_id))
+        self._unindex(old_id)
+        self.bm.adopt_prefix(seq.seq_id, old_id, len(self.bm.block_table(old_id)), n)
+        self.states.transfer(seq.seq_id, old_id)
+        seq.num_processed = n
+        self.continuation_hits += 1
+        self.continuation_tokens_saved += n
+
     def _preempt(self, seq: Sequence) -> None:
         """Recompute-style preemption: blocks freed, prompt grows to include
         generated tokens, back to the head of the waiting queue."""
         if self.bm.has_seq(seq.seq_id):
-            self.bm.free_seq(seq.seq_id)
+            self._free_seq(seq.seq_id)
         seq.prompt_ids = seq.prompt_ids + seq.output_ids
         # keep outputs in the request — generation continues from here
         seq.output_ids = []
@@ -594,6 +653,6 @@ class Scheduler:
         if seq in self.waiting:
             self.waiting.remove(seq)
         if self.bm.has_seq(seq.seq_id):
-            self.bm.free_seq(seq.seq_id)
+            self._free_seq(seq.seq_id)
         self._by_id.pop(seq.seq_id, None)
         seq.request.fail(err)

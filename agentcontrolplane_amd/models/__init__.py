@@ -1,12 +1,14 @@
 from .fetolix import FetolixForCausalLM  # noqa: F401
 from .llama import LlamaForCausalLM  # noqa: F401
 from .mixtral import MixtralForCausalLM  # noqa: F401
+from .tezinex import TezinexForCausalLM  # noqa: F401
 
 #: ModelConfig.architecture -> model class
 MODEL_CLASSES = {
     "llama": LlamaForCausalLM,
     "mixtral": MixtralForCausalLM,
     "Fetolix": FetolixForCausalLM,
+    "Tezinex": TezinexForCausalLM,
 }
 
 

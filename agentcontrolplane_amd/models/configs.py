@@ -7,11 +7,16 @@ from __future__ import annotations
 
 import json
 import os
-from typing import Callable, Dict, Optional
+from typing import Callable, Dict, Optional, Tuple
 
 from ..engine.config import (
-    ClampedGluSpec, LatentAttentionSpec, LayerSpec, LoopSpec, ModelConfig,
+    ChannelDeltaSpec, ClampedGluSpec, GroupedAttentionSpec, LatentAttentionSpec, LayerSpec,
+    LoopSpec, ModelConfig, silu_glu,
 )
+from .weights import tensor_shape
+
+#: a tensor's shape in the checkpoint, by name: for sizes only the weights have
+Shape = Callable[[str], Tuple[int, ...]]
 
 #: the rotation tables bound positions; the design itself sets no limit, so
 #: the engine's max_model_len decides
@@ -44,7 +49,7 @@ def _fetolix_mlp(mlp: Optional[dict]) -> Optional[ClampedGluSpec]:
     return ClampedGluSpec(width=mlp["ff"], limit=mlp["limit"])
 
 
-def _fetolix(d: dict) -> ModelConfig:
+def _fetolix(d: dict, shape: Shape) -> ModelConfig:
     layers = []
     for entry in d["layers"]:
         if entry["type"] not in _FETOLIX_MIXERS:
@@ -67,7 +72,71 @@ def _fetolix(d: dict) -> ModelConfig:
     )
 
 
-CONFIG_READERS: Dict[str, Callable[[dict], ModelConfig]] = {"Fetolix": _fetolix}
+def _channel_delta(m: dict, shape: Shape, p: str) -> ChannelDeltaSpec:
+    return ChannelDeltaSpec(
+        heads=m["heads"], kv_heads=m["kv_heads"], dim=m["dim"], vdim=m["vdim"],
+        conv=m["conv"], decay_rank=shape(p + "a1")[0], gate_rank=shape(p + "g1")[0],
+    )
+
+
+def _grouped_attention(m: dict, shape: Shape, p: str) -> GroupedAttentionSpec:
+    return GroupedAttentionSpec(
+        heads=m["heads"], kv_heads=m["kv_heads"], dim=m["dim"], vdim=m["vdim"],
+        scale=m["scale"], softcap=m["softcap"], window=m["mask"]["size"],
+        keep_first=m["mask"]["keep_first"], kv_from=m.get("kv_from"),
+    )
+
+
+#: Tezinex mixer type -> spec reader
+_TEZINEX_MIXERS = {"channel_delta": _channel_delta, "attention": _grouped_attention}
+
+
+def _tezinex_mlp(mlp: Optional[dict]) -> Optional[ClampedGluSpec]:
+    if mlp is None:
+        return None
+    if mlp["kind"] != "dense":
+        raise ValueError(f"unknown feed-forward kind {mlp['kind']!r}")
+    return silu_glu(mlp["ff"])
+
+
+def _check_borrowed_keys(layers) -> None:
+    for i, layer in enumerate(layers):
+        j = getattr(layer.mixer, "kv_from", None)
+        if j is None:
+            continue
+        m, owner = layer.mixer, layers[j].mixer if 0 <= j < i else None
+        if not isinstance(owner, GroupedAttentionSpec) or owner.kv_from is not None:
+            raise ValueError(f"layer {i}: layer {j} has no keys and values to use")
+        if (m.kv_heads, m.dim, m.vdim) != (owner.kv_heads, owner.dim, owner.vdim):
+            raise ValueError(f"layer {i}: its key/value heads differ from layer {j}'s")
+
+
+def _tezinex(d: dict, shape: Shape) -> ModelConfig:
+    layers = []
+    for i, entry in enumerate(d["layers"]):
+        if entry["type"] not in _TEZINEX_MIXERS:
+            raise ValueError(f"unknown mixer type {entry['type']!r}")
+        m = _TEZINEX_MIXERS[entry["type"]](entry["mixer"], shape, f"l{i}.mix.")
+        if m.heads % m.kv_heads:
+            raise ValueError(f"layer {i}: kv_heads must divide heads")
+        layers.append(LayerSpec(mixer=m, mlp=_tezinex_mlp(entry.get("mlp")), sandwich=True))
+    _check_borrowed_keys(layers)
+    first = layers[0].mixer
+    return ModelConfig(
+        name="Tezinex", architecture="Tezinex", vocab_size=d["vocab"],
+        hidden_size=d["width"], num_layers=len(layers), num_heads=first.heads,
+        num_kv_heads=first.kv_heads, head_dim=first.dim,
+        intermediate_size=max((x.mlp.width for x in layers if x.mlp), default=0),
+        rms_eps=d["norm"]["eps"], max_position=_UNBOUNDED, tie_embeddings=True,
+        layers=tuple(layers), residual_mult=d["residual_mult"], depth_average=True,
+        position_base=10000.0, logit_softcap=d["logit_softcap"],
+    )
+
+
+CONFIG_READERS: Dict[str, Callable[[dict, Shape], ModelConfig]] = {
+    "Fetolix": _fetolix,
+    "Tezinex": _tezinex,
+}
 
 
 def read_architecture(path: str) -> Optional[str]:
@@ -88,4 +157,4 @@ def read_model_config(path: str) -> ModelConfig:
         raise ValueError(
             f"{path}/config.json names architecture {name!r}; have {sorted(CONFIG_READERS)}"
         )
-    return CONFIG_READERS[name](d)
+    return CONFIG_READERS[name](d, lambda tensor: tensor_shape(path, tensor))

@@ -31,7 +31,8 @@ from .. import ops
 from ..engine.batch import FlatBatch
 from ..engine.config import EngineConfig, LayerSpec, ModelConfig
 from ..ops.reference import build_cos_sin
-from .latent_attention import Get, LatentAttention, pad_to, round_up
+from .latent_attention import LatentAttention
+from .layout import Get, pad_to, round_up
 from .llama import _dtype_of
 
 _ALIGN = 16  # rows between sections of the fused input projection

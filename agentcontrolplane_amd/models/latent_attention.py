@@ -23,28 +23,14 @@ fused output projection's input, both owned by the layer.
 """
 from __future__ import annotations
 
-from typing import Callable, Dict, List, Tuple
+from typing import Dict, List, Tuple
 
 import torch
 
 from .. import ops
 from ..engine.batch import FlatBatch
 from ..engine.config import LatentAttentionSpec
-
-Get = Callable[[str], torch.Tensor]
-
-
-def round_up(n: int, m: int) -> int:
-    return -(-n // m) * m
-
-
-def pad_to(t: torch.Tensor, *shape: int) -> torch.Tensor:
-    """Zero-pad each leading corner of t to shape."""
-    if tuple(t.shape) == tuple(shape):
-        return t
-    out = t.new_zeros(shape)
-    out[tuple(slice(0, n) for n in t.shape)] = t
-    return out
+from .layout import Get, pad_to, round_up
 
 
 class LatentAttention:

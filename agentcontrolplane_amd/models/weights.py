@@ -10,7 +10,7 @@ from __future__ import annotations
 
 import json
 import os
-from typing import Dict
+from typing import Dict, List, Tuple
 
 import torch
 
@@ -94,22 +94,33 @@ def save_checkpoint(model, path: str, max_shard_bytes: int = 4 << 30) -> None:
         json.dump(index, f)
 
 
-def _read_tensors(path: str) -> Dict[str, torch.Tensor]:
-    from safetensors.torch import load_file
-
+def _checkpoint_files(path: str) -> List[str]:
     idx_path = os.path.join(path, "model.safetensors.index.json")
     if os.path.exists(idx_path):
         with open(idx_path) as f:
             weight_map = json.load(f)["weight_map"]
-        files = sorted(set(weight_map.values()))
-    else:
-        files = sorted(
-            f for f in os.listdir(path) if f.endswith(".safetensors")
-        )
+        return sorted(set(weight_map.values()))
+    return sorted(f for f in os.listdir(path) if f.endswith(".safetensors"))
+
+
+def _read_tensors(path: str) -> Dict[str, torch.Tensor]:
+    from safetensors.torch import load_file
+
     tensors: Dict[str, torch.Tensor] = {}
-    for fname in files:
+    for fname in _checkpoint_files(path):
         tensors.update(load_file(os.path.join(path, fname)))
     return tensors
+
+
+def tensor_shape(path: str, name: str) -> Tuple[int, ...]:
+    """A tensor's shape in a safetensors directory, from the file headers."""
+    from safetensors import safe_open
+
+    for fname in _checkpoint_files(path):
+        with safe_open(os.path.join(path, fname), framework="pt") as f:
+            if name in f.keys():
+                return tuple(f.get_slice(name).get_shape())
+    raise ValueError(f"checkpoint missing {name}")
 
 
 def load_checkpoint(model, path: str) -> None:

@@ -52,12 +52,13 @@ import os
 _GEMM_MIN_M = int(os.environ.get("ACP_GEMM_MIN_M", str(1 << 30)))
 
 
-def linear(x, w):
-    """x[*, K] @ w[N, K]^T → [*, N].  Large-M bf16 shapes go to the
+def linear(x, w, bias=None):
+    """x[*, K] @ w[N, K]^T (+ bias[N]) → [*, N].  Large-M bf16 shapes go to the
     hand-written 8-phase MFMA GEMM (csrc/gemm_bf16.hip); everything else
     (decode-sized M, ragged shards, CPU) to torch.nn.functional.linear."""
     if (
         x.is_cuda
+        and bias is None
         and x.dtype == torch.bfloat16
         and x.dim() == 2
         and x.shape[0] >= _GEMM_MIN_M
@@ -65,7 +66,7 @@ def linear(x, w):
         and w.shape[1] % 128 == 0
     ):
         return _hip().gemm_bf16(x, w)
-    return torch.nn.functional.linear(x, w)
+    return torch.nn.functional.linear(x, w, bias)
 
 
 def linear_add_(y, x, w):
@@ -119,10 +120,28 @@ def layernorm(x, weight, eps: float, dtype):
     return _impl(x).layernorm(x, weight, eps, dtype)
 
 
-def residual_norm(x, y, eps: float, y_norm=None, x_norm=None, out=None):
-    """x += y, or x += rmsnorm(y) * y_norm, in the fp32 residual x; then
-    out = layernorm(x) * x_norm, or x itself without x_norm."""
-    return _impl(x).residual_norm(x, y, eps, y_norm, x_norm, out)
+def residual_norm(x, y, eps: float, y_norm=None, x_norm=None, out=None, *, center=True,
+                  offset: float = 0.0, mult: float = 1.0, depth=None, depth_coef=None):
+    """x += mult * y, or x += mult * rmsnorm(y) * y_norm, in the fp32 residual x;
+    then, with depth_coef [n + 1] (fp32), x becomes state n in ``depth``
+    [states, N, K] (fp32) and is replaced by sum_j depth_coef[j] * depth[j];
+    then out = norm(x) * x_norm, or x itself without x_norm.  The norm of x is a
+    layer norm, an RMS norm if not ``center``; ``offset`` is added to both norm
+    weights."""
+    return _impl(x).residual_norm(
+        x, y, eps, y_norm, x_norm, out, center, offset, mult, depth, depth_coef
+    )
+
+
+def embed_positions(token_ids, positions, table, cos_sin, x, copy=None):
+    """x = copy = table[token] plus sin (even entries) and cos (odd entries) of the
+    position's angles, cos_sin [2, P, ceil(K / 2)]; x, copy fp32 [N, K]."""
+    return _impl(x).embed_positions(token_ids, positions, table, cos_sin, x, copy)
+
+
+def softcap(logits, cap):
+    """cap * tanh(logits / cap) in fp32; the logits in fp32 without a cap."""
+    return logits.float() if cap is None else _impl(logits).softcap(logits, cap)
 
 
 def clamped_glu(gate_up, limit: float, alpha: float, offset: float, out):
@@ -205,6 +224,44 @@ def latent_expanded_prefill(q, w_ukv, gate, cos_sin, rot_dim: int, cache, batch,
     Writes the chunks' rows of out [N, H, v], gated."""
     _hip().latent_expanded_prefill(
         q, w_ukv, gate, cos_sin, rot_dim, cache, batch, chunks, rank, scale, window, out
+    )
+
+
+# ---------------------------------------- grouped attention: caps, windows, sinks
+
+
+def cache_keys_values(k, v, slot_mapping, k_cache, v_cache):
+    """Scatter k [N, G, d], v [N, G, e] (row-strided) into paged caches
+    [blocks, block, G, d or e]."""
+    return _impl(k).cache_keys_values(k, v, slot_mapping, k_cache, v_cache)
+
+
+def grouped_attention(q, k_cache, v_cache, batch, scale: float, cap, window, keep_first: int,
+                      sink, out):
+    """Attention of a FlatBatch's rows over the paged cache; query head n uses
+    key/value head n // (H / G).  Scores are capped if ``cap``; a query sees itself
+    and the ``window`` - 1 tokens before it (None = all) and the ``keep_first``
+    first tokens; ``sink`` [H] (fp32) or None joins the softmax denominator.
+    q [N, H, d] (row-strided) -> out [N, H, e]."""
+    return _impl(q).grouped_attention(
+        q, k_cache, v_cache, batch, scale, cap, window, keep_first, sink, out
+    )
+
+
+# ----------------------------------------------------------------- delta rule
+
+
+def channel_delta(qkv, conv, b, z, A_log, dt_bias, gate, norm, eps: float, unit_eps: float,
+                  kv_heads: int, state, conv_state, batch):
+    """Gated delta rule over a FlatBatch's rows, each sequence from the state in its
+    slot (zero at position 0), which is advanced.  Row-strided inputs: qkv
+    [N, 2*G*D + H*V] before the convolution, b [N, H] before its sigmoid, z [N, H*D]
+    the decays' input, gate [N, H*V] before its sigmoid.  conv [channels, taps];
+    fp32: A_log [H], dt_bias [H*D], norm [V], state [slots, H, D, V]; conv_state
+    [slots, taps - 1, channels].  Returns [N, H*V]: normed per head and gated."""
+    return _impl(qkv).channel_delta(
+        qkv, conv, b, z, A_log, dt_bias, gate, norm, eps, unit_eps, kv_heads, state,
+        conv_state, batch,
     )
 
 

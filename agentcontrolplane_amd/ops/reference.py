@@ -168,13 +168,40 @@ def layernorm(x, weight, eps: float, dtype):
     return (xc * torch.rsqrt(var + eps) * weight.float()).to(dtype)
 
 
-def residual_norm(x, y, eps: float, y_norm=None, x_norm=None, out=None):
-    yf = y.float()
-    if y_norm is not None:
-        yf = yf * torch.rsqrt(yf.pow(2).mean(-1, keepdim=True) + eps) * y_norm.float()
-    x += yf
-    if out is not None:
-        out.copy_(layernorm(x, x_norm, eps, out.dtype) if x_norm is not None else x)
+def residual_norm(x, y, eps: float, y_norm=None, x_norm=None, out=None, center=True,
+                  offset=0.0, mult=1.0, depth=None, depth_coef=None):
+    if y is not None:
+        yf = y.float()
+        if y_norm is not None:
+            yf = yf * torch.rsqrt(yf.pow(2).mean(-1, keepdim=True) + eps)
+            yf = yf * (offset + y_norm.float())
+        x += mult * yf
+    if depth_coef is not None:
+        n = depth_coef.numel()
+        depth[n - 1] = x
+        x.copy_(torch.einsum("j,jnk->nk", depth_coef, depth[:n]))
+    if out is None:
+        return
+    if x_norm is None:
+        out.copy_(x)
+        return
+    xc = x - x.mean(-1, keepdim=True) if center else x
+    xc = xc * torch.rsqrt(xc.pow(2).mean(-1, keepdim=True) + eps)
+    out.copy_(xc * (offset + x_norm.float()))
+
+
+def embed_positions(token_ids, positions, table, cos_sin, x, copy=None):
+    x.copy_(table[token_ids].float())
+    if cos_sin is not None:
+        w = x.shape[1]
+        x[:, 0::2] += cos_sin[1][positions]
+        x[:, 1::2] += cos_sin[0][positions][:, : w // 2]
+    if copy is not None:
+        copy.copy_(x)
+
+
+def softcap(logits, cap):
+    return cap * torch.tanh(logits.float() / cap)
 
 
 def clamped_glu(gate_up, limit: float, alpha: float, offset: float, out):
@@ -259,6 +286,107 @@ def latent_attention(q, q_rot, cos_sin, rot_dim: int, cache, batch, scale: float
             int(batch.decode_seq_lens[b]) - 1, rank, scale, window,
         )
         row += 1
+    return out
+
+
+# ---------------------------------------- grouped attention: caps, windows, sinks
+
+
+def cache_keys_values(k, v, slot_mapping, k_cache, v_cache):
+    _flat(k_cache)[slot_mapping] = k
+    _flat(v_cache)[slot_mapping] = v
+
+
+def _grouped_attention_seq(q, k_cache, v_cache, block_table, ctx_len: int, scale, cap, window,
+                           keep_first, sink):
+    """One sequence's rows at positions ctx_len..; q [L, H, d] -> [L, H, e]."""
+    L, H, bs = q.shape[0], q.shape[1], k_cache.shape[1]
+    j = torch.arange(ctx_len + L, device=q.device)
+    rows = torch.as_tensor(block_table, device=q.device)[j // bs] * bs + j % bs
+    group = H // k_cache.shape[2]
+    k = _flat(k_cache)[rows].float().repeat_interleave(group, 1).transpose(0, 1)
+    v = _flat(v_cache)[rows].float().repeat_interleave(group, 1).transpose(0, 1)
+    scores = torch.matmul(q.float().transpose(0, 1), k.transpose(1, 2)) * scale  # [H, L, S]
+    if cap is not None:
+        scores = cap * torch.tanh(scores / cap)
+    i = torch.arange(ctx_len, ctx_len + L, device=q.device).view(-1, 1)
+    hidden = j > i
+    if window is not None:
+        hidden |= ((i - j) >= window) & (j >= keep_first)
+    scores = scores.masked_fill(hidden, float("-inf"))
+    if sink is not None:
+        scores = torch.cat([scores, sink.float().view(H, 1, 1).expand(H, L, 1)], -1)
+    probs = torch.softmax(scores, -1)[..., : len(j)]
+    return torch.matmul(probs, v).transpose(0, 1).to(q.dtype)
+
+
+def grouped_attention(q, k_cache, v_cache, batch, scale: float, cap, window, keep_first: int,
+                      sink, out):
+    rest = (scale, cap, window, keep_first, sink)
+    row = 0
+    for m in batch.prefills:
+        out[row : row + m.query_len] = _grouped_attention_seq(
+            q[row : row + m.query_len], k_cache, v_cache, m.block_table, m.ctx_len, *rest
+        )
+        row += m.query_len
+    for n in range(batch.num_decode):
+        out[row] = _grouped_attention_seq(
+            q[row : row + 1], k_cache, v_cache, batch.decode_block_tables[n],
+            int(batch.decode_seq_lens[n]) - 1, *rest,
+        )[0]
+        row += 1
+
+
+# ----------------------------------------------------------------- delta rule
+
+
+def _channel_delta_seq(qkv, conv, b, z, A_log, dt_bias, gate, norm, eps, unit_eps, G, S, tail):
+    """One sequence's rows from state S [H, D, V] and convolution inputs tail
+    [taps - 1, C]; returns the rows, S and tail after them."""
+    T, (H, D, V), taps = qkv.shape[0], S.shape, conv.shape[1]
+    x = torch.cat([tail, qkv])
+    y = sum(x[n : n + T].float() * conv[:, n].float() for n in range(taps))
+    y = torch.nn.functional.silu(y).to(qkv.dtype).float()
+    q, k, v = y.split([G * D, G * D, H * V], 1)
+
+    def unit(t):
+        t = t.reshape(T, G, D)
+        t = t * torch.rsqrt(t.pow(2).sum(-1, keepdim=True) + unit_eps)
+        return t.repeat_interleave(H // G, 1)
+
+    q, k, v = unit(q) * D ** -0.5, unit(k), v.reshape(T, H, V)
+    beta = torch.sigmoid(b.float())
+    step = torch.nn.functional.softplus((z.float() + dt_bias).view(T, H, D), threshold=40.0)
+    g = torch.exp(-torch.exp(A_log).view(H, 1) * step)
+    out = torch.empty(T, H, V, device=S.device)
+    for t in range(T):
+        S = g[t].unsqueeze(-1) * S
+        u = beta[t].unsqueeze(-1) * (v[t] - torch.matmul(k[t].unsqueeze(1), S).squeeze(1))
+        S = S + k[t].unsqueeze(-1) * u.unsqueeze(1)
+        out[t] = torch.matmul(q[t].unsqueeze(1), S).squeeze(1)
+    out = out * torch.rsqrt(out.pow(2).mean(-1, keepdim=True) + eps) * norm
+    out = out.reshape(T, H * V) * torch.sigmoid(gate.float())
+    return out.to(qkv.dtype), S, x[T:]
+
+
+def channel_delta(qkv, conv, b, z, A_log, dt_bias, gate, norm, eps, unit_eps, kv_heads,
+                  state, conv_state, batch):
+    out = torch.empty(gate.shape, dtype=qkv.dtype, device=qkv.device)
+    runs, row = [], 0
+    for m in batch.prefills:
+        runs.append((row, m.query_len, m.state_slot, m.ctx_len == 0))
+        row += m.query_len
+    for n in range(batch.num_decode):
+        runs.append((row + n, 1, int(batch.decode_state_slots[n]), False))
+    for row, n, slot, fresh in runs:
+        r = slice(row, row + n)
+        S, tail = state[slot], conv_state[slot]
+        if fresh:
+            S, tail = torch.zeros_like(S), torch.zeros_like(tail)
+        out[r], state[slot], conv_state[slot] = _channel_delta_seq(
+            qkv[r], conv, b[r], z[r], A_log, dt_bias, gate[r], norm, eps, unit_eps, kv_heads,
+            S, tail,
+        )
     return out
 
 

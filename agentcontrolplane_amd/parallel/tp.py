@@ -157,6 +157,9 @@ def _pack_wire(wire: Optional[dict]) -> torch.Tensor:
     ss = wire["sample_seq_ids"]
     out.append(len(ss))
     out.extend(ss)
+    # models with recurrent state: a slot per prefill chunk and decode row
+    if "state_slots" in wire:
+        out.extend(wire["state_slots"])
     return torch.tensor(out, dtype=torch.int64)
 
 
@@ -194,7 +197,7 @@ def _unpack_wire(t: torch.Tensor) -> Optional[dict]:
     lens = take(n_lens) if n_lens >= 0 else None
     logit_rows = take(one())
     sample_seq_ids = take(one())
-    return {
+    step = {
         "token_ids": token_ids,
         "positions": positions,
         "slot_mapping": slot_mapping,
@@ -206,6 +209,9 @@ def _unpack_wire(t: torch.Tensor) -> Optional[dict]:
         "logit_rows": logit_rows,
         "sample_seq_ids": sample_seq_ids,
     }
+    if pos < len(data):
+        step["state_slots"] = take(len(prefills) + n_dec)
+    return step
 
 
 def broadcast_step(wire: Optional[dict], src: int = 0, group=None) -> Optional[dict]:
