@@ -275,7 +275,7 @@ class Scheduler:
                     avail += self.bm.free_blocks - before
                     if not self.states.free:
                         break
-                self._add_seq(s)
+                self.reserve(s)
                 s.num_processed = 0
             self.waiting.pop(0)
             cur = self.bm.seq_len(s.seq_id)
@@ -339,7 +339,7 @@ class Scheduler:
                     raise RuntimeError("more live sequences than max_batch_size")
                 self.waiting.remove(s)
                 self.running.append(s)
-                self._add_seq(s)
+                self.reserve(s)
             index[s.seq_id] = n
             wanted[s.seq_id] = want
             if count == 1 and s.num_processed > 0:
@@ -481,7 +481,7 @@ class Scheduler:
 
     # ------------------------------------------------------------ storage
 
-    def _add_seq(self, seq: Sequence) -> None:
+    def reserve(self, seq: Sequence) -> None:
         """Pages, and a state slot if the model keeps state."""
         if self.states is not None:
             self.states.acquire(seq.seq_id)

@@ -6,8 +6,8 @@
     S <- diag(g) S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q
     out = W_o (rmsnorm(o) * w * sigmoid(W_g2 W_g1 h))
 
-A sequence's state is S [heads, dim, vdim] in fp32 and the convolutions' last
-taps - 1 inputs, both in the slot the scheduler gave it (engine/state.py).
+A sequence's state is S [heads, dim, vdim] in fp32 and the convolutions' last inputs
+in a ring by position, both in the slot the scheduler gave it (engine/state.py).
 
 One GEMM makes [q | k | v | b | a1 | g1]; the convolution, the recurrence and the
 output norm work on its sections in place.
@@ -116,12 +116,12 @@ class ChannelDelta:
         s = self.spec
         return (
             torch.empty(num_slots, self.heads, s.dim, s.vdim, dtype=torch.float32, device=device),
-            torch.empty(num_slots, s.conv - 1, self.channels, dtype=dtype, device=device),
+            torch.empty(num_slots, s.conv, self.channels, dtype=dtype, device=device),
         )
 
     def state_bytes(self, itemsize: int) -> int:
         s = self.spec
-        return 4 * self.heads * s.dim * s.vdim + (s.conv - 1) * self.channels * itemsize
+        return 4 * self.heads * s.dim * s.vdim + s.conv * self.channels * itemsize
 
     # ------------------------------------------------------------- forward
 

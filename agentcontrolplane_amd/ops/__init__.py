@@ -258,7 +258,7 @@ def channel_delta(qkv, conv, b, z, A_log, dt_bias, gate, norm, eps: float, unit_
     [N, 2*G*D + H*V] before the convolution, b [N, H] before its sigmoid, z [N, H*D]
     the decays' input, gate [N, H*V] before its sigmoid.  conv [channels, taps];
     fp32: A_log [H], dt_bias [H*D], norm [V], state [slots, H, D, V]; conv_state
-    [slots, taps - 1, channels].  Returns [N, H*V]: normed per head and gated."""
+    [slots, taps, channels], the last convolution inputs in a ring by position.  Returns [N, H*V]: normed per head and gated."""
     return _impl(qkv).channel_delta(
         qkv, conv, b, z, A_log, dt_bias, gate, norm, eps, unit_eps, kv_heads, state,
         conv_state, batch,

@@ -113,12 +113,23 @@ def swiglu(gate_up):
 
 def layernorm(x, weight, eps: float, dtype):
     out = torch.empty(x.shape, dtype=dtype, device=x.device)
-    _C.residual_norm(x, None, None, weight, out, eps)
+    _C.residual_norm(x, None, None, weight, out, eps, True, 0.0, 1.0, None, None)
     return out
 
 
-def residual_norm(x, y, eps: float, y_norm=None, x_norm=None, out=None):
-    _C.residual_norm(x, y, y_norm, x_norm, out, eps)
+def residual_norm(x, y, eps: float, y_norm=None, x_norm=None, out=None, center=True,
+                  offset=0.0, mult=1.0, depth=None, depth_coef=None):
+    _C.residual_norm(x, y, y_norm, x_norm, out, eps, center, offset, mult, depth, depth_coef)
+
+
+def embed_positions(token_ids, positions, table, cos_sin, x, copy=None):
+    _C.embed_positions(x, copy, token_ids, positions, table, cos_sin)
+
+
+def softcap(logits, cap):
+    out = torch.empty(logits.shape, dtype=torch.float32, device=logits.device)
+    _C.softcap(out, logits, cap)
+    return out
 
 
 def clamped_glu(gate_up, limit: float, alpha: float, offset: float, out):
@@ -267,6 +278,94 @@ def latent_expanded_prefill(q, w_ukv, gate, cos_sin, rot_dim: int, cache, batch,
             meta.seq_lens, meta.ctx_lens, meta.row_starts, meta.tile_seq, meta.tile_q0,
             meta.key_first, meta.key_starts, scale, window,
         )
+
+
+# ---------------------------------------- grouped attention: caps, windows, sinks
+
+_PLAIN, _DECODE, _PREFILL = 0, 1, 2
+
+
+def cache_keys_values(k, v, slot_mapping, k_cache, v_cache):
+    _C.cache_keys_values(k_cache, v_cache, k, v, slot_mapping)
+
+
+def grouped_attention(q, k_cache, v_cache, batch, scale: float, cap, window, keep_first: int,
+                      sink, out):
+    from . import LATENT_HEADS
+
+    H, d, v, G = q.shape[1], q.shape[2], out.shape[2], k_cache.shape[2]
+    rest = (scale, cap or 0.0, window or _NO_WINDOW, keep_first)
+    tiled = q.dtype == torch.bfloat16 and d in LATENT_HEADS and v in LATENT_HEADS
+    P = batch.num_prefill_tokens
+    if batch.prefills:
+        meta = batch.prefill_meta(128 if tiled else 1)
+        _C.grouped_attn(
+            out[:P], q[:P], k_cache, v_cache, meta.block_tables, meta.seq_lens, meta.ctx_lens,
+            meta.row_starts, meta.tile_seq, meta.tile_q0, sink, None, None, *rest,
+            _PREFILL if tiled else _PLAIN, 1, 1,
+        )
+    if not batch.num_decode:
+        return
+    tables, rows = batch.decode_tables_i32(), batch.num_decode * H
+    gm, n_split, part, ml = 1, 1, None, None
+    if tiled:
+        most = 8 if d + v <= 256 else 4  # query heads a workgroup holds
+        gm = next((n for n in (1, 2, 4) if n >= min(H // G, most)), most)
+        # workgroups that fill the chip; every split has work for its 16 lane groups
+        keys = min(tables.shape[1] * k_cache.shape[1], rest[2] + keep_first)
+        groups = batch.num_decode * G * -(-(H // G) // gm)
+        n_split = max(1, min(_MAX_SPLIT, 1024 // groups, -(-keys // 128)))
+    if n_split > 1:
+        part = torch.empty(n_split * rows * v, dtype=torch.float32, device=q.device)
+        ml = torch.empty(2 * n_split * rows, dtype=torch.float32, device=q.device)
+    _C.grouped_attn(
+        out[P:], q[P:], k_cache, v_cache, tables, batch.decode_lens_i32(), None, None, None,
+        None, sink, part, ml, *rest, _DECODE if tiled else _PLAIN, gm, n_split,
+    )
+
+
+# ----------------------------------------------------------------- delta rule
+
+
+def _step_threads(D: int, V: int) -> int:
+    """Threads of a decode workgroup: at most 16 rows of the state per thread."""
+    columns = V // 4 if V % 4 == 0 else V
+    for n in (256, 512):
+        if n >= columns and n // columns * 16 >= D:
+            return n
+    return 1024
+
+
+def channel_delta(qkv, conv, b, z, A_log, dt_bias, gate, norm, eps, unit_eps, kv_heads,
+                  state, conv_state, batch):
+    H, D, V = state.shape[1:]
+    out = torch.empty(gate.shape, dtype=qkv.dtype, device=qkv.device)
+    P = batch.num_prefill_tokens
+
+    def rows(r):
+        return (out[r], qkv[r], conv, b[r], z[r], A_log, dt_bias, gate[r], norm, state,
+                conv_state)
+
+    if batch.prefills:
+        meta = batch.prefill_meta(16)
+        seqs = len(batch.prefills)
+
+        def space(n, dtype=torch.float32):
+            return torch.empty(P * n, dtype=dtype, device=qkv.device)
+
+        # two columns a lane once one still fills the chip's SIMDs
+        cpl = 2 if seqs * H * V >= 4 * 4096 else 1
+        _C.delta_prompts(
+            *rows(slice(0, P)), meta.seq_lens, meta.state_slots, kv_heads, eps, unit_eps,
+            meta.ctx_lens, meta.row_starts, meta.tile_seq, meta.tile_q0,
+            space(qkv.shape[1], qkv.dtype), space(3 * kv_heads), space(H * D), space(H * V), cpl,
+        )
+    if batch.num_decode:
+        _C.delta_step(
+            *rows(slice(P, None)), batch.decode_lens_i32(), batch.decode_state_slots, kv_heads,
+            eps, unit_eps, _step_threads(D, V),
+        )
+    return out
 
 
 def softmax_sample(logits, temperatures, top_ks, top_ps, gen, mask=None,

@@ -342,7 +342,7 @@ def grouped_attention(q, k_cache, v_cache, batch, scale: float, cap, window, kee
 
 def _channel_delta_seq(qkv, conv, b, z, A_log, dt_bias, gate, norm, eps, unit_eps, G, S, tail):
     """One sequence's rows from state S [H, D, V] and convolution inputs tail
-    [taps - 1, C]; returns the rows, S and tail after them."""
+    [taps - 1, C]; returns the rows and S after them."""
     T, (H, D, V), taps = qkv.shape[0], S.shape, conv.shape[1]
     x = torch.cat([tail, qkv])
     y = sum(x[n : n + T].float() * conv[:, n].float() for n in range(taps))
@@ -366,27 +366,31 @@ def _channel_delta_seq(qkv, conv, b, z, A_log, dt_bias, gate, norm, eps, unit_ep
         out[t] = torch.matmul(q[t].unsqueeze(1), S).squeeze(1)
     out = out * torch.rsqrt(out.pow(2).mean(-1, keepdim=True) + eps) * norm
     out = out.reshape(T, H * V) * torch.sigmoid(gate.float())
-    return out.to(qkv.dtype), S, x[T:]
+    return out.to(qkv.dtype), S
 
 
 def channel_delta(qkv, conv, b, z, A_log, dt_bias, gate, norm, eps, unit_eps, kv_heads,
                   state, conv_state, batch):
     out = torch.empty(gate.shape, dtype=qkv.dtype, device=qkv.device)
-    runs, row = [], 0
+    runs, row, taps = [], 0, conv.shape[1]
     for m in batch.prefills:
-        runs.append((row, m.query_len, m.state_slot, m.ctx_len == 0))
+        runs.append((row, m.query_len, m.state_slot, m.ctx_len))
         row += m.query_len
     for n in range(batch.num_decode):
-        runs.append((row + n, 1, int(batch.decode_state_slots[n]), False))
-    for row, n, slot, fresh in runs:
-        r = slice(row, row + n)
-        S, tail = state[slot], conv_state[slot]
-        if fresh:
-            S, tail = torch.zeros_like(S), torch.zeros_like(tail)
-        out[r], state[slot], conv_state[slot] = _channel_delta_seq(
+        runs.append((row + n, 1, int(batch.decode_state_slots[n]),
+                     int(batch.decode_seq_lens[n]) - 1))
+    for row, n, slot, ctx in runs:
+        r, ring = slice(row, row + n), conv_state[slot]
+        S = state[slot] if ctx else torch.zeros_like(state[slot])
+        tail = torch.zeros(taps - 1, qkv.shape[1], dtype=qkv.dtype, device=qkv.device)
+        for i in range(1, min(taps - 1, ctx) + 1):  # the ring's entry of position p is p % taps
+            tail[-i] = ring[(ctx - i) % taps]
+        out[r], state[slot] = _channel_delta_seq(
             qkv[r], conv, b[r], z[r], A_log, dt_bias, gate[r], norm, eps, unit_eps, kv_heads,
             S, tail,
         )
+        for i in range(max(0, n - taps), n):
+            ring[(ctx + i) % taps] = qkv[row + i]
     return out
 
 

@@ -53,6 +53,8 @@ class Side:
         # decode workloads attend over tokens that were never prefilled
         for c in getattr(m, "caches", None) or m.k_caches + m.v_caches:
             c.normal_(0.0, 0.5)
+        for c in getattr(m, "states", ()):
+            c.normal_(0.0, 0.1)
 
     def _sequence(self, tokens: int):
         ids = [(7 * i) % 250 for i in range(tokens)]
@@ -68,7 +70,7 @@ class Side:
             for s in seqs:  # cached so far: reserve the pages, keep their contents
                 sched.waiting.remove(s)
                 sched.running.append(s)
-                self.engine.bm.add_seq(s.seq_id)
+                sched.reserve(s)
                 self.engine.bm.append_tokens(s.seq_id, tokens - 1)
                 s.num_processed = tokens - 1
             portions = [(s, 1, [0]) for s in seqs]
@@ -129,6 +131,9 @@ def run(name: str, device: str, prefill: List[Tuple[int, int]] = PREFILL,
         "layer_runs": len(cfg.layer_runs),
         "cache_bytes_per_token": {
             k: s.engine.model.kv_block_bytes(1) for k, s in sides.items()
+        },
+        "state_bytes_per_sequence": {
+            k: getattr(s.engine.model, "state_slot_bytes", 0) for k, s in sides.items()
         },
         "workloads": rows,
     }

@@ -36,6 +36,10 @@ def build(verbose: bool = False) -> str:
         os.path.join(CSRC, "latent_proj.hip"),
         os.path.join(CSRC, "latent_attn.hip"),
         os.path.join(CSRC, "latent_prefill.hip"),
+        os.path.join(CSRC, "embedding.hip"),
+        os.path.join(CSRC, "grouped_attn.hip"),
+        os.path.join(CSRC, "grouped_prefill.hip"),
+        os.path.join(CSRC, "channel_delta.hip"),
         os.path.join(CSRC, "sampling.hip"),
         os.path.join(CSRC, "sampling_fullvocab.hip"),
     ]

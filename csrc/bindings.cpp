@@ -6,7 +6,12 @@
 #include <c10/hip/HIPStream.h>
 #include <hip/hip_runtime.h>
 
+#include <cmath>
+
+#include "channel_delta.h"
+#include "grouped_attn.h"
 #include "latent_attn.h"
+#include "residual_norm.h"
 
 namespace py = pybind11;
 
@@ -35,7 +40,17 @@ void launch_prefill_attn_mfma(void*, const void*, const void*, const void*, cons
                               const int*, const int*, const int*, const int*, const int*,
                               float, int, int, int, int, int, int, int64_t, hipStream_t);
 void launch_residual_norm(bool, float*, const void*, const void*, const void*, void*, float,
-                          int, int, int64_t, hipStream_t);
+                          int, int, int64_t, const NormForm*, hipStream_t);
+void launch_embed_positions(bool, float*, float*, const int64_t*, const int64_t*, const void*,
+                            const float*, int, int, int64_t, int64_t, hipStream_t);
+void launch_softcap(bool, float*, const void*, float, int64_t, hipStream_t);
+bool launch_grouped_decode(const GroupedArgs*, int, int, int, int, hipStream_t);
+bool launch_grouped_plain(bool, const GroupedArgs*, int, int, int, hipStream_t);
+bool launch_grouped_prefill(const GroupedArgs*, int, int, hipStream_t);
+void launch_cache_keys_values(void*, void*, const void*, const void*, const int64_t*, int, int,
+                              int64_t, int, hipStream_t);
+void launch_delta_prompts(bool, const DeltaArgs*, int, hipStream_t);
+void launch_delta_step(bool, const DeltaArgs*, int, hipStream_t);
 void launch_side_gate(bool, float*, const float*, const void*, const void*, const int64_t*, const void*,
                       void*, int, int, int, int64_t, hipStream_t);
 void launch_add_to_residual(bool, float*, const void*, void*, int64_t, hipStream_t);
@@ -283,7 +298,8 @@ static void check_aligned(const torch::Tensor& t) {
 }
 
 static void residual_norm(torch::Tensor x, OptTensor y, OptTensor y_norm, OptTensor x_norm,
-                          OptTensor out, double eps) {
+                          OptTensor out, double eps, bool center, double offset, double mult,
+                          OptTensor depth, OptTensor depth_coef) {
   CHECK_CUDA(x); CHECK_CONT(x);
   TORCH_CHECK(x.scalar_type() == at::kFloat && x.dim() == 2);
   TORCH_CHECK(y || out, "nothing to do");
@@ -294,12 +310,61 @@ static void residual_norm(torch::Tensor x, OptTensor y, OptTensor y_norm, OptTen
   if (y_norm) check_vec(*y_norm, dt, w);
   if (x_norm) check_vec(*x_norm, dt, w);
   if (out) check_rows(*out, dt, n, w);
+  NormForm f{};
+  f.center = center;
+  f.offset = (float)offset;
+  f.mult = (float)mult;
+  if (depth_coef) {
+    TORCH_CHECK(depth && y, "depth states");
+    CHECK_CUDA((*depth)); CHECK_CONT((*depth));
+    check_vec(*depth_coef, at::kFloat, depth_coef->numel());
+    TORCH_CHECK(depth->scalar_type() == at::kFloat && depth->dim() == 3 &&
+                depth->size(0) >= depth_coef->numel() && depth_coef->numel() > 0 &&
+                depth->size(1) == n && depth->size(2) == w, "depth states");
+    f.n_depth = depth_coef->numel();
+    f.depth = depth->data_ptr<float>();
+    f.depth_coef = depth_coef->data_ptr<float>();
+    f.depth_stride = depth->stride(0);
+  }
   if (n == 0) return;
   launch_residual_norm(is_bf16(y ? *y : *out), x.data_ptr<float>(),
                        y ? y->data_ptr() : nullptr, y_norm ? y_norm->data_ptr() : nullptr,
                        x_norm ? x_norm->data_ptr() : nullptr,
                        out ? out->data_ptr() : nullptr, (float)eps, n, w,
-                       out ? out->stride(0) : w, cur_stream());
+                       out ? out->stride(0) : w, &f, cur_stream());
+}
+
+static void check_ids(const torch::Tensor& t, int64_t n) {
+  CHECK_CUDA(t); CHECK_CONT(t);
+  TORCH_CHECK(t.scalar_type() == at::kLong && t.numel() == n, "want int64 per row");
+}
+
+static void embed_positions(torch::Tensor x, OptTensor copy, torch::Tensor token_ids,
+                            torch::Tensor positions, torch::Tensor table, OptTensor cos_sin) {
+  const int n = x.size(0), w = x.size(1);
+  check_rows(x, at::kFloat, n, w); CHECK_CONT(x);
+  if (copy) { check_rows(*copy, at::kFloat, n, w); CHECK_CONT((*copy)); }
+  check_ids(token_ids, n); check_ids(positions, n);
+  check_rows(table, table.scalar_type(), table.size(0), w); CHECK_CONT(table);
+  if (cos_sin) {
+    CHECK_CUDA((*cos_sin)); CHECK_CONT((*cos_sin));
+    TORCH_CHECK(cos_sin->scalar_type() == at::kFloat && cos_sin->dim() == 3 &&
+                cos_sin->size(0) == 2 && cos_sin->size(2) == (w + 1) / 2, "position table");
+  }
+  if (n == 0) return;
+  launch_embed_positions(is_bf16(table), x.data_ptr<float>(),
+                         copy ? copy->data_ptr<float>() : nullptr,
+                         token_ids.data_ptr<int64_t>(), positions.data_ptr<int64_t>(),
+                         table.data_ptr(), cos_sin ? cos_sin->data_ptr<float>() : nullptr, n, w,
+                         table.size(0), cos_sin ? cos_sin->size(1) : 1, cur_stream());
+}
+
+static void softcap(torch::Tensor out, torch::Tensor x, double cap) {
+  CHECK_CUDA(x); CHECK_CONT(x); CHECK_CUDA(out); CHECK_CONT(out);
+  TORCH_CHECK(out.scalar_type() == at::kFloat && out.numel() == x.numel() && cap > 0);
+  if (x.numel() == 0) return;
+  launch_softcap(is_bf16(x), out.data_ptr<float>(), x.data_ptr(), (float)cap, x.numel(),
+                 cur_stream());
 }
 
 // x_out = x + y; s = gelu_tanh(gate x_out) * table[token, offset:]
@@ -578,6 +643,217 @@ static void latent_prefill(torch::Tensor out, torch::Tensor q, torch::Tensor kv,
               "latent prefill: unsupported sizes d ", d, " v ", v);
 }
 
+// ---- grouped attention, delta rule
+
+// [N, heads, size] with dense heads and vectors, any token stride, 16-byte aligned
+static void check_token_heads(const torch::Tensor& t, at::ScalarType dtype, int64_t n,
+                              int64_t heads, int64_t size) {
+  CHECK_CUDA(t);
+  TORCH_CHECK(t.dim() == 3 && t.size(0) == n && t.size(1) == heads && t.size(2) == size,
+              "head shape mismatch");
+  TORCH_CHECK(t.stride(2) == 1 && (heads == 1 || t.stride(1) == size), "heads must be dense");
+  TORCH_CHECK(t.scalar_type() == dtype, "dtype mismatch");
+  check_aligned(t);
+}
+
+static void check_cache(const torch::Tensor& t, at::ScalarType dtype) {
+  CHECK_CUDA(t); CHECK_CONT(t);
+  TORCH_CHECK(t.dim() == 4 && t.scalar_type() == dtype, "cache layout");
+  TORCH_CHECK(t.size(3) * t.element_size() % 16 == 0, "cache rows must be 16-byte multiples");
+}
+
+static void cache_keys_values(torch::Tensor k_cache, torch::Tensor v_cache, torch::Tensor k,
+                              torch::Tensor v, torch::Tensor slots) {
+  const auto dt = k.scalar_type();
+  const int n = k.size(0), G = k.size(1);
+  check_cache(k_cache, dt); check_cache(v_cache, dt);
+  check_token_heads(k, dt, n, G, k_cache.size(3));
+  check_token_heads(v, dt, n, G, v_cache.size(3));
+  TORCH_CHECK(k_cache.size(2) == G && v_cache.size(2) == G && k_cache.size(0) == v_cache.size(0) &&
+              k_cache.size(1) == v_cache.size(1), "cache shapes");
+  TORCH_CHECK(k.stride(0) == v.stride(0), "k and v must share a row stride");
+  check_ids(slots, n);
+  if (n == 0) return;
+  const int unit = 16 / (int)k.element_size();
+  launch_cache_keys_values(k_cache.data_ptr(), v_cache.data_ptr(), k.data_ptr(), v.data_ptr(),
+                           slots.data_ptr<int64_t>(), G * k.size(2) / unit, G * v.size(2) / unit,
+                           k.stride(0) / unit, n, cur_stream());
+}
+
+// q [tokens, H, d] -> out [tokens, H, v].  Prefill chunks bring ctx_lens, row_starts and
+// tiles; decode (one token per table row) brings none of them.
+// kind: 0 plain, 1 decode, 2 prefill on the matrix cores
+static void grouped_attn(torch::Tensor out, torch::Tensor q, torch::Tensor k_cache,
+                         torch::Tensor v_cache, torch::Tensor tables, torch::Tensor seq_lens,
+                         OptTensor ctx_lens, OptTensor row_starts, OptTensor tile_seq,
+                         OptTensor tile_q0, OptTensor sink, OptTensor part, OptTensor part_ml,
+                         double scale, double cap, int64_t window, int64_t keep, int64_t kind,
+                         int64_t gm, int64_t n_split) {
+  const auto dt = q.scalar_type();
+  const bool bf16 = is_bf16(q);
+  const int tokens = q.size(0), H = q.size(1), d = q.size(2), v = out.size(2);
+  check_token_heads(q, dt, tokens, H, d);
+  check_token_heads(out, dt, tokens, H, v); CHECK_CONT(out);
+  check_cache(k_cache, dt); check_cache(v_cache, dt);
+  const int G = k_cache.size(2);
+  TORCH_CHECK(k_cache.size(3) == d && v_cache.size(3) == v && v_cache.size(2) == G &&
+              k_cache.size(0) == v_cache.size(0) && k_cache.size(1) == v_cache.size(1) &&
+              H % G == 0, "cache shapes");
+  CHECK_CUDA(tables); CHECK_CONT(tables);
+  TORCH_CHECK(tables.scalar_type() == at::kInt && tables.dim() == 2);
+  const int seqs = tables.size(0);
+  TORCH_CHECK(window > 0 && keep >= 0 && cap >= 0 && n_split >= 1 && n_split <= 64);
+  TORCH_CHECK(kind == 0 || bf16, "the matrix-core kernels take bf16");
+  TORCH_CHECK(kind == 1 || n_split == 1, "only decode splits keys");
+  TORCH_CHECK((kind == 2) <= (bool)tile_seq && !(kind == 1 && tile_seq), "tiles");
+  if (tokens == 0 || seqs == 0) return;
+  GroupedArgs a{};
+  a.out = out.data_ptr();
+  if (n_split > 1) {
+    TORCH_CHECK(part && part_ml && part->is_contiguous() && part_ml->is_contiguous());
+    TORCH_CHECK(part->scalar_type() == at::kFloat && part_ml->scalar_type() == at::kFloat);
+    TORCH_CHECK(part->numel() >= n_split * tokens * H * v &&
+                part_ml->numel() >= 2 * n_split * tokens * H, "split workspace");
+    a.part = part->data_ptr<float>();
+    a.part_ml = (float2*)part_ml->data_ptr<float>();
+  }
+  a.q = q.data_ptr();
+  a.k_cache = k_cache.data_ptr();
+  a.v_cache = v_cache.data_ptr();
+  if (sink) { check_vec(*sink, at::kFloat, H); a.sink = sink->data_ptr<float>(); }
+  a.tables = tables.data_ptr<int>();
+  a.seq_lens = opt_int(seq_lens, seqs);
+  a.ctx_lens = opt_int(ctx_lens, seqs);
+  a.row_starts = opt_int(row_starts, seqs);
+  if (tile_seq) {
+    TORCH_CHECK(ctx_lens && row_starts && tile_q0, "prefill metadata");
+    a.n_tiles = tile_seq->numel();
+    TORCH_CHECK(kind == 2 || a.n_tiles == tokens, "the plain kernel takes a token per tile");
+  } else {
+    TORCH_CHECK(tokens == seqs, "decode has one token per sequence");
+  }
+  a.tile_seq = opt_int(tile_seq, a.n_tiles);
+  a.tile_q0 = opt_int(tile_q0, a.n_tiles);
+  a.q_stride = q.stride(0);
+  a.H = H;
+  a.G = G;
+  a.max_blocks = tables.size(1);
+  a.kv_block = k_cache.size(1);
+  a.window = (int)window;
+  a.keep = (int)keep;
+  a.n_split = (int)n_split;
+  a.rows = tokens * H;
+  a.scale = (float)scale;
+  a.cap = (float)cap;
+  const bool ok = kind == 2   ? launch_grouped_prefill(&a, d, v, cur_stream())
+                  : kind == 1 ? launch_grouped_decode(&a, d, v, seqs, (int)gm, cur_stream())
+                              : launch_grouped_plain(bf16, &a, d, v, tokens, cur_stream());
+  TORCH_CHECK(ok, "grouped attention: unsupported sizes d ", d, " v ", v);
+}
+
+static DeltaArgs delta_args(const torch::Tensor& out, const torch::Tensor& qkv,
+                            const torch::Tensor& conv, const torch::Tensor& b,
+                            const torch::Tensor& z, const torch::Tensor& A_log,
+                            const torch::Tensor& dt_bias, const torch::Tensor& gate,
+                            const torch::Tensor& norm, const torch::Tensor& state,
+                            const torch::Tensor& ring, const torch::Tensor& seq_lens,
+                            const torch::Tensor& slots, int64_t kv_heads, double eps,
+                            double unit_eps) {
+  const auto dt = qkv.scalar_type();
+  DeltaArgs a{};
+  CHECK_CUDA(state); CHECK_CONT(state);
+  TORCH_CHECK(state.scalar_type() == at::kFloat && state.dim() == 4, "state layout");
+  a.N = qkv.size(0);
+  a.H = state.size(1);
+  a.D = state.size(2);
+  a.V = state.size(3);
+  a.G = (int)kv_heads;
+  TORCH_CHECK(a.G > 0 && a.H % a.G == 0 && a.D <= 1024 && a.V <= 1024, "delta rule: head sizes");
+  a.C = 2 * a.G * a.D + a.H * a.V;
+  a.taps = conv.size(1);
+  check_rows(qkv, dt, a.N, a.C);
+  check_rows(conv, dt, a.C, a.taps); CHECK_CONT(conv);
+  check_rows(b, dt, a.N, a.H);
+  check_rows(z, dt, a.N, (int64_t)a.H * a.D);
+  check_rows(gate, dt, a.N, (int64_t)a.H * a.V);
+  check_rows(out, dt, a.N, (int64_t)a.H * a.V); CHECK_CONT(out);
+  check_vec(A_log, at::kFloat, a.H);
+  check_vec(dt_bias, at::kFloat, (int64_t)a.H * a.D);
+  check_vec(norm, at::kFloat, a.V);
+  CHECK_CUDA(ring); CHECK_CONT(ring);
+  TORCH_CHECK(ring.scalar_type() == dt && ring.dim() == 3 && ring.size(0) == state.size(0) &&
+              ring.size(1) == a.taps && ring.size(2) == a.C, "convolution state");
+  TORCH_CHECK((uintptr_t)qkv.data_ptr() % 4 == 0 && (uintptr_t)z.data_ptr() % 4 == 0);
+  is_bf16(qkv);
+  a.seqs = seq_lens.numel();
+  a.qkv = qkv.data_ptr();
+  a.conv = conv.data_ptr();
+  a.b = b.data_ptr();
+  a.z = z.data_ptr();
+  a.gate = gate.data_ptr();
+  a.A_log = A_log.data_ptr<float>();
+  a.dt_bias = dt_bias.data_ptr<float>();
+  a.norm = norm.data_ptr<float>();
+  a.state = state.data_ptr<float>();
+  a.ring = ring.data_ptr();
+  a.out = out.data_ptr();
+  a.seq_lens = opt_int(seq_lens, a.seqs);
+  a.slots = opt_int(slots, a.seqs);
+  a.qkv_stride = qkv.stride(0);
+  a.b_stride = b.stride(0);
+  a.z_stride = z.stride(0);
+  a.gate_stride = gate.stride(0);
+  a.eps = (float)eps;
+  a.unit_eps = (float)unit_eps;
+  a.q_scale = 1.f / std::sqrt((float)a.D);
+  return a;
+}
+
+// The rows of every chunk; y, unit, g, o: workspace (channel_delta.h)
+static void delta_prompts(torch::Tensor out, torch::Tensor qkv, torch::Tensor conv,
+                          torch::Tensor b, torch::Tensor z, torch::Tensor A_log,
+                          torch::Tensor dt_bias, torch::Tensor gate, torch::Tensor norm,
+                          torch::Tensor state, torch::Tensor ring, torch::Tensor seq_lens,
+                          torch::Tensor slots, int64_t kv_heads, double eps, double unit_eps,
+                          torch::Tensor ctx_lens, torch::Tensor row_starts,
+                          torch::Tensor tile_seq, torch::Tensor tile_q0, torch::Tensor y,
+                          torch::Tensor unit, torch::Tensor g, torch::Tensor o, int64_t cpl) {
+  DeltaArgs a = delta_args(out, qkv, conv, b, z, A_log, dt_bias, gate, norm, state, ring,
+                           seq_lens, slots, kv_heads, eps, unit_eps);
+  check_vec(y, qkv.scalar_type(), (int64_t)a.N * a.C);
+  check_vec(unit, at::kFloat, (int64_t)a.N * a.G * 3);
+  check_vec(g, at::kFloat, (int64_t)a.N * a.H * a.D);
+  check_vec(o, at::kFloat, (int64_t)a.N * a.H * a.V);
+  a.y = y.data_ptr();
+  a.unit = unit.data_ptr<float>();
+  a.g = g.data_ptr<float>();
+  a.o = o.data_ptr<float>();
+  a.n_tiles = tile_seq.numel();
+  a.ctx_lens = opt_int(ctx_lens, a.seqs);
+  a.row_starts = opt_int(row_starts, a.seqs);
+  a.tile_seq = opt_int(tile_seq, a.n_tiles);
+  a.tile_q0 = opt_int(tile_q0, a.n_tiles);
+  TORCH_CHECK(a.seqs <= 65535 && a.H <= 16384, "grid");
+  if (a.N == 0 || a.n_tiles == 0) return;
+  launch_delta_prompts(is_bf16(qkv), &a, (int)cpl, cur_stream());
+}
+
+// One token per sequence, row i of sequence i.
+static void delta_step(torch::Tensor out, torch::Tensor qkv, torch::Tensor conv,
+                       torch::Tensor b, torch::Tensor z, torch::Tensor A_log,
+                       torch::Tensor dt_bias, torch::Tensor gate, torch::Tensor norm,
+                       torch::Tensor state, torch::Tensor ring, torch::Tensor seq_lens,
+                       torch::Tensor slots, int64_t kv_heads, double eps, double unit_eps,
+                       int64_t threads) {
+  DeltaArgs a = delta_args(out, qkv, conv, b, z, A_log, dt_bias, gate, norm, state, ring,
+                           seq_lens, slots, kv_heads, eps, unit_eps);
+  TORCH_CHECK(a.seqs == a.N && a.seqs <= 65535, "one token per sequence");
+  TORCH_CHECK(threads % 64 == 0 && threads >= 64 && threads <= 1024 &&
+              (a.V % 4 ? a.V : a.V / 4) <= threads, "threads");
+  if (a.N == 0) return;
+  launch_delta_step(is_bf16(qkv), &a, (int)threads, cur_stream());
+}
+
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.doc() = "MI355X-native runtime: paged-KV block manager + CDNA4 kernels";
   register_block_manager(m);
@@ -600,6 +876,12 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("latent_attn", &latent_attn);
   m.def("latent_gather", &latent_gather);
   m.def("latent_prefill", &latent_prefill);
+  m.def("embed_positions", &embed_positions);
+  m.def("softcap", &softcap);
+  m.def("cache_keys_values", &cache_keys_values);
+  m.def("grouped_attn", &grouped_attn);
+  m.def("delta_prompts", &delta_prompts);
+  m.def("delta_step", &delta_step);
   m.def("sample", &sample);
   m.def("sample_fullvocab", &sample_fullvocab);
 }

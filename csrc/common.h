@@ -50,6 +50,18 @@ DEV float group16_sum(float v) {
   return v;
 }
 
+// the same sum by lane rotations in the VALU; all 16 lanes end with equal bits
+template <int CTRL>
+DEV float dpp_add(float v) {
+  return v + __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), CTRL, 0xf, 0xf, true));
+}
+DEV float row16_sum(float v) {
+  v = dpp_add<0x128>(v);  // row_ror:8
+  v = dpp_add<0x124>(v);
+  v = dpp_add<0x122>(v);
+  return dpp_add<0x121>(v);
+}
+
 // block-wide sum across waves through LDS; `scratch` must hold
 // blockDim.x/64 floats.  Every thread returns the total.
 DEV float block_sum(float v, float* scratch) {

@@ -1,0 +1,22 @@
+// Launch arguments of grouped attention (grouped_attn.hip, grouped_prefill.hip).
+#pragma once
+#include <hip/hip_runtime.h>
+
+struct GroupedArgs {
+  void* out;              // [tokens, H, v]
+  float* part;            // [n_split, rows, v]
+  float2* part_ml;        // [n_split, rows]
+  const void* q;          // [tokens, H, d], tokens q_stride apart
+  const void* k_cache;    // [slots, G, d]
+  const void* v_cache;    // [slots, G, v]
+  const float* sink;      // [H] or null
+  const int* tables;      // [seqs, max_blocks]
+  const int* seq_lens;    // [seqs] cached tokens, this step's included
+  const int* ctx_lens;    // [seqs] before this step; null: seq_len - 1 (decode)
+  const int* row_starts;  // [seqs] first token row; null: seq
+  const int* tile_seq;    // [tiles]; null: decode, one token per sequence
+  const int* tile_q0;     // [tiles] first token of the tile within the chunk
+  int64_t q_stride;
+  int H, G, n_tiles, max_blocks, kv_block, window, keep, n_split, rows;
+  float scale, cap;       // cap 0: none
+};

@@ -37,3 +37,9 @@ struct LatentPrefillArgs {
   int H, n_tiles, rot_dim, window;
   float scale;
 };
+
+// out [rows, width] bf16 from n_split (at most 64) partial sums [n_split, rows, width]
+// with their (maximum in the exp2 domain, sum) [n_split, rows]; an empty split has sum
+// -1 and is one of a row's last
+extern "C" void launch_split_combine(void* out, const float* part, const float2* part_ml,
+                                     int rows, int width, int n_split, hipStream_t stream);

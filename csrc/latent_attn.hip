@@ -19,7 +19,7 @@
 // the transposed reads (4 keys, two units) off each other's banks.
 //
 // Keys past a sequence's end are clamped to its last key and masked; split-K
-// partials are merged by latent_combine_kernel.  The grid depends on host
+// partials are merged by split_combine_kernel.  The grid depends on host
 // values only (capture-safe); lengths are read on the device.
 #include "common_t.h"
 #include "latent_attn.h"
@@ -283,7 +283,7 @@ __global__ __launch_bounds__(256) void latent_attn_kernel(const LatentArgs a) {
 }
 
 // Merge the splits (at most 64) of one row.
-__global__ __launch_bounds__(128) void latent_combine_kernel(
+__global__ __launch_bounds__(128) void split_combine_kernel(
     bf16_t* __restrict__ out, const float* __restrict__ part,
     const float2* __restrict__ part_ml, const int rows, const int rank,
     const int n_split) {
@@ -419,6 +419,12 @@ static bool launch_plain(const LatentArgs& a, int rank, int row, int tiles,
 
 extern "C" {
 
+void launch_split_combine(void* out, const float* part, const float2* part_ml, int rows,
+                          int width, int n_split, hipStream_t stream) {
+  split_combine_kernel<<<rows, 128, 0, stream>>>((bf16_t*)out, part, part_ml, rows, width,
+                                                  n_split);
+}
+
 bool launch_latent_attn(bool bf16, bool mfma, const LatentArgs* a, int rank, int row,
                         int mg, int tiles, hipStream_t stream) {
   if (!mfma)
@@ -432,8 +438,7 @@ bool launch_latent_attn(bool bf16, bool mfma, const LatentArgs* a, int rank, int
     default: return false;
   }
   if (a->n_split > 1)
-    latent_combine_kernel<<<a->rows, 128, 0, stream>>>(
-        (bf16_t*)a->out, a->part, a->part_ml, a->rows, rank, a->n_split);
+    launch_split_combine(a->out, a->part, a->part_ml, a->rows, rank, a->n_split, stream);
   return true;
 }
 

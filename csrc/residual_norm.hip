@@ -1,11 +1,13 @@
 // Norms around an fp32 residual stream (gfx950).
 //
-// residual_norm is one pass over a row: optionally add y, or rmsnorm(y) * w_y,
-// to the residual, then emit layernorm(x) * w_x or x itself for the next GEMM.
-// The row lives in LDS between the reductions (each thread re-reads only what
+// residual_norm is one pass over a row: optionally add mult * y, or mult *
+// rmsnorm(y) * w_y, to the residual, optionally file the result as the newest depth
+// state and replace it by a weighted sum of all states, then emit norm(x) * w_x (layer
+// or RMS norm) or x itself for the next GEMM.  The row lives in LDS between the reductions (each thread re-reads only what
 // it wrote, so the row itself needs no barrier).  Mean first, then the squared
 // deviations: no cancellation.
 #include "common_t.h"
+#include "residual_norm.h"
 
 template <typename T, int V>
 __global__ __launch_bounds__(1024) void residual_norm_kernel(
@@ -14,7 +16,7 @@ __global__ __launch_bounds__(1024) void residual_norm_kernel(
     const T* __restrict__ y_norm,     // [w] or null: plain add
     const T* __restrict__ x_norm,     // [w] or null: out = x
     T* __restrict__ out,              // [n, w] rows out_stride apart, or null
-    const float eps, const int w, const int64_t out_stride) {
+    const float eps, const int w, const int64_t out_stride, const NormForm f) {
   extern __shared__ float row[];
   __shared__ float scratch[3][16];
   float* xr = x + (int64_t)blockIdx.x * w;
@@ -45,14 +47,30 @@ __global__ __launch_bounds__(1024) void residual_norm_kernel(
       if (y_norm) {
         load_f<V>(d, y_norm + i);
 #pragma unroll
-        for (int k = 0; k < V; ++k) d[k] *= row[i + k] * y_scale;
+        for (int k = 0; k < V; ++k) d[k] = (f.offset + d[k]) * row[i + k] * y_scale;
       } else {
         load_f<V>(d, y + (int64_t)blockIdx.x * w + i);
       }
 #pragma unroll
-      for (int k = 0; k < V; ++k) t[k] += d[k];
-      store_f<V>(xr + i, t);
+      for (int k = 0; k < V; ++k) t[k] += f.mult * d[k];
     }
+    if (f.n_depth) {
+      float* state = f.depth + (int64_t)blockIdx.x * w + i;
+      const int last = f.n_depth - 1;
+      store_f<V>(state + last * f.depth_stride, t);
+      const float c = f.depth_coef[last];
+#pragma unroll
+      for (int k = 0; k < V; ++k) t[k] *= c;
+#pragma unroll 8
+      for (int j = 0; j < last; ++j) {
+        float s[V];
+        load_f<V>(s, state + j * f.depth_stride);
+        const float cj = f.depth_coef[j];
+#pragma unroll
+        for (int k = 0; k < V; ++k) t[k] += cj * s[k];
+      }
+    }
+    if (y || f.n_depth) store_f<V>(xr + i, t);
 #pragma unroll
     for (int k = 0; k < V; ++k) {
       sum += t[k];
@@ -63,7 +81,7 @@ __global__ __launch_bounds__(1024) void residual_norm_kernel(
   T* orow = out + (int64_t)blockIdx.x * out_stride;
   float mean = 0.f, inv = 1.f;
   if (x_norm) {
-    mean = block_sum(sum, scratch[1]) / w;
+    if (f.center) mean = block_sum(sum, scratch[1]) / w;
     float ss = 0.f;
     for (int i = i0; i < w; i += step)
 #pragma unroll
@@ -81,7 +99,7 @@ __global__ __launch_bounds__(1024) void residual_norm_kernel(
       float g[V];
       load_f<V>(g, x_norm + i);
 #pragma unroll
-      for (int k = 0; k < V; ++k) t[k] *= g[k];
+      for (int k = 0; k < V; ++k) t[k] *= f.offset + g[k];
     }
     store_f<V>(orow + i, t);
   }
@@ -106,23 +124,24 @@ __global__ __launch_bounds__(256) void add_to_residual_kernel(
 template <typename T>
 static void residual_norm_t(float* x, const void* y, const void* y_norm,
                             const void* x_norm, void* out, float eps, int n,
-                            int w, int64_t out_stride, hipStream_t stream) {
+                            int w, int64_t out_stride, const NormForm& f,
+                            hipStream_t stream) {
   const bool vec = w % 4 == 0 && out_stride % 4 == 0;
   int threads = w >= 1024 ? 256 : w >= 512 ? 128 : 64;
   // few rows: the latency of one counts
   while (n <= 512 && threads < 1024 && threads * 4 < w) threads *= 2;
   auto k = vec ? residual_norm_kernel<T, 4> : residual_norm_kernel<T, 1>;
   k<<<n, threads, w * sizeof(float), stream>>>(
-      x, (const T*)y, (const T*)y_norm, (const T*)x_norm, (T*)out, eps, w, out_stride);
+      x, (const T*)y, (const T*)y_norm, (const T*)x_norm, (T*)out, eps, w, out_stride, f);
 }
 
 extern "C" {
 
 void launch_residual_norm(bool bf16, float* x, const void* y, const void* y_norm,
                           const void* x_norm, void* out, float eps, int n, int w,
-                          int64_t out_stride, hipStream_t stream) {
+                          int64_t out_stride, const NormForm* f, hipStream_t stream) {
   (bf16 ? residual_norm_t<bf16_t> : residual_norm_t<float>)(
-      x, y, y_norm, x_norm, out, eps, n, w, out_stride, stream);
+      x, y, y_norm, x_norm, out, eps, n, w, out_stride, *f, stream);
 }
 
 void launch_add_to_residual(bool bf16, float* x, const void* y, void* out,
