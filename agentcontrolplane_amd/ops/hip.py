@@ -327,11 +327,13 @@ def grouped_attention(q, k_cache, v_cache, batch, scale: float, cap, window, kee
 # ----------------------------------------------------------------- delta rule
 
 
-def _step_threads(D: int, V: int) -> int:
-    """Threads of a decode workgroup: at most 16 rows of the state per thread."""
+def _step_threads(D: int, V: int, workgroups: int) -> int:
+    """Threads of a decode workgroup: at most 16 rows of the state per thread, fewer
+    while the workgroups do not fill the chip."""
     columns = V // 4 if V % 4 == 0 else V
+    rows = 16 if workgroups >= 512 else 4
     for n in (256, 512):
-        if n >= columns and n // columns * 16 >= D:
+        if n >= columns and n // columns * rows >= D:
             return n
     return 1024
 
@@ -363,7 +365,7 @@ def channel_delta(qkv, conv, b, z, A_log, dt_bias, gate, norm, eps, unit_eps, kv
     if batch.num_decode:
         _C.delta_step(
             *rows(slice(P, None)), batch.decode_lens_i32(), batch.decode_state_slots, kv_heads,
-            eps, unit_eps, _step_threads(D, V),
+            eps, unit_eps, _step_threads(D, V, batch.num_decode * H),
         )
     return out
 

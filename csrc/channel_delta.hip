@@ -21,27 +21,65 @@
 #include "common_t.h"
 #include "channel_delta.h"
 
-DEV float silu_f(float x) { return x / (1.f + expf(-x)); }
-DEV float softplus_f(float x) { return x > 20.f ? x : log1pf(expf(x)); }
-DEV float decay_f(float z, float A_log) { return expf(-expf(A_log) * softplus_f(z)); }
+DEV float silu_f(float x) { return x * __builtin_amdgcn_rcpf(1.f + __expf(-x)); }
 
-// convolution of channels c .. c + VW - 1 at position p, rounded as the model stores it;
-// row: the token's input row, ``back`` rows before it are this step's
-template <typename T, int VW>
-DEV void conv_silu(float* y, const DeltaArgs& a, const T* row, const T* ring, int c, int p,
-                   int back) {
-  const T* w = (const T*)a.conv + (int64_t)c * a.taps;
+// log(1 + e^x) with a small relative error everywhere: log(u) e / (u - 1), u = 1 + e
+DEV float softplus_f(float x) {
+  if (x > 20.f) return x;
+  const float e = __expf(x), u = 1.f + e;
+  return u == 1.f ? e : __logf(u) * e * __builtin_amdgcn_rcpf(u - 1.f);
+}
+
+// rate = exp(A_log)
+DEV float decay_f(float z, float rate) { return __expf(-rate * softplus_f(z)); }
+
+// Where a token's convolution finds its inputs: ``back`` rows before ``row`` belong to
+// this step, older ones are in the ring.  p: the token's position.
+template <typename T>
+struct ConvInput {
+  const T* row;
+  const T* ring;
+  int p, back, taps, C;
+  int64_t stride;
+  // input ``ago`` tokens earlier, or null before the start
+  DEV const T* at(int ago) const {
+    if (ago <= back) return row - ago * stride;
+    return ago > p ? nullptr : ring + (int64_t)((p - ago) % taps) * C;
+  }
+};
+
+// convolution of channels c .. c + VW - 1, rounded as the model stores it; TAPS = 0:
+// any number
+template <typename T, int VW, int TAPS>
+DEV void conv_silu(float* y, const T* conv, const ConvInput<T>& in, int c) {
 #pragma unroll
   for (int k = 0; k < VW; ++k) y[k] = 0.f;
-  for (int n = 0; n < a.taps; ++n) {
-    const int ago = a.taps - 1 - n;  // tokens before this one
-    if (ago > p) continue;
-    const T* src = ago <= back ? row - ago * a.qkv_stride
-                               : ring + (int64_t)((p - ago) % a.taps) * a.C;
-    float x[VW];
-    load_f<VW>(x, src + c);
+  if constexpr (TAPS > 0) {
+    // all loads first
+    Pack<T, VW> x[TAPS];
+    Pack<T, TAPS> w[VW];
+    bool have[TAPS];
 #pragma unroll
-    for (int k = 0; k < VW; ++k) y[k] += to_f(w[k * a.taps + n]) * x[k];
+    for (int n = 0; n < TAPS; ++n) {
+      const T* src = in.at(TAPS - 1 - n);
+      have[n] = src;
+      x[n] = *(const Pack<T, VW>*)((src ? src : in.row) + c);
+    }
+#pragma unroll
+    for (int k = 0; k < VW; ++k) w[k] = *(const Pack<T, TAPS>*)(conv + (int64_t)(c + k) * TAPS);
+#pragma unroll
+    for (int n = 0; n < TAPS; ++n)
+#pragma unroll
+      for (int k = 0; k < VW; ++k) y[k] += have[n] ? to_f(w[k].v[n]) * to_f(x[n].v[k]) : 0.f;
+  } else {
+    for (int n = 0; n < in.taps; ++n) {
+      const T* src = in.at(in.taps - 1 - n);
+      if (!src) continue;
+      float x[VW];
+      load_f<VW>(x, src + c);
+#pragma unroll
+      for (int k = 0; k < VW; ++k) y[k] += to_f(conv[(int64_t)(c + k) * in.taps + n]) * x[k];
+    }
   }
 #pragma unroll
   for (int k = 0; k < VW; ++k) y[k] = to_f(from_f<T>(silu_f(y[k])));
@@ -58,32 +96,33 @@ __global__ __launch_bounds__(256) void delta_inputs_kernel(const DeltaArgs a) {
   const int ctx = a.ctx_lens[seq], len = a.seq_lens[seq] - ctx;
   const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
   const T* ring = (const T*)a.ring + (int64_t)a.slots[seq] * a.taps * a.C;
+  const T* conv = (const T*)a.conv;
   for (int i = wid; i < 16; i += 4) {
     const int t = q0 + i;
     if (t >= len) return;
     const int64_t n = a.row_starts[seq] + t;
     if (job >= a.G + a.H) {
       const int h = job - a.G - a.H;
-      const float A_log = a.A_log[h];
+      const float rate = expf(a.A_log[h]);
       const T* z = (const T*)a.z + n * a.z_stride + (int64_t)h * a.D;
       float* g = a.g + (n * a.H + h) * a.D;
       for (int d = lane * VW; d < a.D; d += 64 * VW) {
         float v[VW];
         load_f<VW>(v, z + d);
 #pragma unroll
-        for (int k = 0; k < VW; ++k) v[k] = decay_f(v[k] + a.dt_bias[h * a.D + d + k], A_log);
+        for (int k = 0; k < VW; ++k) v[k] = decay_f(v[k] + a.dt_bias[h * a.D + d + k], rate);
         store_f<VW>(g + d, v);
       }
       continue;
     }
-    const T* row = (const T*)a.qkv + n * a.qkv_stride;
+    const ConvInput<T> in = {(const T*)a.qkv + n * a.qkv_stride, ring, ctx + t, t, a.taps, a.C,
+                             a.qkv_stride};
     T* y = (T*)a.y + n * a.C;
-    const int p = ctx + t;
     if (job >= a.G) {
       const int c0 = 2 * a.G * a.D + (job - a.G) * a.V;
       for (int d = lane * VW; d < a.V; d += 64 * VW) {
         float v[VW];
-        conv_silu<T, VW>(v, a, row, ring, c0 + d, p, t);
+        conv_silu<T, VW, 0>(v, conv, in, c0 + d);
         store_f<VW>(y + c0 + d, v);
       }
       continue;
@@ -92,8 +131,8 @@ __global__ __launch_bounds__(256) void delta_inputs_kernel(const DeltaArgs a) {
     float qq = 0.f, kk = 0.f, kq = 0.f;
     for (int d = lane * VW; d < a.D; d += 64 * VW) {
       float q[VW], k[VW];
-      conv_silu<T, VW>(q, a, row, ring, cq + d, p, t);
-      conv_silu<T, VW>(k, a, row, ring, ck + d, p, t);
+      conv_silu<T, VW, 0>(q, conv, in, cq + d);
+      conv_silu<T, VW, 0>(k, conv, in, ck + d);
       store_f<VW>(y + cq + d, q);
       store_f<VW>(y + ck + d, k);
 #pragma unroll
@@ -110,9 +149,142 @@ __global__ __launch_bounds__(256) void delta_inputs_kernel(const DeltaArgs a) {
   }
 }
 
+// The same for the usual sizes: 4 taps, heads of at most 16 vectors of VW channels.  A
+// thread owns VW channels (16 of them a key head, q and k together) and walks the tile's
+// tokens, so that every input is loaded once, a token ahead.
+template <typename T, int VW>
+__global__ __launch_bounds__(256) void delta_inputs_wide_kernel(const DeltaArgs a) {
+  const int tile = blockIdx.x;
+  const int seq = a.tile_seq[tile], q0 = a.tile_q0[tile];
+  const int ctx = a.ctx_lens[seq], n = min(16, a.seq_lens[seq] - ctx - q0);
+  const int64_t row0 = a.row_starts[seq] + q0;
+  int unit = blockIdx.y * 256 + threadIdx.x;
+
+  if (unit >= a.G * 16 + a.H * a.V / VW) {  // decays
+    const int c = (unit - a.G * 16 - a.H * a.V / VW) * VW;
+    if (c >= a.H * a.D) return;
+    const float rate = expf(a.A_log[c / a.D]);
+    float bias[VW];
+#pragma unroll
+    for (int k = 0; k < VW; ++k) bias[k] = a.dt_bias[c + k];
+    const T* z = (const T*)a.z + row0 * a.z_stride + c;
+    float* g = a.g + row0 * a.H * a.D + c;
+    Pack<T, VW> next = *(const Pack<T, VW>*)z;
+    for (int t = 0; t < n; ++t) {
+      const Pack<T, VW> x = next;
+      if (t + 1 < n) next = *(const Pack<T, VW>*)(z + (t + 1) * a.z_stride);
+      float v[VW];
+#pragma unroll
+      for (int k = 0; k < VW; ++k) v[k] = decay_f(to_f(x.v[k]) + bias[k], rate);
+#pragma unroll
+      for (int k = 0; k < VW; k += 4) store_f<4>(g + (int64_t)t * a.H * a.D + k, v + k);
+    }
+    return;
+  }
+
+  const ConvInput<T> in = {(const T*)a.qkv + row0 * a.qkv_stride,
+                           (const T*)a.ring + (int64_t)a.slots[seq] * 4 * a.C, ctx + q0, q0, 4,
+                           a.C, a.qkv_stride};
+  struct Channels {
+    float w[4][VW], past[3][VW];
+    Pack<T, VW> next;
+    int c;
+  };
+  auto open = [&](Channels& s, int c) {
+    s.c = c;
+    const T* w = (const T*)a.conv + (int64_t)c * 4;
+#pragma unroll
+    for (int k = 0; k < VW; ++k) {
+      float t[4];
+      load_f<4>(t, w + 4 * k);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) s.w[i][k] = t[i];
+    }
+#pragma unroll
+    for (int i = 0; i < 3; ++i) {
+      const T* src = in.at(3 - i);
+#pragma unroll
+      for (int k = 0; k < VW; ++k) s.past[i][k] = 0.f;
+      if (src) load_f<VW>(s.past[i], src + c);
+    }
+    s.next = *(const Pack<T, VW>*)(in.row + c);
+  };
+  auto advance = [&](Channels& s, float* y, int t) {
+    const Pack<T, VW> x = s.next;
+    if (t + 1 < n) s.next = *(const Pack<T, VW>*)(in.row + (t + 1) * a.qkv_stride + s.c);
+#pragma unroll
+    for (int k = 0; k < VW; ++k) {
+      const float v = to_f(x.v[k]);
+      y[k] = 0.f;
+#pragma unroll
+      for (int i = 0; i < 3; ++i) y[k] += s.w[i][k] * s.past[i][k];
+      y[k] += s.w[3][k] * v;
+      s.past[0][k] = s.past[1][k];
+      s.past[1][k] = s.past[2][k];
+      s.past[2][k] = v;
+      y[k] = to_f(from_f<T>(silu_f(y[k])));
+    }
+    store_f<VW>((T*)a.y + (row0 + t) * a.C + s.c, y);
+  };
+
+  if (unit >= a.G * 16) {  // v
+    Channels v;
+    open(v, 2 * a.G * a.D + (unit - a.G * 16) * VW);
+    float y[VW];
+    for (int t = 0; t < n; ++t) advance(v, y, t);
+    return;
+  }
+  const int head = unit >> 4, j = unit & 15;
+  const bool live = j * VW < a.D;
+  const int d = head * a.D + (live ? j * VW : 0);
+  Channels q, k;
+  open(q, d);
+  open(k, a.G * a.D + d);
+  for (int t = 0; t < n; ++t) {
+    float yq[VW], yk[VW], qq = 0.f, kk = 0.f, kq = 0.f;
+    if (live) {
+      advance(q, yq, t);
+      advance(k, yk, t);
+#pragma unroll
+      for (int e = 0; e < VW; ++e) {
+        qq += yq[e] * yq[e];
+        kk += yk[e] * yk[e];
+        kq += yk[e] * yq[e];
+      }
+    }
+    const float rq = a.q_scale * rsqrtf(row16_sum(qq) + a.unit_eps);
+    const float rk = rsqrtf(row16_sum(kk) + a.unit_eps);
+    kq = row16_sum(kq) * rq * rk;
+    if (j < 3)
+      a.unit[((row0 + t) * a.G + head) * 3 + j] = j == 0 ? rq : j == 1 ? rk : kq;
+  }
+}
+
+// N elements as they were loaded, in whole words: taking them apart any earlier than
+// needed would wait for the load.
+template <typename T, int N>
+struct Words {
+  static constexpr int COUNT = (N * sizeof(T) + 3) / 4;
+  unsigned w[COUNT];
+  DEV void load(const T* p) {
+    if constexpr (N * sizeof(T) == 2) {
+      w[0] = *(const unsigned short*)p;
+    } else {
+      const Pack<unsigned, COUNT> x = *(const Pack<unsigned, COUNT>*)p;
+#pragma unroll
+      for (int i = 0; i < COUNT; ++i) w[i] = x.v[i];
+    }
+  }
+  DEV float at(int i) const {
+    if (sizeof(T) == 4) return __uint_as_float(w[i]);
+    return __uint_as_float(i & 1 ? w[i >> 1] & 0xffff0000u : w[i >> 1] << 16);
+  }
+};
+
 // grid (column blocks, H, seqs).  Lane j of a column's 16 holds the dims
 // (e / VW) * 16 VW + j VW + e % VW: its LDS reads are VW wide and 16 lanes contiguous.
-template <typename T, int DPL, int CPL>
+// FULL: D = 16 DPL and rows are aligned to VW channels.
+template <typename T, int DPL, int CPL, bool FULL>
 __global__ __launch_bounds__(256) void delta_scan_kernel(const DeltaArgs a) {
   constexpr int TT = DPL <= 16 ? 16 : 256 / DPL;  // tokens staged at a time
   constexpr int DP = 16 * DPL;
@@ -139,50 +311,49 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(const DeltaArgs a) {
 
   // staging: a thread brings its dims and columns of one token (16 threads a token)
   const int tok = tid >> 4;
-  const bool wide = a.D % VW == 0 && a.C % VW == 0;
-  Pack<T, VW> rq[NV], rk[NV];
-  Pack<float, VW> rg[NV];
-  float rv[CPL], fq, fk, fb, fkq;
+  constexpr int PW = FULL ? VW : 1, PV = DPL / PW;  // pieces of a thread's dims
+  Words<T, PW> rq[PV], rk[PV];
+  Words<float, PW> rg[PV];
+  Words<T, 1> rv[CPL], fb;
+  float fq, fk, fkq;
+  const int t_in = min(tok, len - 1);  // where this thread reads on past the end
+  const T* py = (const T*)a.y + (row0 + t_in) * a.C;
+  const T* pq = py + kvh * a.D;
+  const T* pk = py + (a.G + kvh) * a.D;
+  const T* pv = py + 2 * a.G * a.D + h * a.V;
+  const float* pg = a.g + ((row0 + t_in) * a.H + h) * a.D;
+  const float* pu = a.unit + ((row0 + t_in) * a.G + kvh) * 3;
+  const T* pb = (const T*)a.b + (row0 + t_in) * a.b_stride + h;
+  const int64_t y_step = (int64_t)TT * a.C, g_step = (int64_t)TT * a.H * a.D;
+  const int64_t b_step = TT * a.b_stride;
+  const int u_step = TT * a.G * 3;
   auto fetch = [&](int t0) {
-    const int t = t0 + tok;
-    const bool in = tok < TT && t < len;
-    const int64_t n = row0 + (in ? t : 0);
-    const T* y = (const T*)a.y + n * a.C;
-    const T* yq = y + kvh * a.D;
-    const T* yk = y + (a.G + kvh) * a.D;
-    const float* g = a.g + (n * a.H + h) * a.D;
 #pragma unroll
-    for (int i = 0; i < NV; ++i) {
-      const int d = dim(i * VW);
-      if (wide) {
-        if (d < a.D) {
-          rq[i] = *(const Pack<T, VW>*)(yq + d);
-          rk[i] = *(const Pack<T, VW>*)(yk + d);
-          rg[i] = *(const Pack<float, VW>*)(g + d);
-        }
-      } else {
-#pragma unroll
-        for (int k = 0; k < VW; ++k)
-          if (d + k < a.D) {
-            rq[i].v[k] = yq[d + k];
-            rk[i].v[k] = yk[d + k];
-            rg[i].v[k] = g[d + k];
-          }
-      }
+    for (int i = 0; i < PV; ++i) {
+      const int d = FULL ? dim(i * PW) : min(dim(i * PW), a.D - 1);
+      rq[i].load(pq + d);
+      rk[i].load(pk + d);
+      rg[i].load(pg + d);
     }
 #pragma unroll
-    for (int c = 0; c < CPL; ++c) {
-      const int col = min(col0 + j * CPL + c, a.V - 1);
-      rv[c] = to_f(y[2 * a.G * a.D + h * a.V + col]);
+    for (int c = 0; c < CPL; ++c) rv[c].load(pv + min(col0 + j * CPL + c, a.V - 1));
+    fq = pu[0];
+    fk = pu[1];
+    fkq = pu[2];
+    fb.load(pb);
+    if (t0 + TT + tok < len) {
+      pq += y_step;
+      pk += y_step;
+      pv += y_step;
+      pg += g_step;
+      pu += u_step;
+      pb += b_step;
     }
-    const float* u = a.unit + (n * a.G + kvh) * 3;
-    fq = u[0];
-    fk = u[1];
-    fkq = u[2];
-    fb = to_f(((const T*)a.b)[n * a.b_stride + h]);
   };
-  auto put = [&](int buf) {
+  // tokens past the end change nothing: g = 1, k = q = beta = 0
+  auto put = [&](int buf, int t0) {
     if (tok >= TT) return;
+    const bool in = t0 + tok < len;
     float* at = lds + (buf * 3 * TT + tok) * DP;
 #pragma unroll
     for (int i = 0; i < NV; ++i) {
@@ -190,10 +361,11 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(const DeltaArgs a) {
       Pack<float, VW> q, k, g;
 #pragma unroll
       for (int e = 0; e < VW; ++e) {
-        const bool in = d + e < a.D;
-        q.v[e] = in ? to_f(rq[i].v[e]) * fq : 0.f;
-        k.v[e] = in ? to_f(rk[i].v[e]) * fk : 0.f;
-        g.v[e] = in ? rg[i].v[e] : 0.f;
+        const int p = (i * VW + e) / PW, o = e % PW;
+        const bool has = in && (FULL || d + e < a.D);
+        q.v[e] = has ? rq[p].at(o) * fq : 0.f;
+        k.v[e] = has ? rk[p].at(o) * fk : 0.f;
+        g.v[e] = has ? rg[p].at(o) : 1.f;
       }
       *(Pack<float, VW>*)(at + d) = q;
       *(Pack<float, VW>*)(at + TT * DP + d) = k;
@@ -201,57 +373,76 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(const DeltaArgs a) {
     }
     float* side = side0 + (buf * TT + tok) * SIDE;
 #pragma unroll
-    for (int c = 0; c < CPL; ++c) side[j * CPL + c] = rv[c];
+    for (int c = 0; c < CPL; ++c) side[j * CPL + c] = rv[c].at(0);
     if (j == 0) {
-      side[COLS] = sigmoid_f(fb);
-      side[COLS + 1] = fkq;
+      side[COLS] = in ? sigmoid_f(fb.at(0)) : 0.f;
+      side[COLS + 1] = in ? fkq : 0.f;
     }
   };
 
+  struct Token {
+    float q[DPL], k[DPL], g[DPL], v[CPL], beta, kq;
+  };
+  float* po = a.o + ((row0 + j) * a.H + h) * a.V + col0 + mine;  // token j of a chunk
   fetch(0);
-  put(0);
+  put(0, 0);
   __syncthreads();
   for (int t0 = 0, buf = 0; t0 < len; t0 += TT, buf ^= 1) {
     const bool more = t0 + TT < len;
     if (more) fetch(t0 + TT);
     const int n = min(TT, len - t0);
     float keep[CPL] = {};  // lane j: the output of token j
-    for (int t = 0; t < n; ++t) {
+    auto load = [&](Token& x, int t) {
       const float* at = lds + (buf * 3 * TT + t) * DP + j * VW;
       const float* side = side0 + (buf * TT + t) * SIDE;
-      float q[DPL], k[DPL], g[DPL];
 #pragma unroll
       for (int i = 0; i < NV; ++i) {
-        load_f<VW>(q + i * VW, at + i * 16 * VW);
-        load_f<VW>(k + i * VW, at + TT * DP + i * 16 * VW);
-        load_f<VW>(g + i * VW, at + 2 * TT * DP + i * 16 * VW);
+        load_f<VW>(x.q + i * VW, at + i * 16 * VW);
+        load_f<VW>(x.k + i * VW, at + TT * DP + i * 16 * VW);
+        load_f<VW>(x.g + i * VW, at + 2 * TT * DP + i * 16 * VW);
       }
-      const float beta = side[COLS], kq = side[COLS + 1];
+#pragma unroll
+      for (int c = 0; c < CPL; ++c) x.v[c] = side[mine + c];
+      x.beta = side[COLS];
+      x.kq = side[COLS + 1];
+    };
+    auto run = [&](const Token& x, int t) {
 #pragma unroll
       for (int c = 0; c < CPL; ++c) {
         float sk = 0.f, sq = 0.f;
 #pragma unroll
         for (int e = 0; e < DPL; ++e) {
-          s[c][e] *= g[e];
-          sk += k[e] * s[c][e];
-          sq += q[e] * s[c][e];
+          s[c][e] *= x.g[e];
+          sk += x.k[e] * s[c][e];
+          sq += x.q[e] * s[c][e];
         }
         sk = row16_sum(sk);
         sq = row16_sum(sq);
-        const float u = beta * (side[mine + c] - sk);
-        const float o = sq + kq * u;
+        const float u = x.beta * (x.v[c] - sk);
+        const float o = sq + x.kq * u;
         keep[c] = j == t ? o : keep[c];
 #pragma unroll
-        for (int e = 0; e < DPL; ++e) s[c][e] += k[e] * u;
+        for (int e = 0; e < DPL; ++e) s[c][e] += x.k[e] * u;
       }
+    };
+    // a token's operands are read while the one before is worked on
+    Token even, odd;
+    load(even, 0);
+    for (int t = 0; t < n; t += 2) {
+      load(odd, t + 1);
+      __builtin_amdgcn_sched_barrier(0);
+      run(even, t);
+      load(even, min(t + 2, TT - 1));
+      __builtin_amdgcn_sched_barrier(0);
+      run(odd, t + 1);
     }
     if (j < n) {
-      float* o = a.o + ((row0 + t0 + j) * a.H + h) * a.V + col0 + mine;
 #pragma unroll
       for (int c = 0; c < CPL; ++c)
-        if (col0 + mine + c < a.V) o[c] = keep[c];
+        if (col0 + mine + c < a.V) po[c] = keep[c];
     }
-    if (more) put(buf ^ 1);
+    po += (int64_t)TT * a.H * a.V;
+    if (more) put(buf ^ 1, t0 + TT);
     __syncthreads();
   }
 
@@ -279,27 +470,38 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(const DeltaArgs a) {
 }
 
 // A wave per token and head.
-template <typename T>
+template <typename T, int VW>
 __global__ __launch_bounds__(256) void delta_output_kernel(const DeltaArgs a) {
   const int64_t i = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
   if (i >= (int64_t)a.N * a.H) return;
   const int64_t n = i / a.H;
   const int h = (int)(i - n * a.H), lane = threadIdx.x & 63;
   const float* o = a.o + i * a.V;
-  float ss = 0.f;
-  for (int d = lane; d < a.V; d += 64) ss += o[d] * o[d];
-  const float inv = rsqrtf(wave_sum(ss) / a.V + a.eps);
   const T* gate = (const T*)a.gate + n * a.gate_stride + (int64_t)h * a.V;
+  float ss = 0.f;
+  for (int d = lane * VW; d < a.V; d += 64 * VW) {
+    float x[VW];
+    load_f<VW>(x, o + d);
+#pragma unroll
+    for (int k = 0; k < VW; ++k) ss += x[k] * x[k];
+  }
+  const float inv = rsqrtf(wave_sum(ss) / a.V + a.eps);
   T* out = (T*)a.out + i * a.V;
-  for (int d = lane; d < a.V; d += 64)
-    out[d] = from_f<T>(o[d] * inv * a.norm[d] * sigmoid_f(to_f(gate[d])));
+  for (int d = lane * VW; d < a.V; d += 64 * VW) {
+    float x[VW], g[VW];
+    load_f<VW>(x, o + d);
+    load_f<VW>(g, gate + d);
+#pragma unroll
+    for (int k = 0; k < VW; ++k) x[k] *= inv * a.norm[d + k] * sigmoid_f(g[k]);
+    store_f<VW>(out + d, x);
+  }
 }
 
 // ----------------------------------------------------------------- decode
 
 // grid (H, seqs): a thread owns VW columns of every RG-th row of S, at most ROWS rows;
 // ROWS = 0: any number, S is read twice.
-template <typename T, int VW, int ROWS>
+template <typename T, int VW, int ROWS, int TAPS>
 __global__ __launch_bounds__(1024) void delta_step_kernel(const DeltaArgs a) {
   extern __shared__ float lds[];
   const int h = blockIdx.x, seq = blockIdx.y;
@@ -331,26 +533,34 @@ __global__ __launch_bounds__(1024) void delta_step_kernel(const DeltaArgs a) {
   // convolutions; the input joins the ring
   const int p = a.seq_lens[seq] - 1;
   const T* row = (const T*)a.qkv + seq * a.qkv_stride;
+  const T* conv = (const T*)a.conv;
   T* ring = (T*)a.ring + slot * a.taps * a.C;
+  T* entry = ring + (int64_t)(p % a.taps) * a.C;
+  const ConvInput<T> in = {row, ring, p, 0, a.taps, a.C, 0};
   float qq = 0.f, kk = 0.f, kq = 0.f;
+  const float rate = expf(a.A_log[h]);
   for (int d = tid; d < a.D; d += threads) {
-    const int cq = kvh * a.D + d, ck = (a.G + kvh) * a.D + d;
-    conv_silu<T, 1>(q + d, a, row, ring, cq, p, 0);
-    conv_silu<T, 1>(k + d, a, row, ring, ck, p, 0);
+    const int cq = kvh * a.D + d, ck = (a.G + kvh) * a.D + d, hd = h * a.D + d;
+    float y[2];
+    conv_silu<T, 1, TAPS>(y, conv, in, cq);
+    conv_silu<T, 1, TAPS>(y + 1, conv, in, ck);
+    g[d] = decay_f(to_f(((const T*)a.z)[seq * a.z_stride + hd]) + a.dt_bias[hd], rate);
+    q[d] = y[0];
+    k[d] = y[1];
     if (h == kvh * group) {
-      ring[(int64_t)(p % a.taps) * a.C + cq] = row[cq];
-      ring[(int64_t)(p % a.taps) * a.C + ck] = row[ck];
+      entry[cq] = row[cq];
+      entry[ck] = row[ck];
     }
-    qq += q[d] * q[d];
-    kk += k[d] * k[d];
-    kq += k[d] * q[d];
-    const int hd = h * a.D + d;
-    g[d] = decay_f(to_f(((const T*)a.z)[seq * a.z_stride + hd]) + a.dt_bias[hd], a.A_log[h]);
+    qq += y[0] * y[0];
+    kk += y[1] * y[1];
+    kq += y[1] * y[0];
   }
-  for (int d = tid; d < a.V; d += threads) {
+  for (int d = threads - 1 - tid; d < a.V; d += threads) {  // from the other end
     const int c = 2 * a.G * a.D + h * a.V + d;
-    conv_silu<T, 1>(v + d, a, row, ring, c, p, 0);
-    ring[(int64_t)(p % a.taps) * a.C + c] = row[c];
+    float y;
+    conv_silu<T, 1, TAPS>(&y, conv, in, c);
+    v[d] = y;
+    entry[c] = row[c];
   }
   qq = wave_sum(qq);
   kk = wave_sum(kk);
@@ -451,36 +661,48 @@ __global__ __launch_bounds__(1024) void delta_step_kernel(const DeltaArgs a) {
 
 // ---------------------------------------------------------------- launches
 
-template <typename T, int DPL, int CPL>
+template <typename T, int DPL, int CPL, bool FULL>
 static void launch_scan(const DeltaArgs& a, hipStream_t stream) {
   constexpr int TT = DPL <= 16 ? 16 : 256 / DPL;
   constexpr int bytes = 4 * (2 * 3 * TT * 16 * DPL + 2 * TT * (16 * CPL + 4));
   static_assert(bytes <= 160 * 1024, "LDS");
   static bool attr_set = false;
   if (!attr_set) {
-    (void)hipFuncSetAttribute((const void*)delta_scan_kernel<T, DPL, CPL>,
+    (void)hipFuncSetAttribute((const void*)delta_scan_kernel<T, DPL, CPL, FULL>,
                               hipFuncAttributeMaxDynamicSharedMemorySize, bytes);
     attr_set = true;
   }
   const dim3 grid((a.V + 16 * CPL - 1) / (16 * CPL), a.H, a.seqs);
-  delta_scan_kernel<T, DPL, CPL><<<grid, 256, bytes, stream>>>(a);
+  delta_scan_kernel<T, DPL, CPL, FULL><<<grid, 256, bytes, stream>>>(a);
 }
 
 template <typename T, int DPL>
 static void launch_scan_cols(const DeltaArgs& a, int cpl, hipStream_t stream) {
-  if (cpl == 1 || DPL > 8)
-    launch_scan<T, DPL, 1>(a, stream);
+  constexpr int VW = DPL < 4 ? DPL : 4;
+  if (a.D != 16 * DPL || a.C % VW != 0)
+    launch_scan<T, DPL, 1, false>(a, stream);
+  else if (cpl == 1 || DPL > 8)
+    launch_scan<T, DPL, 1, true>(a, stream);
   else if constexpr (DPL <= 8)
-    launch_scan<T, DPL, 2>(a, stream);
+    launch_scan<T, DPL, 2, true>(a, stream);
 }
 
 template <typename T>
 static void prompts(const DeltaArgs& a, int cpl, hipStream_t stream) {
-  const dim3 grid(a.n_tiles, a.G + 2 * a.H);
-  // pairs of channels: every head then starts at an even one
-  const bool even = a.D % 2 == 0 && a.V % 2 == 0 && a.z_stride % 2 == 0 && a.qkv_stride % 2 == 0;
-  auto inputs = even ? delta_inputs_kernel<T, 2> : delta_inputs_kernel<T, 1>;
-  inputs<<<grid, 256, 0, stream>>>(a);
+  constexpr int W = 16 / sizeof(T);
+  auto all = [&](int n) {  // every head and row starts at a multiple of n channels
+    return a.D % n == 0 && a.V % n == 0 && a.z_stride % n == 0 && a.qkv_stride % n == 0 &&
+           a.gate_stride % n == 0;
+  };
+  const bool aligned = ((uintptr_t)a.qkv | (uintptr_t)a.z | (uintptr_t)a.gate) % 16 == 0;
+  if (aligned && all(W) && a.taps == 4 && a.D <= 16 * W) {
+    const int units = a.G * 16 + a.H * (a.V + a.D) / W;
+    delta_inputs_wide_kernel<T, W><<<dim3(a.n_tiles, (units + 255) / 256), 256, 0, stream>>>(a);
+  } else {
+    const dim3 grid(a.n_tiles, a.G + 2 * a.H);
+    auto inputs = all(2) ? delta_inputs_kernel<T, 2> : delta_inputs_kernel<T, 1>;
+    inputs<<<grid, 256, 0, stream>>>(a);
+  }
   if (a.D <= 16) launch_scan_cols<T, 1>(a, cpl, stream);
   else if (a.D <= 32) launch_scan_cols<T, 2>(a, cpl, stream);
   else if (a.D <= 64) launch_scan_cols<T, 4>(a, cpl, stream);
@@ -489,19 +711,29 @@ static void prompts(const DeltaArgs& a, int cpl, hipStream_t stream) {
   else if (a.D <= 512) launch_scan_cols<T, 32>(a, cpl, stream);
   else launch_scan_cols<T, 64>(a, cpl, stream);
   const int64_t heads = (int64_t)a.N * a.H;
-  delta_output_kernel<T><<<(heads + 3) / 4, 256, 0, stream>>>(a);
+  auto output = aligned && all(4)   ? delta_output_kernel<T, 4>
+                : aligned && all(2) ? delta_output_kernel<T, 2> : delta_output_kernel<T, 1>;
+  output<<<(heads + 3) / 4, 256, 0, stream>>>(a);
 }
 
-template <typename T, int VW>
+template <typename T, int VW, int TAPS>
 static void step(const DeltaArgs& a, int threads, hipStream_t stream) {
   const int ct = a.V / VW, RG = threads / ct, rows = (a.D + RG - 1) / RG;
   const int bytes = 4 * (3 * a.D + 2 * a.V + 2 * RG * a.V + threads / 64 * 4);
   const dim3 grid(a.H, a.seqs);
-  auto k = rows <= 4    ? delta_step_kernel<T, VW, 4>
-           : rows <= 8  ? delta_step_kernel<T, VW, 8>
-           : rows <= 16 ? delta_step_kernel<T, VW, 16>
-                        : delta_step_kernel<T, VW, 0>;
+  auto k = rows <= 4    ? delta_step_kernel<T, VW, 4, TAPS>
+           : rows <= 8  ? delta_step_kernel<T, VW, 8, TAPS>
+           : rows <= 16 ? delta_step_kernel<T, VW, 16, TAPS>
+                        : delta_step_kernel<T, VW, 0, TAPS>;
   k<<<grid, threads, bytes, stream>>>(a);
+}
+
+template <typename T>
+static void step_any(const DeltaArgs& a, int threads, hipStream_t stream) {
+  if (a.V % 4 == 0)
+    a.taps == 4 ? step<T, 4, 4>(a, threads, stream) : step<T, 4, 0>(a, threads, stream);
+  else
+    a.taps == 4 ? step<T, 1, 4>(a, threads, stream) : step<T, 1, 0>(a, threads, stream);
 }
 
 extern "C" {
@@ -513,10 +745,7 @@ void launch_delta_prompts(bool bf16, const DeltaArgs* a, int cpl, hipStream_t st
 
 // V % 4 == 0 or V <= threads
 void launch_delta_step(bool bf16, const DeltaArgs* a, int threads, hipStream_t stream) {
-  if (a->V % 4 == 0)
-    (bf16 ? step<bf16_t, 4> : step<float, 4>)(*a, threads, stream);
-  else
-    (bf16 ? step<bf16_t, 1> : step<float, 1>)(*a, threads, stream);
+  (bf16 ? step_any<bf16_t> : step_any<float>)(*a, threads, stream);
 }
 
 }  // extern "C"

@@ -7,8 +7,8 @@
 // merge of partial sums nor the output knows about it.
 //
 // Decode: a workgroup owns one (sequence, key/value head) and up to GM of its query
-// heads; its 16 lane groups of 16 take every 16th visible key, 4 keys in flight, a
-// lane KE dims of the key and VE of the value.  Kept and window keys form one list
+// heads; its 16 lane groups of 16 take every 16th visible key, a few of them in
+// flight, a lane KE dims of the key and VE of the value.  Kept and window keys form one list
 // without gaps, so nothing is masked.  Few workgroups split the list (grid.y).
 #include "common_t.h"
 #include "grouped_attn.h"
@@ -16,7 +16,6 @@
 
 #define NEG -1e30f
 #define LOG2E 1.44269504088896f
-#define KEYS 4   // keys in flight per lane group
 
 struct KeyList {  // of one query: position of the i-th visible key
   int keep, lo, n;
@@ -32,8 +31,10 @@ static DEV KeyList visible_keys(int pos, int window, int keep) {
 }
 
 template <int KE, int VE, int GM>
-__global__ __launch_bounds__(256) void grouped_decode_kernel(const GroupedArgs a) {
+__global__ __launch_bounds__(256, GM * (KE + VE) <= 32 ? 4 : GM * (KE + VE) <= 64 ? 3 : 2) void grouped_decode_kernel(
+    const GroupedArgs a) {
   constexpr int D = 16 * KE, V = 16 * VE;
+  constexpr int KEYS = GM * (KE + VE) <= 32 ? 4 : 2;  // in flight per lane group
   __shared__ float lds_acc[4][GM][V];
   __shared__ float2 lds_ml[4][GM];
   const int group = a.H / a.G, per = (group + GM - 1) / GM;  // workgroups per kv head
