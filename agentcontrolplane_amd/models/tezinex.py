@@ -57,7 +57,7 @@ class TezinexLayer:
         self.norm1 = self.norm1b = self.norm2 = self.norm2b = None
         self.gate_up: torch.Tensor = None
         self.down: torch.Tensor = None
-        self.depth: Optional[torch.Tensor] = None   # fp32, one per state so far
+        self.depth: Optional[torch.Tensor] = None   # depth weights, one per state so far
 
     def shapes(self, index: int, depth_average: bool) -> List[Tuple[str, Tuple[int, ...]]]:
         w = self.width
@@ -83,7 +83,7 @@ class TezinexLayer:
             ])
             self.down = pad_to(get(p + "mlp.down")[:, mine], self.width, self.ff_pad).contiguous()
         if depth_average:
-            self.depth = get(p + "dwa").float().contiguous()
+            self.depth = get(p + "dwa")
 
     def export(self, p: str) -> Dict[str, torch.Tensor]:
         out = {p + "norm1": self.norm1, p + "norm1b": self.norm1b}
@@ -94,7 +94,7 @@ class TezinexLayer:
             out[p + "mlp.up"] = self.gate_up[self.ff_pad : self.ff_pad + self.ff]
             out[p + "mlp.down"] = self.down[:, : self.ff]
         if self.depth is not None:
-            out[p + "dwa"] = self.depth.to(self.norm1.dtype)
+            out[p + "dwa"] = self.depth
         return out
 
     def feed_forward(self, h: torch.Tensor) -> torch.Tensor:
@@ -125,6 +125,7 @@ class TezinexForCausalLM:
             )
         self.embed: Optional[torch.Tensor] = None
         self.final_norm: Optional[torch.Tensor] = None
+        self.depth_coef: Optional[torch.Tensor] = None  # [layers, layers + 1] fp32
         # per layer: (keys, values), the owner's for borrowed ones, or (S, conv inputs)
         self.stores: List[Tuple[torch.Tensor, torch.Tensor]] = [None] * len(self.layers)
         # TP all-reduce hook installed by the engine
@@ -154,6 +155,11 @@ class TezinexForCausalLM:
         self.final_norm = mine("final.norm")
         for i, layer in enumerate(self.layers):
             layer.load(mine, f"l{i}.", self.cfg.depth_average)
+        if self.cfg.depth_average:
+            n = len(self.layers)
+            self.depth_coef = torch.zeros(n, n + 1, dtype=torch.float32, device=self.device)
+            for i, layer in enumerate(self.layers):
+                self.depth_coef[i, : i + 2] = layer.depth.float()
 
     def random_init(self, seed: int = 0) -> None:
         """Random weights of the config's shapes.  Every rank draws the same
@@ -233,14 +239,10 @@ class TezinexForCausalLM:
         every layer hands on."""
         cfg, eps, w, N = self.cfg, self.cfg.rms_eps, self.cfg.hidden_size, batch.num_tokens
         x = torch.empty(N, w, dtype=torch.float32, device=self.device)
-        depth = None
-        if cfg.depth_average:
-            depth = torch.empty(
-                len(self.layers) + 1, N, w, dtype=torch.float32, device=self.device
-            )
+        depth = None if self.depth_coef is None else ops.Depth.new(self.depth_coef, N, w)
         ops.embed_positions(
             batch.token_ids, batch.positions, self.embed, self.pos_table, x,
-            None if depth is None else depth[0],
+            None if depth is None else depth.states[0],
         )
         kw = dict(center=False, offset=_NORM_OFFSET, mult=cfg.residual_mult)
         h = torch.empty(N, w, dtype=self.dtype, device=self.device)
@@ -255,7 +257,7 @@ class TezinexForCausalLM:
             last = i + 1 == len(self.layers)
             ops.residual_norm(
                 x, y, eps, norm_y, None if last else self.layers[i + 1].norm1,
-                None if last else h, depth=depth, depth_coef=layer.depth, **kw,
+                None if last else h, depth=depth, layer=i, **kw,
             )
             if trace is not None:
                 trace.append(x.clone())

@@ -11,6 +11,8 @@ Two implementations of every engine op:
 """
 from __future__ import annotations
 
+from typing import NamedTuple, Optional
+
 import torch
 
 _HIP = None
@@ -120,16 +122,36 @@ def layernorm(x, weight, eps: float, dtype):
     return _impl(x).layernorm(x, weight, eps, dtype)
 
 
+class Depth(NamedTuple):
+    """States of a depth average: X_0 (the embedding output) and every layer's result."""
+
+    states: torch.Tensor   # [layers + 1, N, K] fp32
+    coef: torch.Tensor     # [layers, layers + 1] fp32: row i weighs the states after layer i
+    partial: torch.Tensor  # [DEPTH_AHEAD, N, K] fp32 workspace
+
+    @staticmethod
+    def new(coef: torch.Tensor, N: int, K: int) -> "Depth":
+        planes = torch.empty(
+            coef.shape[1] + DEPTH_AHEAD, N, K, dtype=torch.float32, device=coef.device
+        )
+        return Depth(planes[: coef.shape[1]], coef, planes[coef.shape[1] :])
+
+
+#: sums the first layer of a block prepares for the block's others (csrc/residual_norm.h)
+DEPTH_AHEAD = 3
+
+
 def residual_norm(x, y, eps: float, y_norm=None, x_norm=None, out=None, *, center=True,
-                  offset: float = 0.0, mult: float = 1.0, depth=None, depth_coef=None):
+                  offset: float = 0.0, mult: float = 1.0, depth: Optional[Depth] = None,
+                  layer: int = 0):
     """x += mult * y, or x += mult * rmsnorm(y) * y_norm, in the fp32 residual x;
-    then, with depth_coef [n + 1] (fp32), x becomes state n in ``depth``
-    [states, N, K] (fp32) and is replaced by sum_j depth_coef[j] * depth[j];
-    then out = norm(x) * x_norm, or x itself without x_norm.  The norm of x is a
-    layer norm, an RMS norm if not ``center``; ``offset`` is added to both norm
-    weights."""
+    then, with ``depth``, x is filed as layer ``layer``'s state and replaced by
+    sum_j coef[layer, j] * states[j] (layers in order: later ones use sums made by
+    earlier ones); then out = norm(x) * x_norm, or x itself without x_norm.  The norm
+    of x is a layer norm, an RMS norm if not ``center``; ``offset`` is added to both
+    norm weights."""
     return _impl(x).residual_norm(
-        x, y, eps, y_norm, x_norm, out, center, offset, mult, depth, depth_coef
+        x, y, eps, y_norm, x_norm, out, center, offset, mult, depth, layer
     )
 
 

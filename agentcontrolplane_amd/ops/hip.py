@@ -113,13 +113,16 @@ def swiglu(gate_up):
 
 def layernorm(x, weight, eps: float, dtype):
     out = torch.empty(x.shape, dtype=dtype, device=x.device)
-    _C.residual_norm(x, None, None, weight, out, eps, True, 0.0, 1.0, None, None)
+    _C.residual_norm(x, None, None, weight, out, eps, True, 0.0, 1.0, None, None, None, 0)
     return out
 
 
 def residual_norm(x, y, eps: float, y_norm=None, x_norm=None, out=None, center=True,
-                  offset=0.0, mult=1.0, depth=None, depth_coef=None):
-    _C.residual_norm(x, y, y_norm, x_norm, out, eps, center, offset, mult, depth, depth_coef)
+                  offset=0.0, mult=1.0, depth=None, layer=0):
+    states, coef, partial = depth or (None, None, None)
+    _C.residual_norm(
+        x, y, y_norm, x_norm, out, eps, center, offset, mult, states, coef, partial, layer
+    )
 
 
 def embed_positions(token_ids, positions, table, cos_sin, x, copy=None):

@@ -169,17 +169,17 @@ def layernorm(x, weight, eps: float, dtype):
 
 
 def residual_norm(x, y, eps: float, y_norm=None, x_norm=None, out=None, center=True,
-                  offset=0.0, mult=1.0, depth=None, depth_coef=None):
+                  offset=0.0, mult=1.0, depth=None, layer=0):
     if y is not None:
         yf = y.float()
         if y_norm is not None:
             yf = yf * torch.rsqrt(yf.pow(2).mean(-1, keepdim=True) + eps)
             yf = yf * (offset + y_norm.float())
         x += mult * yf
-    if depth_coef is not None:
-        n = depth_coef.numel()
-        depth[n - 1] = x
-        x.copy_(torch.einsum("j,jnk->nk", depth_coef, depth[:n]))
+    if depth is not None:
+        n = layer + 2
+        depth.states[n - 1] = x
+        x.copy_(torch.einsum("j,jnk->nk", depth.coef[layer, :n], depth.states[:n]))
     if out is None:
         return
     if x_norm is None:

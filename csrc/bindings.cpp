@@ -6,6 +6,7 @@
 #include <c10/hip/HIPStream.h>
 #include <hip/hip_runtime.h>
 
+#include <algorithm>
 #include <cmath>
 
 #include "channel_delta.h"
@@ -299,7 +300,8 @@ static void check_aligned(const torch::Tensor& t) {
 
 static void residual_norm(torch::Tensor x, OptTensor y, OptTensor y_norm, OptTensor x_norm,
                           OptTensor out, double eps, bool center, double offset, double mult,
-                          OptTensor depth, OptTensor depth_coef) {
+                          OptTensor states, OptTensor coef, OptTensor partial,
+                          int64_t layer) {
   CHECK_CUDA(x); CHECK_CONT(x);
   TORCH_CHECK(x.scalar_type() == at::kFloat && x.dim() == 2);
   TORCH_CHECK(y || out, "nothing to do");
@@ -314,17 +316,28 @@ static void residual_norm(torch::Tensor x, OptTensor y, OptTensor y_norm, OptTen
   f.center = center;
   f.offset = (float)offset;
   f.mult = (float)mult;
-  if (depth_coef) {
-    TORCH_CHECK(depth && y, "depth states");
-    CHECK_CUDA((*depth)); CHECK_CONT((*depth));
-    check_vec(*depth_coef, at::kFloat, depth_coef->numel());
-    TORCH_CHECK(depth->scalar_type() == at::kFloat && depth->dim() == 3 &&
-                depth->size(0) >= depth_coef->numel() && depth_coef->numel() > 0 &&
-                depth->size(1) == n && depth->size(2) == w, "depth states");
-    f.n_depth = depth_coef->numel();
-    f.depth = depth->data_ptr<float>();
-    f.depth_coef = depth_coef->data_ptr<float>();
-    f.depth_stride = depth->stride(0);
+  if (states) {
+    TORCH_CHECK(coef && partial && y, "depth states");
+    for (const auto* t : {&*states, &*coef, &*partial}) {
+      CHECK_CUDA((*t)); CHECK_CONT((*t));
+      TORCH_CHECK(t->scalar_type() == at::kFloat, "depth states are fp32");
+    }
+    TORCH_CHECK(coef->dim() == 2 && layer >= 0 && layer < coef->size(0) &&
+                coef->size(1) >= layer + 2, "depth coefficients");
+    TORCH_CHECK(states->dim() == 3 && states->size(0) >= layer + 2 && states->size(1) == n &&
+                states->size(2) == w, "depth states");
+    TORCH_CHECK(partial->dim() == 3 && partial->size(0) == DEPTH_AHEAD &&
+                partial->size(1) == n && partial->size(2) == w, "depth sums");
+    const int at = (int)layer % (DEPTH_AHEAD + 1);
+    f.n_states = (int)layer + 2;
+    f.first = at ? (int)layer - at + 2 : 0;
+    f.ready = at - 1;
+    f.ahead = std::min(DEPTH_AHEAD, (int)(coef->size(0) - 1 - layer));
+    f.states = states->data_ptr<float>();
+    f.partial = partial->data_ptr<float>();
+    f.coef = coef->data_ptr<float>() + layer * coef->size(1);
+    f.coef_stride = coef->size(1);
+    f.plane = (int64_t)n * w;
   }
   if (n == 0) return;
   launch_residual_norm(is_bf16(y ? *y : *out), x.data_ptr<float>(),
@@ -866,6 +879,7 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("prefill_attn_mfma", &prefill_attn_mfma);
   m.def("mfma_probe", &mfma_probe);
   m.def("gemm_bf16", &gemm_bf16);
+  m.attr("DEPTH_AHEAD") = DEPTH_AHEAD;
   m.def("residual_norm", &residual_norm);
   m.def("side_gate", &side_gate);
   m.def("add_to_residual", &add_to_residual);

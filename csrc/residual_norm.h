@@ -2,12 +2,21 @@
 #pragma once
 #include <stdint.h>
 
+// partial sums a depth block prepares for its later layers
+#define DEPTH_AHEAD 3
+
 struct NormForm {
   bool center;              // layer norm of x, else RMS norm
   float offset;             // added to both norm weights
   float mult;               // on what is added to x
-  int n_depth;              // states averaged, the new one included; 0 = none
-  float* depth;             // [states, n, w], states depth_stride apart
-  const float* depth_coef;  // [n_depth]
-  int64_t depth_stride;
+  // depth average: x becomes state n_states - 1 and then sum_j coef[j] * state_j
+  int n_states;             // 0 = none
+  int first;                // states before it are in partial[ready]; 0: none are
+  int ready;
+  int ahead;                // sums over the n_states for the next layers, coefficients
+                            // in the rows after coef's: partial[0 .. ahead - 1]
+  float* states;            // [.., n, w]
+  float* partial;           // [DEPTH_AHEAD, n, w]
+  const float* coef;
+  int64_t coef_stride, plane;  // plane = n * w
 };

@@ -9,7 +9,55 @@
 #include "common_t.h"
 #include "residual_norm.h"
 
-template <typename T, int V>
+// The depth average would read every state once per layer.  In blocks of
+// DEPTH_AHEAD + 1 layers, the first one reads them all, for itself and for the others,
+// which then read their partial sum and the few states made since.
+template <int V>
+DEV void depth_average(float* t, const NormForm& f, const int64_t at) {
+  const int last = f.n_states - 1;
+  store_f<V>(f.states + last * f.plane + at, t);
+  float sum[V];
+#pragma unroll
+  for (int k = 0; k < V; ++k) sum[k] = f.coef[last] * t[k];
+  if (f.first > 0) {
+    float s[V];
+    load_f<V>(s, f.partial + f.ready * f.plane + at);
+#pragma unroll
+    for (int k = 0; k < V; ++k) sum[k] += s[k];
+    for (int j = f.first; j < last; ++j) {
+      load_f<V>(s, f.states + j * f.plane + at);
+#pragma unroll
+      for (int k = 0; k < V; ++k) sum[k] += f.coef[j] * s[k];
+    }
+  } else {
+    const float* c[DEPTH_AHEAD];
+    float p[DEPTH_AHEAD][V];
+#pragma unroll
+    for (int a = 0; a < DEPTH_AHEAD; ++a) {
+      c[a] = f.coef + (a < f.ahead ? (a + 1) * f.coef_stride : 0);
+#pragma unroll
+      for (int k = 0; k < V; ++k) p[a][k] = c[a][last] * t[k];
+    }
+#pragma unroll 8
+    for (int j = 0; j < last; ++j) {
+      float s[V];
+      load_f<V>(s, f.states + j * f.plane + at);
+#pragma unroll
+      for (int k = 0; k < V; ++k) {
+        sum[k] += f.coef[j] * s[k];
+#pragma unroll
+        for (int a = 0; a < DEPTH_AHEAD; ++a) p[a][k] += c[a][j] * s[k];
+      }
+    }
+#pragma unroll
+    for (int a = 0; a < DEPTH_AHEAD; ++a)
+      if (a < f.ahead) store_f<V>(f.partial + a * f.plane + at, p[a]);
+  }
+#pragma unroll
+  for (int k = 0; k < V; ++k) t[k] = sum[k];
+}
+
+template <typename T, int V, bool DEPTH>
 __global__ __launch_bounds__(1024) void residual_norm_kernel(
     float* __restrict__ x,            // [n, w], updated if y
     const T* __restrict__ y,          // [n, w] or null
@@ -54,23 +102,8 @@ __global__ __launch_bounds__(1024) void residual_norm_kernel(
 #pragma unroll
       for (int k = 0; k < V; ++k) t[k] += f.mult * d[k];
     }
-    if (f.n_depth) {
-      float* state = f.depth + (int64_t)blockIdx.x * w + i;
-      const int last = f.n_depth - 1;
-      store_f<V>(state + last * f.depth_stride, t);
-      const float c = f.depth_coef[last];
-#pragma unroll
-      for (int k = 0; k < V; ++k) t[k] *= c;
-#pragma unroll 8
-      for (int j = 0; j < last; ++j) {
-        float s[V];
-        load_f<V>(s, state + j * f.depth_stride);
-        const float cj = f.depth_coef[j];
-#pragma unroll
-        for (int k = 0; k < V; ++k) t[k] += cj * s[k];
-      }
-    }
-    if (y || f.n_depth) store_f<V>(xr + i, t);
+    if (DEPTH) depth_average<V>(t, f, (int64_t)blockIdx.x * w + i);
+    if (y || DEPTH) store_f<V>(xr + i, t);
 #pragma unroll
     for (int k = 0; k < V; ++k) {
       sum += t[k];
@@ -130,7 +163,8 @@ static void residual_norm_t(float* x, const void* y, const void* y_norm,
   int threads = w >= 1024 ? 256 : w >= 512 ? 128 : 64;
   // few rows: the latency of one counts
   while (n <= 512 && threads < 1024 && threads * 4 < w) threads *= 2;
-  auto k = vec ? residual_norm_kernel<T, 4> : residual_norm_kernel<T, 1>;
+  auto k = f.n_states ? (vec ? residual_norm_kernel<T, 4, true> : residual_norm_kernel<T, 1, true>)
+                      : (vec ? residual_norm_kernel<T, 4, false> : residual_norm_kernel<T, 1, false>);
   k<<<n, threads, w * sizeof(float), stream>>>(
       x, (const T*)y, (const T*)y_norm, (const T*)x_norm, (T*)out, eps, w, out_stride, f);
 }
