@@ -796,7 +796,6 @@ static DeltaArgs delta_args(const torch::Tensor& out, const torch::Tensor& qkv,
   CHECK_CUDA(ring); CHECK_CONT(ring);
   TORCH_CHECK(ring.scalar_type() == dt && ring.dim() == 3 && ring.size(0) == state.size(0) &&
               ring.size(1) == a.taps && ring.size(2) == a.C, "convolution state");
-  TORCH_CHECK((uintptr_t)qkv.data_ptr() % 8 == 0 && (uintptr_t)z.data_ptr() % 8 == 0, "alignment");
   is_bf16(qkv);
   a.seqs = seq_lens.numel();
   a.qkv = qkv.data_ptr();

@@ -700,7 +700,8 @@ static void prompts(const DeltaArgs& a, int cpl, hipStream_t stream) {
     delta_inputs_wide_kernel<T, W><<<dim3(a.n_tiles, (units + 255) / 256), 256, 0, stream>>>(a);
   } else {
     const dim3 grid(a.n_tiles, a.G + 2 * a.H);
-    auto inputs = all(2) ? delta_inputs_kernel<T, 2> : delta_inputs_kernel<T, 1>;
+    const bool even = all(2) && ((uintptr_t)a.qkv | (uintptr_t)a.z) % (2 * sizeof(T)) == 0;
+    auto inputs = even ? delta_inputs_kernel<T, 2> : delta_inputs_kernel<T, 1>;
     inputs<<<grid, 256, 0, stream>>>(a);
   }
   if (a.D <= 16) launch_scan_cols<T, 1>(a, cpl, stream);
