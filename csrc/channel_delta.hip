@@ -469,30 +469,31 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(const DeltaArgs a) {
   }
 }
 
-// A wave per token and head.
-template <typename T, int VW>
+// LANES lanes per token and head, 16 or a wave.
+template <typename T, int VW, int LANES>
 __global__ __launch_bounds__(256) void delta_output_kernel(const DeltaArgs a) {
-  const int64_t i = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
+  const int64_t i = (int64_t)blockIdx.x * (256 / LANES) + threadIdx.x / LANES;
   if (i >= (int64_t)a.N * a.H) return;
   const int64_t n = i / a.H;
-  const int h = (int)(i - n * a.H), lane = threadIdx.x & 63;
+  const int h = (int)(i - n * a.H), lane = threadIdx.x % LANES;
   const float* o = a.o + i * a.V;
   const T* gate = (const T*)a.gate + n * a.gate_stride + (int64_t)h * a.V;
   float ss = 0.f;
-  for (int d = lane * VW; d < a.V; d += 64 * VW) {
+  for (int d = lane * VW; d < a.V; d += LANES * VW) {
     float x[VW];
     load_f<VW>(x, o + d);
 #pragma unroll
     for (int k = 0; k < VW; ++k) ss += x[k] * x[k];
   }
-  const float inv = rsqrtf(wave_sum(ss) / a.V + a.eps);
+  const float inv = rsqrtf((LANES == 16 ? row16_sum(ss) : wave_sum(ss)) / a.V + a.eps);
   T* out = (T*)a.out + i * a.V;
-  for (int d = lane * VW; d < a.V; d += 64 * VW) {
-    float x[VW], g[VW];
+  for (int d = lane * VW; d < a.V; d += LANES * VW) {
+    float x[VW], g[VW], w[VW];
     load_f<VW>(x, o + d);
     load_f<VW>(g, gate + d);
+    load_f<VW>(w, a.norm + d);
 #pragma unroll
-    for (int k = 0; k < VW; ++k) x[k] *= inv * a.norm[d + k] * sigmoid_f(g[k]);
+    for (int k = 0; k < VW; ++k) x[k] *= inv * w[k] * sigmoid_f(g[k]);
     store_f<VW>(out + d, x);
   }
 }
@@ -712,9 +713,11 @@ static void prompts(const DeltaArgs& a, int cpl, hipStream_t stream) {
   else if (a.D <= 512) launch_scan_cols<T, 32>(a, cpl, stream);
   else launch_scan_cols<T, 64>(a, cpl, stream);
   const int64_t heads = (int64_t)a.N * a.H;
-  auto output = aligned && all(4)   ? delta_output_kernel<T, 4>
-                : aligned && all(2) ? delta_output_kernel<T, 2> : delta_output_kernel<T, 1>;
-  output<<<(heads + 3) / 4, 256, 0, stream>>>(a);
+  const bool short_heads = aligned && all(W) && a.V <= 16 * W;
+  auto output = short_heads       ? delta_output_kernel<T, W, 16>
+                : aligned && all(4) ? delta_output_kernel<T, 4, 64> : delta_output_kernel<T, 1, 64>;
+  const int per = short_heads ? 16 : 4;
+  output<<<(heads + per - 1) / per, 256, 0, stream>>>(a);
 }
 
 template <typename T, int VW, int TAPS>
