@@ -226,8 +226,10 @@ class InferenceEngine:
         """Bytes the caches may take on the GPU."""
         free, total = torch.cuda.mem_get_info(self.device)
         budget = int(total * self.cfg.gpu_memory_utilization) - (total - free)
-        # keep headroom for activations: 4 GB or 5% of total
-        return budget - max(4 << 30, int(0.05 * total))
+        # keep headroom for activations: 4 GB or 5% of total, and what the model says
+        # it holds for a whole step
+        held = getattr(self.model, "step_bytes", lambda tokens: 0)
+        return budget - max(4 << 30, int(0.05 * total)) - held(self.cfg.max_prefill_tokens)
 
     def _size_state_pool(self) -> int:
         if self.cfg.num_state_slots is not None:

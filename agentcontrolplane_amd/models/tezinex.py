@@ -229,6 +229,12 @@ class TezinexForCausalLM:
             t for layer, store in zip(self.layers, self.stores) if layer.recurrent for t in store
         ]
 
+    def step_bytes(self, tokens: int) -> int:
+        """What a step of so many tokens holds beyond a layer's activations: the
+        depth states."""
+        planes = len(self.layers) + 1 + ops.DEPTH_AHEAD if self.cfg.depth_average else 0
+        return 4 * planes * tokens * self.cfg.hidden_size
+
     # -------------------------------------------------------------- forward
 
     def _reduced(self, y: torch.Tensor) -> torch.Tensor:
