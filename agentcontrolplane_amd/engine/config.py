@@ -14,6 +14,58 @@ from typing import Optional, Tuple, Union
 
 
 @dataclasses.dataclass(frozen=True)
+class WavelengthScaling:
+    """Rotation slowed by ``factor`` at wavelengths beyond original / low, unchanged
+    below original / high, blended in between (models/rotary.py)."""
+
+    factor: float
+    low: float
+    high: float
+    original: float
+
+
+@dataclasses.dataclass(frozen=True)
+class YarnScaling:
+    """Rotation slowed by ``factor`` along a ramp over the dimensions, from the one that
+    makes ``fast`` turns over the original length to the one that makes ``slow``; cos
+    and sin grow by 0.1 ln(factor) + 1 (models/rotary.py)."""
+
+    factor: float
+    original: float
+    fast: float
+    slow: float
+
+
+RotaryScaling = Union[None, WavelengthScaling, YarnScaling]
+
+
+@dataclasses.dataclass(frozen=True)
+class RotarySpec:
+    """Rotation of a head's first ``dims`` dimensions, i with i + dims/2."""
+
+    base: float
+    dims: int
+    scaling: RotaryScaling = None
+
+
+@dataclasses.dataclass(frozen=True)
+class QueryTemperature:
+    """Queries at position p times 1 + coef ln(floor((p + 1) / every) + 1)."""
+
+    coef: float
+    every: float
+
+
+@dataclasses.dataclass(frozen=True)
+class DistanceBias:
+    """Learned score bias per head and bucket of the distance: half of the buckets
+    hold one distance each, the others widen geometrically up to ``reach``."""
+
+    buckets: int
+    reach: float
+
+
+@dataclasses.dataclass(frozen=True)
 class LatentAttentionSpec:
     """Attention over one cached low-rank latent per token plus one rotated
     key part shared by all heads (models/latent_attention.py)."""
@@ -28,19 +80,22 @@ class LatentAttentionSpec:
     q_rank: Optional[int] = None  # low-rank query; None = direct projection
     window: Optional[int] = None  # keys visible, self included; None = all
     head_gate: bool = True        # sigmoid gate per head on the output
+    rope_scaling: RotaryScaling = None
+    rope_half: bool = False       # dimension i turns with i + rot_dim/2, else 2i with 2i + 1
+    sink: bool = False            # learned logit per head in the denominator
 
     def params(self, w: int) -> int:
         qdim = self.heads * (self.dim + self.rot_dim)
         n = self.q_rank * (w + 1 + qdim) if self.q_rank else w * qdim
         n += w * (self.kv_rank + self.rot_dim) + self.kv_rank
         n += self.kv_rank * self.heads * (self.dim + self.vdim) + self.heads * self.vdim * w
-        return n + (w * self.heads if self.head_gate else 0)
+        return n + (w * self.heads if self.head_gate else 0) + (self.heads if self.sink else 0)
 
 
 @dataclasses.dataclass(frozen=True)
 class GroupedAttentionSpec:
-    """Attention without rotation over cached keys and values shared by groups of
-    query heads (models/grouped_attention.py)."""
+    """Attention over cached keys and values shared by groups of query heads
+    (models/grouped_attention.py)."""
 
     heads: int
     kv_heads: int
@@ -53,11 +108,25 @@ class GroupedAttentionSpec:
     bias: bool = True               # on the query, key and value projections
     sink: bool = True               # learned logit per head in the denominator
     kv_from: Optional[int] = None   # the layer whose keys and values are used
+    conv: int = 0                   # taps of the short convolutions on q, k, v; 0 = none
+    qk_norm: bool = False           # RMS norm of query and key heads, learned weight
+    v_norm: bool = False            # RMS norm of value heads, no weight
+    rotary: Optional[RotarySpec] = None
+    q_temp: Optional[QueryTemperature] = None
+    head_temp: bool = False         # learned factor per head on the scores
+    distance_bias: Optional[DistanceBias] = None
+    sigmoid: bool = False           # weights sigmoid(score + learned offset), not normalized
+    head_gate: bool = False         # sigmoid gate per head on the output
+    out_bias: bool = False
 
     def params(self, w: int) -> int:
         q, o = self.heads * self.dim, self.heads * self.vdim
         kv = 0 if self.kv_from is not None else self.kv_heads * (self.dim + self.vdim)
-        return (q + kv) * (w + self.bias) + o * w + (self.heads if self.sink else 0)
+        n = (q + kv) * (w + self.bias + self.conv) + o * w + (w if self.out_bias else 0)
+        n += 2 * self.dim if self.qk_norm else 0
+        n += self.heads * (self.sink + self.head_temp + self.sigmoid)
+        n += self.heads * self.distance_bias.buckets if self.distance_bias else 0
+        return n + (self.heads * w if self.head_gate else 0)
 
 
 @dataclasses.dataclass(frozen=True)
@@ -83,12 +152,14 @@ class ChannelDeltaSpec:
 
 @dataclasses.dataclass(frozen=True)
 class ClampedGluSpec:
-    """min(gate, limit) * sigmoid(alpha * .) * (clamp(up, +-limit) + offset)."""
+    """g * sigmoid(alpha (g + cubic g^3)) * (clamp(up, +-limit) + offset),
+    g = min(gate, limit)."""
 
     width: int
     limit: float
     alpha: float = 1.702
     offset: float = 1.0
+    cubic: float = 0.0
 
 
 def silu_glu(width: int) -> ClampedGluSpec:
@@ -96,11 +167,40 @@ def silu_glu(width: int) -> ClampedGluSpec:
     return ClampedGluSpec(width, limit=math.inf, alpha=1.0, offset=0.0)
 
 
+def gelu_glu(width: int) -> ClampedGluSpec:
+    """gelu(gate) * up, the tanh form: 1 + tanh(z) = 2 sigmoid(2z)."""
+    return ClampedGluSpec(
+        width, limit=math.inf, alpha=2 * math.sqrt(2 / math.pi), offset=0.0, cubic=0.044715
+    )
+
+
+@dataclasses.dataclass(frozen=True)
+class ExpertsSpec:
+    """Mixture of experts: each token uses ``top`` of ``experts`` GLUs, weighted by the
+    softmax over the chosen router logits, and the shared one (models/experts.py)."""
+
+    experts: int
+    top: int
+    expert: ClampedGluSpec
+    shared: Optional[ClampedGluSpec] = None
+    router_bias: bool = True
+
+    @property
+    def width(self) -> int:
+        """Feed-forward width a token uses."""
+        return self.top * self.expert.width + (self.shared.width if self.shared else 0)
+
+    def params(self, w: int) -> int:
+        n = self.experts * (w + self.router_bias + 3 * w * self.expert.width)
+        return n + (3 * w * self.shared.width if self.shared else 0)
+
+
 @dataclasses.dataclass(frozen=True)
 class LayerSpec:
     mixer: Union[LatentAttentionSpec, GroupedAttentionSpec, ChannelDeltaSpec]
-    mlp: Optional[ClampedGluSpec] = None
+    mlp: Union[None, ClampedGluSpec, ExpertsSpec] = None
     sandwich: bool = False  # mixer, then mlp, each normed on its way in and out
+    mlp_norm: bool = False  # side by side, the mlp on a norm of its own
 
 
 @dataclasses.dataclass(frozen=True)
@@ -146,6 +246,8 @@ class ModelConfig:
     depth_average: bool = False
     # sinusoidal positions added to the embedding: the base, None = none
     position_base: Optional[float] = None
+    # on the token embedding
+    embed_scale: float = 1.0
     # logits -> cap * tanh(logits / cap)
     logit_softcap: Optional[float] = None
 
@@ -182,10 +284,14 @@ class ModelConfig:
 
     def _listed_layer_params(self) -> int:
         w, v = self.hidden_size, self.vocab_size
-        total = v * w + w
+        total = v * w * (1 if self.tie_embeddings else 2) + w
         for i, layer in enumerate(self.layers):
             total += w + layer.mixer.params(w)
-            total += 3 * w * layer.mlp.width if layer.mlp else 0
+            if isinstance(layer.mlp, ExpertsSpec):
+                total += layer.mlp.params(w)
+            elif layer.mlp:
+                total += 3 * w * layer.mlp.width
+            total += w if layer.mlp and layer.mlp_norm else 0
             if layer.sandwich:
                 total += w + (2 * w if layer.mlp else 0)
             if self.depth_average:

@@ -1,5 +1,6 @@
 from .fetolix import FetolixForCausalLM  # noqa: F401
 from .llama import LlamaForCausalLM  # noqa: F401
+from .lobuvik import LobuvikForCausalLM  # noqa: F401
 from .mixtral import MixtralForCausalLM  # noqa: F401
 from .tezinex import TezinexForCausalLM  # noqa: F401
 
@@ -9,6 +10,7 @@ MODEL_CLASSES = {
     "mixtral": MixtralForCausalLM,
     "Fetolix": FetolixForCausalLM,
     "Tezinex": TezinexForCausalLM,
+    "Lobuvik": LobuvikForCausalLM,
 }
 
 

@@ -10,8 +10,9 @@ import os
 from typing import Callable, Dict, Optional, Tuple
 
 from ..engine.config import (
-    ChannelDeltaSpec, ClampedGluSpec, GroupedAttentionSpec, LatentAttentionSpec, LayerSpec,
-    LoopSpec, ModelConfig, silu_glu,
+    ChannelDeltaSpec, ClampedGluSpec, DistanceBias, ExpertsSpec, GroupedAttentionSpec,
+    LatentAttentionSpec, LayerSpec, LoopSpec, ModelConfig, QueryTemperature, RotarySpec,
+    WavelengthScaling, YarnScaling, gelu_glu, silu_glu,
 )
 from .weights import tensor_shape
 
@@ -133,9 +134,96 @@ def _tezinex(d: dict, shape: Shape) -> ModelConfig:
     )
 
 
+def _biased_attention(m: dict, shape: Shape, p: str) -> GroupedAttentionSpec:
+    reach, buckets = m["bias_max"], shape(p + "rel")[0]
+    if buckets < 2 or reach <= buckets // 2:
+        raise ValueError("distance buckets must reach beyond their first half")
+    return GroupedAttentionSpec(
+        heads=m["heads"], kv_heads=m["kv_heads"], dim=m["dim"], vdim=m["vdim"],
+        scale=m["scale"], bias=True, out_bias=True, sink=False, sigmoid=True, conv=m["conv"],
+        qk_norm=True, v_norm=True, distance_bias=DistanceBias(buckets, reach),
+        q_temp=QueryTemperature(m["q_temp"]["coef"], m["q_temp"]["every"]),
+    )
+
+
+def _yarn_latent_attention(m: dict, shape: Shape, p: str) -> LatentAttentionSpec:
+    rot, s = m["rot"], m["rot"]["scaling"]
+    if rot["dims"] != m["rot_dim"]:
+        raise ValueError("latent attention rotates all of its rot_dim dimensions")
+    return LatentAttentionSpec(
+        heads=m["heads"], dim=m["dim"], rot_dim=m["rot_dim"], vdim=m["vdim"],
+        kv_rank=m["kv_rank"], scale=m["scale"], rope_base=rot["base"], rope_half=True,
+        rope_scaling=YarnScaling(s["factor"], s["original"], s["fast"], s["slow"]),
+        window=m["mask"]["size"], head_gate=False, sink=True,
+    )
+
+
+def _rotated_attention(m: dict, shape: Shape, p: str) -> GroupedAttentionSpec:
+    rot, s = m["rot"], m["rot"]["scaling"]
+    if rot["dims"] % 2 or rot["dims"] > m["dim"]:
+        raise ValueError("rot.dims must be even and at most dim")
+    return GroupedAttentionSpec(
+        heads=m["heads"], kv_heads=m["kv_heads"], dim=m["dim"], vdim=m["vdim"],
+        scale=m["scale"], softcap=m["softcap"], window=m["mask"]["size"], bias=False,
+        sink=False, head_temp=True, head_gate=True, rotary=RotarySpec(
+            rot["base"], rot["dims"],
+            WavelengthScaling(s["factor"], s["low"], s["high"], s["original"]),
+        ),
+    )
+
+
+#: Lobuvik mixer type -> spec reader
+_LOBUVIK_MIXERS = {
+    "attention": _biased_attention,
+    "latent_attention": _yarn_latent_attention,
+    "attention_2": _rotated_attention,
+}
+
+
+def _lobuvik_mlp(mlp: Optional[dict]):
+    if mlp is None:
+        return None
+    if mlp["kind"] == "dense":
+        return gelu_glu(mlp["ff"])
+    if mlp["kind"] != "moe":
+        raise ValueError(f"unknown feed-forward kind {mlp['kind']!r}")
+
+    def glu(d: dict) -> ClampedGluSpec:
+        return ClampedGluSpec(width=d["ff"], limit=d["limit"])
+
+    router, shared = mlp["router"], mlp.get("shared")
+    if not 0 < router["top"] <= router["experts"]:
+        raise ValueError("a token uses between 1 and all experts")
+    return ExpertsSpec(
+        experts=router["experts"], top=router["top"], expert=glu(mlp["expert"]),
+        shared=glu(shared) if shared else None,
+    )
+
+
+def _lobuvik(d: dict, shape: Shape) -> ModelConfig:
+    layers = []
+    for i, entry in enumerate(d["layers"]):
+        if entry["type"] not in _LOBUVIK_MIXERS:
+            raise ValueError(f"unknown mixer type {entry['type']!r}")
+        m = _LOBUVIK_MIXERS[entry["type"]](entry["mixer"], shape, f"l{i}.mix.")
+        if isinstance(m, GroupedAttentionSpec) and m.heads % m.kv_heads:
+            raise ValueError(f"layer {i}: kv_heads must divide heads")
+        layers.append(LayerSpec(mixer=m, mlp=_lobuvik_mlp(entry.get("mlp")), mlp_norm=True))
+    first = layers[0].mixer
+    return ModelConfig(
+        name="Lobuvik", architecture="Lobuvik", vocab_size=d["vocab"],
+        hidden_size=d["width"], num_layers=len(layers), num_heads=first.heads,
+        num_kv_heads=getattr(first, "kv_heads", 1), head_dim=first.dim,
+        intermediate_size=max((x.mlp.width for x in layers if x.mlp), default=0),
+        rms_eps=d["norm"]["eps"], max_position=_UNBOUNDED, layers=tuple(layers),
+        embed_scale=d["embedding"]["scale"],
+    )
+
+
 CONFIG_READERS: Dict[str, Callable[[dict, Shape], ModelConfig]] = {
     "Fetolix": _fetolix,
     "Tezinex": _tezinex,
+    "Lobuvik": _lobuvik,
 }
 
 

@@ -32,13 +32,10 @@ from ..engine.batch import FlatBatch
 from ..engine.config import EngineConfig, LayerSpec, ModelConfig
 from ..ops.reference import build_cos_sin
 from .latent_attention import LatentAttention
-from .layout import Get, pad_to, round_up
+from .layout import Get, fuse_columns, pad_to, round_up, summed_linear
 from .llama import _dtype_of
 
 _ALIGN = 16  # rows between sections of the fused input projection
-#: the longest inner dimension of a fused output projection: beyond it the library's
-#: small-batch kernels slow down more than a second GEMM costs
-_FUSED_OUT = 16384
 
 
 class FetolixLayer:
@@ -93,9 +90,7 @@ class FetolixLayer:
             w_in[at + self.ff_pad : at + self.ff_pad + self.ff] = get(p + "mlp.up")[mine]
             outs.append(pad_to(get(p + "mlp.down")[:, mine], self.width, self.ff_pad))
         self.w_in = w_in
-        if m.out_dim + self.ff_pad <= _FUSED_OUT:
-            outs = [torch.cat(outs, 1)]
-        self.w_out = [o.contiguous() for o in outs]
+        self.w_out = fuse_columns(outs)
         if side_dim:
             self.side_gate = get(p + "side.gate")
             self.side_proj = get(p + "side.proj")
@@ -140,11 +135,7 @@ class FetolixLayer:
             section("q"), section("kv"), section("gate"), batch, cache,
             mixed[:, : m.out_dim],
         )
-        at = self.w_out[0].shape[1]
-        y = ops.linear(mixed[:, :at], self.w_out[0])
-        if len(self.w_out) > 1:
-            ops.linear_add_(y, mixed[:, at:], self.w_out[1])
-        return y
+        return summed_linear(mixed, self.w_out)
 
 
 class FetolixForCausalLM:

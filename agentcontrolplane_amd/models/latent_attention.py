@@ -6,6 +6,10 @@ cached per token; keys and values are linear in the latent.
     score  = (q_nope . W_uk c + rotate(q_rot) . k_rot) * scale
     out    = sigmoid(W_g h) * sum_j p_j W_uv c_j
 
+The query may be low-rank, the head gate absent, and a learned logit per head may
+join the softmax denominator.  The rotation pairs dimension 2i with 2i + 1; a design
+that pairs i with i + rot_dim/2 has its weight rows reordered at load time.
+
 Two equal evaluations.  *Absorbed*: q' = W_uk^T q_nope, so a score is one dot
 product with the cached row and the weighted sum is taken over latents, W_uv
 applied once per query.  It reads one short row per key for all heads: decode
@@ -30,7 +34,7 @@ import torch
 from .. import ops
 from ..engine.batch import FlatBatch
 from ..engine.config import LatentAttentionSpec
-from .layout import Get, pad_to, round_up
+from .layout import Get, pad_to, pair_halves, round_up, unpair_halves
 
 
 class LatentAttention:
@@ -57,6 +61,7 @@ class LatentAttention:
         self.w_uk: torch.Tensor = None           # [H, rank, d]: q_nope -> q'
         self.w_ukv: torch.Tensor = None          # [H*d + H*v, rank]: c -> k | v
         self.w_uv: torch.Tensor = None           # [H, v, rank] view of w_ukv
+        self.sink = None                         # [H] fp32
         self.cos_sin: torch.Tensor = None
 
     # ------------------------------------------------------------- weights
@@ -75,6 +80,8 @@ class LatentAttention:
         ]
         if s.head_gate:
             out.append(("g", (s.heads, w)))
+        if s.sink:
+            out.append(("sink", (s.heads,)))
         return out + [("o", (w, s.heads * s.vdim))]
 
     def _mine(self, t: torch.Tensor, per_head: int) -> torch.Tensor:
@@ -84,16 +91,29 @@ class LatentAttention:
     def _pad_query(self, t: torch.Tensor) -> torch.Tensor:
         s, k = self.spec, t.shape[1]
         t = self._mine(t, s.dim + s.rot_dim).view(self.heads, s.dim + s.rot_dim, k)
+        rot = t[:, s.dim :]
+        if s.rope_half:
+            rot = pair_halves(rot, s.rot_dim, 1)
         out = t.new_zeros(self.heads, self.d + self.rot, k)
         out[:, : s.dim] = t[:, : s.dim]
-        out[:, self.d : self.d + s.rot_dim] = t[:, s.dim :]
+        out[:, self.d : self.d + s.rot_dim] = rot
         return out.view(self.q_dim, k)
 
     def _unpad_query(self, t: torch.Tensor) -> torch.Tensor:
         s = self.spec
         t = t.view(self.heads, self.d + self.rot, t.shape[1])
-        t = torch.cat([t[:, : s.dim], t[:, self.d : self.d + s.rot_dim]], 1)
+        rot = t[:, self.d : self.d + s.rot_dim]
+        if s.rope_half:
+            rot = unpair_halves(rot, s.rot_dim, 1)
+        t = torch.cat([t[:, : s.dim], rot], 1)
         return t.reshape(-1, t.shape[2])
+
+    def _shared_key(self, dkv: torch.Tensor, reorder) -> torch.Tensor:
+        """dkv with its rotated rows reordered."""
+        if not self.spec.rope_half:
+            return dkv
+        rank = self.spec.kv_rank
+        return torch.cat([dkv[:rank], reorder(dkv[rank:], self.spec.rot_dim, 0)])
 
     def load(self, get: Get, p: str) -> Dict[str, torch.Tensor]:
         """Install the mixer's own weights; returns its rows of the layer's
@@ -108,9 +128,11 @@ class LatentAttention:
             self.uq = pad_to(uq, uq.shape[0], self.q_rank)
         else:
             sections["q"] = self._pad_query(get(p + "q"))
-        sections["kv"] = get(p + "dkv")
+        sections["kv"] = self._shared_key(get(p + "dkv"), pair_halves)
         if s.head_gate:
             sections["gate"] = self._mine(get(p + "g"), 1)
+        if s.sink:
+            self.sink = self._mine(get(p + "sink"), 1).float().contiguous()
         self.kv_norm = get(p + "dkv.norm").contiguous()
         uk = self._mine(get(p + "uk"), s.dim).view(H, s.dim, s.kv_rank)
         uv = self._mine(get(p + "uv"), s.vdim).view(H, s.vdim, s.kv_rank)
@@ -135,13 +157,15 @@ class LatentAttention:
             out[p + "uq"] = self._unpad_query(self.uq)[:, : s.q_rank]
         else:
             out[p + "q"] = self._unpad_query(sections["q"])
-        out[p + "dkv"] = sections["kv"]
+        out[p + "dkv"] = self._shared_key(sections["kv"], unpair_halves)
         out[p + "dkv.norm"] = self.kv_norm
         k = self.w_ukv[: H * self.d].view(H, self.d, self.rank)
         out[p + "uk"] = k[:, : s.dim, : s.kv_rank].reshape(H * s.dim, s.kv_rank)
         out[p + "uv"] = self.w_uv[:, : s.vdim, : s.kv_rank].reshape(H * s.vdim, s.kv_rank)
         if s.head_gate:
             out[p + "g"] = sections["gate"]
+        if s.sink:
+            out[p + "sink"] = self.sink.to(self.w_uk.dtype)
         o = sections["o"].view(self.width, H, self.v)[:, :, : s.vdim]
         out[p + "o"] = o.reshape(self.width, H * s.vdim)
         return out
@@ -176,13 +200,13 @@ class LatentAttention:
             ops.head_linear(q[row0:, :, : self.d], self.w_uk, qa)
             latent = ops.latent_attention(
                 qa, q[row0:, :, self.d :], self.cos_sin, s.rot_dim, cache, batch, s.scale,
-                s.window, row0, expanded,
+                s.window, row0, expanded, self.sink,
             )
             ops.head_linear(latent, self.w_uv, out[row0:], None if gate is None else gate[row0:])
         if expanded:  # after: the rows above may include expanded chunks'
             ops.latent_expanded_prefill(
                 q, self.w_ukv, gate, self.cos_sin, s.rot_dim, cache, batch, expanded,
-                self.rank, s.scale, s.window, out,
+                self.rank, s.scale, s.window, out, self.sink,
             )
 
     def _split(self, q: torch.Tensor, batch: FlatBatch) -> Tuple[Tuple[int, ...], int]:

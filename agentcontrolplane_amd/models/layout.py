@@ -2,9 +2,11 @@
 sizes the kernels take."""
 from __future__ import annotations
 
-from typing import Callable
+from typing import Callable, List, Optional
 
 import torch
+
+from .. import ops
 
 #: name -> the whole checkpoint tensor, in the model's dtype and on its device
 Get = Callable[[str], torch.Tensor]
@@ -34,3 +36,42 @@ def stack_rows(sections, width: int, align: int = 16):
     for name, t in sections:
         out[places[name][0] : places[name][0] + t.shape[0]] = t
     return out, places
+
+
+def pair_halves(t: torch.Tensor, dims: int, axis: int = -1) -> torch.Tensor:
+    """Reorder the first ``dims`` entries of an axis from [u.. | v..] to (u, v) pairs: a
+    rotation of i with i + dims/2 becomes one of 2i with 2i + 1.  Scores do not change
+    if query and key dimensions move alike."""
+    at = torch.arange(t.shape[axis], device=t.device)
+    at[:dims] = at[:dims].view(2, -1).t().flatten()
+    return t.index_select(axis, at)
+
+
+def unpair_halves(t: torch.Tensor, dims: int, axis: int = -1) -> torch.Tensor:
+    """Inverse of pair_halves()."""
+    at = torch.arange(t.shape[axis], device=t.device)
+    at[:dims] = at[:dims].view(-1, 2).t().flatten()
+    return t.index_select(axis, at)
+
+
+#: the longest inner dimension of a fused output projection: beyond it the library's
+#: small-batch kernels slow down more than a second GEMM costs
+_FUSED_OUT = 16384
+
+
+def fuse_columns(blocks: List[torch.Tensor]) -> List[torch.Tensor]:
+    """Weights [width, k] whose products are summed: one weight if it is not too long."""
+    if sum(b.shape[1] for b in blocks) <= _FUSED_OUT:
+        blocks = [torch.cat(blocks, 1)]
+    return [b.contiguous() for b in blocks]
+
+
+def summed_linear(x: torch.Tensor, blocks: List[torch.Tensor],
+                  bias: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """x [N, sum of k] times the blocks of fuse_columns()."""
+    at = blocks[0].shape[1]
+    y = ops.linear(x[:, :at], blocks[0], bias)
+    for b in blocks[1:]:
+        ops.linear_add_(y, x[:, at : at + b.shape[1]], b)
+        at += b.shape[1]
+    return y

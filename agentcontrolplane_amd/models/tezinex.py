@@ -45,7 +45,9 @@ class TezinexLayer:
         if self.recurrent:
             self.mixer = ChannelDelta(spec.mixer, self.width, cfg.rms_eps, tp_rank, tp_world)
         else:
-            self.mixer = GroupedAttention(spec.mixer, self.width, tp_rank, tp_world)
+            self.mixer = GroupedAttention(
+                spec.mixer, self.width, cfg.rms_eps, tp_rank, tp_world
+            )
         self.mlp = spec.mlp
         self.tp_rank = tp_rank
         if self.mlp:

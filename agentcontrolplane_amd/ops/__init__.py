@@ -143,22 +143,24 @@ DEPTH_AHEAD = 3
 
 def residual_norm(x, y, eps: float, y_norm=None, x_norm=None, out=None, *, center=True,
                   offset: float = 0.0, mult: float = 1.0, depth: Optional[Depth] = None,
-                  layer: int = 0):
-    """x += mult * y, or x += mult * rmsnorm(y) * y_norm, in the fp32 residual x;
-    then, with ``depth``, x is filed as layer ``layer``'s state and replaced by
+                  layer: int = 0, x_norm2=None, out2=None, experts=None):
+    """x += mult * y, or x += mult * rmsnorm(y) * y_norm, in the fp32 residual x, where
+    ``experts`` (rows [N, k, K], weights [N, k] fp32; no y_norm) joins y as
+    sum_j weights[:, j] * rows[:, j]; then, with ``depth``, x is filed as layer ``layer``'s state and replaced by
     sum_j coef[layer, j] * states[j] (layers in order: later ones use sums made by
     earlier ones); then out = norm(x) * x_norm, or x itself without x_norm.  The norm
-    of x is a layer norm, an RMS norm if not ``center``; ``offset`` is added to both
-    norm weights."""
+    of x is a layer norm, an RMS norm if not ``center``; ``offset`` is added to the
+    norm weights.  out2 is the same norm under the weight x_norm2."""
     return _impl(x).residual_norm(
-        x, y, eps, y_norm, x_norm, out, center, offset, mult, depth, layer
+        x, y, eps, y_norm, x_norm, out, center, offset, mult, depth, layer, x_norm2, out2,
+        experts,
     )
 
 
-def embed_positions(token_ids, positions, table, cos_sin, x, copy=None):
-    """x = copy = table[token] plus sin (even entries) and cos (odd entries) of the
-    position's angles, cos_sin [2, P, ceil(K / 2)]; x, copy fp32 [N, K]."""
-    return _impl(x).embed_positions(token_ids, positions, table, cos_sin, x, copy)
+def embed_positions(token_ids, positions, table, cos_sin, x, copy=None, scale: float = 1.0):
+    """x = copy = scale * table[token] plus, with cos_sin [2, P, ceil(K / 2)], sin (even
+    entries) and cos (odd entries) of the position's angles; x, copy fp32 [N, K]."""
+    return _impl(x).embed_positions(token_ids, positions, table, cos_sin, x, copy, scale)
 
 
 def softcap(logits, cap):
@@ -166,10 +168,10 @@ def softcap(logits, cap):
     return logits.float() if cap is None else _impl(logits).softcap(logits, cap)
 
 
-def clamped_glu(gate_up, limit: float, alpha: float, offset: float, out):
+def clamped_glu(gate_up, limit: float, alpha: float, offset: float, out, cubic: float = 0.0):
     """gate_up [N, 2I] (row-strided halves) -> out [N, I] (row-strided):
-    g * sigmoid(alpha g) * (u + offset), g capped at limit, u at +-limit."""
-    return _impl(gate_up).clamped_glu(gate_up, limit, alpha, offset, out)
+    g * sigmoid(alpha (g + cubic g^3)) * (u + offset), g capped at limit, u at +-limit."""
+    return _impl(gate_up).clamped_glu(gate_up, limit, alpha, offset, out, cubic)
 
 
 def side_gate(x, y, gate, token_ids, table, offset: int):
@@ -223,14 +225,14 @@ def head_linear(x, w, out, gate=None):
 
 
 def latent_attention(q, q_rot, cos_sin, rot_dim: int, cache, batch, scale: float, window,
-                     row0: int = 0, skip=()):
-    """Softmax attention of absorbed queries over cached rows, for a FlatBatch's
-    token rows row0.. except the prefill chunks in ``skip`` (left undefined).
+                     row0: int = 0, skip=(), sink=None):
+    """Softmax attention of absorbed queries over cached rows (``sink`` [H], fp32, or None
+    joins the denominator), for a FlatBatch's token rows row0.. except the prefill chunks in ``skip`` (left undefined).
     q [N, H, rank] and its part q_rot [N, H, rot] still to be rotated by the
     row's position; values are a cache row's first ``rank`` dims.
     window = visible keys per query, None = all.  Returns [N, H, rank]."""
     return _impl(q).latent_attention(
-        q, q_rot, cos_sin, rot_dim, cache, batch, scale, window, row0, skip
+        q, q_rot, cos_sin, rot_dim, cache, batch, scale, window, row0, skip, sink
     )
 
 
@@ -240,12 +242,12 @@ def can_expand(t, d: int, v: int, rot: int) -> bool:
 
 
 def latent_expanded_prefill(q, w_ukv, gate, cos_sin, rot_dim: int, cache, batch, chunks,
-                            rank: int, scale: float, window, out):
+                            rank: int, scale: float, window, out, sink=None):
     """The prefill chunks ``chunks`` with keys and values expanded from their
     cached latents by w_ukv [H*d + H*v, rank]; q [N, H, d + rot] not rotated.
     Writes the chunks' rows of out [N, H, v], gated."""
     _hip().latent_expanded_prefill(
-        q, w_ukv, gate, cos_sin, rot_dim, cache, batch, chunks, rank, scale, window, out
+        q, w_ukv, gate, cos_sin, rot_dim, cache, batch, chunks, rank, scale, window, out, sink
     )
 
 
@@ -258,16 +260,54 @@ def cache_keys_values(k, v, slot_mapping, k_cache, v_cache):
     return _impl(k).cache_keys_values(k, v, slot_mapping, k_cache, v_cache)
 
 
+def attention_inputs(proj, heads: int, dim: int, vdim: int, k_cache, v_cache, batch, eps: float,
+                     *, conv=None, ring=None, q_norm=None, k_norm=None, v_norm: bool = False,
+                     cos_sin=None, head_mult=None, q_temp=None):
+    """From projected rows [N, q | k | v channels] (row-strided; heads padded from dim and
+    vdim to the caches' d and e) to queries [N, heads, d], which are returned, and keys
+    and values in their cache slots (batch.slot_mapping).  In this order, each optional:
+
+    conv [taps, channels]: causal convolution per channel; the last inputs of a
+        sequence are kept by position in its slot of ``ring`` [slots, taps, channels]
+    q_norm, k_norm [d], v_norm: RMS norm per head over dim or vdim
+    cos_sin [2, P, n]: rotate a query's and key's first n pairs (2i, 2i + 1)
+    head_mult [heads] fp32, q_temp (coef, every): queries times the head's factor, and
+        times 1 + coef ln(floor((p + 1) / every) + 1) at position p"""
+    return _impl(proj).attention_inputs(
+        proj, heads, dim, vdim, k_cache, v_cache, batch, eps, conv, ring, q_norm, k_norm,
+        v_norm, cos_sin, head_mult, q_temp,
+    )
+
+
 def grouped_attention(q, k_cache, v_cache, batch, scale: float, cap, window, keep_first: int,
-                      sink, out):
+                      sink, out, bias=None, sigmoid: bool = False, gate=None):
     """Attention of a FlatBatch's rows over the paged cache; query head n uses
     key/value head n // (H / G).  Scores are capped if ``cap``; a query sees itself
     and the ``window`` - 1 tokens before it (None = all) and the ``keep_first``
     first tokens; ``sink`` [H] (fp32) or None joins the softmax denominator.
-    q [N, H, d] (row-strided) -> out [N, H, e]."""
+    ``bias`` [H, D] (fp32) adds bias[h, min(distance, D - 1)] to the capped scores;
+    ``sigmoid``: weights are the scores' sigmoids, not a softmax; ``gate`` [N, H]
+    (row-strided) multiplies a head's output by its sigmoid.
+    q [N, H, d], out [N, H, e], both row-strided."""
     return _impl(q).grouped_attention(
-        q, k_cache, v_cache, batch, scale, cap, window, keep_first, sink, out
+        q, k_cache, v_cache, batch, scale, cap, window, keep_first, sink, out, bias, sigmoid,
+        gate,
     )
+
+
+# -------------------------------------------------------------------- experts
+
+
+def moe_route(h, router, bias, top: int):
+    """The ``top`` experts with the largest logits router @ h + bias (fp32) of every row:
+    ids [N, top] int32 and the softmax over the chosen logits [N, top] fp32."""
+    return _impl(h).moe_route(h, router, bias, top)
+
+
+def moe_experts(h, gate_up, down, ids, glu):
+    """Every chosen expert's GLU of its row: h [N, K], gate_up [E, 2I, K], down [E, W, I],
+    ids [N, k] -> [N, k, W].  ``glu`` has limit, alpha, offset and cubic."""
+    return _impl(h).moe_experts(h, gate_up, down, ids, glu)
 
 
 # ----------------------------------------------------------------- delta rule

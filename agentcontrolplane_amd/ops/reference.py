@@ -169,9 +169,13 @@ def layernorm(x, weight, eps: float, dtype):
 
 
 def residual_norm(x, y, eps: float, y_norm=None, x_norm=None, out=None, center=True,
-                  offset=0.0, mult=1.0, depth=None, layer=0):
+                  offset=0.0, mult=1.0, depth=None, layer=0, x_norm2=None, out2=None,
+                  experts=None):
     if y is not None:
         yf = y.float()
+        if experts is not None:
+            rows, weights = experts
+            yf = yf + (rows.float() * weights.unsqueeze(-1)).sum(1)
         if y_norm is not None:
             yf = yf * torch.rsqrt(yf.pow(2).mean(-1, keepdim=True) + eps)
             yf = yf * (offset + y_norm.float())
@@ -188,10 +192,12 @@ def residual_norm(x, y, eps: float, y_norm=None, x_norm=None, out=None, center=T
     xc = x - x.mean(-1, keepdim=True) if center else x
     xc = xc * torch.rsqrt(xc.pow(2).mean(-1, keepdim=True) + eps)
     out.copy_(xc * (offset + x_norm.float()))
+    if out2 is not None:
+        out2.copy_(xc * (offset + x_norm2.float()))
 
 
-def embed_positions(token_ids, positions, table, cos_sin, x, copy=None):
-    x.copy_(table[token_ids].float())
+def embed_positions(token_ids, positions, table, cos_sin, x, copy=None, scale=1.0):
+    x.copy_(table[token_ids].float() * scale)
     if cos_sin is not None:
         w = x.shape[1]
         x[:, 0::2] += cos_sin[1][positions]
@@ -204,10 +210,11 @@ def softcap(logits, cap):
     return cap * torch.tanh(logits.float() / cap)
 
 
-def clamped_glu(gate_up, limit: float, alpha: float, offset: float, out):
+def clamped_glu(gate_up, limit: float, alpha: float, offset: float, out, cubic=0.0):
     g, u = gate_up.float().chunk(2, dim=-1)
     g = g.clamp(max=limit)
-    out.copy_(g * torch.sigmoid(alpha * g) * (u.clamp(-limit, limit) + offset))
+    z = alpha * (g + cubic * g ** 3) if cubic else alpha * g
+    out.copy_(g * torch.sigmoid(z) * (u.clamp(-limit, limit) + offset))
 
 
 def side_gate(x, y, gate, token_ids, table, offset: int):
@@ -248,7 +255,16 @@ def head_linear(x, w, out, gate=None):
     return out
 
 
-def _latent_attention_seq(q, cache, block_table, ctx_len: int, rank: int, scale: float, window):
+def _sink_softmax(scores, sink):
+    """Weights of scores [.., keys]; sink, broadcast over the keys, joins the denominator."""
+    if sink is None:
+        return torch.softmax(scores, -1)
+    scores = torch.cat([scores, sink.expand(*scores.shape[:-1], 1)], -1)
+    return torch.softmax(scores, -1)[..., :-1]
+
+
+def _latent_attention_seq(q, cache, block_table, ctx_len: int, rank: int, scale: float, window,
+                          sink):
     """One sequence's rows at positions ctx_len..; q [L, H, row] -> [L, H, rank]."""
     L, bs = q.shape[0], cache.shape[1]
     j = torch.arange(ctx_len + L, device=q.device)
@@ -259,12 +275,13 @@ def _latent_attention_seq(q, cache, block_table, ctx_len: int, rank: int, scale:
     if window is not None:
         hidden |= (i - j) >= window
     scores = torch.matmul(q.float(), rows.t()) * scale        # [L, H, S]
-    probs = torch.softmax(scores.masked_fill(hidden.unsqueeze(1), float("-inf")), dim=-1)
+    scores = scores.masked_fill(hidden.unsqueeze(1), float("-inf"))
+    probs = _sink_softmax(scores, None if sink is None else sink.view(1, -1, 1))
     return torch.matmul(probs, rows[:, :rank]).to(q.dtype)
 
 
 def latent_attention(q, q_rot, cos_sin, rot_dim: int, cache, batch, scale: float, window,
-                     row0: int = 0, skip=()):
+                     row0: int = 0, skip=(), sink=None):
     N, H, rank = q.shape
     pos = batch.positions[row0:]
     rot = torch.zeros(N, H, cache.shape[-1] - rank, dtype=q.dtype, device=q.device)
@@ -277,13 +294,14 @@ def latent_attention(q, q_rot, cos_sin, rot_dim: int, cache, batch, scale: float
     for n, m in enumerate(batch.prefills):
         if row >= 0 and n not in skip:
             out[row : row + m.query_len] = _latent_attention_seq(
-                q[row : row + m.query_len], cache, m.block_table, m.ctx_len, rank, scale, window
+                q[row : row + m.query_len], cache, m.block_table, m.ctx_len, rank, scale, window,
+                sink,
             )
         row += m.query_len
     for b in range(batch.num_decode):
         out[row : row + 1] = _latent_attention_seq(
             q[row : row + 1], cache, batch.decode_block_tables[b],
-            int(batch.decode_seq_lens[b]) - 1, rank, scale, window,
+            int(batch.decode_seq_lens[b]) - 1, rank, scale, window, sink,
         )
         row += 1
     return out
@@ -297,9 +315,65 @@ def cache_keys_values(k, v, slot_mapping, k_cache, v_cache):
     _flat(v_cache)[slot_mapping] = v
 
 
+def _portions(batch):
+    """(first row, rows, cached tokens before them, state slot, pages) per sequence."""
+    row = 0
+    for m in batch.prefills:
+        yield row, m.query_len, m.ctx_len, m.state_slot, m.block_table
+        row += m.query_len
+    slots = batch.decode_state_slots
+    for n in range(batch.num_decode):
+        yield (row + n, 1, int(batch.decode_seq_lens[n]) - 1,
+               0 if slots is None else int(slots[n]), batch.decode_block_tables[n])
+
+
+def _short_conv(proj, conv, ring, batch):
+    """Causal convolution of every sequence's rows, its ring advanced; fp32."""
+    taps, out = conv.shape[0], torch.empty(proj.shape, device=proj.device)
+    for row, n, ctx, slot, _ in _portions(batch):
+        u = proj[row : row + n]
+        past = [ring[slot, p % taps] if p >= 0 else torch.zeros_like(u[0])
+                for p in range(ctx - taps + 1, ctx)]
+        x = torch.cat([torch.stack(past), u]) if past else u
+        out[row : row + n] = sum(x[j : j + n].float() * conv[j].float() for j in range(taps))
+        for i in range(max(0, n - taps), n):
+            ring[slot, (ctx + i) % taps] = u[i]
+    return out
+
+
+def attention_inputs(proj, heads, dim, vdim, k_cache, v_cache, batch, eps, conv, ring, q_norm,
+                     k_norm, v_norm, cos_sin, head_mult, q_temp):
+    N, d, e, G = proj.shape[0], k_cache.shape[-1], v_cache.shape[-1], k_cache.shape[2]
+    x = proj.float() if conv is None else _short_conv(proj, conv, ring, batch)
+    q, k, v = x.split([heads * d, G * d, G * e], 1)
+    q, k, v = q.reshape(N, heads, d), k.reshape(N, G, d), v.reshape(N, G, e)
+
+    def rms(t, size):  # the padding is zero
+        return t * torch.rsqrt(t.pow(2).sum(-1, keepdim=True) / size + eps)
+
+    if q_norm is not None:
+        q, k = rms(q, dim) * q_norm.float(), rms(k, dim) * k_norm.float()
+    if v_norm:
+        v = rms(v, vdim)
+    p = batch.positions
+    if cos_sin is not None:
+        n = 2 * cos_sin.shape[2]
+        c, s = (t[p].unsqueeze(1) for t in cos_sin)
+        q, k = (torch.cat([_rotate_interleaved(t[..., :n], c, s), t[..., n:]], -1)
+                for t in (q, k))
+    if head_mult is not None:
+        q = q * head_mult.view(1, -1, 1)
+    if q_temp is not None:
+        coef, every = q_temp
+        t = 1 + coef * torch.log(torch.floor((p + 1) / every) + 1)
+        q = q * t.view(-1, 1, 1)
+    cache_keys_values(k.to(proj.dtype), v.to(proj.dtype), batch.slot_mapping, k_cache, v_cache)
+    return q.to(proj.dtype)
+
+
 def _grouped_attention_seq(q, k_cache, v_cache, block_table, ctx_len: int, scale, cap, window,
-                           keep_first, sink):
-    """One sequence's rows at positions ctx_len..; q [L, H, d] -> [L, H, e]."""
+                           keep_first, sink, bias, sigmoid):
+    """One sequence's rows at positions ctx_len..; q [L, H, d] -> fp32 [L, H, e]."""
     L, H, bs = q.shape[0], q.shape[1], k_cache.shape[1]
     j = torch.arange(ctx_len + L, device=q.device)
     rows = torch.as_tensor(block_table, device=q.device)[j // bs] * bs + j % bs
@@ -310,31 +384,53 @@ def _grouped_attention_seq(q, k_cache, v_cache, block_table, ctx_len: int, scale
     if cap is not None:
         scores = cap * torch.tanh(scores / cap)
     i = torch.arange(ctx_len, ctx_len + L, device=q.device).view(-1, 1)
+    if bias is not None:
+        scores = scores + bias[:, (i - j).clamp(0, bias.shape[1] - 1)]
     hidden = j > i
     if window is not None:
         hidden |= ((i - j) >= window) & (j >= keep_first)
     scores = scores.masked_fill(hidden, float("-inf"))
-    if sink is not None:
-        scores = torch.cat([scores, sink.float().view(H, 1, 1).expand(H, L, 1)], -1)
-    probs = torch.softmax(scores, -1)[..., : len(j)]
-    return torch.matmul(probs, v).transpose(0, 1).to(q.dtype)
+    if sigmoid:
+        probs = torch.sigmoid(scores)
+    else:
+        probs = _sink_softmax(scores, None if sink is None else sink.view(H, 1, 1))
+    return torch.matmul(probs, v).transpose(0, 1)
 
 
 def grouped_attention(q, k_cache, v_cache, batch, scale: float, cap, window, keep_first: int,
-                      sink, out):
-    rest = (scale, cap, window, keep_first, sink)
-    row = 0
-    for m in batch.prefills:
-        out[row : row + m.query_len] = _grouped_attention_seq(
-            q[row : row + m.query_len], k_cache, v_cache, m.block_table, m.ctx_len, *rest
+                      sink, out, bias=None, sigmoid=False, gate=None):
+    for row, n, ctx, _, pages in _portions(batch):
+        y = _grouped_attention_seq(
+            q[row : row + n], k_cache, v_cache, pages, ctx, scale, cap, window, keep_first, sink,
+            bias, sigmoid,
         )
-        row += m.query_len
-    for n in range(batch.num_decode):
-        out[row] = _grouped_attention_seq(
-            q[row : row + 1], k_cache, v_cache, batch.decode_block_tables[n],
-            int(batch.decode_seq_lens[n]) - 1, *rest,
-        )[0]
-        row += 1
+        if gate is not None:
+            y = y * torch.sigmoid(gate[row : row + n].float()).unsqueeze(-1)
+        out[row : row + n] = y
+
+
+# -------------------------------------------------------------------- experts
+
+
+def moe_route(h, router, bias, top: int):
+    z = torch.matmul(h.float(), router.float().t())
+    if bias is not None:
+        z = z + bias
+    best = torch.topk(z, top, -1)
+    return best.indices.int(), torch.softmax(best.values, -1)
+
+
+def moe_experts(h, gate_up, down, ids, glu):
+    N, k = ids.shape
+    rows = torch.empty(N, k, down.shape[1], dtype=h.dtype, device=h.device)
+    for e in range(gate_up.shape[0]):
+        token, choice = (ids == e).nonzero(as_tuple=True)
+        if len(token):
+            x = torch.nn.functional.linear(h[token], gate_up[e])
+            act = x.new_empty(len(token), down.shape[2])
+            clamped_glu(x, glu.limit, glu.alpha, glu.offset, act, glu.cubic)
+            rows[token, choice] = torch.nn.functional.linear(act, down[e])
+    return rows
 
 
 # ----------------------------------------------------------------- delta rule
