@@ -113,20 +113,26 @@ def swiglu(gate_up):
 
 def layernorm(x, weight, eps: float, dtype):
     out = torch.empty(x.shape, dtype=dtype, device=x.device)
-    _C.residual_norm(x, None, None, weight, out, eps, True, 0.0, 1.0, None, None, None, 0)
+    _C.residual_norm(
+        x, None, None, weight, out, eps, True, 0.0, 1.0, None, None, None, 0, None, None, None,
+        None,
+    )
     return out
 
 
 def residual_norm(x, y, eps: float, y_norm=None, x_norm=None, out=None, center=True,
-                  offset=0.0, mult=1.0, depth=None, layer=0):
+                  offset=0.0, mult=1.0, depth=None, layer=0, x_norm2=None, out2=None,
+                  experts=None):
     states, coef, partial = depth or (None, None, None)
+    rows, weights = experts or (None, None)
     _C.residual_norm(
-        x, y, y_norm, x_norm, out, eps, center, offset, mult, states, coef, partial, layer
+        x, y, y_norm, x_norm, out, eps, center, offset, mult, states, coef, partial, layer,
+        x_norm2, out2, rows, weights,
     )
 
 
-def embed_positions(token_ids, positions, table, cos_sin, x, copy=None):
-    _C.embed_positions(x, copy, token_ids, positions, table, cos_sin)
+def embed_positions(token_ids, positions, table, cos_sin, x, copy=None, scale=1.0):
+    _C.embed_positions(x, copy, token_ids, positions, table, cos_sin, scale)
 
 
 def softcap(logits, cap):
@@ -135,8 +141,8 @@ def softcap(logits, cap):
     return out
 
 
-def clamped_glu(gate_up, limit: float, alpha: float, offset: float, out):
-    _C.clamped_glu(out, gate_up, limit, alpha, offset)
+def clamped_glu(gate_up, limit: float, alpha: float, offset: float, out, cubic=0.0):
+    _C.clamped_glu(out, gate_up, limit, alpha, offset, cubic)
 
 
 #: up to this many tokens the fused side_gate kernel beats the GEMM route
@@ -180,7 +186,7 @@ def head_linear(x, w, out, gate=None):
 
 
 def _latent_attn(out, q, q_rot, cos_sin, rot_dim, cache, tables, seq_lens, prefill, tiles,
-                 mg, max_keys, scale, window, mfma):
+                 mg, max_keys, scale, window, mfma, sink):
     """One launch over prefill tiles (prefill = their metadata) or decode
     rows.  Few tiles split their keys over several workgroups."""
     n_split = 1
@@ -200,12 +206,12 @@ def _latent_attn(out, q, q_rot, cos_sin, rot_dim, cache, tables, seq_lens, prefi
     _C.latent_attn(
         out, q, q_rot, cos_sin, rot_dim, cache, tables, seq_lens,
         *((m.ctx_lens, m.row_starts, m.tile_seq, m.tile_q0) if m else (None,) * 4),
-        part, ml, scale, window, mg, n_split, mfma,
+        part, ml, sink, scale, window, mg, n_split, mfma,
     )
 
 
 def latent_attention(q, q_rot, cos_sin, rot_dim: int, cache, batch, scale: float, window,
-                     row0: int = 0, skip=()):
+                     row0: int = 0, skip=(), sink=None):
     from . import LATENT_RANKS
 
     N, H, rank = q.shape
@@ -223,7 +229,7 @@ def latent_attention(q, q_rot, cos_sin, rot_dim: int, cache, batch, scale: float
         _latent_attn(
             out[:P], q[:P], q_rot[:P], *common, meta.block_tables, meta.seq_lens, meta,
             meta.tile_seq.numel(), most, max(batch.prefills[i].seq_len for i in chunks),
-            scale, window, mfma,
+            scale, window, mfma, sink,
         )
     if batch.num_decode:
         mg = 1 if H <= 16 else 2 if H <= 32 else most
@@ -231,7 +237,7 @@ def latent_attention(q, q_rot, cos_sin, rot_dim: int, cache, batch, scale: float
         _latent_attn(
             out[P:], q[P:], q_rot[P:], *common, tables, batch.decode_lens_i32(), None,
             batch.num_decode * -(-H // (16 * mg)), mg,
-            tables.shape[1] * cache.shape[1], scale, window, mfma,
+            tables.shape[1] * cache.shape[1], scale, window, mfma, sink,
         )
     return out
 
@@ -260,7 +266,7 @@ def _expansion_groups(batch, chunks, window: int, bytes_per_key: int):
 
 
 def latent_expanded_prefill(q, w_ukv, gate, cos_sin, rot_dim: int, cache, batch, chunks,
-                            rank: int, scale: float, window, out):
+                            rank: int, scale: float, window, out, sink=None):
     from . import linear
 
     window = window or _NO_WINDOW
@@ -279,7 +285,7 @@ def latent_expanded_prefill(q, w_ukv, gate, cos_sin, rot_dim: int, cache, batch,
         _C.latent_prefill(
             out, q, linear(rows[:, :rank], w_ukv), rows[:, rank:], gate, cos_sin, rot_dim,
             meta.seq_lens, meta.ctx_lens, meta.row_starts, meta.tile_seq, meta.tile_q0,
-            meta.key_first, meta.key_starts, scale, window,
+            meta.key_first, meta.key_starts, sink, scale, window,
         )
 
 
@@ -292,20 +298,73 @@ def cache_keys_values(k, v, slot_mapping, k_cache, v_cache):
     _C.cache_keys_values(k_cache, v_cache, k, v, slot_mapping)
 
 
+def _conv_rows(batch):
+    """Per row of a step: rows of its sequence right before it, its state slot; and the
+    rows that later steps' convolutions read.  None, slots, None: decode rows only."""
+    if not batch.prefills:
+        return None, batch.decode_state_slots, None
+    device, P = batch.positions.device, batch.num_prefill_tokens
+    meta, counts = batch.prefill_meta(16), [m.query_len for m in batch.prefills]
+    times = torch.tensor(counts, device=device)
+    per_row = torch.stack([meta.ctx_lens, meta.state_slots]).repeat_interleave(
+        times, 1, output_size=P
+    )
+    back, slots = batch.positions[:P].int() - per_row[0], per_row[1]
+    if batch.num_decode:
+        back = torch.cat([back, back.new_zeros(batch.num_decode)])
+        slots = torch.cat([slots, batch.decode_state_slots])
+    return back.contiguous(), slots.contiguous(), counts
+
+
+def _ring_rows(batch, taps: int):
+    """The last rows of every portion, as many as a convolution looks back."""
+    rows, at = [], 0
+    for m in batch.prefills:
+        at += m.query_len
+        rows.extend(range(at - min(m.query_len, taps), at))
+    rows.extend(range(at, at + batch.num_decode))
+    return torch.tensor(rows, dtype=torch.int32, device=batch.positions.device)
+
+
+def attention_inputs(proj, heads, dim, vdim, k_cache, v_cache, batch, eps, conv, ring, q_norm,
+                     k_norm, v_norm, cos_sin, head_mult, q_temp):
+    q = torch.empty(proj.shape[0], heads, k_cache.shape[3], dtype=proj.dtype, device=proj.device)
+    back = states = ring_rows = None
+    if conv is not None:
+        back, states, _ = batch.memo("conv_rows", lambda: _conv_rows(batch))
+        if batch.prefills:
+            taps = conv.shape[0]
+            ring_rows = batch.memo(("ring_rows", taps), lambda: _ring_rows(batch, taps))
+    coef, every = q_temp or (0.0, 0.0)
+    _C.attention_inputs(
+        q, k_cache, v_cache, proj, batch.positions, batch.slot_mapping, dim, vdim, eps, conv,
+        ring, back, states, ring_rows, ring_rows is None, q_norm, k_norm, v_norm, cos_sin,
+        head_mult, coef, every,
+    )
+    return q
+
+
 def grouped_attention(q, k_cache, v_cache, batch, scale: float, cap, window, keep_first: int,
-                      sink, out):
+                      sink, out, bias=None, sigmoid=False, gate=None):
     from . import LATENT_HEADS
 
     H, d, v, G = q.shape[1], q.shape[2], out.shape[2], k_cache.shape[2]
-    rest = (scale, cap or 0.0, window or _NO_WINDOW, keep_first)
-    tiled = q.dtype == torch.bfloat16 and d in LATENT_HEADS and v in LATENT_HEADS
+    rest = (scale, cap or 0.0, window or _NO_WINDOW, keep_first, sigmoid)
+    tiled = (q.dtype == torch.bfloat16 and d in LATENT_HEADS and v in LATENT_HEADS
+             and not (sigmoid and cap))
     P = batch.num_prefill_tokens
+    if gate is not None and q.dtype != gate.dtype:
+        raise TypeError("the gate has the queries' dtype")
+
+    def gates(r):
+        return None if gate is None else gate[r]
+
     if batch.prefills:
         meta = batch.prefill_meta(128 if tiled else 1)
         _C.grouped_attn(
             out[:P], q[:P], k_cache, v_cache, meta.block_tables, meta.seq_lens, meta.ctx_lens,
-            meta.row_starts, meta.tile_seq, meta.tile_q0, sink, None, None, *rest,
-            _PREFILL if tiled else _PLAIN, 1, 1,
+            meta.row_starts, meta.tile_seq, meta.tile_q0, sink, bias, gates(slice(0, P)), None,
+            None, *rest, _PREFILL if tiled else _PLAIN, 1, 1,
         )
     if not batch.num_decode:
         return
@@ -323,8 +382,45 @@ def grouped_attention(q, k_cache, v_cache, batch, scale: float, cap, window, kee
         ml = torch.empty(2 * n_split * rows, dtype=torch.float32, device=q.device)
     _C.grouped_attn(
         out[P:], q[P:], k_cache, v_cache, tables, batch.decode_lens_i32(), None, None, None,
-        None, sink, part, ml, *rest, _DECODE if tiled else _PLAIN, gm, n_split,
+        None, sink, bias, gates(slice(P, None)), part, ml, *rest, _DECODE if tiled else _PLAIN, gm, n_split,
     )
+
+
+# -------------------------------------------------------------------- experts
+
+
+def moe_route(h, router, bias, top: int):
+    ids = torch.empty(h.shape[0], top, dtype=torch.int32, device=h.device)
+    weights = torch.empty(h.shape[0], top, dtype=torch.float32, device=h.device)
+    _C.moe_route(ids, weights, h, router, bias)
+    return ids, weights
+
+
+#: rows per expert from which the tiled product is used
+_TILED_ROWS = 64
+
+
+def moe_experts(h, gate_up, down, ids, glu):
+    (N, k), E, inner = ids.shape, gate_up.shape[0], down.shape[2]
+    n, device = N * k, h.device
+    act = torch.empty(n, inner, dtype=h.dtype, device=device)
+    rows = torch.empty(N, k, down.shape[1], dtype=h.dtype, device=device)
+    form = (glu.limit, glu.alpha, glu.offset, glu.cubic)
+    perm = offsets = tile_expert = tile_row = None
+    kind, tt = 0, 1
+    if h.dtype == torch.bfloat16:
+        tiled = n >= _TILED_ROWS * E and gate_up.shape[2] % 128 == 0 and inner % 128 == 0
+        kind, tt = (2, 1) if tiled else (1, 1 if n <= 8 * E else 2 if n <= 32 * E else 4)
+        perm = torch.empty(n, dtype=torch.int32, device=device)
+        offsets = torch.empty(E + 2, dtype=torch.int32, device=device)
+        if tiled:
+            tiles = torch.empty(2, n // _C.EXPERT_TILE + E, dtype=torch.int32, device=device)
+            tile_expert, tile_row = tiles
+        _C.moe_group(perm, offsets, tile_expert, tile_row, ids, E)
+    grouped = (ids, perm, offsets, tile_expert, tile_row)
+    _C.experts_linear(act, h, gate_up, *grouped, True, *form, kind, tt)
+    _C.experts_linear(rows.view(n, -1), act, down, *grouped, False, *form, kind, tt)
+    return rows
 
 
 # ----------------------------------------------------------------- delta rule

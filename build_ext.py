@@ -39,6 +39,9 @@ def build(verbose: bool = False) -> str:
         os.path.join(CSRC, "embedding.hip"),
         os.path.join(CSRC, "grouped_attn.hip"),
         os.path.join(CSRC, "grouped_prefill.hip"),
+        os.path.join(CSRC, "attn_inputs.hip"),
+        os.path.join(CSRC, "experts.hip"),
+        os.path.join(CSRC, "experts_gemm.hip"),
         os.path.join(CSRC, "channel_delta.hip"),
         os.path.join(CSRC, "sampling.hip"),
         os.path.join(CSRC, "sampling_fullvocab.hip"),

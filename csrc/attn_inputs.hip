@@ -1,0 +1,217 @@
+// What happens to q, k and v between their projection and attention, in one pass
+// (gfx950): short convolution, norms per head, rotation, query temperature; keys and
+// values go to their cache slots.
+//
+// A thread owns VW channels of one row.  Heads start at multiples of their size, so a
+// head is a group of d / VW neighbouring lanes, which reduce by shuffles; sections are
+// aligned so that no group straddles a wave.  Rotations pair dimension 2i with 2i + 1,
+// both in one thread.  Everything between load and store is fp32.
+//
+// The convolutions' inputs are kept in a ring by position.  A row that is alone in its
+// sequence's step writes an entry that its own convolution does not read, at once;
+// with longer portions that entry may be one that an earlier row reads, so their last
+// inputs follow in a second launch.
+#include "common_t.h"
+#include "attn_inputs.h"
+
+// input of VW channels ``ago`` tokens before row n, or zeros
+template <typename T, int VW>
+DEV Pack<T, VW> conv_input(const AttnInputsArgs& a, int64_t n, int64_t p, int back, int64_t state,
+                           int ago, int c) {
+  const T* src = (const T*)a.proj + n * a.stride + c;
+  bool have = true;
+  if (ago <= back) {
+    src -= ago * a.stride;
+  } else {
+    have = ago <= p;
+    const int64_t entry = have ? (p - ago) % a.taps : 0;
+    if (have) src = (const T*)a.ring + (state * a.taps + entry) * a.C + c;
+  }
+  Pack<T, VW> x = *(const Pack<T, VW>*)src;
+  if (!have)
+#pragma unroll
+    for (int k = 0; k < VW; ++k) x.v[k] = from_f<T>(0.f);
+  return x;
+}
+
+// TAPS: 0 none, 4 unrolled, -1 any number
+template <typename T, int VW, int TAPS>
+DEV void channels(const AttnInputsArgs& a, int64_t n, int64_t p, int back, int64_t state, int c,
+                  float* y) {
+  if constexpr (TAPS == 0) {
+    load_f<VW>(y, (const T*)a.proj + n * a.stride + c);
+  } else {
+    const int taps = TAPS > 0 ? TAPS : a.taps;
+    const T* w = (const T*)a.conv + c;
+#pragma unroll
+    for (int k = 0; k < VW; ++k) y[k] = 0.f;
+#pragma unroll(TAPS > 0 ? TAPS : 1)
+    for (int j = 0; j < taps; ++j) {
+      const Pack<T, VW> x = conv_input<T, VW>(a, n, p, back, state, taps - 1 - j, c);
+      const Pack<T, VW> f = *(const Pack<T, VW>*)(w + (int64_t)j * a.C);
+#pragma unroll
+      for (int k = 0; k < VW; ++k) y[k] += to_f(f.v[k]) * to_f(x.v[k]);
+    }
+  }
+}
+
+// y: VW channels from i of a head whose squares sum to ss; sect 0 q, 1 k, 2 v
+template <typename T, int VW>
+DEV void finish(const AttnInputsArgs& a, int64_t n, int64_t p, int sect, int head, int i,
+                float ss, float* y) {
+  if (sect < 2 ? a.q_norm != nullptr : a.v_norm) {
+    const float inv = rsqrtf(ss / (sect < 2 ? a.dim : a.vdim) + a.eps);
+#pragma unroll
+    for (int k = 0; k < VW; ++k) y[k] *= inv;
+    if (sect < 2) {
+      float w[VW];
+      load_f<VW>(w, (const T*)(sect == 0 ? a.q_norm : a.k_norm) + i);
+#pragma unroll
+      for (int k = 0; k < VW; ++k) y[k] *= w[k];
+    }
+  }
+  if (a.cos_sin && sect < 2) {
+    const float* ct = a.cos_sin + p * a.pairs;
+    const float* st = ct + a.P * a.pairs;
+#pragma unroll
+    for (int k = 0; k < VW; k += 2) {
+      const int at = (i + k) >> 1;
+      if (at < a.pairs) {
+        const float co = ct[at], si = st[at], u = y[k], v = y[k + 1];
+        y[k] = u * co - v * si;
+        y[k + 1] = v * co + u * si;
+      }
+    }
+  }
+  if (sect == 0) {
+    float f = a.head_mult ? a.head_mult[head] : 1.f;
+    if (a.q_every > 0.f) f *= 1.f + a.q_coef * logf(floorf((float)(p + 1) / a.q_every) + 1.f);
+#pragma unroll
+    for (int k = 0; k < VW; ++k) y[k] *= f;
+    store_f<VW>((T*)a.q + (n * a.H + head) * a.d + i, y);
+  } else if (sect == 1) {
+    store_f<VW>((T*)a.k_cache + (a.slots[n] * a.G + head) * a.d + i, y);
+  } else {
+    store_f<VW>((T*)a.v_cache + (a.slots[n] * a.G + head) * a.v + i, y);
+  }
+}
+
+// Head sizes of at most 64 threads, a power of two.  grid (units / 256, rows): a row has
+// ``units`` threads, a multiple of 64.
+template <typename T, int VW, int TAPS>
+__global__ __launch_bounds__(256) void attn_inputs_kernel(const AttnInputsArgs a, const int units,
+                                                          const int64_t total) {
+  const int64_t id = (int64_t)blockIdx.x * 256 + threadIdx.x;
+  if (id >= total) return;
+  const int64_t n = id / units;
+  int u = (int)(id - n * units);
+  const int lq = a.d / VW, lv = a.v / VW;
+  const int k_at = a.H * lq, v_at = ((a.H + a.G) * lq + lv - 1) / lv * lv;
+  int sect = 0, c0 = 0, lanes = lq;
+  bool live = true;
+  if (u >= v_at) {
+    sect = 2;
+    u -= v_at;
+    c0 = (a.H + a.G) * a.d;
+    lanes = lv;
+    live = u < a.G * lv;
+  } else if (u >= k_at) {
+    sect = 1;
+    u -= k_at;
+    c0 = a.H * a.d;
+    live = u < a.G * lq;
+  }
+  if (!live) u = 0;
+  const int64_t p = a.positions[n];
+  const int back = a.back ? a.back[n] : 0;
+  const int64_t state = TAPS ? a.states[n] : 0;
+  float y[VW];
+  channels<T, VW, TAPS>(a, n, p, back, state, c0 + u * VW, y);
+  if (TAPS && a.write_ring && live)
+    *(Pack<T, VW>*)((T*)a.ring + (state * a.taps + p % a.taps) * a.C + c0 + u * VW) =
+        *(const Pack<T, VW>*)((const T*)a.proj + n * a.stride + c0 + u * VW);
+  float ss = 0.f;
+#pragma unroll
+  for (int k = 0; k < VW; ++k) ss += y[k] * y[k];
+#pragma unroll
+  for (int off = 1; off < 64; off <<= 1) {
+    const float t = __shfl_xor(ss, off, 64);
+    if (off < lanes) ss += t;
+  }
+  if (live) finish<T, VW>(a, n, p, sect, u / lanes, u % lanes * VW, ss, y);
+}
+
+// Any head size (a multiple of VW): a wave per row and head.
+template <typename T, int VW>
+__global__ __launch_bounds__(256) void attn_inputs_any_kernel(const AttnInputsArgs a) {
+  const int64_t n = blockIdx.y;
+  int head = blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (head >= a.H + 2 * a.G) return;
+  const int lane = threadIdx.x & 63;
+  int sect = 0, c0 = head * a.d, size = a.d;
+  if (head >= a.H + a.G) {
+    head -= a.H + a.G;
+    sect = 2;
+    c0 = (a.H + a.G) * a.d + head * a.v;
+    size = a.v;
+  } else if (head >= a.H) {
+    head -= a.H;
+    sect = 1;
+  }
+  const int64_t p = a.positions[n];
+  const int back = a.back ? a.back[n] : 0;
+  const int64_t state = a.conv ? a.states[n] : 0;
+  auto get = [&](int i, float* y) {
+    if (a.conv)
+      channels<T, VW, -1>(a, n, p, back, state, c0 + i, y);
+    else
+      channels<T, VW, 0>(a, n, p, back, state, c0 + i, y);
+  };
+  float ss = 0.f, y[VW];
+  for (int i = lane * VW; i < size; i += 64 * VW) {
+    get(i, y);
+#pragma unroll
+    for (int k = 0; k < VW; ++k) ss += y[k] * y[k];
+  }
+  ss = wave_sum(ss);
+  for (int i = lane * VW; i < size; i += 64 * VW) {
+    get(i, y);
+    if (a.conv && a.write_ring)
+      *(Pack<T, VW>*)((T*)a.ring + (state * a.taps + p % a.taps) * a.C + c0 + i) =
+          *(const Pack<T, VW>*)((const T*)a.proj + n * a.stride + c0 + i);
+    finish<T, VW>(a, n, p, sect, head, i, ss, y);
+  }
+}
+
+// grid (parts of a row, ring rows)
+template <typename T, int VW>
+__global__ __launch_bounds__(256) void attn_ring_kernel(const AttnInputsArgs a) {
+  const int c = (blockIdx.x * 256 + threadIdx.x) * VW;
+  if (c >= a.C) return;
+  const int64_t n = a.ring_rows[blockIdx.y];
+  *(Pack<T, VW>*)((T*)a.ring + (a.states[n] * (int64_t)a.taps + a.positions[n] % a.taps) * a.C + c) =
+      *(const Pack<T, VW>*)((const T*)a.proj + n * a.stride + c);
+}
+
+template <typename T, int VW>
+static void launch(const AttnInputsArgs& a, hipStream_t stream) {
+  const int lq = a.d / VW, lv = a.v / VW;
+  auto fits = [](int lanes) { return lanes <= 64 && (lanes & (lanes - 1)) == 0; };
+  if (fits(lq) && fits(lv)) {
+    const int v_at = ((a.H + a.G) * lq + lv - 1) / lv * lv;
+    const int units = (v_at + a.G * lv + 63) / 64 * 64;
+    const int64_t total = (int64_t)a.N * units;
+    auto k = !a.conv         ? attn_inputs_kernel<T, VW, 0>
+             : a.taps == 4   ? attn_inputs_kernel<T, VW, 4>
+                             : attn_inputs_kernel<T, VW, -1>;
+    k<<<(unsigned)((total + 255) / 256), 256, 0, stream>>>(a, units, total);
+  } else {
+    attn_inputs_any_kernel<T, VW><<<dim3((a.H + 2 * a.G + 3) / 4, a.N), 256, 0, stream>>>(a);
+  }
+  if (a.n_ring_rows)
+    attn_ring_kernel<T, VW><<<dim3((a.C / VW + 255) / 256, a.n_ring_rows), 256, 0, stream>>>(a);
+}
+
+extern "C" void launch_attn_inputs(bool bf16, const AttnInputsArgs* a, hipStream_t stream) {
+  bf16 ? launch<bf16_t, 8>(*a, stream) : launch<float, 4>(*a, stream);
+}

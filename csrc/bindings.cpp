@@ -9,7 +9,9 @@
 #include <algorithm>
 #include <cmath>
 
+#include "attn_inputs.h"
 #include "channel_delta.h"
+#include "experts.h"
 #include "grouped_attn.h"
 #include "latent_attn.h"
 #include "residual_norm.h"
@@ -43,7 +45,14 @@ void launch_prefill_attn_mfma(void*, const void*, const void*, const void*, cons
 void launch_residual_norm(bool, float*, const void*, const void*, const void*, void*, float,
                           int, int, int64_t, const NormForm*, hipStream_t);
 void launch_embed_positions(bool, float*, float*, const int64_t*, const int64_t*, const void*,
-                            const float*, int, int, int64_t, int64_t, hipStream_t);
+                            const float*, float, int, int, int64_t, int64_t, hipStream_t);
+void launch_attn_inputs(bool, const AttnInputsArgs*, hipStream_t);
+void launch_moe_route(bool, int*, float*, const void*, const void*, const float*, int, int, int,
+                      int, int64_t, hipStream_t);
+void launch_moe_group(int*, int*, int*, int*, const int*, int, int, hipStream_t);
+void launch_experts_small(bool, const ExpertsArgs*, int, hipStream_t);
+void launch_experts_f32(bool, const ExpertsArgs*, hipStream_t);
+void launch_experts_gemm(bool, const ExpertsArgs*, hipStream_t);
 void launch_softcap(bool, float*, const void*, float, int64_t, hipStream_t);
 bool launch_grouped_decode(const GroupedArgs*, int, int, int, int, hipStream_t);
 bool launch_grouped_plain(bool, const GroupedArgs*, int, int, int, hipStream_t);
@@ -55,7 +64,7 @@ void launch_delta_step(bool, const DeltaArgs*, int, hipStream_t);
 void launch_side_gate(bool, float*, const float*, const void*, const void*, const int64_t*, const void*,
                       void*, int, int, int, int64_t, hipStream_t);
 void launch_add_to_residual(bool, float*, const void*, void*, int64_t, hipStream_t);
-void launch_clamped_glu(bool, void*, const void*, float, float, float, int, int, int64_t,
+void launch_clamped_glu(bool, void*, const void*, float, float, float, float, int, int, int64_t,
                         int64_t, hipStream_t);
 void launch_gelu_gate(bool, void*, const int64_t*, const void*, int, int, int64_t,
                       hipStream_t);
@@ -301,7 +310,8 @@ static void check_aligned(const torch::Tensor& t) {
 static void residual_norm(torch::Tensor x, OptTensor y, OptTensor y_norm, OptTensor x_norm,
                           OptTensor out, double eps, bool center, double offset, double mult,
                           OptTensor states, OptTensor coef, OptTensor partial,
-                          int64_t layer) {
+                          int64_t layer, OptTensor x_norm2, OptTensor out2, OptTensor rows,
+                          OptTensor weights) {
   CHECK_CUDA(x); CHECK_CONT(x);
   TORCH_CHECK(x.scalar_type() == at::kFloat && x.dim() == 2);
   TORCH_CHECK(y || out, "nothing to do");
@@ -316,6 +326,23 @@ static void residual_norm(torch::Tensor x, OptTensor y, OptTensor y_norm, OptTen
   f.center = center;
   f.offset = (float)offset;
   f.mult = (float)mult;
+  if (rows) {
+    TORCH_CHECK(y && !y_norm && weights && rows->dim() == 3, "expert rows");
+    f.top = rows->size(1);
+    TORCH_CHECK(rows->size(0) == n && rows->size(2) == w && rows->scalar_type() == dt &&
+                weights->dim() == 2 && weights->size(0) == n && weights->size(1) == f.top &&
+                weights->scalar_type() == at::kFloat, "expert rows");
+    CHECK_CUDA((*rows)); CHECK_CONT((*rows)); CHECK_CUDA((*weights)); CHECK_CONT((*weights));
+    f.rows = rows->data_ptr();
+    f.weights = weights->data_ptr<float>();
+  }
+  if (out2) {
+    TORCH_CHECK(out && x_norm && x_norm2, "second norm");
+    check_rows(*out2, dt, n, w); check_vec(*x_norm2, dt, w);
+    f.x_norm2 = x_norm2->data_ptr();
+    f.out2 = out2->data_ptr();
+    f.out2_stride = out2->stride(0);
+  }
   if (states) {
     TORCH_CHECK(coef && partial && y, "depth states");
     for (const auto* t : {&*states, &*coef, &*partial}) {
@@ -353,7 +380,8 @@ static void check_ids(const torch::Tensor& t, int64_t n) {
 }
 
 static void embed_positions(torch::Tensor x, OptTensor copy, torch::Tensor token_ids,
-                            torch::Tensor positions, torch::Tensor table, OptTensor cos_sin) {
+                            torch::Tensor positions, torch::Tensor table, OptTensor cos_sin,
+                            double scale) {
   const int n = x.size(0), w = x.size(1);
   check_rows(x, at::kFloat, n, w); CHECK_CONT(x);
   if (copy) { check_rows(*copy, at::kFloat, n, w); CHECK_CONT((*copy)); }
@@ -368,8 +396,8 @@ static void embed_positions(torch::Tensor x, OptTensor copy, torch::Tensor token
   launch_embed_positions(is_bf16(table), x.data_ptr<float>(),
                          copy ? copy->data_ptr<float>() : nullptr,
                          token_ids.data_ptr<int64_t>(), positions.data_ptr<int64_t>(),
-                         table.data_ptr(), cos_sin ? cos_sin->data_ptr<float>() : nullptr, n, w,
-                         table.size(0), cos_sin ? cos_sin->size(1) : 1, cur_stream());
+                         table.data_ptr(), cos_sin ? cos_sin->data_ptr<float>() : nullptr,
+                         (float)scale, n, w, table.size(0), cos_sin ? cos_sin->size(1) : 1, cur_stream());
 }
 
 static void softcap(torch::Tensor out, torch::Tensor x, double cap) {
@@ -416,7 +444,7 @@ static void add_to_residual(torch::Tensor x, torch::Tensor y, OptTensor out) {
 }
 
 static void clamped_glu(torch::Tensor out, torch::Tensor gate_up, double limit,
-                        double alpha, double offset) {
+                        double alpha, double offset, double cubic) {
   const int rows = out.size(0), inter = out.size(1);
   check_rows(out, gate_up.scalar_type(), rows, inter);
   check_rows(gate_up, gate_up.scalar_type(), rows, 2 * (int64_t)inter);
@@ -424,7 +452,7 @@ static void clamped_glu(torch::Tensor out, torch::Tensor gate_up, double limit,
   TORCH_CHECK(inter % 8 == 0, "padded width must be a multiple of 8");
   if (rows == 0) return;
   launch_clamped_glu(is_bf16(out), out.data_ptr(), gate_up.data_ptr(), (float)limit,
-                     (float)alpha, (float)offset, rows, inter, gate_up.stride(0),
+                     (float)alpha, (float)offset, (float)cubic, rows, inter, gate_up.stride(0),
                      out.stride(0), cur_stream());
 }
 
@@ -522,8 +550,8 @@ static void latent_attn(torch::Tensor out, torch::Tensor q, torch::Tensor q_rot,
                         torch::Tensor cos_sin, int64_t rot_dim, torch::Tensor cache,
                         torch::Tensor tables, torch::Tensor seq_lens, OptTensor ctx_lens,
                         OptTensor row_starts, OptTensor tile_seq, OptTensor tile_r0,
-                        OptTensor part, OptTensor part_ml, double scale, int64_t window,
-                        int64_t mg, int64_t n_split, bool mfma) {
+                        OptTensor part, OptTensor part_ml, OptTensor sink, double scale,
+                        int64_t window, int64_t mg, int64_t n_split, bool mfma) {
   CHECK_CUDA(q); CHECK_CONT(q); CHECK_CONT(out); CHECK_CUDA(cache); CHECK_CONT(cache);
   CHECK_CUDA(tables); CHECK_CONT(tables); CHECK_CUDA(seq_lens); CHECK_CONT(seq_lens);
   const bool bf16 = is_bf16(q);
@@ -571,6 +599,7 @@ static void latent_attn(torch::Tensor out, torch::Tensor q, torch::Tensor q_rot,
   a.cos_sin = cos_sin.data_ptr<float>();
   a.positions = cos_sin.size(1);
   a.cache = cache.data_ptr();
+  if (sink) { check_vec(*sink, at::kFloat, H); a.sink = sink->data_ptr<float>(); }
   a.tables = tables.data_ptr<int>();
   a.seq_lens = seq_lens.data_ptr<int>();
   a.ctx_lens = opt_int(ctx_lens, seqs);
@@ -611,7 +640,8 @@ static void latent_prefill(torch::Tensor out, torch::Tensor q, torch::Tensor kv,
                            int64_t rot_dim, torch::Tensor seq_lens, torch::Tensor ctx_lens,
                            torch::Tensor row_starts, torch::Tensor tile_seq,
                            torch::Tensor tile_q0, torch::Tensor key_first,
-                           torch::Tensor key_starts, double scale, int64_t window) {
+                           torch::Tensor key_starts, OptTensor sink, double scale,
+                           int64_t window) {
   const int tokens = q.size(0), H = q.size(1), d = q.size(2) - 64, v = out.size(2);
   check_heads(q, at::kBFloat16, tokens, H);
   check_heads(out, at::kBFloat16, tokens, H);
@@ -632,6 +662,7 @@ static void latent_prefill(torch::Tensor out, torch::Tensor q, torch::Tensor kv,
   a.kv = kv.data_ptr();
   a.k_rot = k_rot.data_ptr();
   a.gate = gate ? gate->data_ptr() : nullptr;
+  if (sink) { check_vec(*sink, at::kFloat, H); a.sink = sink->data_ptr<float>(); }
   a.cos_sin = cos_sin.data_ptr<float>();
   a.n_tiles = tile_seq.numel();
   a.seq_lens = opt_int(seq_lens, seqs);
@@ -699,14 +730,15 @@ static void cache_keys_values(torch::Tensor k_cache, torch::Tensor v_cache, torc
 static void grouped_attn(torch::Tensor out, torch::Tensor q, torch::Tensor k_cache,
                          torch::Tensor v_cache, torch::Tensor tables, torch::Tensor seq_lens,
                          OptTensor ctx_lens, OptTensor row_starts, OptTensor tile_seq,
-                         OptTensor tile_q0, OptTensor sink, OptTensor part, OptTensor part_ml,
-                         double scale, double cap, int64_t window, int64_t keep, int64_t kind,
-                         int64_t gm, int64_t n_split) {
+                         OptTensor tile_q0, OptTensor sink, OptTensor bias, OptTensor gate,
+                         OptTensor part, OptTensor part_ml, double scale, double cap,
+                         int64_t window, int64_t keep, bool sigmoid, int64_t kind, int64_t gm,
+                         int64_t n_split) {
   const auto dt = q.scalar_type();
   const bool bf16 = is_bf16(q);
   const int tokens = q.size(0), H = q.size(1), d = q.size(2), v = out.size(2);
   check_token_heads(q, dt, tokens, H, d);
-  check_token_heads(out, dt, tokens, H, v); CHECK_CONT(out);
+  check_token_heads(out, dt, tokens, H, v);
   check_cache(k_cache, dt); check_cache(v_cache, dt);
   const int G = k_cache.size(2);
   TORCH_CHECK(k_cache.size(3) == d && v_cache.size(3) == v && v_cache.size(2) == G &&
@@ -734,6 +766,21 @@ static void grouped_attn(torch::Tensor out, torch::Tensor q, torch::Tensor k_cac
   a.k_cache = k_cache.data_ptr();
   a.v_cache = v_cache.data_ptr();
   if (sink) { check_vec(*sink, at::kFloat, H); a.sink = sink->data_ptr<float>(); }
+  TORCH_CHECK(!(sink && sigmoid), "a sink belongs to the softmax");
+  if (bias) {
+    TORCH_CHECK(bias->dim() == 2 && bias->size(0) == H && bias->size(1) > 0 &&
+                bias->scalar_type() == at::kFloat, "bias by head and distance");
+    CHECK_CUDA((*bias)); CHECK_CONT((*bias));
+    a.bias = bias->data_ptr<float>();
+    a.n_bias = bias->size(1);
+  }
+  if (gate) {
+    check_rows(*gate, dt, tokens, H);
+    a.gate = gate->data_ptr();
+    a.gate_stride = gate->stride(0);
+  }
+  a.sigmoid = sigmoid;
+  a.out_stride = out.stride(0);
   a.tables = tables.data_ptr<int>();
   a.seq_lens = opt_int(seq_lens, seqs);
   a.ctx_lens = opt_int(ctx_lens, seqs);
@@ -762,6 +809,169 @@ static void grouped_attn(torch::Tensor out, torch::Tensor q, torch::Tensor k_cac
                   : kind == 1 ? launch_grouped_decode(&a, d, v, seqs, (int)gm, cur_stream())
                               : launch_grouped_plain(bf16, &a, d, v, tokens, cur_stream());
   TORCH_CHECK(ok, "grouped attention: unsupported sizes d ", d, " v ", v);
+}
+
+// proj [N, (H + G) d + G v] -> q [N, H, d] and the rows' cache slots.  back, states: per row;
+// ring_rows: rows that join the ring after all others have read it.
+static void attention_inputs(torch::Tensor q, torch::Tensor k_cache, torch::Tensor v_cache,
+                             torch::Tensor proj, torch::Tensor positions, torch::Tensor slots,
+                             int64_t dim, int64_t vdim, double eps, OptTensor conv,
+                             OptTensor ring, OptTensor back, OptTensor states,
+                             OptTensor ring_rows, bool write_ring, OptTensor q_norm,
+                             OptTensor k_norm, bool v_norm, OptTensor cos_sin,
+                             OptTensor head_mult, double q_coef, double q_every) {
+  const auto dt = proj.scalar_type();
+  const bool bf16 = is_bf16(proj);
+  AttnInputsArgs a{};
+  a.N = q.size(0);
+  a.H = q.size(1);
+  a.d = q.size(2);
+  check_token_heads(q, dt, a.N, a.H, a.d); CHECK_CONT(q);
+  check_cache(k_cache, dt); check_cache(v_cache, dt);
+  a.G = k_cache.size(2);
+  a.v = v_cache.size(3);
+  TORCH_CHECK(k_cache.size(3) == a.d && v_cache.size(2) == a.G &&
+              k_cache.size(0) == v_cache.size(0) && k_cache.size(1) == v_cache.size(1),
+              "cache shapes");
+  a.C = (a.H + a.G) * a.d + a.G * a.v;
+  check_rows(proj, dt, a.N, a.C); check_aligned(proj);
+  check_ids(positions, a.N); check_ids(slots, a.N);
+  TORCH_CHECK(dim > 0 && dim <= a.d && vdim > 0 && vdim <= a.v && a.d % 8 == 0 && a.v % 8 == 0,
+              "head sizes");
+  if (conv) {
+    a.taps = conv->size(0);
+    TORCH_CHECK(a.taps > 0 && ring && states, "convolution state");
+    check_rows(*conv, dt, a.taps, a.C); CHECK_CONT((*conv));
+    CHECK_CUDA((*ring)); CHECK_CONT((*ring));
+    TORCH_CHECK(ring->dim() == 3 && ring->size(1) == a.taps && ring->size(2) == a.C &&
+                ring->scalar_type() == dt, "convolution state");
+    a.conv = conv->data_ptr();
+    a.ring = ring->data_ptr();
+    a.back = opt_int(back, a.N);
+    a.states = opt_int(states, a.N);
+    a.write_ring = write_ring;
+    if (ring_rows) {
+      a.n_ring_rows = ring_rows->numel();
+      a.ring_rows = opt_int(ring_rows, a.n_ring_rows);
+      TORCH_CHECK(a.n_ring_rows <= 65535, "grid");
+    }
+  }
+  if (q_norm) {
+    TORCH_CHECK(k_norm, "q and k are normed alike");
+    check_vec(*q_norm, dt, a.d); check_vec(*k_norm, dt, a.d);
+    a.q_norm = q_norm->data_ptr();
+    a.k_norm = k_norm->data_ptr();
+  }
+  a.v_norm = v_norm;
+  if (cos_sin) {
+    check_rotation(*cos_sin, positions, a.N, 2 * cos_sin->size(2));
+    a.pairs = cos_sin->size(2);
+    TORCH_CHECK(2 * a.pairs <= a.d, "rotated dimensions");
+    a.cos_sin = cos_sin->data_ptr<float>();
+    a.P = cos_sin->size(1);
+  }
+  if (head_mult) {
+    check_vec(*head_mult, at::kFloat, a.H);
+    a.head_mult = head_mult->data_ptr<float>();
+  }
+  TORCH_CHECK(q_every >= 0);
+  a.q_coef = (float)q_coef;
+  a.q_every = (float)q_every;
+  a.q = q.data_ptr();
+  a.k_cache = k_cache.data_ptr();
+  a.v_cache = v_cache.data_ptr();
+  a.proj = proj.data_ptr();
+  a.positions = positions.data_ptr<int64_t>();
+  a.slots = slots.data_ptr<int64_t>();
+  a.stride = proj.stride(0);
+  a.dim = (int)dim;
+  a.vdim = (int)vdim;
+  a.eps = (float)eps;
+  TORCH_CHECK(a.N <= 65535 * 16, "grid");
+  if (a.N == 0) return;
+  launch_attn_inputs(bf16, &a, cur_stream());
+}
+
+// ---- mixture of experts
+
+static void moe_route(torch::Tensor ids, torch::Tensor weights, torch::Tensor h, torch::Tensor w,
+                      OptTensor bias) {
+  const int N = h.size(0), K = h.size(1), E = w.size(0), top = ids.size(1);
+  check_rows(h, h.scalar_type(), N, K); check_aligned(h);
+  check_rows(w, h.scalar_type(), E, K); CHECK_CONT(w);
+  check_rows(ids, at::kInt, N, top); CHECK_CONT(ids);
+  check_rows(weights, at::kFloat, N, top); CHECK_CONT(weights);
+  if (bias) check_vec(*bias, at::kFloat, E);
+  TORCH_CHECK(K % 64 == 0 && E <= 512 && top > 0 && top <= E && top <= 64, "router sizes");
+  if (N == 0) return;
+  launch_moe_route(is_bf16(h), ids.data_ptr<int>(), weights.data_ptr<float>(), h.data_ptr(),
+                   w.data_ptr(), bias ? bias->data_ptr<float>() : nullptr, N, E, K, top,
+                   h.stride(0), cur_stream());
+}
+
+// perm [n], offsets [E + 2]; tiles of EXPERT_TILE rows: at most ceil(n / tile) + E
+static void moe_group(torch::Tensor perm, torch::Tensor offsets, OptTensor tile_expert,
+                      OptTensor tile_row, torch::Tensor ids, int64_t E) {
+  const int64_t n = ids.numel();
+  CHECK_CUDA(ids); CHECK_CONT(ids);
+  TORCH_CHECK(ids.scalar_type() == at::kInt && E > 0 && E <= 512 && n < (1 << 30));
+  const int64_t tiles = tile_expert ? n / EXPERT_TILE + E : 0;
+  int* te = (int*)opt_int(tile_expert, tiles);
+  int* tr = (int*)opt_int(tile_row, tiles);
+  TORCH_CHECK(!te == !tr, "tiles");
+  launch_moe_group((int*)opt_int(perm, n), (int*)opt_int(offsets, E + 2), te, tr,
+                   ids.data_ptr<int>(), (int)n, (int)E, cur_stream());
+}
+
+// One product of the routed experts (experts.h).  kind: 0 fp32, 1 few rows, 2 tiles
+static void experts_linear(torch::Tensor out, torch::Tensor x, torch::Tensor w, torch::Tensor ids,
+                           OptTensor perm, OptTensor offsets, OptTensor tile_expert,
+                           OptTensor tile_row, bool glu, double limit, double alpha,
+                           double offset, double cubic, int64_t kind, int64_t tt) {
+  const auto dt = x.scalar_type();
+  ExpertsArgs a{};
+  CHECK_CUDA(w); CHECK_CONT(w); CHECK_CUDA(ids); CHECK_CONT(ids);
+  TORCH_CHECK(w.dim() == 3 && w.scalar_type() == dt && ids.dim() == 2 &&
+              ids.scalar_type() == at::kInt, "experts");
+  a.entries = ids.numel();
+  a.top = ids.size(1);
+  a.E = w.size(0);
+  a.O = (int)(glu ? w.size(1) / 2 : w.size(1));
+  a.K = w.size(2);
+  check_rows(x, dt, glu ? ids.size(0) : a.entries, a.K); check_aligned(x);
+  check_rows(out, dt, a.entries, a.O); CHECK_CONT(out);
+  TORCH_CHECK(w.size(1) == (glu ? 2 : 1) * (int64_t)a.O && a.K % 64 == 0 &&
+              (!glu || a.O % 64 == 0), "inner sizes must be padded");
+  TORCH_CHECK((kind == 0) == (dt == at::kFloat), "kernels by dtype");
+  a.out = out.data_ptr();
+  a.x = x.data_ptr();
+  a.w = w.data_ptr();
+  a.ids = ids.data_ptr<int>();
+  a.x_stride = x.stride(0);
+  a.limit = (float)limit;
+  a.alpha = (float)alpha;
+  a.offset = (float)offset;
+  a.cubic = (float)cubic;
+  if (a.entries == 0) return;
+  if (kind == 0) {
+    TORCH_CHECK((a.O + 63) / 64 <= 65535, "grid");
+    launch_experts_f32(glu, &a, cur_stream());
+    return;
+  }
+  is_bf16(x);
+  TORCH_CHECK(perm && offsets, "grouped entries");
+  a.perm = opt_int(perm, a.entries);
+  a.offsets = opt_int(offsets, a.E + 2);
+  if (kind == 1) {
+    TORCH_CHECK(tt == 1 || tt == 2 || tt == 4, "token fragments");
+    launch_experts_small(glu, &a, (int)tt, cur_stream());
+    return;
+  }
+  TORCH_CHECK(tile_expert && a.K % 128 == 0, "tiles");
+  a.tiles = a.entries / EXPERT_TILE + a.E;
+  a.tile_expert = opt_int(tile_expert, a.tiles);
+  a.tile_row = opt_int(tile_row, a.tiles);
+  launch_experts_gemm(glu, &a, cur_stream());
 }
 
 static DeltaArgs delta_args(const torch::Tensor& out, const torch::Tensor& qkv,
@@ -893,6 +1103,11 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("softcap", &softcap);
   m.def("cache_keys_values", &cache_keys_values);
   m.def("grouped_attn", &grouped_attn);
+  m.def("attention_inputs", &attention_inputs);
+  m.attr("EXPERT_TILE") = EXPERT_TILE;
+  m.def("moe_route", &moe_route);
+  m.def("moe_group", &moe_group);
+  m.def("experts_linear", &experts_linear);
   m.def("delta_prompts", &delta_prompts);
   m.def("delta_step", &delta_step);
   m.def("sample", &sample);

@@ -1,4 +1,4 @@
-// The two ends of a model with an fp32 residual (gfx950): token embedding plus
+// The two ends of a model with an fp32 residual (gfx950): scaled token embedding plus
 // sinusoidal positions, and capped logits.
 #include "common_t.h"
 
@@ -8,7 +8,8 @@ template <typename T, int V>
 __global__ __launch_bounds__(256) void embed_positions_kernel(
     float* __restrict__ x, float* __restrict__ copy, const int64_t* __restrict__ token_ids,
     const int64_t* __restrict__ positions, const T* __restrict__ table,
-    const float* __restrict__ cos_sin, const int w, const int64_t vocab, const int64_t P) {
+    const float* __restrict__ cos_sin, const float scale, const int w, const int64_t vocab,
+    const int64_t P) {
   const int64_t n = blockIdx.x;
   const int64_t tok = min(max(token_ids[n], (int64_t)0), vocab - 1);
   const int64_t p = min(max(positions[n], (int64_t)0), P - 1);
@@ -16,6 +17,8 @@ __global__ __launch_bounds__(256) void embed_positions_kernel(
   for (int i = (blockIdx.y * 256 + threadIdx.x) * V; i < w; i += gridDim.y * 256 * V) {
     float v[V];
     load_f<V>(v, table + tok * w + i);
+#pragma unroll
+    for (int k = 0; k < V; ++k) v[k] *= scale;
     if (cos_sin) {
 #pragma unroll
       for (int k = 0; k < V; ++k)
@@ -46,16 +49,16 @@ extern "C" {
 
 void launch_embed_positions(bool bf16, float* x, float* copy, const int64_t* token_ids,
                             const int64_t* positions, const void* table, const float* cos_sin,
-                            int n, int w, int64_t vocab, int64_t P, hipStream_t stream) {
+                            float scale, int n, int w, int64_t vocab, int64_t P, hipStream_t stream) {
   const int v = w % 4 == 0 ? 4 : 1;
   const dim3 grid(n, (w / v + 255) / 256);
   if (bf16) {
     auto k = v == 4 ? embed_positions_kernel<bf16_t, 4> : embed_positions_kernel<bf16_t, 1>;
-    k<<<grid, 256, 0, stream>>>(x, copy, token_ids, positions, (const bf16_t*)table, cos_sin, w,
+    k<<<grid, 256, 0, stream>>>(x, copy, token_ids, positions, (const bf16_t*)table, cos_sin, scale, w,
                                 vocab, P);
   } else {
     auto k = v == 4 ? embed_positions_kernel<float, 4> : embed_positions_kernel<float, 1>;
-    k<<<grid, 256, 0, stream>>>(x, copy, token_ids, positions, (const float*)table, cos_sin, w,
+    k<<<grid, 256, 0, stream>>>(x, copy, token_ids, positions, (const float*)table, cos_sin, scale, w,
                                 vocab, P);
   }
 }

@@ -1,17 +1,18 @@
 // Gated activations over row-strided GEMM outputs (gfx950).
 //
 //   clamped_glu: g = min(gate, limit), u = clamp(up, +-limit);
-//                g * sigmoid(alpha g) * (u + offset)
+//                g * sigmoid(alpha (g + cubic g^3)) * (u + offset)
 //   gelu_gate:   gelu_tanh(s) * table[token, offset + i]
 //   side_gate:   x + y, then gelu_gate of (gate x): for few tokens, where two
 //                elementwise launches and a GEMM of one narrow tile cost more than
 //                reading the small weight once per token from L2
 #include "common_t.h"
+#include "gated_act.h"
 
 template <typename T, int V>
 __global__ __launch_bounds__(256) void clamped_glu_kernel(
     T* __restrict__ out, const T* __restrict__ gate_up, const float limit,
-    const float alpha, const float offset, const int rows, const int inter,
+    const float alpha, const float offset, const float cubic, const int rows, const int inter,
     const int64_t in_stride, const int64_t out_stride) {
   const int per_row = inter / V;
   const int64_t total = (int64_t)rows * per_row;
@@ -23,11 +24,7 @@ __global__ __launch_bounds__(256) void clamped_glu_kernel(
     load_f<V>(g, gate_up + r * in_stride + c);
     load_f<V>(u, gate_up + r * in_stride + inter + c);
 #pragma unroll
-    for (int k = 0; k < V; ++k) {
-      const float gc = fminf(g[k], limit);
-      const float uc = fminf(fmaxf(u[k], -limit), limit);
-      g[k] = gc * sigmoid_f(alpha * gc) * (uc + offset);
-    }
+    for (int k = 0; k < V; ++k) g[k] = clamped_glu_f(g[k], u[k], limit, alpha, offset, cubic);
     store_f<V>(out + r * out_stride + c, g);
   }
 }
@@ -103,18 +100,18 @@ __global__ __launch_bounds__(256) void gelu_gate_kernel(
 extern "C" {
 
 void launch_clamped_glu(bool bf16, void* out, const void* gate_up, float limit,
-                        float alpha, float offset, int rows, int inter,
+                        float alpha, float offset, float cubic, int rows, int inter,
                         int64_t in_stride, int64_t out_stride, hipStream_t stream) {
   const int v = bf16 ? 8 : 4;
   const int64_t want = ((int64_t)rows * (inter / v) + 255) / 256;
   const int grid = (int)(want < 4096 ? want : 4096);
   if (bf16)
     clamped_glu_kernel<bf16_t, 8><<<grid, 256, 0, stream>>>(
-        (bf16_t*)out, (const bf16_t*)gate_up, limit, alpha, offset, rows, inter,
+        (bf16_t*)out, (const bf16_t*)gate_up, limit, alpha, offset, cubic, rows, inter,
         in_stride, out_stride);
   else
     clamped_glu_kernel<float, 4><<<grid, 256, 0, stream>>>(
-        (float*)out, (const float*)gate_up, limit, alpha, offset, rows, inter,
+        (float*)out, (const float*)gate_up, limit, alpha, offset, cubic, rows, inter,
         in_stride, out_stride);
 }
 

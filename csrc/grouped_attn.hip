@@ -2,9 +2,10 @@
 // for every other case (gfx950).
 //
 // A query at position p sees the keys p - window + 1 .. p and the first ``keep``
-// ones; scores may be capped and a sink may join the denominator.  The sink is the
-// softmax's starting state (maximum = sink, sum = 1, no value), so that neither the
-// merge of partial sums nor the output knows about it.
+// ones; scores may be capped, get a bias by distance, and a sink may join the
+// denominator.  The sink is the softmax's starting state (maximum = sink, sum = 1, no
+// value), so that neither the merge of partial sums nor the output knows about it.
+// Sigmoid weights need no such state: their partial results are plain sums.
 //
 // Decode: a workgroup owns one (sequence, key/value head) and up to GM of its query
 // heads; its 16 lane groups of 16 take every 16th visible key, a few of them in
@@ -30,7 +31,7 @@ static DEV KeyList visible_keys(int pos, int window, int keep) {
   return k;
 }
 
-template <int KE, int VE, int GM>
+template <int KE, int VE, int GM, bool SIG>
 __global__ __launch_bounds__(256, GM * (KE + VE) <= 32 ? 4 : GM * (KE + VE) <= 64 ? 3 : 2) void grouped_decode_kernel(
     const GroupedArgs a) {
   constexpr int D = 16 * KE, V = 16 * VE;
@@ -45,7 +46,8 @@ __global__ __launch_bounds__(256, GM * (KE + VE) <= 32 ? 4 : GM * (KE + VE) <= 6
   const int j = lane & 15, gid = wid * 4 + (lane >> 4);
   const int64_t row0 = (int64_t)seq * a.H + h0;
 
-  const KeyList keys = visible_keys(a.seq_lens[seq] - 1, a.window, a.keep);
+  const int pos = a.seq_lens[seq] - 1;
+  const KeyList keys = visible_keys(pos, a.window, a.keep);
   const int per_split = (keys.n + a.n_split - 1) / a.n_split;
   const int x0 = min(keys.n, (int)blockIdx.y * per_split), x1 = min(keys.n, x0 + per_split);
   if (x0 >= x1) {  // an empty split; those are a row's last ones
@@ -82,6 +84,12 @@ __global__ __launch_bounds__(256, GM * (KE + VE) <= 32 ? 4 : GM * (KE + VE) <= 6
       slot[u] = (int64_t)table[k / a.kv_block] * a.kv_block + k % a.kv_block;
     }
   };
+  // biases: distances of n_bias - 1 and more share one
+  const int far = a.n_bias - 1;
+  float b_far[GM];
+#pragma unroll
+  for (int g = 0; g < GM; ++g)
+    b_far[g] = a.bias ? a.bias[(h0 + min(g, heads - 1)) * a.n_bias + far] * LOG2E : 0.f;
   find(x0 + gid);
   for (int x = x0 + gid; x < x1; x += 16 * KEYS) {
     Pack<bf16_t, KE> k[KEYS];
@@ -91,10 +99,25 @@ __global__ __launch_bounds__(256, GM * (KE + VE) <= 32 ? 4 : GM * (KE + VE) <= 6
       k[u] = *(const Pack<bf16_t, KE>*)(kc + slot[u] * a.G * D);
       v[u] = *(const Pack<bf16_t, VE>*)(vc + slot[u] * a.G * V);
     }
+    int dist[KEYS];
+    bool near = false;
+#pragma unroll
+    for (int u = 0; u < KEYS; ++u) {
+      dist[u] = pos - keys.at(min(x + 16 * u, x1 - 1));
+      near |= dist[u] < far;
+    }
+    near &= a.bias != nullptr;
     find(x + 16 * KEYS);
 #pragma unroll
     for (int g = 0; g < GM; ++g) {
-      float s[KEYS], mt = m[g];
+      float s[KEYS], b[KEYS], mt = m[g];
+#pragma unroll
+      for (int u = 0; u < KEYS; ++u) b[u] = b_far[g];
+      if (near) {
+        const float* br = a.bias + (int64_t)(h0 + min(g, heads - 1)) * a.n_bias;
+#pragma unroll
+        for (int u = 0; u < KEYS; ++u) b[u] = br[min(dist[u], far)] * LOG2E;
+      }
 #pragma unroll
       for (int u = 0; u < KEYS; ++u) {
         float dot = 0.f;
@@ -103,8 +126,17 @@ __global__ __launch_bounds__(256, GM * (KE + VE) <= 32 ? 4 : GM * (KE + VE) <= 6
         dot = row16_sum(dot) * mul;
         if (a.cap > 0.f)
           dot = c1 - 2.f * c1 * __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(dot) + 1.f);
-        s[u] = x + 16 * u < x1 ? dot : -INFINITY;
+        s[u] = x + 16 * u < x1 ? dot + b[u] : -INFINITY;
         mt = fmaxf(mt, s[u]);
+      }
+      if constexpr (SIG) {
+#pragma unroll
+        for (int u = 0; u < KEYS; ++u) {
+          const float p = __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(-s[u]));
+#pragma unroll
+          for (int e = 0; e < VE; ++e) acc[g][e] += p * to_f(v[u].v[e]);
+        }
+        continue;
       }
       const float alpha = __builtin_amdgcn_exp2f(m[g] - mt);
       m[g] = mt;
@@ -126,7 +158,7 @@ __global__ __launch_bounds__(256, GM * (KE + VE) <= 32 ? 4 : GM * (KE + VE) <= 6
   for (int g = 0; g < GM; ++g) {
     float mx = fmaxf(m[g], __shfl_xor(m[g], 16, 64));
     mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
-    const float w = __builtin_amdgcn_exp2f(m[g] - mx);
+    const float w = SIG ? 1.f : __builtin_amdgcn_exp2f(m[g] - mx);
     float lg = l[g] * w;
     lg += __shfl_xor(lg, 16, 64);
     lg += __shfl_xor(lg, 32, 64);
@@ -147,16 +179,18 @@ __global__ __launch_bounds__(256, GM * (KE + VE) <= 32 ? 4 : GM * (KE + VE) <= 6
     for (int w = 0; w < 4; ++w) mx = fmaxf(mx, lds_ml[w][g].x);
 #pragma unroll
     for (int w = 0; w < 4; ++w) {
-      const float f = __builtin_amdgcn_exp2f(lds_ml[w][g].x - mx);
+      const float f = SIG ? 1.f : __builtin_amdgcn_exp2f(lds_ml[w][g].x - mx);
       sum += f * lds_ml[w][g].y;
       o += f * lds_acc[w][g][e];
     }
     if (a.n_split == 1) {
-      ((bf16_t*)a.out)[(row0 + g) * V + e] = from_f<bf16_t>(o / sum);
+      if (!SIG) o /= sum;
+      if (a.gate) o *= sigmoid_f(bf2f(((const bf16_t*)a.gate)[seq * a.gate_stride + h0 + g]));
+      ((bf16_t*)a.out)[seq * a.out_stride + (int64_t)(h0 + g) * V + e] = from_f<bf16_t>(o);
     } else {
       const int64_t at = (int64_t)blockIdx.y * a.rows + row0 + g;
       a.part[at * V + e] = o;
-      if (e == 0) a.part_ml[at] = float2{mx, sum};
+      if (e == 0) a.part_ml[at] = SIG ? float2{0.f, 1.f} : float2{mx, sum};
     }
   }
 }
@@ -199,6 +233,13 @@ __global__ __launch_bounds__(256) void grouped_plain_kernel(
     }
     dot = wave_sum(dot) * a.scale;
     if (a.cap > 0.f) dot = a.cap * tanhf(dot / a.cap);
+    if (a.bias) dot += a.bias[(int64_t)h * a.n_bias + min(pos - k, a.n_bias - 1)];
+    if (a.sigmoid) {
+      const float p = 1.f / (1.f + expf(-dot));
+#pragma unroll
+      for (int e = 0; e < NE; ++e) acc[e] += p * val[e];
+      continue;
+    }
     const float mn = fmaxf(m, dot);
     const float alpha = expf(m - mn), p = expf(dot - mn);
     m = mn;
@@ -217,14 +258,16 @@ __global__ __launch_bounds__(256) void grouped_plain_kernel(
   for (int i = 0; i < 4; ++i) mx = fmaxf(mx, ml[i].x);
 #pragma unroll
   for (int i = 0; i < 4; ++i) {
-    w[i] = expf(ml[i].x - mx);
+    w[i] = a.sigmoid ? 1.f : expf(ml[i].x - mx);
     sum += w[i] * ml[i].y;
   }
+  float f = a.sigmoid ? 1.f : 1.f / sum;
+  if (a.gate) f *= sigmoid_f(to_f(((const T*)a.gate)[token * a.gate_stride + h]));
   for (int i = threadIdx.x; i < v; i += 256) {
     float o = 0.f;
 #pragma unroll
     for (int n = 0; n < 4; ++n) o += w[n] * part[n][i];
-    ((T*)a.out)[((int64_t)token * a.H + h) * v + i] = from_f<T>(o / sum);
+    ((T*)a.out)[token * a.out_stride + (int64_t)h * v + i] = from_f<T>(o * f);
   }
 }
 
@@ -245,28 +288,34 @@ __global__ __launch_bounds__(256) void cache_keys_values_kernel(
     v_cache[slots[n] * v_units + u - k_units] = v[n * stride + u - k_units];
 }
 
-template <int KE, int VE>
+template <int KE, int VE, bool SIG>
 static void launch_decode(const GroupedArgs& a, int seqs, int gm, hipStream_t stream) {
   if (KE + VE > 16 && gm > 4) gm = 4;
   const int group = a.H / a.G;
   const dim3 grid(seqs * a.G * ((group + gm - 1) / gm), a.n_split);
   if (gm == 1)
-    grouped_decode_kernel<KE, VE, 1><<<grid, 256, 0, stream>>>(a);
+    grouped_decode_kernel<KE, VE, 1, SIG><<<grid, 256, 0, stream>>>(a);
   else if (gm == 2)
-    grouped_decode_kernel<KE, VE, 2><<<grid, 256, 0, stream>>>(a);
+    grouped_decode_kernel<KE, VE, 2, SIG><<<grid, 256, 0, stream>>>(a);
   else if (gm == 4)
-    grouped_decode_kernel<KE, VE, 4><<<grid, 256, 0, stream>>>(a);
+    grouped_decode_kernel<KE, VE, 4, SIG><<<grid, 256, 0, stream>>>(a);
   else if constexpr (KE + VE <= 16)
-    grouped_decode_kernel<KE, VE, 8><<<grid, 256, 0, stream>>>(a);
+    grouped_decode_kernel<KE, VE, 8, SIG><<<grid, 256, 0, stream>>>(a);
+}
+
+template <int KE, int VE>
+static bool launch_decode(const GroupedArgs& a, int seqs, int gm, hipStream_t stream) {
+  (a.sigmoid ? launch_decode<KE, VE, true> : launch_decode<KE, VE, false>)(a, seqs, gm, stream);
+  return true;
 }
 
 template <int KE>
 static bool launch_decode_v(const GroupedArgs& a, int v, int seqs, int gm,
                             hipStream_t stream) {
   switch (v) {
-    case 64: launch_decode<KE, 4>(a, seqs, gm, stream); return true;
-    case 128: launch_decode<KE, 8>(a, seqs, gm, stream); return true;
-    case 256: launch_decode<KE, 16>(a, seqs, gm, stream); return true;
+    case 64: return launch_decode<KE, 4>(a, seqs, gm, stream);
+    case 128: return launch_decode<KE, 8>(a, seqs, gm, stream);
+    case 256: return launch_decode<KE, 16>(a, seqs, gm, stream);
     default: return false;
   }
 }
@@ -295,8 +344,10 @@ bool launch_grouped_decode(const GroupedArgs* a, int d, int v, int seqs, int gm,
     case 128: ok = launch_decode_v<8>(*a, v, seqs, gm, stream); break;
     case 256: ok = launch_decode_v<16>(*a, v, seqs, gm, stream); break;
   }
-  if (ok && a->n_split > 1)
-    launch_split_combine(a->out, a->part, a->part_ml, a->rows, v, a->n_split, stream);
+  if (ok && a->n_split > 1) {
+    const SplitOut out = {a->out, a->gate, a->out_stride, a->gate_stride, a->H, a->sigmoid};
+    launch_split_combine(&out, a->part, a->part_ml, a->rows, v, a->n_split, stream);
+  }
   return ok;
 }
 

@@ -1,5 +1,6 @@
 // Grouped attention of prompt portions over the paged cache on the matrix cores
-// (gfx950): windows that keep the first tokens, capped scores, a sink.
+// (gfx950): windows that keep the first tokens, capped scores, biases by distance, a
+// sink; softmax or sigmoid weights; a gate per head.
 //
 // A workgroup owns 128 query rows of one head, a wave 32 of them.  Keys and values
 // stream through LDS in tiles of 64, double buffered, loaded straight from their pages;
@@ -9,7 +10,9 @@
 //   QK^T (A = keys, B = queries, 32x32x16): a lane owns one query and, per 32
 //     keys, the rows (r & 3) + 8 (r >> 2) + 4 (lane >> 5)
 //   softmax: 32 registers and one exchange between the lane halves; it starts from
-//     the sink (maximum = sink, sum = 1)
+//     the sink (maximum = sink, sum = 1).  Sigmoid weights need neither
+//   biases: beyond the last distance with one of its own they are one number a head;
+//     only tiles nearer than that look them up
 //   PV (A = values^T, B = probabilities): the product's 16 key slots are taken in
 //     the order the scores already have, so the probabilities never leave their lane;
 //     the value fragments are read transposed (ds_read_b64_tr_b16) in that order
@@ -30,9 +33,11 @@ typedef __attribute__((address_space(1))) const char glob_char;
 #define NEG -1e30f
 #define LOG2E 1.44269504088896f
 
-template <int DN, int VN, bool CAP>
+// FORM: 0 softmax, 1 softmax of capped scores, 2 sigmoid
+template <int DN, int VN, int FORM>
 __global__ __launch_bounds__(256, DN + VN <= 4 ? 2 : 1) void grouped_prefill_kernel(
     const GroupedArgs a) {
+  constexpr bool CAP = FORM == 1, SIG = FORM == 2;
   constexpr int D = 64 * DN, V = 64 * VN;
   constexpr int KU = D / 8, VU = V / 8;       // units per LDS row
   constexpr int STEPS = D / 16, VT = V / 32;
@@ -123,6 +128,9 @@ __global__ __launch_bounds__(256, DN + VN <= 4 ? 2 : 1) void grouped_prefill_ker
   const float mul = CAP ? 2.f * LOG2E * a.scale / a.cap : a.scale * LOG2E;
   float m_run = a.sink ? a.sink[head] * LOG2E : NEG;
   float l_run = a.sink && half == 0 ? 1.f : 0.f;
+  const float* bias = a.bias ? a.bias + (int64_t)head * a.n_bias : nullptr;
+  const int far = a.n_bias - 1;
+  const float b_far = bias ? bias[far] * LOG2E : 0.f;
   f32x16_v o[VT] = {};
   const int w_lo = ctx + q0 + wid * 32;                    // wave's positions
   const int w_hi = min(w_lo + 31, k_end - 1);
@@ -152,38 +160,60 @@ __global__ __launch_bounds__(256, DN + VN <= 4 ? 2 : 1) void grouped_prefill_ker
         }
       }
       const bool edge = key0 + KT - 1 > w_lo || w_hi - key0 >= a.window;
-      float mt = NEG;
 #pragma unroll
       for (int b = 0; b < 2; ++b)
 #pragma unroll
         for (int e = 0; e < 16; ++e) {
           float v = s[b][e] * mul;
           if (CAP) v = c1 - 2.f * c1 * __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(v) + 1.f);
-          if (edge) {
-            const int key = key0 + b * 32 + (e & 3) + 8 * (e >> 2) + 4 * half;
-            if (key > qpos || (qpos - key >= a.window && key >= a.keep)) v = -INFINITY;
-          }
-          s[b][e] = v;
-          mt = fmaxf(mt, v);
+          s[b][e] = v + b_far;
         }
-      mt = fmaxf(mt, __shfl_xor(mt, 32, 64));
-      if (__any(mt > m_run)) {
-        const float m_new = fmaxf(m_run, mt);
-        const float alpha = __builtin_amdgcn_exp2f(m_run - m_new);
-        m_run = m_new;
-        l_run *= alpha;
+      if (bias && w_lo - (key0 + KT - 1) < far) {
 #pragma unroll
-        for (int n = 0; n < VT; ++n) o[n] *= alpha;
+        for (int b = 0; b < 2; ++b)
+#pragma unroll
+          for (int e = 0; e < 16; ++e) {
+            const int key = key0 + b * 32 + (e & 3) + 8 * (e >> 2) + 4 * half;
+            s[b][e] += bias[min(max(qpos - key, 0), far)] * LOG2E - b_far;
+          }
       }
-      float sum = 0.f;
+      float mt = NEG;
 #pragma unroll
       for (int b = 0; b < 2; ++b)
 #pragma unroll
         for (int e = 0; e < 16; ++e) {
-          s[b][e] = __builtin_amdgcn_exp2f(s[b][e] - m_run);
-          sum += s[b][e];
+          if (edge) {
+            const int key = key0 + b * 32 + (e & 3) + 8 * (e >> 2) + 4 * half;
+            if (key > qpos || (qpos - key >= a.window && key >= a.keep)) s[b][e] = -INFINITY;
+          }
+          mt = fmaxf(mt, s[b][e]);
         }
-      l_run += sum;
+      if constexpr (SIG) {
+#pragma unroll
+        for (int b = 0; b < 2; ++b)
+#pragma unroll
+          for (int e = 0; e < 16; ++e)
+            s[b][e] = __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(-s[b][e]));
+      } else {
+        mt = fmaxf(mt, __shfl_xor(mt, 32, 64));
+        if (__any(mt > m_run)) {
+          const float m_new = fmaxf(m_run, mt);
+          const float alpha = __builtin_amdgcn_exp2f(m_run - m_new);
+          m_run = m_new;
+          l_run *= alpha;
+#pragma unroll
+          for (int n = 0; n < VT; ++n) o[n] *= alpha;
+        }
+        float sum = 0.f;
+#pragma unroll
+        for (int b = 0; b < 2; ++b)
+#pragma unroll
+          for (int e = 0; e < 16; ++e) {
+            s[b][e] = __builtin_amdgcn_exp2f(s[b][e] - m_run);
+            sum += s[b][e];
+          }
+        l_run += sum;
+      }
 
       const char* vt = kt + K_BYTES;
 #pragma unroll
@@ -212,8 +242,9 @@ __global__ __launch_bounds__(256, DN + VN <= 4 ? 2 : 1) void grouped_prefill_ker
 
   l_run += __shfl_xor(l_run, 32, 64);
   if (!live) return;
-  const float inv = l_run > 0.f ? 1.f / l_run : 0.f;
-  bf16_t* dst = (bf16_t*)a.out + ((row0 + r) * a.H + head) * V + 4 * half;
+  float inv = SIG ? 1.f : l_run > 0.f ? 1.f / l_run : 0.f;
+  if (a.gate) inv *= sigmoid_f(bf2f(((const bf16_t*)a.gate)[(row0 + r) * a.gate_stride + head]));
+  bf16_t* dst = (bf16_t*)a.out + (row0 + r) * a.out_stride + (int64_t)head * V + 4 * half;
 #pragma unroll
   for (int t = 0; t < VT; ++t)
 #pragma unroll
@@ -224,31 +255,34 @@ __global__ __launch_bounds__(256, DN + VN <= 4 ? 2 : 1) void grouped_prefill_ker
     }
 }
 
-template <int DN, int VN, bool CAP>
+template <int DN, int VN, int FORM>
 static void launch(const GroupedArgs& a, hipStream_t stream) {
   constexpr int bytes = 2 * KT * (64 * DN + 64 * VN) * 2 + 2 * KT * 4;
   static_assert(bytes <= 160 * 1024, "LDS");
   static bool attr_set = false;
   if (!attr_set) {
-    (void)hipFuncSetAttribute((const void*)grouped_prefill_kernel<DN, VN, CAP>,
+    (void)hipFuncSetAttribute((const void*)grouped_prefill_kernel<DN, VN, FORM>,
                               hipFuncAttributeMaxDynamicSharedMemorySize, bytes);
     attr_set = true;
   }
-  grouped_prefill_kernel<DN, VN, CAP><<<a.n_tiles * a.H, 256, bytes, stream>>>(a);
+  grouped_prefill_kernel<DN, VN, FORM><<<a.n_tiles * a.H, 256, bytes, stream>>>(a);
 }
 
 template <int DN, int VN>
-static bool launch_cap(const GroupedArgs& a, hipStream_t stream) {
-  a.cap > 0.f ? launch<DN, VN, true>(a, stream) : launch<DN, VN, false>(a, stream);
+static bool launch_form(const GroupedArgs& a, hipStream_t stream) {
+  if (a.sigmoid && a.cap > 0.f) return false;
+  (a.sigmoid       ? launch<DN, VN, 2>
+   : a.cap > 0.f   ? launch<DN, VN, 1>
+                   : launch<DN, VN, 0>)(a, stream);
   return true;
 }
 
 template <int DN>
 static bool launch_v(const GroupedArgs& a, int v, hipStream_t stream) {
   switch (v) {
-    case 64: return launch_cap<DN, 1>(a, stream);
-    case 128: return launch_cap<DN, 2>(a, stream);
-    case 256: return launch_cap<DN, 4>(a, stream);
+    case 64: return launch_form<DN, 1>(a, stream);
+    case 128: return launch_form<DN, 2>(a, stream);
+    case 256: return launch_form<DN, 4>(a, stream);
     default: return false;
   }
 }

@@ -11,6 +11,7 @@ struct LatentArgs {
   const void* q_rot;      // [tokens, H, rot] not yet rotated, strides below
   const float* cos_sin;   // [2, positions, rot_dim / 2]
   const void* cache;      // [slots, row]
+  const float* sink;      // [H] or null
   const int* tables;      // [seqs, max_blocks]
   const int* seq_lens;    // [seqs] cached tokens, this step's included
   const int* ctx_lens;    // [seqs] before this step; null: seq_len - 1 (decode)
@@ -29,6 +30,7 @@ struct LatentPrefillArgs {
   const void* kv;         // [keys, H * d | H * v], rows kv_stride apart
   const void* k_rot;      // [keys, rot], rows rot_stride apart
   const void* gate;       // [tokens, H], rows gate_stride apart, or null
+  const float* sink;      // [H] or null
   const float* cos_sin;   // [2, positions, rot_dim / 2]
   const int *seq_lens, *ctx_lens, *row_starts, *tile_seq, *tile_q0;
   const int* key_first;   // [seqs] position of a sequence's first key row
@@ -38,8 +40,18 @@ struct LatentPrefillArgs {
   float scale;
 };
 
-// out [rows, width] bf16 from n_split (at most 64) partial sums [n_split, rows, width]
+// Where merged rows go: row r is head r % H of token r / H.
+struct SplitOut {
+  void* out;              // bf16, tokens out_stride apart
+  const void* gate;       // [tokens, H] bf16 before its sigmoid, or null
+  int64_t out_stride, gate_stride;
+  int H;
+  bool sum;               // partial results are summed as they are, no softmax
+};
+
+// bf16 rows of ``width`` from n_split (at most 64) partial sums [n_split, rows, width]
 // with their (maximum in the exp2 domain, sum) [n_split, rows]; an empty split has sum
 // -1 and is one of a row's last
-extern "C" void launch_split_combine(void* out, const float* part, const float2* part_ml,
-                                     int rows, int width, int n_split, hipStream_t stream);
+extern "C" void launch_split_combine(const SplitOut* out, const float* part,
+                                     const float2* part_ml, int rows, int width, int n_split,
+                                     hipStream_t stream);

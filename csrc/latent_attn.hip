@@ -157,11 +157,13 @@ __global__ __launch_bounds__(256) void latent_attn_kernel(const LatentArgs a) {
   stage(t_begin);
 
   f32x4_v o[MG][NR] = {};
+  // a sink is the softmax's starting state: its maximum, one term of the sum, no value
+  const bool sink = a.sink && blockIdx.y == 0;
   float m_run[MG], l_run[MG];
 #pragma unroll
   for (int m = 0; m < MG; ++m) {
-    m_run[m] = NEG;
-    l_run[m] = 0.f;
+    m_run[m] = sink ? a.sink[(tl.r0 + m * 16 + c) % a.H] * 1.44269504088896f : NEG;
+    l_run[m] = sink && wid == 0 && g == 0 ? 1.f : 0.f;
   }
   const float scale2 = a.scale * 1.44269504088896f;  // exp2 domain
   const int sw_c = ((c & 3) << 1) | ((c >> 2) & 1);
@@ -284,9 +286,8 @@ __global__ __launch_bounds__(256) void latent_attn_kernel(const LatentArgs a) {
 
 // Merge the splits (at most 64) of one row.
 __global__ __launch_bounds__(128) void split_combine_kernel(
-    bf16_t* __restrict__ out, const float* __restrict__ part,
-    const float2* __restrict__ part_ml, const int rows, const int rank,
-    const int n_split) {
+    const SplitOut dst, const float* __restrict__ part, const float2* __restrict__ part_ml,
+    const int rows, const int rank, const int n_split) {
   __shared__ float weight[64];
   const int row = blockIdx.x, lane = threadIdx.x & 63;
   const float2 ml = lane < n_split ? part_ml[(int64_t)lane * rows + row] : float2{NEG, -1.f};
@@ -294,7 +295,11 @@ __global__ __launch_bounds__(128) void split_combine_kernel(
   const float m = wave_max(ml.x);
   const float w = ml.y > 0.f ? __builtin_amdgcn_exp2f(ml.x - m) : 0.f;
   const float l = wave_sum(w * fmaxf(ml.y, 0.f));
-  if (threadIdx.x < 64) weight[lane] = l > 0.f ? w / l : 0.f;
+  const int token = row / dst.H, head = row % dst.H;
+  const float gate =
+      dst.gate ? sigmoid_f(bf2f(((const bf16_t*)dst.gate)[token * dst.gate_stride + head])) : 1.f;
+  if (threadIdx.x < 64) weight[lane] = dst.sum ? gate : l > 0.f ? gate * w / l : 0.f;
+  bf16_t* out = (bf16_t*)dst.out + token * dst.out_stride + (int64_t)head * rank;
   __syncthreads();
   for (int i = threadIdx.x * 4; i < rank; i += 512) {
     float acc[4] = {};
@@ -306,7 +311,7 @@ __global__ __launch_bounds__(128) void split_combine_kernel(
 #pragma unroll
       for (int k = 0; k < 4; ++k) acc[k] += weight[s] * v[k];
     }
-    store_f<4>(out + (int64_t)row * rank + i, acc);
+    store_f<4>(out + i, acc);
   }
 }
 
@@ -338,7 +343,8 @@ __global__ __launch_bounds__(256) void latent_attn_plain_kernel(
       q[e] = (d & 1 ? v * co + u * si : u * co - v * si) * a.scale;
     }
   }
-  float m = NEG, l = 0.f;
+  const bool sink = a.sink && wid == 0;
+  float m = sink ? a.sink[qrow % a.H] : NEG, l = sink ? 1.f : 0.f;
   for (int k = max(0, pos - a.window + 1) + wid; k <= pos; k += 4) {
     const int64_t slot = (int64_t)table[k / a.kv_block] * a.kv_block + k % a.kv_block;
     const T* kr = (const T*)a.cache + slot * row;
@@ -419,10 +425,9 @@ static bool launch_plain(const LatentArgs& a, int rank, int row, int tiles,
 
 extern "C" {
 
-void launch_split_combine(void* out, const float* part, const float2* part_ml, int rows,
-                          int width, int n_split, hipStream_t stream) {
-  split_combine_kernel<<<rows, 128, 0, stream>>>((bf16_t*)out, part, part_ml, rows, width,
-                                                  n_split);
+void launch_split_combine(const SplitOut* out, const float* part, const float2* part_ml,
+                          int rows, int width, int n_split, hipStream_t stream) {
+  split_combine_kernel<<<rows, 128, 0, stream>>>(*out, part, part_ml, rows, width, n_split);
 }
 
 bool launch_latent_attn(bool bf16, bool mfma, const LatentArgs* a, int rank, int row,
@@ -437,8 +442,10 @@ bool launch_latent_attn(bool bf16, bool mfma, const LatentArgs* a, int rank, int
     case 512: launch_mg<8>(*a, mg, tiles, stream); break;
     default: return false;
   }
-  if (a->n_split > 1)
-    launch_split_combine(a->out, a->part, a->part_ml, a->rows, rank, a->n_split, stream);
+  if (a->n_split > 1) {
+    const SplitOut out = {a->out, nullptr, (int64_t)a->H * rank, 0, a->H, false};
+    launch_split_combine(&out, a->part, a->part_ml, a->rows, rank, a->n_split, stream);
+  }
   return true;
 }
 

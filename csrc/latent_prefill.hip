@@ -128,7 +128,9 @@ __global__ __launch_bounds__(256, DN + VN <= 4 ? 2 : 1) void latent_prefill_kern
   }
 
   const float scale2 = a.scale * 1.44269504088896f;
-  float m_run = NEG, l_run = 0.f;
+  // a sink is the softmax's starting state: its maximum, one term of the sum, no value
+  float m_run = a.sink ? a.sink[head] * 1.44269504088896f : NEG;
+  float l_run = a.sink && half == 0 ? 1.f : 0.f;
   f32x16_v o[VT] = {};
   const int w_lo = ctx + q0 + wid * 32;                    // wave's positions
   const int w_hi = min(w_lo + 31, ctx + q0 + rows - 1);

@@ -9,6 +9,14 @@ struct NormForm {
   bool center;              // layer norm of x, else RMS norm
   float offset;             // added to both norm weights
   float mult;               // on what is added to x
+  // sum_j weights[n, j] * rows[n, j] joins y
+  int top;                  // 0 = none
+  const void* rows;         // [n, top, w]
+  const float* weights;     // [n, top]
+  // the same norm of x under another weight
+  const void* x_norm2;      // [w]
+  void* out2;               // rows out2_stride apart, or null
+  int64_t out2_stride;
   // depth average: x becomes state n_states - 1 and then sum_j coef[j] * state_j
   int n_states;             // 0 = none
   int first;                // states before it are in partial[ready]; 0: none are

@@ -3,7 +3,9 @@
 // residual_norm is one pass over a row: optionally add mult * y, or mult *
 // rmsnorm(y) * w_y, to the residual, optionally file the result as the newest depth
 // state and replace it by a weighted sum of all states, then emit norm(x) * w_x (layer
-// or RMS norm) or x itself for the next GEMM.  The row lives in LDS between the reductions (each thread re-reads only what
+// or RMS norm) or x itself for the next GEMM.  What is added may include a weighted sum
+// of several rows (chosen experts' results); the norm may be written a second time under
+// another weight.  The row lives in LDS between the reductions (each thread re-reads only what
 // it wrote, so the row itself needs no barrier).  Mean first, then the squared
 // deviations: no cancellation.
 #include "common_t.h"
@@ -98,6 +100,15 @@ __global__ __launch_bounds__(1024) void residual_norm_kernel(
         for (int k = 0; k < V; ++k) d[k] = (f.offset + d[k]) * row[i + k] * y_scale;
       } else {
         load_f<V>(d, y + (int64_t)blockIdx.x * w + i);
+        const T* er = (const T*)f.rows + (int64_t)blockIdx.x * f.top * w + i;
+        const float* ew = f.weights + (int64_t)blockIdx.x * f.top;
+#pragma unroll 4
+        for (int j = 0; j < f.top; ++j) {
+          float e[V];
+          load_f<V>(e, er + (int64_t)j * w);
+#pragma unroll
+          for (int k = 0; k < V; ++k) d[k] += ew[j] * e[k];
+        }
       }
 #pragma unroll
       for (int k = 0; k < V; ++k) t[k] += f.mult * d[k];
@@ -124,10 +135,18 @@ __global__ __launch_bounds__(1024) void residual_norm_kernel(
       }
     inv = rsqrtf(block_sum(ss, scratch[2]) / w + eps);
   }
+  T* orow2 = f.out2 ? (T*)f.out2 + (int64_t)blockIdx.x * f.out2_stride : nullptr;
   for (int i = i0; i < w; i += step) {
     float t[V];
 #pragma unroll
     for (int k = 0; k < V; ++k) t[k] = (row[i + k] - mean) * inv;
+    if (orow2) {
+      float g[V];
+      load_f<V>(g, (const T*)f.x_norm2 + i);
+#pragma unroll
+      for (int k = 0; k < V; ++k) g[k] = (f.offset + g[k]) * t[k];
+      store_f<V>(orow2 + i, g);
+    }
     if (x_norm) {
       float g[V];
       load_f<V>(g, x_norm + i);
@@ -159,7 +178,7 @@ static void residual_norm_t(float* x, const void* y, const void* y_norm,
                             const void* x_norm, void* out, float eps, int n,
                             int w, int64_t out_stride, const NormForm& f,
                             hipStream_t stream) {
-  const bool vec = w % 4 == 0 && out_stride % 4 == 0;
+  const bool vec = w % 4 == 0 && out_stride % 4 == 0 && f.out2_stride % 4 == 0;
   int threads = w >= 1024 ? 256 : w >= 512 ? 128 : 64;
   // few rows: the latency of one counts
   while (n <= 512 && threads < 1024 && threads * 4 < w) threads *= 2;
