@@ -356,6 +356,37 @@ def _tezinex(name: str, *, width: int, layers: int, ff: int, heads: int, kv_head
     )
 
 
+def _lobuvik(name: str, *, width: int, layers: int, heads: int, kv_heads: int, dim: int,
+             vdim: int, conv: int, bias: DistanceBias, kv_rank: int, rot_dim: int, window: int,
+             ff: int, experts: ExpertsSpec, vocab: int, **kw) -> ModelConfig:
+    """Biased, latent and rotated attention in turn; a dense feed-forward in the first
+    layer, experts in the others."""
+    biased = GroupedAttentionSpec(
+        heads=heads, kv_heads=kv_heads, dim=dim, vdim=vdim, scale=dim ** -0.5, bias=True,
+        out_bias=True, sink=False, sigmoid=True, conv=conv, qk_norm=True, v_norm=True,
+        distance_bias=bias, q_temp=QueryTemperature(0.1, 8192),
+    )
+    latent = LatentAttentionSpec(
+        heads=heads, dim=dim, rot_dim=rot_dim, vdim=vdim, kv_rank=kv_rank,
+        scale=(dim + rot_dim) ** -0.5, rope_base=1e6, rope_half=True,
+        rope_scaling=YarnScaling(8.0, 4096, 32.0, 1.0), window=window, head_gate=False, sink=True,
+    )
+    rotated = GroupedAttentionSpec(
+        heads=heads, kv_heads=kv_heads, dim=dim, vdim=vdim, scale=dim ** -0.5, softcap=50.0,
+        window=window, bias=False, sink=False, head_temp=True, head_gate=True,
+        rotary=RotarySpec(5e5, dim // 2, WavelengthScaling(8.0, 1.0, 4.0, 8192)),
+    )
+    mixers = (biased, latent, rotated)
+    return ModelConfig(
+        name=name, architecture="Lobuvik", vocab_size=vocab, hidden_size=width,
+        intermediate_size=ff, num_layers=layers, num_heads=heads, num_kv_heads=kv_heads,
+        head_dim=dim, layers=tuple(
+            LayerSpec(mixers[i % 3], gelu_glu(ff) if i == 0 else experts, mlp_norm=True)
+            for i in range(layers)
+        ), **kw,
+    )
+
+
 PRESETS = {
     "llama3-8b": ModelConfig(),
     # Llama-2 family: same architecture, smaller rope base / context / vocab
@@ -432,6 +463,27 @@ PRESETS = {
         "tiny-tezinex", width=44, layers=6, ff=60, heads=6, kv_heads=3, dim=10, vdim=14,
         window=21, keep_first=3, d_heads=4, d_kv_heads=2, d_dim=12, d_vdim=18, rank=7,
         vocab=300, conv=3, attn_every=2, max_position=4096, dtype="float32",
+    ),
+    # Lobuvik with the layer sizes of an 8B-class dense model per token (random weights):
+    # width, heads and active feed-forward of llama3-8b
+    "lobuvik-8b": _lobuvik(
+        "lobuvik-8b", width=4096, layers=30, heads=32, kv_heads=8, dim=128, vdim=128, conv=4,
+        bias=DistanceBias(64, 512), kv_rank=512, rot_dim=64, window=4096, ff=14336,
+        experts=ExpertsSpec(32, 4, ClampedGluSpec(2560, 7.0), ClampedGluSpec(4096, 7.0)),
+        vocab=128256,
+    ),
+    # half the width, 16 heads
+    "lobuvik-2b": _lobuvik(
+        "lobuvik-2b", width=2048, layers=18, heads=16, kv_heads=8, dim=128, vdim=128, conv=4,
+        bias=DistanceBias(32, 256), kv_rank=512, rot_dim=64, window=1024, ff=8192,
+        experts=ExpertsSpec(16, 4, ClampedGluSpec(1536, 7.0), ClampedGluSpec(2048, 7.0)),
+        vocab=32000,
+    ),
+    "tiny-lobuvik": _lobuvik(
+        "tiny-lobuvik", width=44, layers=4, heads=6, kv_heads=3, dim=12, vdim=10, conv=3,
+        bias=DistanceBias(12, 50), kv_rank=20, rot_dim=6, window=23, ff=52,
+        experts=ExpertsSpec(5, 2, ClampedGluSpec(18, 1.5), ClampedGluSpec(22, 2.0)),
+        vocab=300, max_position=4096, dtype="float32",
     ),
     # tiny GPU config: real head_dim/GQA shape for the CDNA4 kernels at
     # test scale (kernels require head_dim 128)
