@@ -396,8 +396,9 @@ def moe_route(h, router, bias, top: int):
     return ids, weights
 
 
-#: rows per expert from which the tiled product is used
-_TILED_ROWS = 64
+#: average rows per expert from which the tiled product is faster (its weights are read
+#: once, however many rows there are)
+_TILED_ROWS = 12
 
 
 def moe_experts(h, gate_up, down, ids, glu):
@@ -410,7 +411,7 @@ def moe_experts(h, gate_up, down, ids, glu):
     kind, tt = 0, 1
     if h.dtype == torch.bfloat16:
         tiled = n >= _TILED_ROWS * E and gate_up.shape[2] % 128 == 0 and inner % 128 == 0
-        kind, tt = (2, 1) if tiled else (1, 1 if n <= 8 * E else 2 if n <= 32 * E else 4)
+        kind, tt = (2, 1) if tiled else (1, 1 if n <= 8 * E else 2)
         perm = torch.empty(n, dtype=torch.int32, device=device)
         offsets = torch.empty(E + 2, dtype=torch.int32, device=device)
         if tiled:

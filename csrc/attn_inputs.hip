@@ -14,51 +14,58 @@
 #include "common_t.h"
 #include "attn_inputs.h"
 
-// input of VW channels ``ago`` tokens before row n, or zeros
+// input of VW channels ``ago`` > back tokens before row n: from the ring, or zeros
 template <typename T, int VW>
-DEV Pack<T, VW> conv_input(const AttnInputsArgs& a, int64_t n, int64_t p, int back, int64_t state,
-                           int ago, int c) {
-  const T* src = (const T*)a.proj + n * a.stride + c;
-  bool have = true;
-  if (ago <= back) {
-    src -= ago * a.stride;
+DEV Pack<T, VW> ring_input(const AttnInputsArgs& a, int p, int64_t state, int ago, int c) {
+  Pack<T, VW> x;
+  if (ago <= p) {
+    x = *(const Pack<T, VW>*)((const T*)a.ring + (state * a.taps + (p - ago) % a.taps) * a.C + c);
   } else {
-    have = ago <= p;
-    const int64_t entry = have ? (p - ago) % a.taps : 0;
-    if (have) src = (const T*)a.ring + (state * a.taps + entry) * a.C + c;
-  }
-  Pack<T, VW> x = *(const Pack<T, VW>*)src;
-  if (!have)
 #pragma unroll
     for (int k = 0; k < VW; ++k) x.v[k] = from_f<T>(0.f);
+  }
   return x;
 }
 
-// TAPS: 0 none, 4 unrolled, -1 any number
-template <typename T, int VW, int TAPS>
-DEV void channels(const AttnInputsArgs& a, int64_t n, int64_t p, int back, int64_t state, int c,
+template <typename T, int VW>
+DEV Pack<T, VW> row_input(const AttnInputsArgs& a, int64_t n, int c) {
+  return *(const Pack<T, VW>*)((const T*)a.proj + n * a.stride + c);
+}
+
+template <typename T, int VW>
+DEV void add_tap(float* y, const Pack<T, VW>& f, const Pack<T, VW>& x) {
+#pragma unroll
+  for (int k = 0; k < VW; ++k) y[k] += to_f(f.v[k]) * to_f(x.v[k]);
+}
+
+// VW channels of row n, convolved if there is a convolution
+template <typename T, int VW>
+DEV void channels(const AttnInputsArgs& a, int64_t n, int p, int back, int64_t state, int c,
                   float* y) {
-  if constexpr (TAPS == 0) {
+  if (!a.conv) {
     load_f<VW>(y, (const T*)a.proj + n * a.stride + c);
-  } else {
-    const int taps = TAPS > 0 ? TAPS : a.taps;
-    const T* w = (const T*)a.conv + c;
-#pragma unroll
-    for (int k = 0; k < VW; ++k) y[k] = 0.f;
-#pragma unroll(TAPS > 0 ? TAPS : 1)
-    for (int j = 0; j < taps; ++j) {
-      const Pack<T, VW> x = conv_input<T, VW>(a, n, p, back, state, taps - 1 - j, c);
-      const Pack<T, VW> f = *(const Pack<T, VW>*)(w + (int64_t)j * a.C);
-#pragma unroll
-      for (int k = 0; k < VW; ++k) y[k] += to_f(f.v[k]) * to_f(x.v[k]);
-    }
+    return;
   }
+  const T* w = (const T*)a.conv + c;
+#pragma unroll
+  for (int k = 0; k < VW; ++k) y[k] = 0.f;
+  for (int j = 0; j < a.taps; ++j) {
+    const int ago = a.taps - 1 - j;
+    add_tap<T, VW>(y, *(const Pack<T, VW>*)(w + (int64_t)j * a.C),
+                   ago <= back ? row_input<T, VW>(a, n - ago, c)
+                               : ring_input<T, VW>(a, p, state, ago, c));
+  }
+}
+
+template <typename T, int VW>
+DEV void to_ring(const AttnInputsArgs& a, int64_t n, int p, int64_t state, int c) {
+  *(Pack<T, VW>*)((T*)a.ring + (state * a.taps + p % a.taps) * a.C + c) = row_input<T, VW>(a, n, c);
 }
 
 // y: VW channels from i of a head whose squares sum to ss; sect 0 q, 1 k, 2 v
 template <typename T, int VW>
-DEV void finish(const AttnInputsArgs& a, int64_t n, int64_t p, int sect, int head, int i,
-                float ss, float* y) {
+DEV void finish(const AttnInputsArgs& a, int64_t n, int p, int sect, int head, int i, float ss,
+                float* y) {
   if (sect < 2 ? a.q_norm != nullptr : a.v_norm) {
     const float inv = rsqrtf(ss / (sect < 2 ? a.dim : a.vdim) + a.eps);
 #pragma unroll
@@ -71,7 +78,7 @@ DEV void finish(const AttnInputsArgs& a, int64_t n, int64_t p, int sect, int hea
     }
   }
   if (a.cos_sin && sect < 2) {
-    const float* ct = a.cos_sin + p * a.pairs;
+    const float* ct = a.cos_sin + (int64_t)p * a.pairs;
     const float* st = ct + a.P * a.pairs;
 #pragma unroll
     for (int k = 0; k < VW; k += 2) {
@@ -96,15 +103,14 @@ DEV void finish(const AttnInputsArgs& a, int64_t n, int64_t p, int sect, int hea
   }
 }
 
-// Head sizes of at most 64 threads, a power of two.  grid (units / 256, rows): a row has
-// ``units`` threads, a multiple of 64.
-template <typename T, int VW, int TAPS>
-__global__ __launch_bounds__(256) void attn_inputs_kernel(const AttnInputsArgs a, const int units,
-                                                          const int64_t total) {
-  const int64_t id = (int64_t)blockIdx.x * 256 + threadIdx.x;
-  if (id >= total) return;
-  const int64_t n = id / units;
-  int u = (int)(id - n * units);
+// Head sizes of at most 64 threads, a power of two.  grid (threads of a row / 256, rows / R):
+// a row has ``units`` threads, a multiple of 64; a thread does R rows in turn.  TAPS: 0 none,
+// 4: its rows' inputs are loaded once, -1 any number.
+template <typename T, int VW, int TAPS, int R>
+__global__ __launch_bounds__(256) void attn_inputs_kernel(const AttnInputsArgs a, const int units) {
+  int u = blockIdx.x * 256 + threadIdx.x;
+  if (u >= units) return;
+  const int64_t n0 = (int64_t)blockIdx.y * R;
   const int lq = a.d / VW, lv = a.v / VW;
   const int k_at = a.H * lq, v_at = ((a.H + a.G) * lq + lv - 1) / lv * lv;
   int sect = 0, c0 = 0, lanes = lq;
@@ -122,23 +128,62 @@ __global__ __launch_bounds__(256) void attn_inputs_kernel(const AttnInputsArgs a
     live = u < a.G * lq;
   }
   if (!live) u = 0;
-  const int64_t p = a.positions[n];
-  const int back = a.back ? a.back[n] : 0;
-  const int64_t state = TAPS ? a.states[n] : 0;
-  float y[VW];
-  channels<T, VW, TAPS>(a, n, p, back, state, c0 + u * VW, y);
-  if (TAPS && a.write_ring && live)
-    *(Pack<T, VW>*)((T*)a.ring + (state * a.taps + p % a.taps) * a.C + c0 + u * VW) =
-        *(const Pack<T, VW>*)((const T*)a.proj + n * a.stride + c0 + u * VW);
-  float ss = 0.f;
+  const int c = c0 + u * VW, head = u >> (31 - __clz(lanes)), i = (u & (lanes - 1)) * VW;
+
+  constexpr int W = TAPS > 0 ? TAPS : 1;
+  Pack<T, VW> x[R + W - 1], f[W];
+  if constexpr (TAPS >= 0) {  // row n0 + r and the W - 1 before it are x[r .. r + W - 1]
 #pragma unroll
-  for (int k = 0; k < VW; ++k) ss += y[k] * y[k];
-#pragma unroll
-  for (int off = 1; off < 64; off <<= 1) {
-    const float t = __shfl_xor(ss, off, 64);
-    if (off < lanes) ss += t;
+    for (int r = 0; r < R + W - 1; ++r) {
+      const int64_t n = n0 - (W - 1) + r;
+      x[r] = row_input<T, VW>(a, min(max(n, (int64_t)0), (int64_t)a.N - 1), c);
+    }
   }
-  if (live) finish<T, VW>(a, n, p, sect, u / lanes, u % lanes * VW, ss, y);
+  if constexpr (TAPS > 0) {
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j)
+      f[j] = *(const Pack<T, VW>*)((const T*)a.conv + (int64_t)j * a.C + c);
+  }
+#pragma unroll
+  for (int r = 0; r < R; ++r) {
+    const int64_t n = n0 + r;
+    if (n >= a.N) return;
+    const int p = (int)a.positions[n];
+    const int back = TAPS && a.back ? a.back[n] : 0;
+    const int64_t state = TAPS ? a.states[n] : 0;
+    float y[VW];
+    if constexpr (TAPS < 0) {
+      channels<T, VW>(a, n, p, back, state, c, y);
+    } else if constexpr (TAPS == 0) {
+#pragma unroll
+      for (int k = 0; k < VW; ++k) y[k] = to_f(x[r].v[k]);
+    } else {
+#pragma unroll
+      for (int k = 0; k < VW; ++k) y[k] = 0.f;
+      if (back >= TAPS - 1) {
+#pragma unroll
+        for (int j = 0; j < TAPS; ++j) add_tap<T, VW>(y, f[j], x[r + j]);
+      } else {  // some inputs are from earlier steps
+#pragma unroll
+        for (int j = 0; j < TAPS; ++j) {
+          const int ago = TAPS - 1 - j;
+          add_tap<T, VW>(y, f[j], ago <= back ? x[r + j] : ring_input<T, VW>(a, p, state, ago, c));
+        }
+      }
+    }
+    if (TAPS && a.write_ring && live) to_ring<T, VW>(a, n, p, state, c);
+    float ss = 0.f;
+    if (a.q_norm || a.v_norm) {
+#pragma unroll
+      for (int k = 0; k < VW; ++k) ss += y[k] * y[k];
+#pragma unroll
+      for (int off = 1; off < 64; off <<= 1) {
+        const float t = __shfl_xor(ss, off, 64);
+        if (off < lanes) ss += t;
+      }
+    }
+    if (live) finish<T, VW>(a, n, p, sect, head, i, ss, y);
+  }
 }
 
 // Any head size (a multiple of VW): a wave per row and head.
@@ -158,27 +203,19 @@ __global__ __launch_bounds__(256) void attn_inputs_any_kernel(const AttnInputsAr
     head -= a.H;
     sect = 1;
   }
-  const int64_t p = a.positions[n];
+  const int p = (int)a.positions[n];
   const int back = a.back ? a.back[n] : 0;
   const int64_t state = a.conv ? a.states[n] : 0;
-  auto get = [&](int i, float* y) {
-    if (a.conv)
-      channels<T, VW, -1>(a, n, p, back, state, c0 + i, y);
-    else
-      channels<T, VW, 0>(a, n, p, back, state, c0 + i, y);
-  };
   float ss = 0.f, y[VW];
   for (int i = lane * VW; i < size; i += 64 * VW) {
-    get(i, y);
+    channels<T, VW>(a, n, p, back, state, c0 + i, y);
 #pragma unroll
     for (int k = 0; k < VW; ++k) ss += y[k] * y[k];
   }
   ss = wave_sum(ss);
   for (int i = lane * VW; i < size; i += 64 * VW) {
-    get(i, y);
-    if (a.conv && a.write_ring)
-      *(Pack<T, VW>*)((T*)a.ring + (state * a.taps + p % a.taps) * a.C + c0 + i) =
-          *(const Pack<T, VW>*)((const T*)a.proj + n * a.stride + c0 + i);
+    channels<T, VW>(a, n, p, back, state, c0 + i, y);
+    if (a.conv && a.write_ring) to_ring<T, VW>(a, n, p, state, c0 + i);
     finish<T, VW>(a, n, p, sect, head, i, ss, y);
   }
 }
@@ -189,8 +226,15 @@ __global__ __launch_bounds__(256) void attn_ring_kernel(const AttnInputsArgs a) 
   const int c = (blockIdx.x * 256 + threadIdx.x) * VW;
   if (c >= a.C) return;
   const int64_t n = a.ring_rows[blockIdx.y];
-  *(Pack<T, VW>*)((T*)a.ring + (a.states[n] * (int64_t)a.taps + a.positions[n] % a.taps) * a.C + c) =
-      *(const Pack<T, VW>*)((const T*)a.proj + n * a.stride + c);
+  to_ring<T, VW>(a, n, (int)a.positions[n], a.states[n], c);
+}
+
+template <typename T, int VW, int R>
+static void launch_rows(const AttnInputsArgs& a, int units, hipStream_t stream) {
+  auto k = !a.conv       ? attn_inputs_kernel<T, VW, 0, R>
+           : a.taps == 4 ? attn_inputs_kernel<T, VW, 4, R>
+                         : attn_inputs_kernel<T, VW, -1, R>;
+  k<<<dim3((units + 255) / 256, (a.N + R - 1) / R), 256, 0, stream>>>(a, units);
 }
 
 template <typename T, int VW>
@@ -200,11 +244,10 @@ static void launch(const AttnInputsArgs& a, hipStream_t stream) {
   if (fits(lq) && fits(lv)) {
     const int v_at = ((a.H + a.G) * lq + lv - 1) / lv * lv;
     const int units = (v_at + a.G * lv + 63) / 64 * 64;
-    const int64_t total = (int64_t)a.N * units;
-    auto k = !a.conv         ? attn_inputs_kernel<T, VW, 0>
-             : a.taps == 4   ? attn_inputs_kernel<T, VW, 4>
-                             : attn_inputs_kernel<T, VW, -1>;
-    k<<<(unsigned)((total + 255) / 256), 256, 0, stream>>>(a, units, total);
+    if (a.N >= 2048)
+      launch_rows<T, VW, 4>(a, units, stream);
+    else
+      launch_rows<T, VW, 1>(a, units, stream);
   } else {
     attn_inputs_any_kernel<T, VW><<<dim3((a.H + 2 * a.G + 3) / 4, a.N), 256, 0, stream>>>(a);
   }

@@ -887,7 +887,7 @@ static void attention_inputs(torch::Tensor q, torch::Tensor k_cache, torch::Tens
   a.dim = (int)dim;
   a.vdim = (int)vdim;
   a.eps = (float)eps;
-  TORCH_CHECK(a.N <= 65535 * 16, "grid");
+  TORCH_CHECK(a.N <= 65535, "grid");
   if (a.N == 0) return;
   launch_attn_inputs(bf16, &a, cur_stream());
 }
@@ -963,7 +963,7 @@ static void experts_linear(torch::Tensor out, torch::Tensor x, torch::Tensor w, 
   a.perm = opt_int(perm, a.entries);
   a.offsets = opt_int(offsets, a.E + 2);
   if (kind == 1) {
-    TORCH_CHECK(tt == 1 || tt == 2 || tt == 4, "token fragments");
+    TORCH_CHECK(tt == 1 || tt == 2, "token fragments");
     launch_experts_small(glu, &a, (int)tt, cur_stream());
     return;
   }

@@ -10,6 +10,7 @@ typedef __bf16 bf16x8_v __attribute__((ext_vector_type(8)));
 typedef float f32x4_v __attribute__((ext_vector_type(4)));
 
 #define ROUTE_T 16  // tokens per workgroup
+#define AHEAD 8      // turns whose ids are loaded together
 
 // The wave picks the ``top`` largest of logits[0 .. E) (overwritten), the lower index
 // among equals, and their softmax weights.
@@ -51,7 +52,9 @@ static DEV void choose(float* logits, int E, int top, int* ids, float* weights) 
 }
 
 // 16 tokens a workgroup: its waves split K in blocks of 64, partial logits meet in LDS.
-// Dynamic LDS: [waves][E16][16] floats, E16 = E rounded up to 16.
+// NF fragments of 16 experts at a time.
+// Dynamic LDS: [waves][16][E16] floats, E16 = E rounded up to 16.
+template <int NF>
 __global__ __launch_bounds__(1024) void route_mfma_kernel(
     int* __restrict__ ids, float* __restrict__ weights, const bf16_t* __restrict__ h,
     const bf16_t* __restrict__ w, const float* __restrict__ bias, const int N, const int E,
@@ -59,42 +62,40 @@ __global__ __launch_bounds__(1024) void route_mfma_kernel(
   extern __shared__ float part[];
   const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6, waves = blockDim.x >> 6;
   const int c = lane & 15, g = lane >> 4;
-  const int E16 = (E + 15) & ~15;
+  const int E16 = (E + 15) & ~15, logits = ROUTE_T * E16;
   const int n0 = blockIdx.x * ROUTE_T;
   const bf16_t* hp = h + (int64_t)min(n0 + c, N - 1) * h_stride + g * 8;
-  float* mine = part + (int64_t)wid * E16 * ROUTE_T;
-  for (int e0 = 0; e0 < E16; e0 += 64) {
-    const bf16_t* wp[4];
+  float* mine = part + (int64_t)wid * logits;
+  for (int e0 = 0; e0 < E16; e0 += 16 * NF) {
+    const bf16_t* wp[NF];
 #pragma unroll
-    for (int i = 0; i < 4; ++i)
+    for (int i = 0; i < NF; ++i)
       wp[i] = w + (int64_t)min(e0 + i * 16 + c, E - 1) * K + g * 8;
-    f32x4_v acc[4] = {};
-#pragma unroll 2
+    f32x4_v acc[NF] = {};
+#pragma unroll 4
     for (int k = wid * 64; k < K; k += waves * 64) {
 #pragma unroll
       for (int s = 0; s < 64; s += 32) {
         const bf16x8_v b = *(const bf16x8_v*)(hp + k + s);
 #pragma unroll
-        for (int i = 0; i < 4; ++i) {
-          const bf16x8_v a = *(const bf16x8_v*)(wp[i] + k + s);
-          acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, acc[i], 0, 0, 0);
+        for (int i = 0; i < NF; ++i) {
+          const bf16x8_v f = *(const bf16x8_v*)(wp[i] + k + s);
+          acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(f, b, acc[i], 0, 0, 0);
         }
       }
     }
 #pragma unroll
-    for (int i = 0; i < 4; ++i)
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int e = e0 + i * 16 + g * 4 + r;
-        if (e < E16) mine[c * E16 + e] = acc[i][r];
-      }
+    for (int i = 0; i < NF; ++i) {
+      const int e = e0 + i * 16 + g * 4;
+      if (e < E16) *(f32x4_v*)(mine + c * E16 + e) = acc[i];
+    }
   }
   __syncthreads();
   // the first wave's part becomes the logits
-  for (int i = threadIdx.x; i < ROUTE_T * E16; i += blockDim.x) {
+  for (int i = threadIdx.x; i < logits; i += blockDim.x) {
     const int e = i % E16;
     float z = e < E ? (bias ? bias[e] : 0.f) : -INFINITY;
-    for (int p = 0; p < waves; ++p) z += part[(int64_t)p * E16 * ROUTE_T + i];
+    for (int p = 0; p < waves; ++p) z += part[(int64_t)p * logits + i];
     part[i] = z;
   }
   __syncthreads();
@@ -146,12 +147,23 @@ __global__ __launch_bounds__(1024) void group_kernel(
   const int per = ((n + 15) / 16 + 63) / 64 * 64;
   const int i0 = wid * per, i1 = min(n, i0 + per);
   int* mine = counts + wid * E;
-  for (int i = i0; i < i1; i += 64) {
-    const int id = i + lane < i1 ? ids[i + lane] : E;
+  auto turns = [&](auto&& turn) {  // over this wave's entries, their ids loaded ahead
+    for (int i = i0; i < i1; i += 64 * AHEAD) {
+      int id[AHEAD];
+#pragma unroll
+      for (int j = 0; j < AHEAD; ++j) {
+        const int at = i + j * 64 + lane;
+        id[j] = at < i1 ? ids[at] : E;
+      }
+#pragma unroll
+      for (int j = 0; j < AHEAD; ++j) turn(i + j * 64 + lane, id[j]);
+    }
+  };
+  turns([&](int, int id) {
     const uint64_t m = same_id(id, bits);
     if (id < E && lane == __builtin_ctzll(m)) mine[id] += __popcll(m);
     asm volatile("" ::: "memory");  // the next turn reads what other lanes wrote
-  }
+  });
   __syncthreads();
   for (int e = threadIdx.x; e < E; e += 1024) {
     int run = 0;
@@ -195,8 +207,7 @@ __global__ __launch_bounds__(1024) void group_kernel(
     }
   }
   __syncthreads();
-  for (int i = i0; i < i1; i += 64) {
-    const int id = i + lane < i1 ? ids[i + lane] : E;
+  turns([&](int at, int id) {
     const uint64_t m = same_id(id, bits);
     const int leader = __builtin_ctzll(m);
     int base = 0;
@@ -206,8 +217,8 @@ __global__ __launch_bounds__(1024) void group_kernel(
     }
     asm volatile("" ::: "memory");
     base = __shfl(base, leader, 64);
-    if (id < E) perm[total[id] + base + __popcll(m & ((1ull << lane) - 1))] = i + lane;
-  }
+    if (id < E) perm[total[id] + base + __popcll(m & ((1ull << lane) - 1))] = at;
+  });
 }
 
 // Few rows per expert: bound by the weights.  grid (outputs / 16 or 32, E); the 4 waves
@@ -309,11 +320,13 @@ void launch_moe_route(bool bf16, int* ids, float* weights, const void* h, const 
                       const float* bias, int N, int E, int K, int top, int64_t h_stride,
                       hipStream_t stream) {
   const int E16 = (E + 15) & ~15;
-  if (bf16 && E <= 128) {
+  if (bf16 && E <= 128) {  // at most 64 KiB of partial logits
     // few workgroups: more waves share the weights' latency
     const int waves = N <= 4096 && E16 <= 64 ? 16 : 8;
-    const int bytes = waves * E16 * ROUTE_T * 4;  // at most 64 KiB
-    route_mfma_kernel<<<(N + ROUTE_T - 1) / ROUTE_T, 64 * waves, bytes, stream>>>(
+    auto k = E16 <= 16   ? route_mfma_kernel<1>
+             : E16 <= 32 ? route_mfma_kernel<2>
+                         : route_mfma_kernel<4>;
+    k<<<(N + ROUTE_T - 1) / ROUTE_T, 64 * waves, waves * ROUTE_T * E16 * 4, stream>>>(
         ids, weights, (const bf16_t*)h, (const bf16_t*)w, bias, N, E, K, top, h_stride);
   } else if (bf16) {
     route_plain_kernel<bf16_t><<<N, 256, E * 4, stream>>>(
@@ -329,14 +342,12 @@ void launch_moe_group(int* perm, int* offsets, int* tile_expert, int* tile_row, 
   group_kernel<<<1, 1024, 17 * E * 4, stream>>>(perm, offsets, tile_expert, tile_row, ids, n, E);
 }
 
-// tt: token fragments at a time, 1, 2 or 4
+// tt: token fragments at a time, 1 or 2
 void launch_experts_small(bool glu, const ExpertsArgs* a, int tt, hipStream_t stream) {
   const int per = glu ? 16 : 32;
   const dim3 grid((a->O + per - 1) / per, a->E);
-  auto k = glu ? (tt == 1 ? experts_small_kernel<true, 1>
-                  : tt == 2 ? experts_small_kernel<true, 2> : experts_small_kernel<true, 4>)
-               : (tt == 1 ? experts_small_kernel<false, 1>
-                  : tt == 2 ? experts_small_kernel<false, 2> : experts_small_kernel<false, 4>);
+  auto k = glu ? (tt == 1 ? experts_small_kernel<true, 1> : experts_small_kernel<true, 2>)
+               : (tt == 1 ? experts_small_kernel<false, 1> : experts_small_kernel<false, 2>);
   k<<<grid, 256, 0, stream>>>(*a);
 }
 

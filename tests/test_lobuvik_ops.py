@@ -100,19 +100,36 @@ INPUTS = [
 ]
 
 
+#: portions of every sequence, the step it begins in, its state slot: the last sequence
+#: takes over the third one's slot after its end
+SHORT = ([[7, 1, 1, 2, 12], [2, 3, 1, 3], [1, 20, 2, 17], [1, 1]], [0, 1, 0, 4], [2, 0, 1, 1])
+#: enough rows for the kernel's longer turns, sequences that begin within one
+LONG = ([[3, 2042, 2, 1], [2, 3, 1, 5], [1, 9, 2000, 90], [2, 50]], [0, 0, 0, 4], [0, 3, 1, 1])
+
+
 @pytest.mark.parametrize("H,G,dim,vdim,taps,norms,rot,temp,mult", INPUTS)
 def test_attention_inputs(device, dtype, H, G, dim, vdim, taps, norms, rot, temp, mult):
     """Sequences run in steps of unequal portions, down to one token, beside each other;
     state slots are handed on uncleared.  Queries and cached rows are those of the whole
     sequences."""
+    run_attention_inputs(device, dtype, H, G, dim, vdim, taps, norms, rot, temp, mult, SHORT)
+
+
+@pytest.mark.parametrize("H,G,dim,vdim,taps,norms,rot,temp,mult", [
+    (2, 1, 60, 64, 4, True, 0, (0.5, 700), False), (1, 1, 64, 20, 3, True, 64, None, True),
+    (3, 1, 64, 128, 0, False, 10, None, True),
+])
+def test_attention_inputs_of_long_prompts(device, dtype, H, G, dim, vdim, taps, norms, rot, temp,
+                                          mult):
+    run_attention_inputs(device, dtype, H, G, dim, vdim, taps, norms, rot, temp, mult, LONG)
+
+
+def run_attention_inputs(device, dtype, H, G, dim, vdim, taps, norms, rot, temp, mult, steps):
     from agentcontrolplane_amd.engine.batch import FlatBatch, SeqMeta
 
+    sizes, start, slot = steps
     d, e, block, eps = ops.latent_head(dim), ops.latent_head(vdim), 4, 1e-2
-    C, lens = (H + G) * d + G * e, [23, 9, 40, 2]
-    sizes = [[7, 1, 1, 2, 12], [2, 3, 1, 3], [1, 20, 2, 17], [1, 1]]
-    start = [0, 1, 0, 3]          # the step a sequence begins in
-    slot = [2, 0, 1, 1]           # the last one takes over the third's... after its end
-    start[3] = 4
+    C, lens = (H + G) * d + G * e, [sum(z) for z in sizes]
     live = torch.zeros(C, dtype=torch.bool)  # the rest is padding
     for n in range(H + G):
         live[n * d : n * d + dim] = True
@@ -125,7 +142,7 @@ def test_attention_inputs(device, dtype, H, G, dim, vdim, taps, norms, rot, temp
     if norms:
         qn, kn = (1 + 0.3 * rand(d, dtype=dtype, device="cpu", seed=s) for s in (10, 11))
     factor = 1 + rand(H, dtype=F32, device="cpu", seed=12) if mult else None
-    table = rotation_table(64, 300.0, rot, None, "cpu") if rot else None
+    table = rotation_table(2200, 300.0, rot, None, "cpu") if rot else None
 
     def whole(x):  # the mechanisms on a whole sequence, pairs (2i, 2i + 1) put back in halves
         T, x = len(x), x.double()
