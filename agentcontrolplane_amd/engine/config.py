@@ -574,7 +574,7 @@ class EngineConfig:
     num_state_slots: Optional[int] = None
     max_batch_size: int = 2048
     # chunked-prefill token budget per step: 16384 measured ~7% faster
-    # wave p50 than 8192 at 1k concurrency (r02 A/B, gpurun_out/bench3b) —
+    # wave p50 than 8192 at 1k concurrency —
     # fewer, larger steps amortize per-step host+launch cost; activations
     # at 16k tokens are ~1 GB against 288 GB HBM
     max_prefill_tokens: int = 16384

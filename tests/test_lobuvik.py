@@ -80,7 +80,7 @@ CONFIGS = {
     "wide": (config(400, 128, [
         biased(8, 2, 64, 128, 4, 100, moe(4, 2, 128, 1.5, 96)),
         latent(4, 64, 64, 64, 128, 50, dense(96)),
-        rotated(16, 4, 64, 64, 32, 33, moe(8, 4, 64, 1.5, 128)),
+        rotated(16, 4, 64, 64, 32, 33, moe(8, 3, 64, 1.25, 128)),
         biased(2, 1, 128, 64, 2, 64, dense(64)),
     ], scale=1.3), {0: 32, 3: 16}),
     # beyond the matrix-core kernels' sizes

@@ -89,7 +89,7 @@ def test_distance_buckets(B, D):
 
 INPUTS = [
     # heads, kv heads, dim, vdim, taps, norms, rotated dims, temperature, head factor
-    (4, 2, 64, 32, 4, True, 0, (0.5, 7), False),
+    (6, 2, 64, 48, 4, True, 0, (0.7, 7), False),
     (6, 3, 12, 20, 3, True, 8, None, True),
     (8, 1, 128, 128, 2, False, 128, (0.3, 1), True),
     (3, 3, 70, 256, 6, True, 2, (2.0, 100), False),
@@ -116,7 +116,7 @@ def test_attention_inputs(device, dtype, H, G, dim, vdim, taps, norms, rot, temp
 
 
 @pytest.mark.parametrize("H,G,dim,vdim,taps,norms,rot,temp,mult", [
-    (2, 1, 60, 64, 4, True, 0, (0.5, 700), False), (1, 1, 64, 20, 3, True, 64, None, True),
+    (2, 1, 60, 64, 4, True, 0, (0.7, 700), False), (1, 1, 64, 20, 3, True, 64, None, True),
     (3, 1, 64, 128, 0, False, 10, None, True),
 ])
 def test_attention_inputs_of_long_prompts(device, dtype, H, G, dim, vdim, taps, norms, rot, temp,
@@ -242,7 +242,7 @@ def attend(q, k, v, ctx, scale, cap, window, bias, sigmoid, gate):
 
 FORMS = [
     # heads, kv heads, dim, vdim, window, cap, biased distances, sigmoid, gate, block, chunks
-    (4, 2, 64, 32, None, None, 60, True, False, 16, [(0, 40), (200, 2), (17, 3), (300, 1), (59, 1)]),
+    (6, 2, 64, 32, None, None, 60, True, False, 16, [(0, 40), (200, 2), (17, 3), (300, 1), (59, 1)]),
     (6, 3, 12, 20, None, None, 1, True, True, 4, [(0, 5), (0, 1), (9, 2), (130, 1), (63, 1)]),
     (8, 1, 128, 128, 100, None, 300, True, True, 16, [(0, 9), (350, 1), (99, 1), (101, 130)]),
     (8, 8, 128, 64, None, None, 3, True, False, 16, [(0, 260), (1200, 1), (777, 2), (2, 1)]),
@@ -250,7 +250,7 @@ FORMS = [
     (2, 2, 300, 40, None, None, 90, True, True, 16, [(0, 60), (70, 1), (200, 2)]),
     (1, 1, 1, 1, None, None, 2, True, False, 1, [(0, 5), (3, 1), (8, 2)]),
     (16, 4, 64, 128, None, None, 129, True, True, 64, [(0, 130), (1, 1), (64, 1), (65, 64)]),
-    (8, 4, 64, 64, 40, 20.0, 0, False, True, 16, [(0, 100), (39, 1), (40, 1), (41, 1), (600, 3)]),
+    (12, 4, 64, 64, 43, 20.0, 0, False, True, 16, [(0, 100), (42, 1), (43, 1), (44, 1), (600, 3)]),
     (4, 4, 96, 70, None, None, 33, False, True, 16, [(0, 70), (500, 1), (31, 2)]),
     (4, 2, 64, 64, 70, 3.0, 50, False, True, 16, [(0, 170), (500, 1), (70, 1), (31, 2)]),
     (4, 2, 64, 64, None, 2.0, 30, True, False, 16, [(0, 50), (500, 1), (31, 2)]),
@@ -354,7 +354,7 @@ def still(positions, device):
 SINKS = [
     # heads, latent, window, chunks
     (3, 24, None, [(0, 5), (0, 20), (100, 3), (130, 1), (0, 1)]),
-    (8, 64, 40, [(0, 100), (39, 1), (40, 1), (700, 1), (300, 2)]),
+    (6, 64, 40, [(0, 100), (39, 1), (40, 1), (700, 1), (300, 2)]),
     (20, 500, 33, [(0, 40), (500, 1), (32, 1)]),
     (40, 130, 1, [(0, 9), (17, 1)]),
     (2, 600, 20, [(0, 30), (90, 1)]),
@@ -506,7 +506,7 @@ def test_route_ties_and_order(device, dtype):
 
 EXPERTS = [
     # tokens, experts, top, K, inner, W: few and many rows per expert, padded inner sizes
-    (1, 4, 2, 64, 64, 40), (3, 8, 3, 192, 64, 192), (50, 8, 4, 128, 128, 96),
+    (1, 4, 2, 64, 64, 40), (3, 6, 3, 192, 64, 160), (50, 8, 4, 128, 128, 96),
     (70, 3, 2, 64, 192, 31), (300, 4, 2, 128, 128, 130), (700, 2, 1, 256, 256, 258),
     (260, 3, 3, 128, 384, 512), (40, 40, 1, 64, 64, 64), (1030, 5, 2, 512, 128, 72),
 ]
