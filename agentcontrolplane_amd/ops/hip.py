@@ -299,30 +299,30 @@ def cache_keys_values(k, v, slot_mapping, k_cache, v_cache):
 
 
 def _conv_rows(batch):
-    """Per row of a step: rows of its sequence right before it, its state slot; and the
-    rows that later steps' convolutions read.  None, slots, None: decode rows only."""
+    """Per row of a step: rows of its sequence right before it, and its state slot.
+    None, slots: every row is alone in its sequence's step."""
     if not batch.prefills:
-        return None, batch.decode_state_slots, None
-    device, P = batch.positions.device, batch.num_prefill_tokens
-    meta, counts = batch.prefill_meta(16), [m.query_len for m in batch.prefills]
-    times = torch.tensor(counts, device=device)
-    per_row = torch.stack([meta.ctx_lens, meta.state_slots]).repeat_interleave(
-        times, 1, output_size=P
+        return None, batch.decode_state_slots
+    P, meta = batch.num_prefill_tokens, batch.prefill_meta(16)
+    ctx, slots = torch.stack([meta.ctx_lens, meta.state_slots]).repeat_interleave(
+        meta.seq_lens - meta.ctx_lens, 1, output_size=P
     )
-    back, slots = batch.positions[:P].int() - per_row[0], per_row[1]
+    back = batch.positions[:P].int() - ctx
     if batch.num_decode:
         back = torch.cat([back, back.new_zeros(batch.num_decode)])
         slots = torch.cat([slots, batch.decode_state_slots])
-    return back.contiguous(), slots.contiguous(), counts
+    return back, slots.contiguous()
 
 
 def _ring_rows(batch, taps: int):
-    """The last rows of every portion, as many as a convolution looks back."""
+    """The last rows of every portion, as many as a ring holds."""
     rows, at = [], 0
     for m in batch.prefills:
         at += m.query_len
         rows.extend(range(at - min(m.query_len, taps), at))
     rows.extend(range(at, at + batch.num_decode))
+    if batch._stager is not None:
+        return batch._stager.tensor(f"ring_rows{taps}", rows, "int32")
     return torch.tensor(rows, dtype=torch.int32, device=batch.positions.device)
 
 
@@ -331,7 +331,7 @@ def attention_inputs(proj, heads, dim, vdim, k_cache, v_cache, batch, eps, conv,
     q = torch.empty(proj.shape[0], heads, k_cache.shape[3], dtype=proj.dtype, device=proj.device)
     back = states = ring_rows = None
     if conv is not None:
-        back, states, _ = batch.memo("conv_rows", lambda: _conv_rows(batch))
+        back, states = batch.memo("conv_rows", lambda: _conv_rows(batch))
         if batch.prefills:
             taps = conv.shape[0]
             ring_rows = batch.memo(("ring_rows", taps), lambda: _ring_rows(batch, taps))
@@ -353,8 +353,6 @@ def grouped_attention(q, k_cache, v_cache, batch, scale: float, cap, window, kee
     tiled = (q.dtype == torch.bfloat16 and d in LATENT_HEADS and v in LATENT_HEADS
              and not (sigmoid and cap))
     P = batch.num_prefill_tokens
-    if gate is not None and q.dtype != gate.dtype:
-        raise TypeError("the gate has the queries' dtype")
 
     def gates(r):
         return None if gate is None else gate[r]
