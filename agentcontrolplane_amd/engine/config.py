@@ -104,16 +104,19 @@ class GroupedAttentionSpec:
     scale: float                    # on the scores
     softcap: Optional[float] = None  # scores -> softcap * tanh(score / softcap)
     window: Optional[int] = None    # keys visible, self included; None = all
+    chunk: Optional[int] = None     # only keys of the query's own chunk, positions / chunk
     keep_first: int = 0             # first tokens that stay visible beyond the window
     bias: bool = True               # on the query, key and value projections
     sink: bool = True               # learned logit per head in the denominator
     kv_from: Optional[int] = None   # the layer whose keys and values are used
     conv: int = 0                   # taps of the short convolutions on q, k, v; 0 = none
     qk_norm: bool = False           # RMS norm of query and key heads, learned weight
+    row_norm: bool = False          # the same over all query (key) heads at once
     v_norm: bool = False            # RMS norm of value heads, no weight
     rotary: Optional[RotarySpec] = None
     q_temp: Optional[QueryTemperature] = None
     head_temp: bool = False         # learned factor per head on the scores
+    talk: bool = False              # a head's scores are a learned mix of all heads'
     distance_bias: Optional[DistanceBias] = None
     sigmoid: bool = False           # weights sigmoid(score + learned offset), not normalized
     head_gate: bool = False         # sigmoid gate per head on the output
@@ -124,30 +127,39 @@ class GroupedAttentionSpec:
         kv = 0 if self.kv_from is not None else self.kv_heads * (self.dim + self.vdim)
         n = (q + kv) * (w + self.bias + self.conv) + o * w + (w if self.out_bias else 0)
         n += 2 * self.dim if self.qk_norm else 0
+        n += (self.heads + self.kv_heads) * self.dim if self.row_norm else 0
+        n += self.heads ** 2 if self.talk else 0
         n += self.heads * (self.sink + self.head_temp + self.sigmoid)
         n += self.heads * self.distance_bias.buckets if self.distance_bias else 0
         return n + (self.heads * w if self.head_gate else 0)
 
 
 @dataclasses.dataclass(frozen=True)
-class ChannelDeltaSpec:
-    """Gated delta rule with one decay per head and key channel
-    (models/channel_delta.py)."""
+class GatedDeltaSpec:
+    """Gated delta rule with one decay per head, or per head and key channel
+    (models/gated_delta.py)."""
 
     heads: int                      # value heads, one state each
     kv_heads: int                   # query/key heads
     dim: int                        # query/key size per head
     vdim: int                       # value size per head
     conv: int                       # taps of the short convolutions
-    decay_rank: int                 # inner size of the decay projection
-    gate_rank: int                  # inner size of the output gate's projection
+    decay_rank: int = 0             # inner size of the decay projection; 0 = direct
+    gate_rank: int = 0              # inner size of the output gate's projection; 0 = direct
+    head_decay: bool = False        # one decay per head, else one per head and key channel
+    gate_silu: bool = False         # output gate silu, else sigmoid
     unit_eps: float = 1e-6          # in the unit vectors' sum of squares
+
+    @property
+    def decays(self) -> int:
+        return self.heads * (1 if self.head_decay else self.dim)
 
     def params(self, w: int) -> int:
         qk, v = 2 * self.kv_heads * self.dim, self.heads * self.vdim
         n = (qk + v) * (w + self.conv) + self.heads * (w + 1) + self.vdim + v * w
-        n += self.decay_rank * (w + self.heads * self.dim) + self.heads * self.dim
-        return n + self.gate_rank * (w + v)
+        r, g = self.decay_rank, self.gate_rank
+        n += (r * (w + self.decays) if r else w * self.decays) + self.decays
+        return n + (g * (w + v) if g else w * v)
 
 
 @dataclasses.dataclass(frozen=True)
@@ -160,6 +172,10 @@ class ClampedGluSpec:
     alpha: float = 1.702
     offset: float = 1.0
     cubic: float = 0.0
+    bias: bool = False              # on all three projections
+
+    def params(self, w: int) -> int:
+        return 3 * w * self.width + (2 * self.width + w if self.bias else 0)
 
 
 def silu_glu(width: int) -> ClampedGluSpec:
@@ -167,23 +183,28 @@ def silu_glu(width: int) -> ClampedGluSpec:
     return ClampedGluSpec(width, limit=math.inf, alpha=1.0, offset=0.0)
 
 
-def gelu_glu(width: int) -> ClampedGluSpec:
+def gelu_glu(width: int, bias: bool = False) -> ClampedGluSpec:
     """gelu(gate) * up, the tanh form: 1 + tanh(z) = 2 sigmoid(2z)."""
     return ClampedGluSpec(
-        width, limit=math.inf, alpha=2 * math.sqrt(2 / math.pi), offset=0.0, cubic=0.044715
+        width, limit=math.inf, alpha=2 * math.sqrt(2 / math.pi), offset=0.0, cubic=0.044715,
+        bias=bias,
     )
 
 
 @dataclasses.dataclass(frozen=True)
 class ExpertsSpec:
     """Mixture of experts: each token uses ``top`` of ``experts`` GLUs, weighted by the
-    softmax over the chosen router logits, and the shared one (models/experts.py)."""
+    softmax over the chosen router logits or by their normed sigmoids, and the shared one
+    (models/experts.py)."""
 
     experts: int
     top: int
     expert: ClampedGluSpec
     shared: Optional[ClampedGluSpec] = None
     router_bias: bool = True
+    sigmoid: bool = False           # scores are the logits' sigmoids
+    correction: bool = False        # learned, on the scores in the choice only
+    scale: float = 1.0              # on the weights
 
     @property
     def width(self) -> int:
@@ -191,16 +212,19 @@ class ExpertsSpec:
         return self.top * self.expert.width + (self.shared.width if self.shared else 0)
 
     def params(self, w: int) -> int:
-        n = self.experts * (w + self.router_bias + 3 * w * self.expert.width)
-        return n + (3 * w * self.shared.width if self.shared else 0)
+        each = w + self.router_bias + self.correction + self.expert.params(w)
+        return self.experts * each + (self.shared.params(w) if self.shared else 0)
 
 
 @dataclasses.dataclass(frozen=True)
 class LayerSpec:
-    mixer: Union[LatentAttentionSpec, GroupedAttentionSpec, ChannelDeltaSpec]
+    mixer: Union[LatentAttentionSpec, GroupedAttentionSpec, GatedDeltaSpec]
     mlp: Union[None, ClampedGluSpec, ExpertsSpec] = None
     sandwich: bool = False  # mixer, then mlp, each normed on its way in and out
     mlp_norm: bool = False  # side by side, the mlp on a norm of its own
+    norm_out: bool = False  # mixer, then mlp, each normed on its way out only
+    gated: bool = False     # sigmoid gates on both results, from what they were made of
+    weights_of: Optional[int] = None  # the layer whose weights are used
 
 
 @dataclasses.dataclass(frozen=True)
@@ -250,6 +274,8 @@ class ModelConfig:
     embed_scale: float = 1.0
     # logits -> cap * tanh(logits / cap)
     logit_softcap: Optional[float] = None
+    # on the logits
+    logit_scale: float = 1.0
 
     @property
     def layer_runs(self) -> Tuple[Tuple[int, bool], ...]:
@@ -286,12 +312,12 @@ class ModelConfig:
         w, v = self.hidden_size, self.vocab_size
         total = v * w * (1 if self.tie_embeddings else 2) + w
         for i, layer in enumerate(self.layers):
+            if layer.weights_of is not None:
+                continue
             total += w + layer.mixer.params(w)
-            if isinstance(layer.mlp, ExpertsSpec):
-                total += layer.mlp.params(w)
-            elif layer.mlp:
-                total += 3 * w * layer.mlp.width
-            total += w if layer.mlp and layer.mlp_norm else 0
+            total += layer.mlp.params(w) if layer.mlp else 0
+            total += w if layer.mlp and (layer.mlp_norm or layer.norm_out) else 0
+            total += (w * w + w) * (2 if layer.mlp else 1) if layer.gated else 0
             if layer.sandwich:
                 total += w + (2 * w if layer.mlp else 0)
             if self.depth_average:
@@ -333,7 +359,7 @@ def _tezinex(name: str, *, width: int, layers: int, ff: int, heads: int, kv_head
              attn_every: int = 4, share: int = 2, **kw) -> ModelConfig:
     """Every ``attn_every``-th layer is windowed attention, the others delta
     layers; of ``share`` consecutive attention layers all use the first one's keys."""
-    delta = ChannelDeltaSpec(d_heads, d_kv_heads, d_dim, d_vdim, conv, rank, rank)
+    delta = GatedDeltaSpec(d_heads, d_kv_heads, d_dim, d_vdim, conv, rank, rank)
 
     def mixer(i: int):
         nth, at = divmod(i, attn_every)
@@ -384,6 +410,40 @@ def _lobuvik(name: str, *, width: int, layers: int, heads: int, kv_heads: int, d
             LayerSpec(mixers[i % 3], gelu_glu(ff) if i == 0 else experts, mlp_norm=True)
             for i in range(layers)
         ), **kw,
+    )
+
+
+def _noganex(name: str, *, width: int, layers: int, heads: int, kv_heads: int, dim: int,
+             vdim: int, chunk: int, rotary: RotarySpec, d_heads: int, d_kv_heads: int,
+             d_dim: int, d_vdim: int, ff: int, experts: ExpertsSpec, vocab: int, conv: int = 4,
+             logit_scale: float = 0.5, **kw) -> ModelConfig:
+    """Chunked attention with a dense feed-forward and delta layers with experts in turn;
+    every second delta layer uses the one before's weights."""
+    attention = LayerSpec(GroupedAttentionSpec(
+        heads=heads, kv_heads=kv_heads, dim=dim, vdim=vdim, scale=dim ** -0.5, chunk=chunk,
+        bias=False, sink=False, row_norm=True, rotary=rotary, talk=True,
+    ), gelu_glu(ff, bias=True), norm_out=True, gated=True)
+    delta = LayerSpec(GatedDeltaSpec(
+        d_heads, d_kv_heads, d_dim, d_vdim, conv, head_decay=True, gate_silu=True,
+    ), experts, norm_out=True, gated=True)
+
+    def layer(i: int) -> LayerSpec:
+        if i % 2 == 0:
+            return attention
+        return delta if i % 4 == 1 else dataclasses.replace(delta, weights_of=i - 2)
+
+    return ModelConfig(
+        name=name, architecture="Noganex", vocab_size=vocab, hidden_size=width,
+        intermediate_size=ff, num_layers=layers, num_heads=heads, num_kv_heads=kv_heads,
+        head_dim=dim, layers=tuple(layer(i) for i in range(layers)), logit_scale=logit_scale,
+        **kw,
+    )
+
+
+def _corrected_experts(experts: int, top: int, ff: int, shared: int, scale: float) -> ExpertsSpec:
+    return ExpertsSpec(
+        experts, top, silu_glu(ff), silu_glu(shared), router_bias=False, sigmoid=True,
+        correction=True, scale=scale,
     )
 
 
@@ -483,6 +543,27 @@ PRESETS = {
         "tiny-lobuvik", width=44, layers=4, heads=6, kv_heads=3, dim=12, vdim=10, conv=3,
         bias=DistanceBias(12, 50), kv_rank=20, rot_dim=6, window=23, ff=52,
         experts=ExpertsSpec(5, 2, ClampedGluSpec(18, 1.5), ClampedGluSpec(22, 2.0)),
+        vocab=300, max_position=4096, dtype="float32",
+    ),
+    # Noganex with the layer sizes of an 8B-class dense model per token (random weights):
+    # width, heads and active feed-forward of llama3-8b
+    "noganex-8b": _noganex(
+        "noganex-8b", width=4096, layers=28, heads=32, kv_heads=8, dim=128, vdim=128,
+        chunk=4096, rotary=RotarySpec(5e5, 128, YarnScaling(4.0, 8192, 32.0, 1.0)), d_heads=32,
+        d_kv_heads=16, d_dim=128, d_vdim=128, ff=14336,
+        experts=_corrected_experts(32, 4, 2560, 4096, 2.5), vocab=128256,
+    ),
+    # half the width, 16 heads
+    "noganex-2b": _noganex(
+        "noganex-2b", width=2048, layers=18, heads=16, kv_heads=8, dim=128, vdim=128,
+        chunk=1024, rotary=RotarySpec(5e5, 64, YarnScaling(4.0, 4096, 32.0, 1.0)), d_heads=16,
+        d_kv_heads=8, d_dim=128, d_vdim=128, ff=8192,
+        experts=_corrected_experts(16, 4, 1536, 2048, 2.5), vocab=32000,
+    ),
+    "tiny-noganex": _noganex(
+        "tiny-noganex", width=44, layers=4, heads=6, kv_heads=2, dim=12, vdim=10, chunk=23,
+        rotary=RotarySpec(1e4, 8, YarnScaling(3.0, 64, 8.0, 1.0)), d_heads=6, d_kv_heads=3,
+        d_dim=10, d_vdim=14, conv=3, ff=52, experts=_corrected_experts(5, 2, 18, 22, 1.7),
         vocab=300, max_position=4096, dtype="float32",
     ),
     # tiny GPU config: real head_dim/GQA shape for the CDNA4 kernels at

@@ -2,6 +2,7 @@ from .fetolix import FetolixForCausalLM  # noqa: F401
 from .llama import LlamaForCausalLM  # noqa: F401
 from .lobuvik import LobuvikForCausalLM  # noqa: F401
 from .mixtral import MixtralForCausalLM  # noqa: F401
+from .noganex import NoganexForCausalLM  # noqa: F401
 from .tezinex import TezinexForCausalLM  # noqa: F401
 
 #: ModelConfig.architecture -> model class
@@ -11,6 +12,7 @@ MODEL_CLASSES = {
     "Fetolix": FetolixForCausalLM,
     "Tezinex": TezinexForCausalLM,
     "Lobuvik": LobuvikForCausalLM,
+    "Noganex": NoganexForCausalLM,
 }
 
 

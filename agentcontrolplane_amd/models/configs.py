@@ -5,12 +5,13 @@ A reader per architecture name; the name also picks the model class
 """
 from __future__ import annotations
 
+import dataclasses
 import json
 import os
 from typing import Callable, Dict, Optional, Tuple
 
 from ..engine.config import (
-    ChannelDeltaSpec, ClampedGluSpec, DistanceBias, ExpertsSpec, GroupedAttentionSpec,
+    ClampedGluSpec, DistanceBias, ExpertsSpec, GatedDeltaSpec, GroupedAttentionSpec,
     LatentAttentionSpec, LayerSpec, LoopSpec, ModelConfig, QueryTemperature, RotarySpec,
     WavelengthScaling, YarnScaling, gelu_glu, silu_glu,
 )
@@ -73,10 +74,17 @@ def _fetolix(d: dict, shape: Shape) -> ModelConfig:
     )
 
 
-def _channel_delta(m: dict, shape: Shape, p: str) -> ChannelDeltaSpec:
-    return ChannelDeltaSpec(
+def _channel_delta(m: dict, shape: Shape, p: str) -> GatedDeltaSpec:
+    return GatedDeltaSpec(
         heads=m["heads"], kv_heads=m["kv_heads"], dim=m["dim"], vdim=m["vdim"],
         conv=m["conv"], decay_rank=shape(p + "a1")[0], gate_rank=shape(p + "g1")[0],
+    )
+
+
+def _head_delta(m: dict) -> GatedDeltaSpec:
+    return GatedDeltaSpec(
+        heads=m["heads"], kv_heads=m["kv_heads"], dim=m["dim"], vdim=m["vdim"],
+        conv=m["conv"], head_decay=True, gate_silu=True,
     )
 
 
@@ -220,10 +228,82 @@ def _lobuvik(d: dict, shape: Shape) -> ModelConfig:
     )
 
 
+def _talking_attention(m: dict) -> GroupedAttentionSpec:
+    rot, s = m["rot"], m["rot"]["scaling"]
+    if rot["dims"] % 2 or rot["dims"] > m["dim"]:
+        raise ValueError("rot.dims must be even and at most dim")
+    return GroupedAttentionSpec(
+        heads=m["heads"], kv_heads=m["kv_heads"], dim=m["dim"], vdim=m["vdim"],
+        scale=m["scale"], chunk=m["mask"]["size"], bias=False, sink=False, row_norm=True,
+        talk=True, rotary=RotarySpec(
+            rot["base"], rot["dims"],
+            YarnScaling(s["factor"], s["original"], s["fast"], s["slow"]),
+        ),
+    )
+
+
+#: Noganex mixer type -> spec reader
+_NOGANEX_MIXERS = {"attention": _talking_attention, "delta": _head_delta}
+
+
+def _noganex_mlp(mlp: Optional[dict]):
+    if mlp is None:
+        return None
+    if mlp["kind"] == "dense":
+        return gelu_glu(mlp["ff"], bias=True)
+    if mlp["kind"] != "moe":
+        raise ValueError(f"unknown feed-forward kind {mlp['kind']!r}")
+    router, shared = mlp["router"], mlp.get("shared")
+    if not 0 < router["top"] <= router["experts"]:
+        raise ValueError("a token uses between 1 and all experts")
+    return ExpertsSpec(
+        experts=router["experts"], top=router["top"], expert=silu_glu(mlp["expert"]["ff"]),
+        shared=silu_glu(shared["ff"]) if shared else None, router_bias=False, sigmoid=True,
+        correction=True, scale=router["scale"],
+    )
+
+
+def _check_shared_weights(layers) -> None:
+    for i, layer in enumerate(layers):
+        j = layer.weights_of
+        if j is None:
+            continue
+        owner = layers[j] if 0 <= j < len(layers) else None
+        if owner is None or owner.weights_of is not None:
+            raise ValueError(f"layer {i}: layer {j} has no weights to use")
+        if dataclasses.replace(layer, weights_of=None) != owner:
+            raise ValueError(f"layer {i} differs from layer {j}, whose weights it uses")
+
+
+def _noganex(d: dict, shape: Shape) -> ModelConfig:
+    layers = []
+    for i, entry in enumerate(d["layers"]):
+        if entry["type"] not in _NOGANEX_MIXERS:
+            raise ValueError(f"unknown mixer type {entry['type']!r}")
+        m = _NOGANEX_MIXERS[entry["type"]](entry["mixer"])
+        if m.heads % m.kv_heads:
+            raise ValueError(f"layer {i}: kv_heads must divide heads")
+        layers.append(LayerSpec(
+            mixer=m, mlp=_noganex_mlp(entry.get("mlp")), norm_out=True, gated=True,
+            weights_of=entry.get("weights_of"),
+        ))
+    _check_shared_weights(layers)
+    first = layers[0].mixer
+    return ModelConfig(
+        name="Noganex", architecture="Noganex", vocab_size=d["vocab"],
+        hidden_size=d["width"], num_layers=len(layers), num_heads=first.heads,
+        num_kv_heads=first.kv_heads, head_dim=first.dim,
+        intermediate_size=max((x.mlp.width for x in layers if x.mlp), default=0),
+        rms_eps=d["norm"]["eps"], max_position=_UNBOUNDED, layers=tuple(layers),
+        logit_scale=d["logit_scale"],
+    )
+
+
 CONFIG_READERS: Dict[str, Callable[[dict, Shape], ModelConfig]] = {
     "Fetolix": _fetolix,
     "Tezinex": _tezinex,
     "Lobuvik": _lobuvik,
+    "Noganex": _noganex,
 }
 
 

@@ -1,10 +1,12 @@
 """Grouped attention over paged keys and values, with the parts a design picks.
 
     q, k, v = conv(W h + b);  query head n uses key/value head n // (heads / kv_heads)
-    q, k = rmsnorm(.) w, rotated;  v = rmsnorm(v)
+    q, k = rmsnorm(.) w, per head or over all heads, rotated;  v = rmsnorm(v)
     q_i *= 1 + coef ln(floor((i + 1) / every) + 1),  times a learned factor per head
-    s_ij = cap(scale * q_i . k_j) + bias[bucket(i - j)]
+    s_ij = scale * q_i . k_j,  mixed over the heads:  s_h <- sum_g T[h, g] s_g
+    s_ij = cap(s_ij) + bias[bucket(i - j)]
     i sees j:  j <= i and (i - j < window or j < keep_first)
+               and floor(i / chunk) = floor(j / chunk)
     out_i = sum_j exp(s_ij) v_j / (exp(sink) + sum_j exp(s_ij))
          or sum_j sigmoid(s_ij + offset) v_j,  times sigmoid(W_g h) per head
 
@@ -52,6 +54,12 @@ class GroupedAttention:
             raise ValueError("TP degree must divide the key/value head count")
         if spec.kv_from is not None and (spec.conv or spec.qk_norm or spec.rotary):
             raise ValueError("borrowed keys are used as their owner cached them")
+        if tp_world > 1 and (spec.row_norm or spec.talk):
+            raise ValueError("norms and score mixes over all heads need them on one rank")
+        if spec.row_norm and (spec.qk_norm or spec.conv):
+            raise ValueError("a norm over all heads goes with neither head norms nor convolutions")
+        if spec.chunk and spec.keep_first:
+            raise ValueError("chunks keep no first tokens")
         self.spec, self.width, self.eps = spec, width, eps
         self.heads, self.kv_heads = spec.heads // tp_world, spec.kv_heads // tp_world
         self.tp_rank = tp_rank
@@ -61,16 +69,18 @@ class GroupedAttention:
         kv = 0 if spec.kv_from is not None else self.kv_heads * (self.d + self.v)
         self.channels = self.heads * self.d + kv
         #: is there more between the projection and the cache than a copy?
-        self.shaped = bool(spec.conv or spec.qk_norm or spec.v_norm or spec.rotary
-                           or spec.q_temp or spec.head_temp)
-        self.w_in: torch.Tensor = None   # [q | k | v | head gates rows, width]
+        self.shaped = bool(spec.conv or spec.qk_norm or spec.row_norm or spec.v_norm
+                           or spec.rotary or spec.q_temp or spec.head_temp)
+        self.w_in: torch.Tensor = None   # [q | k | v | head gates | beside rows, width]
+        self.beside_at: Optional[Tuple[int, int]] = None  # first row and rows of beside
         self.bias: Optional[torch.Tensor] = None
         self.conv: Optional[torch.Tensor] = None       # [taps, channels]
-        self.q_norm = self.k_norm = None               # [d]
+        self.q_norm = self.k_norm = None               # [d], or of all heads
         self.w_out: torch.Tensor = None
         self.out_bias: Optional[torch.Tensor] = None   # on the first rank
         # fp32
         self.sink = self.temp = None                   # [heads]
+        self.talk: Optional[torch.Tensor] = None       # [heads, heads]
         self.rel = self.offset = None                  # [buckets, heads], [heads]
         self.dist_bias: Optional[torch.Tensor] = None  # [heads, distances], offset included
         self.cos_sin: Optional[torch.Tensor] = None    # set by the model if spec.rotary
@@ -96,6 +106,10 @@ class GroupedAttention:
                 out.append((name + ".conv", (heads * size, s.conv)))
         if s.qk_norm:
             out += [("q.norm", (s.dim,)), ("k.norm", (s.dim,))]
+        if s.row_norm:
+            out += [("q.norm", (s.heads * s.dim,)), ("k.norm", (s.kv_heads * s.dim,))]
+        if s.talk:
+            out.append(("talk", (s.heads, s.heads)))
         if s.distance_bias:
             out.append(("rel", (s.distance_bias.buckets, s.heads)))
         if s.sigmoid:
@@ -134,9 +148,14 @@ class GroupedAttention:
             t = pair_halves(t, self.spec.rotary.dims)
         return pad_to(t, self.d).contiguous()
 
-    def load(self, get: Get, p: str) -> None:
-        s, rows, biases, taps = self.spec, [], [], []
+    def load(self, get: Get, p: str,
+             beside: Optional[Tuple[torch.Tensor, torch.Tensor]] = None) -> None:
+        """``beside``: rows and bias of another product of the same input."""
+        s, rows, biases, taps, row_norms = self.spec, [], [], [], {}
         for part in self._parts():
+            if s.row_norm and part[0] != "v":
+                w = get(p + part[0] + ".norm").unsqueeze(1)
+                row_norms[part[0]] = self._laid_out(w, *part).flatten().contiguous()
             rows.append(self._laid_out(get(p + part[0]), *part))
             if s.bias:
                 biases.append(self._laid_out(get(p + part[0] + ".b").unsqueeze(1), *part))
@@ -145,14 +164,26 @@ class GroupedAttention:
         if s.head_gate:
             gate = self._mine(get(p + "g"), s.heads)
             rows.append(pad_to(gate, round_up(self.heads, 16), self.width))
+        if beside:
+            self.beside_at = (sum(len(r) for r in rows), beside[0].shape[0])
+            rows.append(pad_to(beside[0], round_up(beside[0].shape[0], 16), self.width))
         self.w_in = torch.cat(rows).contiguous()
+        if s.bias or beside:
+            self.bias = self.w_in.new_zeros(self.w_in.shape[0])
         if s.bias:
-            self.bias = pad_to(torch.cat(biases).flatten(), self.w_in.shape[0])
+            self.bias[: self.channels] = torch.cat(biases).flatten()
+        if beside:
+            at, n = self.beside_at
+            self.bias[at : at + n] = beside[1]
         if s.conv:
             self.conv = torch.cat(taps).t().contiguous()
         if s.qk_norm:
             self.q_norm = self._head_norm(get(p + "q.norm"))
             self.k_norm = self._head_norm(get(p + "k.norm"))
+        if s.row_norm:
+            self.q_norm, self.k_norm = row_norms["q"], row_norms["k"]
+        if s.talk:
+            self.talk = get(p + "talk").float().contiguous()
 
         def per_head(name):
             return self._mine(get(p + name), s.heads).float().contiguous()
@@ -186,6 +217,9 @@ class GroupedAttention:
             if s.bias:
                 b = self.bias[at : at + n].unsqueeze(1)
                 out[p + name + ".b"] = self._restored(b, name, size, padded).flatten()
+            if s.row_norm and name != "v":
+                t = (self.q_norm if name == "q" else self.k_norm).unsqueeze(1)
+                out[p + name + ".norm"] = self._restored(t, name, size, padded).flatten()
             if s.conv:
                 taps = self.conv[:, at : at + n].t()
                 out[p + name + ".conv"] = self._restored(taps, name, size, padded)
@@ -196,7 +230,8 @@ class GroupedAttention:
                 out[p + name] = unpair_halves(t, s.rotary.dims) if s.rotary else t
         if s.distance_bias:
             out[p + "rel"] = self.rel.to(dt)
-        for name, t in (("sink", self.sink), ("temp", self.temp), ("pb", self.offset)):
+        for name, t in (("sink", self.sink), ("temp", self.temp), ("pb", self.offset),
+                        ("talk", self.talk)):
             if t is not None:
                 out[p + name] = t.to(dt)
         if s.head_gate:
@@ -206,6 +241,10 @@ class GroupedAttention:
         if s.out_bias:
             out[p + "o.b"] = self.out_bias
         return out
+
+    def beside(self) -> Tuple[torch.Tensor, torch.Tensor]:
+        at, n = self.beside_at
+        return self.w_in[at : at + n], self.bias[at : at + n]
 
     # ----------------------------------------------------- pages and state
 
@@ -235,8 +274,9 @@ class GroupedAttention:
     # ------------------------------------------------------------- forward
 
     def attend(self, h: torch.Tensor, batch: FlatBatch, cache: Tuple[torch.Tensor, torch.Tensor],
-               ring: Optional[torch.Tensor], out: torch.Tensor) -> None:
-        """h [N, width] -> out [N, heads * v] (row-strided): the heads ahead of W_o."""
+               ring: Optional[torch.Tensor], out: torch.Tensor) -> Optional[torch.Tensor]:
+        """h [N, width] -> out [N, heads * v] (row-strided): the heads ahead of W_o.
+        Returns the product beside the mixer's, if there is one."""
         s, N = self.spec, h.shape[0]
         proj = ops.linear(h, self.w_in, self.bias)
         row, at = proj.stride(0), self.heads * self.d
@@ -257,12 +297,20 @@ class GroupedAttention:
         out = out.as_strided((N, self.heads, self.v), (out.stride(0), self.v, 1))
         ops.grouped_attention(
             q, *cache, batch, s.scale, s.softcap, s.window, s.keep_first, self.sink, out,
-            bias=self.dist_bias, sigmoid=s.sigmoid, gate=gate,
+            bias=self.dist_bias, sigmoid=s.sigmoid, gate=gate, chunk=s.chunk, talk=self.talk,
         )
+        if self.beside_at is None:
+            return None
+        at, n = self.beside_at
+        return proj[:, at : at + n]
+
+    def mix(self, h: torch.Tensor, batch: FlatBatch, cache: Tuple[torch.Tensor, torch.Tensor]):
+        """h [N, width] -> the heads ahead of W_o [N, heads * v] and, if there is one, the
+        product beside the mixer's."""
+        out = torch.empty(h.shape[0], self.out_dim, dtype=h.dtype, device=h.device)
+        return out, self.attend(h, batch, cache, None, out)
 
     def forward(self, h: torch.Tensor, batch: FlatBatch,
                 cache: Tuple[torch.Tensor, torch.Tensor]) -> torch.Tensor:
         """h [N, width] -> this rank's part of [N, width]."""
-        out = torch.empty(h.shape[0], self.out_dim, dtype=h.dtype, device=h.device)
-        self.attend(h, batch, cache, None, out)
-        return ops.linear(out, self.w_out, self.out_bias)
+        return ops.linear(self.mix(h, batch, cache)[0], self.w_out, self.out_bias)

@@ -38,6 +38,15 @@ def stack_rows(sections, width: int, align: int = 16):
     return out, places
 
 
+def section_bias(w: torch.Tensor, places, biases) -> torch.Tensor:
+    """Bias over the rows of a stack_rows() weight, zero in sections without one."""
+    out = w.new_zeros(w.shape[0])
+    for name, b in biases.items():
+        at = places[name][0]
+        out[at : at + b.shape[0]] = b
+    return out
+
+
 def pair_halves(t: torch.Tensor, dims: int, axis: int = -1) -> torch.Tensor:
     """Reorder the first ``dims`` entries of an axis from [u.. | v..] to (u, v) pairs: a
     rotation of i with i + dims/2 becomes one of 2i with 2i + 1.  Scores do not change

@@ -27,9 +27,9 @@ import torch
 
 from .. import ops
 from ..engine.batch import FlatBatch
-from ..engine.config import ChannelDeltaSpec, EngineConfig, LayerSpec, ModelConfig
+from ..engine.config import EngineConfig, GatedDeltaSpec, LayerSpec, ModelConfig
 from ..ops.reference import build_cos_sin
-from .channel_delta import ChannelDelta
+from .gated_delta import GatedDelta
 from .grouped_attention import GroupedAttention
 from .layout import Get, pad_to, round_up
 from .llama import _dtype_of
@@ -41,9 +41,9 @@ _NORM_OFFSET = 1.0
 class TezinexLayer:
     def __init__(self, spec: LayerSpec, cfg: ModelConfig, tp_rank: int, tp_world: int):
         self.width = cfg.hidden_size
-        self.recurrent = isinstance(spec.mixer, ChannelDeltaSpec)
+        self.recurrent = isinstance(spec.mixer, GatedDeltaSpec)
         if self.recurrent:
-            self.mixer = ChannelDelta(spec.mixer, self.width, cfg.rms_eps, tp_rank, tp_world)
+            self.mixer = GatedDelta(spec.mixer, self.width, cfg.rms_eps, tp_rank, tp_world)
         else:
             self.mixer = GroupedAttention(
                 spec.mixer, self.width, cfg.rms_eps, tp_rank, tp_world

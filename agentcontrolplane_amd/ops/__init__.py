@@ -143,17 +143,18 @@ DEPTH_AHEAD = 3
 
 def residual_norm(x, y, eps: float, y_norm=None, x_norm=None, out=None, *, center=True,
                   offset: float = 0.0, mult: float = 1.0, depth: Optional[Depth] = None,
-                  layer: int = 0, x_norm2=None, out2=None, experts=None):
+                  layer: int = 0, x_norm2=None, out2=None, experts=None, gate=None):
     """x += mult * y, or x += mult * rmsnorm(y) * y_norm, in the fp32 residual x, where
-    ``experts`` (rows [N, k, K], weights [N, k] fp32; no y_norm) joins y as
-    sum_j weights[:, j] * rows[:, j]; then, with ``depth``, x is filed as layer ``layer``'s state and replaced by
+    ``experts`` (rows [N, k, K], weights [N, k] fp32) joins y as
+    sum_j weights[:, j] * rows[:, j] and then ``gate`` [N, K] (row-strided) multiplies it
+    by its sigmoid; then, with ``depth``, x is filed as layer ``layer``'s state and replaced by
     sum_j coef[layer, j] * states[j] (layers in order: later ones use sums made by
     earlier ones); then out = norm(x) * x_norm, or x itself without x_norm.  The norm
     of x is a layer norm, an RMS norm if not ``center``; ``offset`` is added to the
     norm weights.  out2 is the same norm under the weight x_norm2."""
     return _impl(x).residual_norm(
         x, y, eps, y_norm, x_norm, out, center, offset, mult, depth, layer, x_norm2, out2,
-        experts,
+        experts, gate,
     )
 
 
@@ -269,7 +270,8 @@ def attention_inputs(proj, heads: int, dim: int, vdim: int, k_cache, v_cache, ba
 
     conv [taps, channels]: causal convolution per channel; the last inputs of a
         sequence are kept by position in its slot of ``ring`` [slots, taps, channels]
-    q_norm, k_norm [d], v_norm: RMS norm per head over dim or vdim
+    q_norm, k_norm [d], v_norm: RMS norm per head over dim or vdim; [heads * d] and
+        [G * d]: over all heads at once (no conv, no v_norm)
     cos_sin [2, P, n]: rotate a query's and key's first n pairs (2i, 2i + 1)
     head_mult [heads] fp32, q_temp (coef, every): queries times the head's factor, and
         times 1 + coef ln(floor((p + 1) / every) + 1) at position p"""
@@ -280,28 +282,33 @@ def attention_inputs(proj, heads: int, dim: int, vdim: int, k_cache, v_cache, ba
 
 
 def grouped_attention(q, k_cache, v_cache, batch, scale: float, cap, window, keep_first: int,
-                      sink, out, bias=None, sigmoid: bool = False, gate=None):
+                      sink, out, bias=None, sigmoid: bool = False, gate=None, chunk=None,
+                      talk=None):
     """Attention of a FlatBatch's rows over the paged cache; query head n uses
-    key/value head n // (H / G).  Scores are capped if ``cap``; a query sees itself
-    and the ``window`` - 1 tokens before it (None = all) and the ``keep_first``
-    first tokens; ``sink`` [H] (fp32) or None joins the softmax denominator.
+    key/value head n // (H / G).  ``talk`` [H, H] (fp32) mixes the scores over the heads:
+    head h's are sum_g talk[h, g] * head g's.  Scores are capped if ``cap``; a query sees
+    itself and the ``window`` - 1 tokens before it (None = all) and the ``keep_first``
+    first tokens, with ``chunk`` (no keep_first) only those of its own chunk, position
+    // chunk; ``sink`` [H] (fp32) or None joins the softmax denominator.
     ``bias`` [H, D] (fp32) adds bias[h, min(distance, D - 1)] to the capped scores;
     ``sigmoid``: weights are the scores' sigmoids, not a softmax; ``gate`` [N, H]
     (row-strided) multiplies a head's output by its sigmoid.
     q [N, H, d], out [N, H, e], both row-strided."""
     return _impl(q).grouped_attention(
         q, k_cache, v_cache, batch, scale, cap, window, keep_first, sink, out, bias, sigmoid,
-        gate,
+        gate, chunk, talk,
     )
 
 
 # -------------------------------------------------------------------- experts
 
 
-def moe_route(h, router, bias, top: int):
+def moe_route(h, router, bias, top: int, sigmoid: bool = False, scale: float = 1.0):
     """The ``top`` experts with the largest logits router @ h + bias (fp32) of every row:
-    ids [N, top] int32 and the softmax over the chosen logits [N, top] fp32."""
-    return _impl(h).moe_route(h, router, bias, top)
+    ids [N, top] int32 and scale * the softmax over the chosen logits [N, top] fp32.
+    ``sigmoid``: the choice is by sigmoid(router @ h) + bias, the weights are
+    scale * the chosen sigmoids over their sum."""
+    return _impl(h).moe_route(h, router, bias, top, sigmoid, scale)
 
 
 def moe_experts(h, gate_up, down, ids, glu):
@@ -313,17 +320,18 @@ def moe_experts(h, gate_up, down, ids, glu):
 # ----------------------------------------------------------------- delta rule
 
 
-def channel_delta(qkv, conv, b, z, A_log, dt_bias, gate, norm, eps: float, unit_eps: float,
-                  kv_heads: int, state, conv_state, batch):
+def gated_delta(qkv, conv, b, z, A_log, dt_bias, gate, norm, eps: float, unit_eps: float,
+                kv_heads: int, state, conv_state, batch, gate_silu: bool = False):
     """Gated delta rule over a FlatBatch's rows, each sequence from the state in its
     slot (zero at position 0), which is advanced.  Row-strided inputs: qkv
     [N, 2*G*D + H*V] before the convolution, b [N, H] before its sigmoid, z [N, H*D]
-    the decays' input, gate [N, H*V] before its sigmoid.  conv [channels, taps];
-    fp32: A_log [H], dt_bias [H*D], norm [V], state [slots, H, D, V]; conv_state
-    [slots, taps, channels], the last convolution inputs in a ring by position.  Returns [N, H*V]: normed per head and gated."""
-    return _impl(qkv).channel_delta(
+    or [N, H] (one decay per head) the decays' input, gate [N, H*V] before its sigmoid or
+    silu.  conv [channels, taps]; fp32: A_log [H], dt_bias like z, norm [V], state
+    [slots, H, D, V]; conv_state [slots, taps, channels], the last convolution inputs in a
+    ring by position.  Returns [N, H*V]: normed per head and gated."""
+    return _impl(qkv).gated_delta(
         qkv, conv, b, z, A_log, dt_bias, gate, norm, eps, unit_eps, kv_heads, state,
-        conv_state, batch,
+        conv_state, batch, gate_silu,
     )
 
 

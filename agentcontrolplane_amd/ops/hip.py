@@ -436,7 +436,7 @@ def _step_threads(D: int, V: int, workgroups: int) -> int:
     return 1024
 
 
-def channel_delta(qkv, conv, b, z, A_log, dt_bias, gate, norm, eps, unit_eps, kv_heads,
+def gated_delta(qkv, conv, b, z, A_log, dt_bias, gate, norm, eps, unit_eps, kv_heads,
                   state, conv_state, batch):
     H, D, V = state.shape[1:]
     out = torch.empty(gate.shape, dtype=qkv.dtype, device=qkv.device)

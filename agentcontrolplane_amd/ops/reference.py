@@ -170,12 +170,14 @@ def layernorm(x, weight, eps: float, dtype):
 
 def residual_norm(x, y, eps: float, y_norm=None, x_norm=None, out=None, center=True,
                   offset=0.0, mult=1.0, depth=None, layer=0, x_norm2=None, out2=None,
-                  experts=None):
+                  experts=None, gate=None):
     if y is not None:
         yf = y.float()
         if experts is not None:
             rows, weights = experts
             yf = yf + (rows.float() * weights.unsqueeze(-1)).sum(1)
+        if gate is not None:
+            yf = yf * torch.sigmoid(gate.float())
         if y_norm is not None:
             yf = yf * torch.rsqrt(yf.pow(2).mean(-1, keepdim=True) + eps)
             yf = yf * (offset + y_norm.float())
@@ -346,6 +348,12 @@ def attention_inputs(proj, heads, dim, vdim, k_cache, v_cache, batch, eps, conv,
     N, d, e, G = proj.shape[0], k_cache.shape[-1], v_cache.shape[-1], k_cache.shape[2]
     x = proj.float() if conv is None else _short_conv(proj, conv, ring, batch)
     q, k, v = x.split([heads * d, G * d, G * e], 1)
+    if q_norm is not None and q_norm.numel() > d:  # over all heads; the padding is zero
+        q, k = (
+            t * torch.rsqrt(t.pow(2).sum(-1, keepdim=True) / (n * dim) + eps) * w.float()
+            for t, n, w in ((q, heads, q_norm), (k, G, k_norm))
+        )
+        q_norm = None
     q, k, v = q.reshape(N, heads, d), k.reshape(N, G, d), v.reshape(N, G, e)
 
     def rms(t, size):  # the padding is zero
@@ -372,7 +380,7 @@ def attention_inputs(proj, heads, dim, vdim, k_cache, v_cache, batch, eps, conv,
 
 
 def _grouped_attention_seq(q, k_cache, v_cache, block_table, ctx_len: int, scale, cap, window,
-                           keep_first, sink, bias, sigmoid):
+                           keep_first, sink, bias, sigmoid, chunk, talk):
     """One sequence's rows at positions ctx_len..; q [L, H, d] -> fp32 [L, H, e]."""
     L, H, bs = q.shape[0], q.shape[1], k_cache.shape[1]
     j = torch.arange(ctx_len + L, device=q.device)
@@ -381,6 +389,8 @@ def _grouped_attention_seq(q, k_cache, v_cache, block_table, ctx_len: int, scale
     k = _flat(k_cache)[rows].float().repeat_interleave(group, 1).transpose(0, 1)
     v = _flat(v_cache)[rows].float().repeat_interleave(group, 1).transpose(0, 1)
     scores = torch.matmul(q.float().transpose(0, 1), k.transpose(1, 2)) * scale  # [H, L, S]
+    if talk is not None:
+        scores = torch.matmul(talk, scores.flatten(1)).view_as(scores)
     if cap is not None:
         scores = cap * torch.tanh(scores / cap)
     i = torch.arange(ctx_len, ctx_len + L, device=q.device).view(-1, 1)
@@ -389,6 +399,8 @@ def _grouped_attention_seq(q, k_cache, v_cache, block_table, ctx_len: int, scale
     hidden = j > i
     if window is not None:
         hidden |= ((i - j) >= window) & (j >= keep_first)
+    if chunk is not None:
+        hidden |= (i // chunk) != (j // chunk)
     scores = scores.masked_fill(hidden, float("-inf"))
     if sigmoid:
         probs = torch.sigmoid(scores)
@@ -398,11 +410,11 @@ def _grouped_attention_seq(q, k_cache, v_cache, block_table, ctx_len: int, scale
 
 
 def grouped_attention(q, k_cache, v_cache, batch, scale: float, cap, window, keep_first: int,
-                      sink, out, bias=None, sigmoid=False, gate=None):
+                      sink, out, bias=None, sigmoid=False, gate=None, chunk=None, talk=None):
     for row, n, ctx, _, pages in _portions(batch):
         y = _grouped_attention_seq(
             q[row : row + n], k_cache, v_cache, pages, ctx, scale, cap, window, keep_first, sink,
-            bias, sigmoid,
+            bias, sigmoid, chunk, talk,
         )
         if gate is not None:
             y = y * torch.sigmoid(gate[row : row + n].float()).unsqueeze(-1)
@@ -412,12 +424,14 @@ def grouped_attention(q, k_cache, v_cache, batch, scale: float, cap, window, kee
 # -------------------------------------------------------------------- experts
 
 
-def moe_route(h, router, bias, top: int):
+def moe_route(h, router, bias, top: int, sigmoid=False, scale=1.0):
     z = torch.matmul(h.float(), router.float().t())
-    if bias is not None:
-        z = z + bias
-    best = torch.topk(z, top, -1)
-    return best.indices.int(), torch.softmax(best.values, -1)
+    s = torch.sigmoid(z) if sigmoid else z
+    best = torch.topk(s if bias is None else s + bias, top, -1)
+    if not sigmoid:
+        return best.indices.int(), scale * torch.softmax(best.values, -1)
+    w = s.gather(-1, best.indices)
+    return best.indices.int(), scale * w / (w.sum(-1, keepdim=True) + 1e-20)
 
 
 def moe_experts(h, gate_up, down, ids, glu):
@@ -436,7 +450,8 @@ def moe_experts(h, gate_up, down, ids, glu):
 # ----------------------------------------------------------------- delta rule
 
 
-def _channel_delta_seq(qkv, conv, b, z, A_log, dt_bias, gate, norm, eps, unit_eps, G, S, tail):
+def _gated_delta_seq(qkv, conv, b, z, A_log, dt_bias, gate, norm, eps, unit_eps, G, S, tail,
+                     gate_silu):
     """One sequence's rows from state S [H, D, V] and convolution inputs tail
     [taps - 1, C]; returns the rows and S after them."""
     T, (H, D, V), taps = qkv.shape[0], S.shape, conv.shape[1]
@@ -452,7 +467,8 @@ def _channel_delta_seq(qkv, conv, b, z, A_log, dt_bias, gate, norm, eps, unit_ep
 
     q, k, v = unit(q) * D ** -0.5, unit(k), v.reshape(T, H, V)
     beta = torch.sigmoid(b.float())
-    step = torch.nn.functional.softplus((z.float() + dt_bias).view(T, H, D), threshold=40.0)
+    # one decay per head and channel, or one per head
+    step = torch.nn.functional.softplus((z.float() + dt_bias).view(T, H, -1), threshold=40.0)
     g = torch.exp(-torch.exp(A_log).view(H, 1) * step)
     out = torch.empty(T, H, V, device=S.device)
     for t in range(T):
@@ -461,12 +477,14 @@ def _channel_delta_seq(qkv, conv, b, z, A_log, dt_bias, gate, norm, eps, unit_ep
         S = S + k[t].unsqueeze(-1) * u.unsqueeze(1)
         out[t] = torch.matmul(q[t].unsqueeze(1), S).squeeze(1)
     out = out * torch.rsqrt(out.pow(2).mean(-1, keepdim=True) + eps) * norm
-    out = out.reshape(T, H * V) * torch.sigmoid(gate.float())
+    gate = gate.float()
+    gate = torch.nn.functional.silu(gate) if gate_silu else torch.sigmoid(gate)
+    out = out.reshape(T, H * V) * gate
     return out.to(qkv.dtype), S
 
 
-def channel_delta(qkv, conv, b, z, A_log, dt_bias, gate, norm, eps, unit_eps, kv_heads,
-                  state, conv_state, batch):
+def gated_delta(qkv, conv, b, z, A_log, dt_bias, gate, norm, eps, unit_eps, kv_heads,
+                state, conv_state, batch, gate_silu=False):
     out = torch.empty(gate.shape, dtype=qkv.dtype, device=qkv.device)
     runs, row, taps = [], 0, conv.shape[1]
     for m in batch.prefills:
@@ -481,9 +499,9 @@ def channel_delta(qkv, conv, b, z, A_log, dt_bias, gate, norm, eps, unit_eps, kv
         tail = torch.zeros(taps - 1, qkv.shape[1], dtype=qkv.dtype, device=qkv.device)
         for i in range(1, min(taps - 1, ctx) + 1):  # the ring's entry of position p is p % taps
             tail[-i] = ring[(ctx - i) % taps]
-        out[r], state[slot] = _channel_delta_seq(
+        out[r], state[slot] = _gated_delta_seq(
             qkv[r], conv, b[r], z[r], A_log, dt_bias, gate[r], norm, eps, unit_eps, kv_heads,
-            S, tail,
+            S, tail, gate_silu,
         )
         for i in range(max(0, n - taps), n):
             ring[(ctx + i) % taps] = qkv[row + i]

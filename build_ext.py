@@ -42,7 +42,7 @@ def build(verbose: bool = False) -> str:
         os.path.join(CSRC, "attn_inputs.hip"),
         os.path.join(CSRC, "experts.hip"),
         os.path.join(CSRC, "experts_gemm.hip"),
-        os.path.join(CSRC, "channel_delta.hip"),
+        os.path.join(CSRC, "gated_delta.hip"),
         os.path.join(CSRC, "sampling.hip"),
         os.path.join(CSRC, "sampling_fullvocab.hip"),
     ]

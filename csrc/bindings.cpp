@@ -10,7 +10,7 @@
 #include <cmath>
 
 #include "attn_inputs.h"
-#include "channel_delta.h"
+#include "gated_delta.h"
 #include "experts.h"
 #include "grouped_attn.h"
 #include "latent_attn.h"
@@ -1031,7 +1031,7 @@ static DeltaArgs delta_args(const torch::Tensor& out, const torch::Tensor& qkv,
   return a;
 }
 
-// The rows of every chunk; y, unit, g, o: workspace (channel_delta.h)
+// The rows of every chunk; y, unit, g, o: workspace (gated_delta.h)
 static void delta_prompts(torch::Tensor out, torch::Tensor qkv, torch::Tensor conv,
                           torch::Tensor b, torch::Tensor z, torch::Tensor A_log,
                           torch::Tensor dt_bias, torch::Tensor gate, torch::Tensor norm,

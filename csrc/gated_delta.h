@@ -1,4 +1,4 @@
-// Launch arguments of the gated delta rule (channel_delta.hip).
+// Launch arguments of the gated delta rule (gated_delta.hip).
 #pragma once
 #include <hip/hip_runtime.h>
 

@@ -19,7 +19,7 @@
 // never hits an entry that the token's own convolution reads, whichever workgroup
 // comes first.
 #include "common_t.h"
-#include "channel_delta.h"
+#include "gated_delta.h"
 
 DEV float silu_f(float x) { return x * __builtin_amdgcn_rcpf(1.f + __expf(-x)); }
 

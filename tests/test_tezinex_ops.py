@@ -313,7 +313,7 @@ class DeltaCase:
         pad = -(-self.C // 16) * 16
         wide = torch.zeros(len(rows), pad + 16 * -(-H // 16), dtype=self.dtype, device=self.device)
         wide[:, : self.C], wide[:, pad : pad + H] = dev(self.qkv), dev(self.b)
-        out = ops.channel_delta(
+        out = ops.gated_delta(
             wide[:, : self.C], self.conv.to(self.device), wide[:, pad : pad + H], dev(self.z),
             self.A_log.to(self.device), self.dt_bias.to(self.device), dev(self.gate),
             self.norm.to(self.device), self.eps, self.unit_eps, G, self.state, self.ring, batch,
