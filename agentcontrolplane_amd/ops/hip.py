@@ -115,19 +115,19 @@ def layernorm(x, weight, eps: float, dtype):
     out = torch.empty(x.shape, dtype=dtype, device=x.device)
     _C.residual_norm(
         x, None, None, weight, out, eps, True, 0.0, 1.0, None, None, None, 0, None, None, None,
-        None,
+        None, None,
     )
     return out
 
 
 def residual_norm(x, y, eps: float, y_norm=None, x_norm=None, out=None, center=True,
                   offset=0.0, mult=1.0, depth=None, layer=0, x_norm2=None, out2=None,
-                  experts=None):
+                  experts=None, gate=None):
     states, coef, partial = depth or (None, None, None)
     rows, weights = experts or (None, None)
     _C.residual_norm(
         x, y, y_norm, x_norm, out, eps, center, offset, mult, states, coef, partial, layer,
-        x_norm2, out2, rows, weights,
+        x_norm2, out2, rows, weights, gate,
     )
 
 
@@ -345,12 +345,12 @@ def attention_inputs(proj, heads, dim, vdim, k_cache, v_cache, batch, eps, conv,
 
 
 def grouped_attention(q, k_cache, v_cache, batch, scale: float, cap, window, keep_first: int,
-                      sink, out, bias=None, sigmoid=False, gate=None):
+                      sink, out, bias=None, sigmoid=False, gate=None, chunk=None, talk=None):
     from . import LATENT_HEADS
 
     H, d, v, G = q.shape[1], q.shape[2], out.shape[2], k_cache.shape[2]
-    rest = (scale, cap or 0.0, window or _NO_WINDOW, keep_first, sigmoid)
-    tiled = (q.dtype == torch.bfloat16 and d in LATENT_HEADS and v in LATENT_HEADS
+    rest = (scale, cap or 0.0, window or _NO_WINDOW, chunk or _NO_WINDOW, keep_first, sigmoid)
+    tiled = (talk is None and q.dtype == torch.bfloat16 and d in LATENT_HEADS and v in LATENT_HEADS
              and not (sigmoid and cap))
     P = batch.num_prefill_tokens
 
@@ -361,8 +361,8 @@ def grouped_attention(q, k_cache, v_cache, batch, scale: float, cap, window, kee
         meta = batch.prefill_meta(128 if tiled else 1)
         _C.grouped_attn(
             out[:P], q[:P], k_cache, v_cache, meta.block_tables, meta.seq_lens, meta.ctx_lens,
-            meta.row_starts, meta.tile_seq, meta.tile_q0, sink, bias, gates(slice(0, P)), None,
-            None, *rest, _PREFILL if tiled else _PLAIN, 1, 1,
+            meta.row_starts, meta.tile_seq, meta.tile_q0, sink, bias, gates(slice(0, P)), talk,
+            None, None, *rest, _PREFILL if tiled else _PLAIN, 1, 1,
         )
     if not batch.num_decode:
         return
@@ -372,7 +372,7 @@ def grouped_attention(q, k_cache, v_cache, batch, scale: float, cap, window, kee
         most = 8 if d + v <= 256 else 4  # query heads a workgroup holds
         gm = next((n for n in (1, 2, 4) if n >= min(H // G, most)), most)
         # workgroups that fill the chip; every split has work for its 16 lane groups
-        keys = min(tables.shape[1] * k_cache.shape[1], rest[2] + keep_first)
+        keys = min(tables.shape[1] * k_cache.shape[1], rest[2] + keep_first, rest[3])
         groups = batch.num_decode * G * -(-(H // G) // gm)
         n_split = max(1, min(_MAX_SPLIT, 1024 // groups, -(-keys // 128)))
     if n_split > 1:
@@ -380,17 +380,18 @@ def grouped_attention(q, k_cache, v_cache, batch, scale: float, cap, window, kee
         ml = torch.empty(2 * n_split * rows, dtype=torch.float32, device=q.device)
     _C.grouped_attn(
         out[P:], q[P:], k_cache, v_cache, tables, batch.decode_lens_i32(), None, None, None,
-        None, sink, bias, gates(slice(P, None)), part, ml, *rest, _DECODE if tiled else _PLAIN, gm, n_split,
+        None, sink, bias, gates(slice(P, None)), talk, part, ml, *rest,
+        _DECODE if tiled else _PLAIN, gm, n_split,
     )
 
 
 # -------------------------------------------------------------------- experts
 
 
-def moe_route(h, router, bias, top: int):
+def moe_route(h, router, bias, top: int, sigmoid=False, scale=1.0):
     ids = torch.empty(h.shape[0], top, dtype=torch.int32, device=h.device)
     weights = torch.empty(h.shape[0], top, dtype=torch.float32, device=h.device)
-    _C.moe_route(ids, weights, h, router, bias)
+    _C.moe_route(ids, weights, h, router, bias, sigmoid, scale)
     return ids, weights
 
 
@@ -437,7 +438,7 @@ def _step_threads(D: int, V: int, workgroups: int) -> int:
 
 
 def gated_delta(qkv, conv, b, z, A_log, dt_bias, gate, norm, eps, unit_eps, kv_heads,
-                  state, conv_state, batch):
+                state, conv_state, batch, gate_silu=False):
     H, D, V = state.shape[1:]
     out = torch.empty(gate.shape, dtype=qkv.dtype, device=qkv.device)
     P = batch.num_prefill_tokens
@@ -457,13 +458,14 @@ def gated_delta(qkv, conv, b, z, A_log, dt_bias, gate, norm, eps, unit_eps, kv_h
         cpl = 2 if seqs * H * V >= 4 * 4096 else 1
         _C.delta_prompts(
             *rows(slice(0, P)), meta.seq_lens, meta.state_slots, kv_heads, eps, unit_eps,
-            meta.ctx_lens, meta.row_starts, meta.tile_seq, meta.tile_q0,
-            space(qkv.shape[1], qkv.dtype), space(3 * kv_heads), space(H * D), space(H * V), cpl,
+            gate_silu, meta.ctx_lens, meta.row_starts, meta.tile_seq, meta.tile_q0,
+            space(qkv.shape[1], qkv.dtype), space(3 * kv_heads),
+            None if z.shape[1] == H else space(H * D), space(H * V), cpl,
         )
     if batch.num_decode:
         _C.delta_step(
             *rows(slice(P, None)), batch.decode_lens_i32(), batch.decode_state_slots, kv_heads,
-            eps, unit_eps, _step_threads(D, V, batch.num_decode * H),
+            eps, unit_eps, gate_silu, _step_threads(D, V, batch.num_decode * H),
         )
     return out
 

@@ -1,11 +1,12 @@
 // What happens to q, k and v between their projection and attention, in one pass
-// (gfx950): short convolution, norms per head, rotation, query temperature; keys and
-// values go to their cache slots.
+// (gfx950): short convolution, norms per head or over all heads, rotation, query
+// temperature; keys and values go to their cache slots.
 //
 // A thread owns VW channels of one row.  Heads start at multiples of their size, so a
 // head is a group of d / VW neighbouring lanes, which reduce by shuffles; sections are
 // aligned so that no group straddles a wave.  Rotations pair dimension 2i with 2i + 1,
-// both in one thread.  Everything between load and store is fp32.
+// both in one thread.  Norms over all heads take a workgroup per row.  Everything between
+// load and store is fp32.
 //
 // The convolutions' inputs are kept in a ring by position.  A row that is alone in its
 // sequence's step writes an entry that its own convolution does not read, at once;
@@ -62,17 +63,19 @@ DEV void to_ring(const AttnInputsArgs& a, int64_t n, int p, int64_t state, int c
   *(Pack<T, VW>*)((T*)a.ring + (state * a.taps + p % a.taps) * a.C + c) = row_input<T, VW>(a, n, c);
 }
 
-// y: VW channels from i of a head whose squares sum to ss; sect 0 q, 1 k, 2 v
+// y: VW channels from i of a head whose norm's squares sum to ss; sect 0 q, 1 k, 2 v
 template <typename T, int VW>
 DEV void finish(const AttnInputsArgs& a, int64_t n, int p, int sect, int head, int i, float ss,
                 float* y) {
   if (sect < 2 ? a.q_norm != nullptr : a.v_norm) {
-    const float inv = rsqrtf(ss / (sect < 2 ? a.dim : a.vdim) + a.eps);
+    const int heads = !a.row_norm ? 1 : sect == 0 ? a.H : a.G;
+    const float inv = rsqrtf(ss / (sect < 2 ? heads * a.dim : a.vdim) + a.eps);
 #pragma unroll
     for (int k = 0; k < VW; ++k) y[k] *= inv;
     if (sect < 2) {
       float w[VW];
-      load_f<VW>(w, (const T*)(sect == 0 ? a.q_norm : a.k_norm) + i);
+      const int at = a.row_norm ? head * a.d + i : i;
+      load_f<VW>(w, (const T*)(sect == 0 ? a.q_norm : a.k_norm) + at);
 #pragma unroll
       for (int k = 0; k < VW; ++k) y[k] *= w[k];
     }
@@ -220,6 +223,46 @@ __global__ __launch_bounds__(256) void attn_inputs_any_kernel(const AttnInputsAr
   }
 }
 
+// Norms over all heads: a workgroup per row, a thread has every blockDim.x-th VW
+// channels, at most PER of them.  No convolution, no norm of v.
+template <typename T, int VW, int PER>
+__global__ __launch_bounds__(1024) void attn_inputs_row_kernel(const AttnInputsArgs a) {
+  __shared__ float scratch[2][16];
+  const int64_t n = blockIdx.x;
+  const int p = (int)a.positions[n];
+  const int units = a.C / VW, q_end = a.H * a.d, k_end = q_end + a.G * a.d;
+  Pack<T, VW> x[PER];
+#pragma unroll
+  for (int j = 0; j < PER; ++j) {
+    const int u = threadIdx.x + j * blockDim.x;
+    x[j] = row_input<T, VW>(a, n, min(u, units - 1) * VW);
+  }
+  float qq = 0.f, kk = 0.f;
+#pragma unroll
+  for (int j = 0; j < PER; ++j) {
+    const int c = (threadIdx.x + j * blockDim.x) * VW;
+    float ss = 0.f;
+#pragma unroll
+    for (int k = 0; k < VW; ++k) ss += to_f(x[j].v[k]) * to_f(x[j].v[k]);
+    qq += c < q_end ? ss : 0.f;
+    kk += c >= q_end && c < k_end ? ss : 0.f;
+  }
+  qq = block_sum(qq, scratch[0]);
+  kk = block_sum(kk, scratch[1]);
+#pragma unroll
+  for (int j = 0; j < PER; ++j) {
+    int c = (threadIdx.x + j * blockDim.x) * VW;
+    if (c >= a.C) return;
+    const int sect = c < q_end ? 0 : c < k_end ? 1 : 2;
+    c -= sect == 0 ? 0 : sect == 1 ? q_end : k_end;
+    const int size = sect < 2 ? a.d : a.v, head = c / size;
+    float y[VW];
+#pragma unroll
+    for (int k = 0; k < VW; ++k) y[k] = to_f(x[j].v[k]);
+    finish<T, VW>(a, n, p, sect, head, c - head * size, sect == 0 ? qq : kk, y);
+  }
+}
+
 // grid (parts of a row, ring rows)
 template <typename T, int VW>
 __global__ __launch_bounds__(256) void attn_ring_kernel(const AttnInputsArgs a) {
@@ -241,6 +284,18 @@ template <typename T, int VW>
 static void launch(const AttnInputsArgs& a, hipStream_t stream) {
   const int lq = a.d / VW, lv = a.v / VW;
   auto fits = [](int lanes) { return lanes <= 64 && (lanes & (lanes - 1)) == 0; };
+  if (a.row_norm) {
+    const int units = a.C / VW;
+    int threads = 256;
+    while (threads < 1024 && units > 4 * threads) threads *= 2;
+    if (units <= threads)
+      attn_inputs_row_kernel<T, VW, 1><<<a.N, threads, 0, stream>>>(a);
+    else if (units <= 4 * threads)
+      attn_inputs_row_kernel<T, VW, 4><<<a.N, threads, 0, stream>>>(a);
+    else
+      attn_inputs_row_kernel<T, VW, 16><<<a.N, threads, 0, stream>>>(a);
+    return;
+  }
   if (fits(lq) && fits(lv)) {
     const int v_at = ((a.H + a.G) * lq + lv - 1) / lv * lv;
     const int units = (v_at + a.G * lv + 63) / 64 * 64;

@@ -48,7 +48,7 @@ void launch_embed_positions(bool, float*, float*, const int64_t*, const int64_t*
                             const float*, float, int, int, int64_t, int64_t, hipStream_t);
 void launch_attn_inputs(bool, const AttnInputsArgs*, hipStream_t);
 void launch_moe_route(bool, int*, float*, const void*, const void*, const float*, int, int, int,
-                      int, int64_t, hipStream_t);
+                      int, int64_t, bool, float, hipStream_t);
 void launch_moe_group(int*, int*, int*, int*, const int*, int, int, hipStream_t);
 void launch_experts_small(bool, const ExpertsArgs*, int, hipStream_t);
 void launch_experts_f32(bool, const ExpertsArgs*, hipStream_t);
@@ -311,7 +311,7 @@ static void residual_norm(torch::Tensor x, OptTensor y, OptTensor y_norm, OptTen
                           OptTensor out, double eps, bool center, double offset, double mult,
                           OptTensor states, OptTensor coef, OptTensor partial,
                           int64_t layer, OptTensor x_norm2, OptTensor out2, OptTensor rows,
-                          OptTensor weights) {
+                          OptTensor weights, OptTensor gate) {
   CHECK_CUDA(x); CHECK_CONT(x);
   TORCH_CHECK(x.scalar_type() == at::kFloat && x.dim() == 2);
   TORCH_CHECK(y || out, "nothing to do");
@@ -327,7 +327,7 @@ static void residual_norm(torch::Tensor x, OptTensor y, OptTensor y_norm, OptTen
   f.offset = (float)offset;
   f.mult = (float)mult;
   if (rows) {
-    TORCH_CHECK(y && !y_norm && weights && rows->dim() == 3, "expert rows");
+    TORCH_CHECK(y && weights && rows->dim() == 3, "expert rows");
     f.top = rows->size(1);
     TORCH_CHECK(rows->size(0) == n && rows->size(2) == w && rows->scalar_type() == dt &&
                 weights->dim() == 2 && weights->size(0) == n && weights->size(1) == f.top &&
@@ -335,6 +335,12 @@ static void residual_norm(torch::Tensor x, OptTensor y, OptTensor y_norm, OptTen
     CHECK_CUDA((*rows)); CHECK_CONT((*rows)); CHECK_CUDA((*weights)); CHECK_CONT((*weights));
     f.rows = rows->data_ptr();
     f.weights = weights->data_ptr<float>();
+  }
+  if (gate) {
+    TORCH_CHECK(y, "a gate belongs to y");
+    check_rows(*gate, dt, n, w);
+    f.gate = gate->data_ptr();
+    f.gate_stride = gate->stride(0);
   }
   if (out2) {
     TORCH_CHECK(out && x_norm && x_norm2, "second norm");
@@ -731,9 +737,9 @@ static void grouped_attn(torch::Tensor out, torch::Tensor q, torch::Tensor k_cac
                          torch::Tensor v_cache, torch::Tensor tables, torch::Tensor seq_lens,
                          OptTensor ctx_lens, OptTensor row_starts, OptTensor tile_seq,
                          OptTensor tile_q0, OptTensor sink, OptTensor bias, OptTensor gate,
-                         OptTensor part, OptTensor part_ml, double scale, double cap,
-                         int64_t window, int64_t keep, bool sigmoid, int64_t kind, int64_t gm,
-                         int64_t n_split) {
+                         OptTensor talk, OptTensor part, OptTensor part_ml, double scale,
+                         double cap, int64_t window, int64_t chunk, int64_t keep, bool sigmoid,
+                         int64_t kind, int64_t gm, int64_t n_split) {
   const auto dt = q.scalar_type();
   const bool bf16 = is_bf16(q);
   const int tokens = q.size(0), H = q.size(1), d = q.size(2), v = out.size(2);
@@ -748,6 +754,8 @@ static void grouped_attn(torch::Tensor out, torch::Tensor q, torch::Tensor k_cac
   TORCH_CHECK(tables.scalar_type() == at::kInt && tables.dim() == 2);
   const int seqs = tables.size(0);
   TORCH_CHECK(window > 0 && keep >= 0 && cap >= 0 && n_split >= 1 && n_split <= 64);
+  TORCH_CHECK(chunk > 0 && chunk <= (1 << 30) && (keep == 0 || chunk == (1 << 30)),
+              "chunks keep no first tokens");
   TORCH_CHECK(kind == 0 || bf16, "the matrix-core kernels take bf16");
   TORCH_CHECK(kind == 1 || n_split == 1, "only decode splits keys");
   TORCH_CHECK((kind == 2) <= (bool)tile_seq && !(kind == 1 && tile_seq), "tiles");
@@ -779,6 +787,11 @@ static void grouped_attn(torch::Tensor out, torch::Tensor q, torch::Tensor k_cac
     a.gate = gate->data_ptr();
     a.gate_stride = gate->stride(0);
   }
+  if (talk) {
+    check_rows(*talk, at::kFloat, H, H); CHECK_CONT((*talk));
+    a.talk = talk->data_ptr<float>();
+  }
+  a.chunk = (int)chunk;
   a.sigmoid = sigmoid;
   a.out_stride = out.stride(0);
   a.tables = tables.data_ptr<int>();
@@ -805,6 +818,7 @@ static void grouped_attn(torch::Tensor out, torch::Tensor q, torch::Tensor k_cac
   a.rows = tokens * H;
   a.scale = (float)scale;
   a.cap = (float)cap;
+  TORCH_CHECK(!talk || kind == 0, "mixed scores");
   const bool ok = kind == 2   ? launch_grouped_prefill(&a, d, v, cur_stream())
                   : kind == 1 ? launch_grouped_decode(&a, d, v, seqs, (int)gm, cur_stream())
                               : launch_grouped_plain(bf16, &a, d, v, tokens, cur_stream());
@@ -858,7 +872,12 @@ static void attention_inputs(torch::Tensor q, torch::Tensor k_cache, torch::Tens
   }
   if (q_norm) {
     TORCH_CHECK(k_norm, "q and k are normed alike");
-    check_vec(*q_norm, dt, a.d); check_vec(*k_norm, dt, a.d);
+    // weights of all heads: a norm over all heads
+    a.row_norm = q_norm->numel() != a.d;
+    check_vec(*q_norm, dt, (a.row_norm ? a.H : 1) * a.d);
+    check_vec(*k_norm, dt, (a.row_norm ? a.G : 1) * a.d);
+    TORCH_CHECK(!a.row_norm || (!conv && !v_norm && a.C <= 16 * 1024 * (bf16 ? 8 : 4)),
+                "norms over all heads");
     a.q_norm = q_norm->data_ptr();
     a.k_norm = k_norm->data_ptr();
   }
@@ -895,7 +914,7 @@ static void attention_inputs(torch::Tensor q, torch::Tensor k_cache, torch::Tens
 // ---- mixture of experts
 
 static void moe_route(torch::Tensor ids, torch::Tensor weights, torch::Tensor h, torch::Tensor w,
-                      OptTensor bias) {
+                      OptTensor bias, bool sigmoid, double scale) {
   const int N = h.size(0), K = h.size(1), E = w.size(0), top = ids.size(1);
   check_rows(h, h.scalar_type(), N, K); check_aligned(h);
   check_rows(w, h.scalar_type(), E, K); CHECK_CONT(w);
@@ -906,7 +925,7 @@ static void moe_route(torch::Tensor ids, torch::Tensor weights, torch::Tensor h,
   if (N == 0) return;
   launch_moe_route(is_bf16(h), ids.data_ptr<int>(), weights.data_ptr<float>(), h.data_ptr(),
                    w.data_ptr(), bias ? bias->data_ptr<float>() : nullptr, N, E, K, top,
-                   h.stride(0), cur_stream());
+                   h.stride(0), sigmoid, (float)scale, cur_stream());
 }
 
 // perm [n], offsets [E + 2]; tiles of EXPERT_TILE rows: at most ceil(n / tile) + E
@@ -981,7 +1000,7 @@ static DeltaArgs delta_args(const torch::Tensor& out, const torch::Tensor& qkv,
                             const torch::Tensor& norm, const torch::Tensor& state,
                             const torch::Tensor& ring, const torch::Tensor& seq_lens,
                             const torch::Tensor& slots, int64_t kv_heads, double eps,
-                            double unit_eps) {
+                            double unit_eps, bool gate_silu) {
   const auto dt = qkv.scalar_type();
   DeltaArgs a{};
   CHECK_CUDA(state); CHECK_CONT(state);
@@ -997,11 +1016,13 @@ static DeltaArgs delta_args(const torch::Tensor& out, const torch::Tensor& qkv,
   check_rows(qkv, dt, a.N, a.C);
   check_rows(conv, dt, a.C, a.taps); CHECK_CONT(conv);
   check_rows(b, dt, a.N, a.H);
-  check_rows(z, dt, a.N, (int64_t)a.H * a.D);
+  a.head_decay = z.size(1) == a.H;
+  const int64_t decays = (int64_t)a.H * (a.head_decay ? 1 : a.D);
+  check_rows(z, dt, a.N, decays);
   check_rows(gate, dt, a.N, (int64_t)a.H * a.V);
   check_rows(out, dt, a.N, (int64_t)a.H * a.V); CHECK_CONT(out);
   check_vec(A_log, at::kFloat, a.H);
-  check_vec(dt_bias, at::kFloat, (int64_t)a.H * a.D);
+  check_vec(dt_bias, at::kFloat, decays);
   check_vec(norm, at::kFloat, a.V);
   CHECK_CUDA(ring); CHECK_CONT(ring);
   TORCH_CHECK(ring.scalar_type() == dt && ring.dim() == 3 && ring.size(0) == state.size(0) &&
@@ -1028,6 +1049,7 @@ static DeltaArgs delta_args(const torch::Tensor& out, const torch::Tensor& qkv,
   a.eps = (float)eps;
   a.unit_eps = (float)unit_eps;
   a.q_scale = 1.f / std::sqrt((float)a.D);
+  a.gate_silu = gate_silu;
   return a;
 }
 
@@ -1037,18 +1059,21 @@ static void delta_prompts(torch::Tensor out, torch::Tensor qkv, torch::Tensor co
                           torch::Tensor dt_bias, torch::Tensor gate, torch::Tensor norm,
                           torch::Tensor state, torch::Tensor ring, torch::Tensor seq_lens,
                           torch::Tensor slots, int64_t kv_heads, double eps, double unit_eps,
-                          torch::Tensor ctx_lens, torch::Tensor row_starts,
+                          bool gate_silu, torch::Tensor ctx_lens, torch::Tensor row_starts,
                           torch::Tensor tile_seq, torch::Tensor tile_q0, torch::Tensor y,
-                          torch::Tensor unit, torch::Tensor g, torch::Tensor o, int64_t cpl) {
+                          torch::Tensor unit, OptTensor g, torch::Tensor o, int64_t cpl) {
   DeltaArgs a = delta_args(out, qkv, conv, b, z, A_log, dt_bias, gate, norm, state, ring,
-                           seq_lens, slots, kv_heads, eps, unit_eps);
+                           seq_lens, slots, kv_heads, eps, unit_eps, gate_silu);
   check_vec(y, qkv.scalar_type(), (int64_t)a.N * a.C);
   check_vec(unit, at::kFloat, (int64_t)a.N * a.G * 3);
-  check_vec(g, at::kFloat, (int64_t)a.N * a.H * a.D);
+  if (!a.head_decay) {
+    TORCH_CHECK(g, "workspace for the decays");
+    check_vec(*g, at::kFloat, (int64_t)a.N * a.H * a.D);
+    a.g = g->data_ptr<float>();
+  }
   check_vec(o, at::kFloat, (int64_t)a.N * a.H * a.V);
   a.y = y.data_ptr();
   a.unit = unit.data_ptr<float>();
-  a.g = g.data_ptr<float>();
   a.o = o.data_ptr<float>();
   a.n_tiles = tile_seq.numel();
   a.ctx_lens = opt_int(ctx_lens, a.seqs);
@@ -1066,9 +1091,9 @@ static void delta_step(torch::Tensor out, torch::Tensor qkv, torch::Tensor conv,
                        torch::Tensor dt_bias, torch::Tensor gate, torch::Tensor norm,
                        torch::Tensor state, torch::Tensor ring, torch::Tensor seq_lens,
                        torch::Tensor slots, int64_t kv_heads, double eps, double unit_eps,
-                       int64_t threads) {
+                       bool gate_silu, int64_t threads) {
   DeltaArgs a = delta_args(out, qkv, conv, b, z, A_log, dt_bias, gate, norm, state, ring,
-                           seq_lens, slots, kv_heads, eps, unit_eps);
+                           seq_lens, slots, kv_heads, eps, unit_eps, gate_silu);
   TORCH_CHECK(a.seqs == a.N && a.seqs <= 65535, "one token per sequence");
   TORCH_CHECK(threads % 64 == 0 && threads >= 64 && threads <= 1024 &&
               (a.V % 4 ? a.V : a.V / 4) <= threads, "threads");

@@ -13,8 +13,10 @@ typedef float f32x4_v __attribute__((ext_vector_type(4)));
 #define AHEAD 8      // turns whose ids are loaded together
 
 // The wave picks the ``top`` largest of logits[0 .. E) (overwritten), the lower index
-// among equals, and their softmax weights.
-static DEV void choose(float* logits, int E, int top, int* ids, float* weights) {
+// among equals, and their weights: scale times their softmax or, with ``scores``, times
+// the chosen scores over their sum.
+static DEV void choose(float* logits, const float* scores, int E, int top, float scale, int* ids,
+                       float* weights) {
   const int lane = threadIdx.x & 63;
   float mine = -INFINITY, first = 0.f;
   int my_id = 0;
@@ -38,16 +40,16 @@ static DEV void choose(float* logits, int E, int top, int* ids, float* weights) 
     at = min(at, E - 1);  // whatever the logits are, an id stays an id
     if (j == 0) first = best;
     if (lane == j) {
-      mine = best;
+      mine = scores ? scores[at] : best;
       my_id = at;
     }
     if (lane == (at & 63)) logits[at] = -INFINITY;
   }
-  const float w = lane < top ? expf(mine - first) : 0.f;
-  const float sum = wave_sum(w);
+  const float w = lane >= top ? 0.f : scores ? mine : expf(mine - first);
+  const float sum = wave_sum(w) + (scores ? 1e-20f : 0.f);
   if (lane < top) {
     ids[lane] = my_id;
-    weights[lane] = w / sum;
+    weights[lane] = scale * w / sum;
   }
 }
 
@@ -58,7 +60,7 @@ template <int NF>
 __global__ __launch_bounds__(1024) void route_mfma_kernel(
     int* __restrict__ ids, float* __restrict__ weights, const bf16_t* __restrict__ h,
     const bf16_t* __restrict__ w, const float* __restrict__ bias, const int N, const int E,
-    const int K, const int top, const int64_t h_stride) {
+    const int K, const int top, const int64_t h_stride, const bool sigmoid, const float scale) {
   extern __shared__ float part[];
   const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6, waves = blockDim.x >> 6;
   const int c = lane & 15, g = lane >> 4;
@@ -91,17 +93,18 @@ __global__ __launch_bounds__(1024) void route_mfma_kernel(
     }
   }
   __syncthreads();
-  // the first wave's part becomes the logits
+  // the first wave's part becomes the logits, the second's the scores
   for (int i = threadIdx.x; i < logits; i += blockDim.x) {
     const int e = i % E16;
-    float z = e < E ? (bias ? bias[e] : 0.f) : -INFINITY;
+    float z = 0.f;
     for (int p = 0; p < waves; ++p) z += part[(int64_t)p * logits + i];
-    part[i] = z;
+    if (sigmoid) part[logits + i] = z = 1.f / (1.f + expf(-z));
+    part[i] = e < E ? z + (bias ? bias[e] : 0.f) : -INFINITY;
   }
   __syncthreads();
   for (int t = wid; t < min(ROUTE_T, N - n0); t += waves)
-    choose(part + t * E16, E, top, ids + (int64_t)(n0 + t) * top,
-           weights + (int64_t)(n0 + t) * top);
+    choose(part + t * E16, sigmoid ? part + logits + t * E16 : nullptr, E, top, scale,
+           ids + (int64_t)(n0 + t) * top, weights + (int64_t)(n0 + t) * top);
 }
 
 // Any dtype: a workgroup per token, a wave per expert in turn.
@@ -109,18 +112,23 @@ template <typename T>
 __global__ __launch_bounds__(256) void route_plain_kernel(
     int* __restrict__ ids, float* __restrict__ weights, const T* __restrict__ h,
     const T* __restrict__ w, const float* __restrict__ bias, const int E, const int K,
-    const int top, const int64_t h_stride) {
-  extern __shared__ float part[];
+    const int top, const int64_t h_stride, const bool sigmoid, const float scale) {
+  extern __shared__ float part[];  // [2][E]
   const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
   const int64_t n = blockIdx.x;
   for (int e = wid; e < E; e += 4) {
     float z = 0.f;
     for (int k = lane; k < K; k += 64) z += to_f(h[n * h_stride + k]) * to_f(w[(int64_t)e * K + k]);
     z = wave_sum(z);
-    if (lane == 0) part[e] = z + (bias ? bias[e] : 0.f);
+    if (sigmoid) z = 1.f / (1.f + expf(-z));
+    if (lane == 0) {
+      part[E + e] = z;
+      part[e] = z + (bias ? bias[e] : 0.f);
+    }
   }
   __syncthreads();
-  if (wid == 0) choose(part, E, top, ids + n * top, weights + n * top);
+  if (wid == 0)
+    choose(part, sigmoid ? part + E : nullptr, E, top, scale, ids + n * top, weights + n * top);
 }
 
 // lanes of the wave whose id (``bits`` bits) equals this lane's
@@ -318,7 +326,7 @@ extern "C" {
 
 void launch_moe_route(bool bf16, int* ids, float* weights, const void* h, const void* w,
                       const float* bias, int N, int E, int K, int top, int64_t h_stride,
-                      hipStream_t stream) {
+                      bool sigmoid, float scale, hipStream_t stream) {
   const int E16 = (E + 15) & ~15;
   if (bf16 && E <= 128) {  // at most 64 KiB of partial logits
     // few workgroups: more waves share the weights' latency
@@ -327,13 +335,16 @@ void launch_moe_route(bool bf16, int* ids, float* weights, const void* h, const 
              : E16 <= 32 ? route_mfma_kernel<2>
                          : route_mfma_kernel<4>;
     k<<<(N + ROUTE_T - 1) / ROUTE_T, 64 * waves, waves * ROUTE_T * E16 * 4, stream>>>(
-        ids, weights, (const bf16_t*)h, (const bf16_t*)w, bias, N, E, K, top, h_stride);
+        ids, weights, (const bf16_t*)h, (const bf16_t*)w, bias, N, E, K, top, h_stride, sigmoid,
+        scale);
   } else if (bf16) {
-    route_plain_kernel<bf16_t><<<N, 256, E * 4, stream>>>(
-        ids, weights, (const bf16_t*)h, (const bf16_t*)w, bias, E, K, top, h_stride);
+    route_plain_kernel<bf16_t><<<N, 256, E * 8, stream>>>(
+        ids, weights, (const bf16_t*)h, (const bf16_t*)w, bias, E, K, top, h_stride, sigmoid,
+        scale);
   } else {
-    route_plain_kernel<float><<<N, 256, E * 4, stream>>>(
-        ids, weights, (const float*)h, (const float*)w, bias, E, K, top, h_stride);
+    route_plain_kernel<float><<<N, 256, E * 8, stream>>>(
+        ids, weights, (const float*)h, (const float*)w, bias, E, K, top, h_stride, sigmoid,
+        scale);
   }
 }
 

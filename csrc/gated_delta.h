@@ -7,10 +7,10 @@ struct DeltaArgs {
   const void* qkv;        // [N, C] before the convolution
   const void* conv;       // [C, taps]
   const void* b;          // [N, H]
-  const void* z;          // [N, H * D]
+  const void* z;          // [N, H * D], or [N, H] with head_decay
   const void* gate;       // [N, H * V]
   const float* A_log;     // [H]
-  const float* dt_bias;   // [H * D]
+  const float* dt_bias;   // like a row of z
   const float* norm;      // [V]
   float* state;           // [slots, H, D, V]
   void* ring;             // [slots, taps, C]: input of position p at p % taps
@@ -18,7 +18,7 @@ struct DeltaArgs {
   // workspace of the prompt kernels
   void* y;                // [N, C] convolved
   float* unit;            // [N, G, 3] factors that make q and k unit vectors, then q . k
-  float* g;               // [N, H * D] decays
+  float* g;               // [N, H * D] decays; null with head_decay
   float* o;               // [N, H, V] before the norm
   const int* seq_lens;    // [seqs] tokens including this step's
   const int* ctx_lens;    // [seqs] before this step; null: decode
@@ -29,4 +29,6 @@ struct DeltaArgs {
   int64_t qkv_stride, b_stride, z_stride, gate_stride;
   int H, G, D, V, C, taps, N, seqs, n_tiles;
   float eps, unit_eps, q_scale;
+  bool head_decay;        // one decay per head
+  bool gate_silu;         // gate silu(x), else sigmoid(x)
 };

@@ -1,14 +1,15 @@
-// Gated delta rule with a decay per head and key channel (gfx950).
+// Gated delta rule with a decay per head and key channel, or one per head (gfx950).
 //
 //   S <- diag(g) S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q
 //
 // per head, S [D, V] in fp32.  With k and q known ahead, both products of a token are
 // taken over the decayed state at once: o = (diag(g) S)^T q + (k . q) u, so a token
-// costs one reduction.  Everything in the recurrence is fp32 (the VALU's rate, since
+// costs one reduction.  One decay per head is a factor on both sums and needs no vector
+// of its own.  Everything in the recurrence is fp32 (the VALU's rate, since
 // the bf16 matrix cores would round q, k and S).
 //
 // Portions of a prompt, three launches:
-//   delta_inputs: short convolution + silu, unit factors, k . q, decays
+//   delta_inputs: short convolution + silu, unit factors, k . q, decays per channel
 //   delta_scan:   the recurrence.  A wave owns 4 * CPL columns of S in registers, 16
 //                 lanes a column; q, k, g of the head's next tokens wait in LDS, shared
 //                 by the workgroup's columns
@@ -29,6 +30,8 @@ DEV float softplus_f(float x) {
   const float e = __expf(x), u = 1.f + e;
   return u == 1.f ? e : __logf(u) * e * __builtin_amdgcn_rcpf(u - 1.f);
 }
+
+DEV float gate_f(float x, bool silu) { return (silu ? x : 1.f) * sigmoid_f(x); }
 
 // rate = exp(A_log)
 DEV float decay_f(float z, float rate) { return __expf(-rate * softplus_f(z)); }
@@ -88,7 +91,7 @@ DEV void conv_silu(float* y, const T* conv, const ConvInput<T>& in, int c) {
 // ---------------------------------------------------------------- prompts
 
 // grid (tiles of 16 tokens, G + 2 H): a wave per token and head.  The first G heads
-// are q and k together, the next H v, the last H the decays.
+// are q and k together, the next H v, the last H the decays per channel.
 template <typename T, int VW>
 __global__ __launch_bounds__(256) void delta_inputs_kernel(const DeltaArgs a) {
   const int tile = blockIdx.x, job = blockIdx.y;
@@ -160,7 +163,8 @@ __global__ __launch_bounds__(256) void delta_inputs_wide_kernel(const DeltaArgs 
   const int64_t row0 = a.row_starts[seq] + q0;
   int unit = blockIdx.y * 256 + threadIdx.x;
 
-  if (unit >= a.G * 16 + a.H * a.V / VW) {  // decays
+  if (unit >= a.G * 16 + a.H * a.V / VW) {  // decays per channel
+    if (a.head_decay) return;
     const int c = (unit - a.G * 16 - a.H * a.V / VW) * VW;
     if (c >= a.H * a.D) return;
     const float rate = expf(a.A_log[c / a.D]);
@@ -283,15 +287,16 @@ struct Words {
 
 // grid (column blocks, H, seqs).  Lane j of a column's 16 holds the dims
 // (e / VW) * 16 VW + j VW + e % VW: its LDS reads are VW wide and 16 lanes contiguous.
-// FULL: D = 16 DPL and rows are aligned to VW channels.
-template <typename T, int DPL, int CPL, bool FULL>
+// FULL: D = 16 DPL and rows are aligned to VW channels.  HEAD: one decay per head.
+template <typename T, int DPL, int CPL, bool FULL, bool HEAD>
 __global__ __launch_bounds__(256) void delta_scan_kernel(const DeltaArgs a) {
   constexpr int TT = DPL <= 16 ? 16 : 256 / DPL;  // tokens staged at a time
   constexpr int DP = 16 * DPL;
   constexpr int VW = DPL < 4 ? DPL : 4, NV = DPL / VW;
   constexpr int COLS = 16 * CPL, SIDE = COLS + 4;
+  constexpr int VECS = HEAD ? 2 : 3;
   extern __shared__ float lds[];
-  float* const side0 = lds + 2 * 3 * TT * DP;  // per token: v columns, beta, k . q
+  float* const side0 = lds + 2 * VECS * TT * DP;  // per token: v columns, beta, k . q, decay
   const int seq = blockIdx.z, h = blockIdx.y, kvh = h / (a.H / a.G);
   const int ctx = a.ctx_lens[seq], len = a.seq_lens[seq] - ctx;
   const int64_t row0 = a.row_starts[seq], slot = a.slots[seq];
@@ -314,18 +319,20 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(const DeltaArgs a) {
   constexpr int PW = FULL ? VW : 1, PV = DPL / PW;  // pieces of a thread's dims
   Words<T, PW> rq[PV], rk[PV];
   Words<float, PW> rg[PV];
-  Words<T, 1> rv[CPL], fb;
+  Words<T, 1> rv[CPL], fb, fz;
+  const float rate = HEAD ? expf(a.A_log[h]) : 0.f, z_bias = HEAD ? a.dt_bias[h] : 0.f;
   float fq, fk, fkq;
   const int t_in = min(tok, len - 1);  // where this thread reads on past the end
   const T* py = (const T*)a.y + (row0 + t_in) * a.C;
   const T* pq = py + kvh * a.D;
   const T* pk = py + (a.G + kvh) * a.D;
   const T* pv = py + 2 * a.G * a.D + h * a.V;
-  const float* pg = a.g + ((row0 + t_in) * a.H + h) * a.D;
+  const float* pg = HEAD ? nullptr : a.g + ((row0 + t_in) * a.H + h) * a.D;
+  const T* pz = (const T*)a.z + (row0 + t_in) * a.z_stride + h;
   const float* pu = a.unit + ((row0 + t_in) * a.G + kvh) * 3;
   const T* pb = (const T*)a.b + (row0 + t_in) * a.b_stride + h;
   const int64_t y_step = (int64_t)TT * a.C, g_step = (int64_t)TT * a.H * a.D;
-  const int64_t b_step = TT * a.b_stride;
+  const int64_t b_step = TT * a.b_stride, z_step = TT * a.z_stride;
   const int u_step = TT * a.G * 3;
   auto fetch = [&](int t0) {
 #pragma unroll
@@ -333,7 +340,7 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(const DeltaArgs a) {
       const int d = FULL ? dim(i * PW) : min(dim(i * PW), a.D - 1);
       rq[i].load(pq + d);
       rk[i].load(pk + d);
-      rg[i].load(pg + d);
+      if (!HEAD) rg[i].load(pg + d);
     }
 #pragma unroll
     for (int c = 0; c < CPL; ++c) rv[c].load(pv + min(col0 + j * CPL + c, a.V - 1));
@@ -341,20 +348,22 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(const DeltaArgs a) {
     fk = pu[1];
     fkq = pu[2];
     fb.load(pb);
+    if (HEAD) fz.load(pz);
     if (t0 + TT + tok < len) {
       pq += y_step;
       pk += y_step;
       pv += y_step;
-      pg += g_step;
+      if (!HEAD) pg += g_step;
       pu += u_step;
       pb += b_step;
+      if (HEAD) pz += z_step;
     }
   };
   // tokens past the end change nothing: g = 1, k = q = beta = 0
   auto put = [&](int buf, int t0) {
     if (tok >= TT) return;
     const bool in = t0 + tok < len;
-    float* at = lds + (buf * 3 * TT + tok) * DP;
+    float* at = lds + (buf * VECS * TT + tok) * DP;
 #pragma unroll
     for (int i = 0; i < NV; ++i) {
       const int d = dim(i * VW);
@@ -365,11 +374,11 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(const DeltaArgs a) {
         const bool has = in && (FULL || d + e < a.D);
         q.v[e] = has ? rq[p].at(o) * fq : 0.f;
         k.v[e] = has ? rk[p].at(o) * fk : 0.f;
-        g.v[e] = has ? rg[p].at(o) : 1.f;
+        if (!HEAD) g.v[e] = has ? rg[p].at(o) : 1.f;
       }
       *(Pack<float, VW>*)(at + d) = q;
       *(Pack<float, VW>*)(at + TT * DP + d) = k;
-      *(Pack<float, VW>*)(at + 2 * TT * DP + d) = g;
+      if (!HEAD) *(Pack<float, VW>*)(at + 2 * TT * DP + d) = g;
     }
     float* side = side0 + (buf * TT + tok) * SIDE;
 #pragma unroll
@@ -377,11 +386,12 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(const DeltaArgs a) {
     if (j == 0) {
       side[COLS] = in ? sigmoid_f(fb.at(0)) : 0.f;
       side[COLS + 1] = in ? fkq : 0.f;
+      if (HEAD) side[COLS + 2] = in ? decay_f(fz.at(0) + z_bias, rate) : 1.f;
     }
   };
 
   struct Token {
-    float q[DPL], k[DPL], g[DPL], v[CPL], beta, kq;
+    float q[DPL], k[DPL], g[HEAD ? 1 : DPL], v[CPL], beta, kq;
   };
   float* po = a.o + ((row0 + j) * a.H + h) * a.V + col0 + mine;  // token j of a chunk
   fetch(0);
@@ -393,18 +403,19 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(const DeltaArgs a) {
     const int n = min(TT, len - t0);
     float keep[CPL] = {};  // lane j: the output of token j
     auto load = [&](Token& x, int t) {
-      const float* at = lds + (buf * 3 * TT + t) * DP + j * VW;
+      const float* at = lds + (buf * VECS * TT + t) * DP + j * VW;
       const float* side = side0 + (buf * TT + t) * SIDE;
 #pragma unroll
       for (int i = 0; i < NV; ++i) {
         load_f<VW>(x.q + i * VW, at + i * 16 * VW);
         load_f<VW>(x.k + i * VW, at + TT * DP + i * 16 * VW);
-        load_f<VW>(x.g + i * VW, at + 2 * TT * DP + i * 16 * VW);
+        if constexpr (!HEAD) load_f<VW>(x.g + i * VW, at + 2 * TT * DP + i * 16 * VW);
       }
 #pragma unroll
       for (int c = 0; c < CPL; ++c) x.v[c] = side[mine + c];
       x.beta = side[COLS];
       x.kq = side[COLS + 1];
+      if (HEAD) x.g[0] = side[COLS + 2];
     };
     auto run = [&](const Token& x, int t) {
 #pragma unroll
@@ -412,17 +423,18 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(const DeltaArgs a) {
         float sk = 0.f, sq = 0.f;
 #pragma unroll
         for (int e = 0; e < DPL; ++e) {
-          s[c][e] *= x.g[e];
+          if (!HEAD) s[c][e] *= x.g[e];
           sk += x.k[e] * s[c][e];
           sq += x.q[e] * s[c][e];
         }
-        sk = row16_sum(sk);
-        sq = row16_sum(sq);
+        sk = row16_sum(sk) * (HEAD ? x.g[0] : 1.f);
+        sq = row16_sum(sq) * (HEAD ? x.g[0] : 1.f);
         const float u = x.beta * (x.v[c] - sk);
         const float o = sq + x.kq * u;
         keep[c] = j == t ? o : keep[c];
 #pragma unroll
-        for (int e = 0; e < DPL; ++e) s[c][e] += x.k[e] * u;
+        for (int e = 0; e < DPL; ++e)
+          s[c][e] = HEAD ? x.g[0] * s[c][e] + x.k[e] * u : s[c][e] + x.k[e] * u;
       }
     };
     // a token's operands are read while the one before is worked on
@@ -493,7 +505,7 @@ __global__ __launch_bounds__(256) void delta_output_kernel(const DeltaArgs a) {
     load_f<VW>(g, gate + d);
     load_f<VW>(w, a.norm + d);
 #pragma unroll
-    for (int k = 0; k < VW; ++k) x[k] *= inv * w[k] * sigmoid_f(g[k]);
+    for (int k = 0; k < VW; ++k) x[k] *= inv * w[k] * gate_f(g[k], a.gate_silu);
     store_f<VW>(out + d, x);
   }
 }
@@ -541,7 +553,8 @@ __global__ __launch_bounds__(1024) void delta_step_kernel(const DeltaArgs a) {
   float qq = 0.f, kk = 0.f, kq = 0.f;
   const float rate = expf(a.A_log[h]);
   for (int d = tid; d < a.D; d += threads) {
-    const int cq = kvh * a.D + d, ck = (a.G + kvh) * a.D + d, hd = h * a.D + d;
+    const int cq = kvh * a.D + d, ck = (a.G + kvh) * a.D + d;
+    const int hd = a.head_decay ? h : h * a.D + d;
     float y[2];
     conv_silu<T, 1, TAPS>(y, conv, in, cq);
     conv_silu<T, 1, TAPS>(y + 1, conv, in, ck);
@@ -657,51 +670,58 @@ __global__ __launch_bounds__(1024) void delta_step_kernel(const DeltaArgs a) {
   const T* gate = (const T*)a.gate + seq * a.gate_stride + (int64_t)h * a.V;
   T* out = (T*)a.out + ((int64_t)seq * a.H + h) * a.V;
   for (int d = tid; d < a.V; d += threads)
-    out[d] = from_f<T>(o[d] * inv * a.norm[d] * sigmoid_f(to_f(gate[d])));
+    out[d] = from_f<T>(o[d] * inv * a.norm[d] * gate_f(to_f(gate[d]), a.gate_silu));
 }
 
 // ---------------------------------------------------------------- launches
 
-template <typename T, int DPL, int CPL, bool FULL>
+template <typename T, int DPL, int CPL, bool FULL, bool HEAD>
 static void launch_scan(const DeltaArgs& a, hipStream_t stream) {
   constexpr int TT = DPL <= 16 ? 16 : 256 / DPL;
-  constexpr int bytes = 4 * (2 * 3 * TT * 16 * DPL + 2 * TT * (16 * CPL + 4));
+  constexpr int bytes = 4 * (2 * (HEAD ? 2 : 3) * TT * 16 * DPL + 2 * TT * (16 * CPL + 4));
   static_assert(bytes <= 160 * 1024, "LDS");
   static bool attr_set = false;
   if (!attr_set) {
-    (void)hipFuncSetAttribute((const void*)delta_scan_kernel<T, DPL, CPL, FULL>,
+    (void)hipFuncSetAttribute((const void*)delta_scan_kernel<T, DPL, CPL, FULL, HEAD>,
                               hipFuncAttributeMaxDynamicSharedMemorySize, bytes);
     attr_set = true;
   }
   const dim3 grid((a.V + 16 * CPL - 1) / (16 * CPL), a.H, a.seqs);
-  delta_scan_kernel<T, DPL, CPL, FULL><<<grid, 256, bytes, stream>>>(a);
+  delta_scan_kernel<T, DPL, CPL, FULL, HEAD><<<grid, 256, bytes, stream>>>(a);
+}
+
+template <typename T, int DPL, bool HEAD>
+static void launch_scan_decay(const DeltaArgs& a, int cpl, hipStream_t stream) {
+  constexpr int VW = DPL < 4 ? DPL : 4;
+  if (a.D != 16 * DPL || a.C % VW != 0)
+    launch_scan<T, DPL, 1, false, HEAD>(a, stream);
+  else if (cpl == 1 || DPL > 8)
+    launch_scan<T, DPL, 1, true, HEAD>(a, stream);
+  else if constexpr (DPL <= 8)
+    launch_scan<T, DPL, 2, true, HEAD>(a, stream);
 }
 
 template <typename T, int DPL>
 static void launch_scan_cols(const DeltaArgs& a, int cpl, hipStream_t stream) {
-  constexpr int VW = DPL < 4 ? DPL : 4;
-  if (a.D != 16 * DPL || a.C % VW != 0)
-    launch_scan<T, DPL, 1, false>(a, stream);
-  else if (cpl == 1 || DPL > 8)
-    launch_scan<T, DPL, 1, true>(a, stream);
-  else if constexpr (DPL <= 8)
-    launch_scan<T, DPL, 2, true>(a, stream);
+  (a.head_decay ? launch_scan_decay<T, DPL, true> : launch_scan_decay<T, DPL, false>)(a, cpl,
+                                                                                      stream);
 }
 
 template <typename T>
 static void prompts(const DeltaArgs& a, int cpl, hipStream_t stream) {
   constexpr int W = 16 / sizeof(T);
   auto all = [&](int n) {  // every head and row starts at a multiple of n channels
-    return a.D % n == 0 && a.V % n == 0 && a.z_stride % n == 0 && a.qkv_stride % n == 0 &&
-           a.gate_stride % n == 0;
+    return a.D % n == 0 && a.V % n == 0 && (a.head_decay || a.z_stride % n == 0) &&
+           a.qkv_stride % n == 0 && a.gate_stride % n == 0;
   };
-  const bool aligned = ((uintptr_t)a.qkv | (uintptr_t)a.z | (uintptr_t)a.gate) % 16 == 0;
+  const uintptr_t z = a.head_decay ? 0 : (uintptr_t)a.z;
+  const bool aligned = ((uintptr_t)a.qkv | z | (uintptr_t)a.gate) % 16 == 0;
   if (aligned && all(W) && a.taps == 4 && a.D <= 16 * W) {
-    const int units = a.G * 16 + a.H * (a.V + a.D) / W;
+    const int units = a.G * 16 + a.H * (a.V + (a.head_decay ? 0 : a.D)) / W;
     delta_inputs_wide_kernel<T, W><<<dim3(a.n_tiles, (units + 255) / 256), 256, 0, stream>>>(a);
   } else {
-    const dim3 grid(a.n_tiles, a.G + 2 * a.H);
-    const bool even = all(2) && ((uintptr_t)a.qkv | (uintptr_t)a.z) % (2 * sizeof(T)) == 0;
+    const dim3 grid(a.n_tiles, a.G + (a.head_decay ? 1 : 2) * a.H);
+    const bool even = all(2) && ((uintptr_t)a.qkv | z) % (2 * sizeof(T)) == 0;
     auto inputs = even ? delta_inputs_kernel<T, 2> : delta_inputs_kernel<T, 1>;
     inputs<<<grid, 256, 0, stream>>>(a);
   }

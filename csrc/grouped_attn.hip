@@ -2,8 +2,9 @@
 // for every other case (gfx950).
 //
 // A query at position p sees the keys p - window + 1 .. p and the first ``keep``
-// ones; scores may be capped, get a bias by distance, and a sink may join the
-// denominator.  The sink is the softmax's starting state (maximum = sink, sum = 1, no
+// ones, or of those only the ones of its own chunk; scores may be mixed over the heads (the
+// plain kernel; talk_attn.hip has the others), capped, get a bias by distance, and a sink
+// may join the denominator.  The sink is the softmax's starting state (maximum = sink, sum = 1, no
 // value), so that neither the merge of partial sums nor the output knows about it.
 // Sigmoid weights need no such state: their partial results are plain sums.
 //
@@ -23,10 +24,10 @@ struct KeyList {  // of one query: position of the i-th visible key
   DEV int at(int i) const { return i < keep ? i : lo + i - keep; }
 };
 
-static DEV KeyList visible_keys(int pos, int window, int keep) {
+static DEV KeyList visible_keys(const GroupedArgs& a, int pos) {
   KeyList k;
-  k.lo = max(0, pos - window + 1);
-  k.keep = min(keep, k.lo);
+  k.lo = first_key(a, pos);
+  k.keep = min(a.keep, k.lo);
   k.n = k.keep + pos + 1 - k.lo;
   return k;
 }
@@ -47,7 +48,7 @@ __global__ __launch_bounds__(256, GM * (KE + VE) <= 32 ? 4 : GM * (KE + VE) <= 6
   const int64_t row0 = (int64_t)seq * a.H + h0;
 
   const int pos = a.seq_lens[seq] - 1;
-  const KeyList keys = visible_keys(pos, a.window, a.keep);
+  const KeyList keys = visible_keys(a, pos);
   const int per_split = (keys.n + a.n_split - 1) / a.n_split;
   const int x0 = min(keys.n, (int)blockIdx.y * per_split), x1 = min(keys.n, x0 + per_split);
   if (x0 >= x1) {  // an empty split; those are a row's last ones
@@ -212,23 +213,37 @@ __global__ __launch_bounds__(256) void grouped_plain_kernel(
   }
   const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
   const int* table = a.tables + (int64_t)seq * a.max_blocks;
-  const T* qr = (const T*)a.q + token * a.q_stride + (int64_t)h * d;
+  const T* qr = (const T*)a.q + token * a.q_stride;
   float q[NE], acc[NE] = {};
+  // mixed scores are those of one long query, the mix of the heads that share a key head,
+  // against all key heads
+  const int dk = a.talk ? a.G * d : d, k_at = a.talk ? 0 : kvh * d, group = a.H / a.G;
 #pragma unroll
-  for (int e = 0; e < NE; ++e) q[e] = e * 64 + lane < d ? to_f(qr[e * 64 + lane]) : 0.f;
+  for (int e = 0; e < NE; ++e) {
+    const int i = e * 64 + lane;
+    q[e] = 0.f;
+    if (i >= dk) continue;
+    if (a.talk) {
+      const int g0 = i / d * group;
+      for (int g = g0; g < g0 + group; ++g)
+        q[e] += a.talk[h * a.H + g] * to_f(qr[(int64_t)g * d + i % d]);
+    } else {
+      q[e] = to_f(qr[(int64_t)h * d + i]);
+    }
+  }
   const bool sink = a.sink && wid == 0;
   float m = sink ? a.sink[h] : NEG, l = sink ? 1.f : 0.f;
-  const KeyList keys = visible_keys(pos, a.window, a.keep);
+  const KeyList keys = visible_keys(a, pos);
   for (int x = wid; x < keys.n; x += 4) {
     const int k = keys.at(x);
     const int64_t slot = (int64_t)table[k / a.kv_block] * a.kv_block + k % a.kv_block;
-    const T* kr = (const T*)a.k_cache + (slot * a.G + kvh) * d;
+    const T* kr = (const T*)a.k_cache + slot * a.G * d + k_at;
     const T* vr = (const T*)a.v_cache + (slot * a.G + kvh) * v;
     float dot = 0.f, val[NE];
 #pragma unroll
     for (int e = 0; e < NE; ++e) {
       const int i = e * 64 + lane;
-      if (i < d) dot += q[e] * to_f(kr[i]);
+      if (i < dk) dot += q[e] * to_f(kr[i]);
       val[e] = i < v ? to_f(vr[i]) : 0.f;
     }
     dot = wave_sum(dot) * a.scale;
@@ -322,13 +337,15 @@ static bool launch_decode_v(const GroupedArgs& a, int v, int seqs, int gm,
 
 template <typename T>
 static bool launch_plain(const GroupedArgs& a, int d, int v, int tokens, hipStream_t stream) {
-  const int ne = ((d > v ? d : v) + 63) / 64;
-  if (ne > 32) return false;
-  auto k = ne <= 1   ? grouped_plain_kernel<T, 1>
-           : ne <= 2 ? grouped_plain_kernel<T, 2>
-           : ne <= 4 ? grouped_plain_kernel<T, 4>
-           : ne <= 8 ? grouped_plain_kernel<T, 8>
-                     : grouped_plain_kernel<T, 32>;
+  const int dk = a.talk ? a.G * d : d;
+  const int ne = ((dk > v ? dk : v) + 63) / 64;
+  if (ne > 64) return false;
+  auto k = ne <= 1    ? grouped_plain_kernel<T, 1>
+           : ne <= 2  ? grouped_plain_kernel<T, 2>
+           : ne <= 4  ? grouped_plain_kernel<T, 4>
+           : ne <= 8  ? grouped_plain_kernel<T, 8>
+           : ne <= 32 ? grouped_plain_kernel<T, 32>
+                      : grouped_plain_kernel<T, 64>;
   k<<<dim3(tokens, a.H), 256, 0, stream>>>(a, d, v);
   return true;
 }

@@ -1,5 +1,5 @@
 // Grouped attention of prompt portions over the paged cache on the matrix cores
-// (gfx950): windows that keep the first tokens, capped scores, biases by distance, a
+// (gfx950): windows that keep the first tokens, chunks, capped scores, biases by distance, a
 // sink; softmax or sigmoid weights; a gate per head.
 //
 // A workgroup owns 128 query rows of one head, a wave 32 of them.  Keys and values
@@ -75,7 +75,7 @@ __global__ __launch_bounds__(256, DN + VN <= 4 ? 2 : 1) void grouped_prefill_ker
   // key tiles: those with kept tokens, then those some row's window reaches
   const int k_end = ctx + q0 + rows;
   const int kept = (min(a.keep, k_end) + KT - 1) / KT;
-  const int first = max(kept, max(0, ctx + q0 - a.window + 1) / KT);
+  const int first = max(kept, first_key(a, ctx + q0) / KT);
   const int n_tiles = kept + max(0, (k_end + KT - 1) / KT - first);
   auto key_of = [&](int t) { return (t < kept ? t : first + t - kept) * KT; };
   // this thread's key of tile t, as a slot
@@ -134,6 +134,8 @@ __global__ __launch_bounds__(256, DN + VN <= 4 ? 2 : 1) void grouped_prefill_ker
   f32x16_v o[VT] = {};
   const int w_lo = ctx + q0 + wid * 32;                    // wave's positions
   const int w_hi = min(w_lo + 31, k_end - 1);
+  const int lo = live ? first_key(a, qpos) : 0;
+  const int lo_lo = first_key(a, w_lo), lo_hi = first_key(a, max(w_lo, w_hi));
   const int sw_k = ((c & 3) << 1) | ((c >> 2) & 1);
   const int i16 = lane & 15, g = lane >> 4;
 
@@ -147,7 +149,7 @@ __global__ __launch_bounds__(256, DN + VN <= 4 ? 2 : 1) void grouped_prefill_ker
     if (t + 1 < n_tiles) stage(t + 1);
     const int key0 = key_of(t);
     // a tile that one of this wave's rows sees
-    if (wid * 32 < rows && key0 <= w_hi && (w_lo - (key0 + KT - 1) < a.window || key0 < a.keep)) {
+    if (wid * 32 < rows && key0 <= w_hi && (key0 + KT - 1 >= lo_lo || key0 < a.keep)) {
       const char* kt = lds + (t & 1) * TILE_BYTES;
       f32x16_v s[2] = {};
 #pragma unroll
@@ -159,7 +161,7 @@ __global__ __launch_bounds__(256, DN + VN <= 4 ? 2 : 1) void grouped_prefill_ker
           s[b] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(kf, qf[st], s[b], 0, 0, 0);
         }
       }
-      const bool edge = key0 + KT - 1 > w_lo || w_hi - key0 >= a.window;
+      const bool edge = key0 + KT - 1 > w_lo || key0 < lo_hi;
 #pragma unroll
       for (int b = 0; b < 2; ++b)
 #pragma unroll
@@ -184,7 +186,7 @@ __global__ __launch_bounds__(256, DN + VN <= 4 ? 2 : 1) void grouped_prefill_ker
         for (int e = 0; e < 16; ++e) {
           if (edge) {
             const int key = key0 + b * 32 + (e & 3) + 8 * (e >> 2) + 4 * half;
-            if (key > qpos || (qpos - key >= a.window && key >= a.keep)) s[b][e] = -INFINITY;
+            if (key > qpos || (key < lo && key >= a.keep)) s[b][e] = -INFINITY;
           }
           mt = fmaxf(mt, s[b][e]);
         }

@@ -13,6 +13,9 @@ struct NormForm {
   int top;                  // 0 = none
   const void* rows;         // [n, top, w]
   const float* weights;     // [n, top]
+  // and then sigmoid(gate[n]) multiplies y
+  const void* gate;         // [n, w] rows gate_stride apart, or null
+  int64_t gate_stride;
   // the same norm of x under another weight
   const void* x_norm2;      // [w]
   void* out2;               // rows out2_stride apart, or null

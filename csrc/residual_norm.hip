@@ -4,8 +4,8 @@
 // rmsnorm(y) * w_y, to the residual, optionally file the result as the newest depth
 // state and replace it by a weighted sum of all states, then emit norm(x) * w_x (layer
 // or RMS norm) or x itself for the next GEMM.  What is added may include a weighted sum
-// of several rows (chosen experts' results); the norm may be written a second time under
-// another weight.  The row lives in LDS between the reductions (each thread re-reads only what
+// of several rows (chosen experts' results) and be gated; the norm may be written a second
+// time under another weight.  The row lives in LDS between the reductions (each thread re-reads only what
 // it wrote, so the row itself needs no barrier).  Mean first, then the squared
 // deviations: no cancellation.
 #include "common_t.h"
@@ -59,6 +59,27 @@ DEV void depth_average(float* t, const NormForm& f, const int64_t at) {
   for (int k = 0; k < V; ++k) t[k] = sum[k];
 }
 
+// what is added to x at i: y, the experts' rows and the gate
+template <typename T, int V>
+DEV void addend(float* d, const T* y, const NormForm& f, const int w, const int i) {
+  load_f<V>(d, y + (int64_t)blockIdx.x * w + i);
+  const T* er = (const T*)f.rows + (int64_t)blockIdx.x * f.top * w + i;
+  const float* ew = f.weights + (int64_t)blockIdx.x * f.top;
+#pragma unroll 4
+  for (int j = 0; j < f.top; ++j) {
+    float e[V];
+    load_f<V>(e, er + (int64_t)j * w);
+#pragma unroll
+    for (int k = 0; k < V; ++k) d[k] += ew[j] * e[k];
+  }
+  if (f.gate) {
+    float g[V];
+    load_f<V>(g, (const T*)f.gate + (int64_t)blockIdx.x * f.gate_stride + i);
+#pragma unroll
+    for (int k = 0; k < V; ++k) d[k] *= sigmoid_f(g[k]);
+  }
+}
+
 template <typename T, int V, bool DEPTH>
 __global__ __launch_bounds__(1024) void residual_norm_kernel(
     float* __restrict__ x,            // [n, w], updated if y
@@ -75,11 +96,10 @@ __global__ __launch_bounds__(1024) void residual_norm_kernel(
 
   float y_scale = 1.f;
   if (y && y_norm) {
-    const T* yr = y + (int64_t)blockIdx.x * w;
     float ss = 0.f;
     for (int i = i0; i < w; i += step) {
       float t[V];
-      load_f<V>(t, yr + i);
+      addend<T, V>(t, y, f, w, i);
 #pragma unroll
       for (int k = 0; k < V; ++k) {
         ss += t[k] * t[k];
@@ -99,16 +119,7 @@ __global__ __launch_bounds__(1024) void residual_norm_kernel(
 #pragma unroll
         for (int k = 0; k < V; ++k) d[k] = (f.offset + d[k]) * row[i + k] * y_scale;
       } else {
-        load_f<V>(d, y + (int64_t)blockIdx.x * w + i);
-        const T* er = (const T*)f.rows + (int64_t)blockIdx.x * f.top * w + i;
-        const float* ew = f.weights + (int64_t)blockIdx.x * f.top;
-#pragma unroll 4
-        for (int j = 0; j < f.top; ++j) {
-          float e[V];
-          load_f<V>(e, er + (int64_t)j * w);
-#pragma unroll
-          for (int k = 0; k < V; ++k) d[k] += ew[j] * e[k];
-        }
+        addend<T, V>(d, y, f, w, i);
       }
 #pragma unroll
       for (int k = 0; k < V; ++k) t[k] += f.mult * d[k];
@@ -178,7 +189,8 @@ static void residual_norm_t(float* x, const void* y, const void* y_norm,
                             const void* x_norm, void* out, float eps, int n,
                             int w, int64_t out_stride, const NormForm& f,
                             hipStream_t stream) {
-  const bool vec = w % 4 == 0 && out_stride % 4 == 0 && f.out2_stride % 4 == 0;
+  const bool vec = w % 4 == 0 && out_stride % 4 == 0 && f.out2_stride % 4 == 0 &&
+                   f.gate_stride % 4 == 0 && (uintptr_t)f.gate % (4 * sizeof(T)) == 0;
   int threads = w >= 1024 ? 256 : w >= 512 ? 128 : 64;
   // few rows: the latency of one counts
   while (n <= 512 && threads < 1024 && threads * 4 < w) threads *= 2;
