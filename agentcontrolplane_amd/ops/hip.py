@@ -291,7 +291,7 @@ def latent_expanded_prefill(q, w_ukv, gate, cos_sin, rot_dim: int, cache, batch,
 
 # ---------------------------------------- grouped attention: caps, windows, sinks
 
-_PLAIN, _DECODE, _PREFILL = 0, 1, 2
+_PLAIN, _DECODE, _PREFILL, _TALK_DECODE, _TALK_PREFILL = range(5)
 
 
 def cache_keys_values(k, v, slot_mapping, k_cache, v_cache):
@@ -350,29 +350,40 @@ def grouped_attention(q, k_cache, v_cache, batch, scale: float, cap, window, kee
 
     H, d, v, G = q.shape[1], q.shape[2], out.shape[2], k_cache.shape[2]
     rest = (scale, cap or 0.0, window or _NO_WINDOW, chunk or _NO_WINDOW, keep_first, sigmoid)
-    tiled = (talk is None and q.dtype == torch.bfloat16 and d in LATENT_HEADS and v in LATENT_HEADS
-             and not (sigmoid and cap))
+    bf16 = q.dtype == torch.bfloat16
+    if talk is None:
+        tiled = bf16 and d in LATENT_HEADS and v in LATENT_HEADS and not (sigmoid and cap)
+        kinds, tile = ((_DECODE, _PREFILL) if tiled else (_PLAIN, _PLAIN)), 128
+    else:
+        tiled = bf16 and not (sigmoid or cap or keep_first) and all(
+            t is None for t in (sink, bias, gate))
+        tile = _C.talk_prefill_tokens(H, G, d, v) if tiled else 0
+        tiled = tiled and _C.talk_decode_fits(H, G, d, v)
+        kinds = (_TALK_DECODE if tiled else _PLAIN, _TALK_PREFILL if tile else _PLAIN)
     P = batch.num_prefill_tokens
 
     def gates(r):
         return None if gate is None else gate[r]
 
     if batch.prefills:
-        meta = batch.prefill_meta(128 if tiled else 1)
+        meta = batch.prefill_meta(tile if kinds[1] != _PLAIN else 1)
         _C.grouped_attn(
             out[:P], q[:P], k_cache, v_cache, meta.block_tables, meta.seq_lens, meta.ctx_lens,
             meta.row_starts, meta.tile_seq, meta.tile_q0, sink, bias, gates(slice(0, P)), talk,
-            None, None, *rest, _PREFILL if tiled else _PLAIN, 1, 1,
+            None, None, *rest, kinds[1], 1, 1,
         )
     if not batch.num_decode:
         return
     tables, rows = batch.decode_tables_i32(), batch.num_decode * H
     gm, n_split, part, ml = 1, 1, None, None
-    if tiled:
+    # keys a row may see
+    keys = min(tables.shape[1] * k_cache.shape[1], rest[2] + keep_first, rest[3])
+    if kinds[0] == _TALK_DECODE:  # a workgroup has all heads, and 4 waves with 32 keys each
+        n_split = max(1, min(_MAX_SPLIT, 1024 // batch.num_decode, -(-keys // 128)))
+    elif kinds[0] == _DECODE:
         most = 8 if d + v <= 256 else 4  # query heads a workgroup holds
         gm = next((n for n in (1, 2, 4) if n >= min(H // G, most)), most)
         # workgroups that fill the chip; every split has work for its 16 lane groups
-        keys = min(tables.shape[1] * k_cache.shape[1], rest[2] + keep_first, rest[3])
         groups = batch.num_decode * G * -(-(H // G) // gm)
         n_split = max(1, min(_MAX_SPLIT, 1024 // groups, -(-keys // 128)))
     if n_split > 1:
@@ -381,7 +392,7 @@ def grouped_attention(q, k_cache, v_cache, batch, scale: float, cap, window, kee
     _C.grouped_attn(
         out[P:], q[P:], k_cache, v_cache, tables, batch.decode_lens_i32(), None, None, None,
         None, sink, bias, gates(slice(P, None)), talk, part, ml, *rest,
-        _DECODE if tiled else _PLAIN, gm, n_split,
+        kinds[0], gm, n_split,
     )
 
 

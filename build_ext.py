@@ -39,6 +39,7 @@ def build(verbose: bool = False) -> str:
         os.path.join(CSRC, "embedding.hip"),
         os.path.join(CSRC, "grouped_attn.hip"),
         os.path.join(CSRC, "grouped_prefill.hip"),
+        os.path.join(CSRC, "talk_attn.hip"),
         os.path.join(CSRC, "attn_inputs.hip"),
         os.path.join(CSRC, "experts.hip"),
         os.path.join(CSRC, "experts_gemm.hip"),

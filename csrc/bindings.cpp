@@ -57,6 +57,10 @@ void launch_softcap(bool, float*, const void*, float, int64_t, hipStream_t);
 bool launch_grouped_decode(const GroupedArgs*, int, int, int, int, hipStream_t);
 bool launch_grouped_plain(bool, const GroupedArgs*, int, int, int, hipStream_t);
 bool launch_grouped_prefill(const GroupedArgs*, int, int, hipStream_t);
+int talk_prefill_tokens(int, int, int, int);
+bool talk_decode_fits(int, int, int, int);
+bool launch_talk_prefill(const GroupedArgs*, int, int, hipStream_t);
+bool launch_talk_decode(const GroupedArgs*, int, int, int, hipStream_t);
 void launch_cache_keys_values(void*, void*, const void*, const void*, const int64_t*, int, int,
                               int64_t, int, hipStream_t);
 void launch_delta_prompts(bool, const DeltaArgs*, int, hipStream_t);
@@ -732,7 +736,7 @@ static void cache_keys_values(torch::Tensor k_cache, torch::Tensor v_cache, torc
 
 // q [tokens, H, d] -> out [tokens, H, v].  Prefill chunks bring ctx_lens, row_starts and
 // tiles; decode (one token per table row) brings none of them.
-// kind: 0 plain, 1 decode, 2 prefill on the matrix cores
+// kind: 0 plain, 1 decode, 2 prefill on the matrix cores, with mixed scores 3 decode, 4 prefill
 static void grouped_attn(torch::Tensor out, torch::Tensor q, torch::Tensor k_cache,
                          torch::Tensor v_cache, torch::Tensor tables, torch::Tensor seq_lens,
                          OptTensor ctx_lens, OptTensor row_starts, OptTensor tile_seq,
@@ -757,8 +761,9 @@ static void grouped_attn(torch::Tensor out, torch::Tensor q, torch::Tensor k_cac
   TORCH_CHECK(chunk > 0 && chunk <= (1 << 30) && (keep == 0 || chunk == (1 << 30)),
               "chunks keep no first tokens");
   TORCH_CHECK(kind == 0 || bf16, "the matrix-core kernels take bf16");
-  TORCH_CHECK(kind == 1 || n_split == 1, "only decode splits keys");
-  TORCH_CHECK((kind == 2) <= (bool)tile_seq && !(kind == 1 && tile_seq), "tiles");
+  const bool decode = kind == 1 || kind == 3, prefill = kind == 2 || kind == 4;
+  TORCH_CHECK(decode || n_split == 1, "only decode splits keys");
+  TORCH_CHECK(prefill <= (bool)tile_seq && !(decode && tile_seq), "tiles");
   if (tokens == 0 || seqs == 0) return;
   GroupedArgs a{};
   a.out = out.data_ptr();
@@ -801,7 +806,7 @@ static void grouped_attn(torch::Tensor out, torch::Tensor q, torch::Tensor k_cac
   if (tile_seq) {
     TORCH_CHECK(ctx_lens && row_starts && tile_q0, "prefill metadata");
     a.n_tiles = tile_seq->numel();
-    TORCH_CHECK(kind == 2 || a.n_tiles == tokens, "the plain kernel takes a token per tile");
+    TORCH_CHECK(prefill || a.n_tiles == tokens, "the plain kernel takes a token per tile");
   } else {
     TORCH_CHECK(tokens == seqs, "decode has one token per sequence");
   }
@@ -818,8 +823,10 @@ static void grouped_attn(torch::Tensor out, torch::Tensor q, torch::Tensor k_cac
   a.rows = tokens * H;
   a.scale = (float)scale;
   a.cap = (float)cap;
-  TORCH_CHECK(!talk || kind == 0, "mixed scores");
-  const bool ok = kind == 2   ? launch_grouped_prefill(&a, d, v, cur_stream())
+  TORCH_CHECK((bool)talk ? kind != 1 && kind != 2 : kind < 3, "mixed scores");
+  const bool ok = kind == 4   ? launch_talk_prefill(&a, d, v, cur_stream())
+                  : kind == 3 ? launch_talk_decode(&a, d, v, seqs, cur_stream())
+                  : kind == 2   ? launch_grouped_prefill(&a, d, v, cur_stream())
                   : kind == 1 ? launch_grouped_decode(&a, d, v, seqs, (int)gm, cur_stream())
                               : launch_grouped_plain(bf16, &a, d, v, tokens, cur_stream());
   TORCH_CHECK(ok, "grouped attention: unsupported sizes d ", d, " v ", v);
@@ -1128,6 +1135,8 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("softcap", &softcap);
   m.def("cache_keys_values", &cache_keys_values);
   m.def("grouped_attn", &grouped_attn);
+  m.def("talk_prefill_tokens", &talk_prefill_tokens);
+  m.def("talk_decode_fits", &talk_decode_fits);
   m.def("attention_inputs", &attention_inputs);
   m.attr("EXPERT_TILE") = EXPERT_TILE;
   m.def("moe_route", &moe_route);

@@ -1,0 +1,647 @@
+// Grouped attention whose heads mix their scores, over the paged cache on the matrix cores
+// (gfx950):
+//
+//   s_h(i, j) = sum_g T[h, g] scale q_g(i) . k_g(j),   softmax over the visible keys
+//
+// Decode.  The mix moves to the query: s_h is one product of a long query, T's mix of the
+// heads that share a key head, side by side for all key heads, with the whole key row.
+// A workgroup owns a sequence, or a run of its keys; it builds the long queries in LDS,
+// in the order of the matrix cores' fragments.  Its waves take 32 keys at a time, each by
+// itself: keys go from memory straight to the matrix cores, weights through a few LDS
+// rows to the lanes that hold the values.  The waves meet once, at the end.
+//
+// Prompts.  There the mix is a product of its own (the long queries would multiply the
+// first product by the number of key heads).  A workgroup owns 32 / group tokens with all
+// their heads; wave g computes what belongs to key/value head g: raw scores, and values
+// times weights.  In between the scores of a tile of 32 keys go through LDS to be mixed,
+// a wave per token: 16 keys x heads times heads x heads.  Scores are fp32 and travel as
+// three bf16 parts, whose products with a bf16 T lose nothing.
+#include "common_t.h"
+#include "grouped_attn.h"
+#include "latent_attn.h"
+
+typedef __bf16 bf16x8_v __attribute__((ext_vector_type(8)));
+typedef __bf16 bf16x4_v __attribute__((ext_vector_type(4)));
+typedef float f32x4_v __attribute__((ext_vector_type(4)));
+typedef __attribute__((address_space(3))) char lds_char;
+typedef __attribute__((address_space(3))) bf16x4_v lds_bf16x4;
+typedef __attribute__((address_space(1))) const char glob_char;
+
+#define NEG -1e30f
+#define LOG2E 1.44269504088896f
+
+// what lanes of this wave wrote to LDS is there for its others
+DEV void wave_sync() {
+  __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+  __builtin_amdgcn_wave_barrier();
+  __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
+}
+
+DEV float quad_max(float v) {  // over the lanes with this lane & 15
+  v = fmaxf(v, __shfl_xor(v, 16, 64));
+  return fmaxf(v, __shfl_xor(v, 32, 64));
+}
+DEV float quad_sum(float v) {
+  v += __shfl_xor(v, 16, 64);
+  return v + __shfl_xor(v, 32, 64);
+}
+
+// ------------------------------------------------------------------ decode
+
+#define DEC_ROWS 16  // keys whose weights are in LDS at a time
+
+// HT: 16-head tiles.  A lane holds UL pieces of 8 value dims and the up to GM heads of
+// their value head.  grid (sequences, splits).
+template <int HT, int GM, int UL>
+__global__ __launch_bounds__(256, 2) void talk_decode_kernel(const GroupedArgs a, const int d,
+                                                             const int v) {
+  extern __shared__ char lds[];
+  const int group = a.H / a.G, DK = a.G * d, steps = DK / 32;
+  const int units = a.G * v / 8, p_row = a.G * GM + 4;
+  const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
+  const int c = lane & 15, quad = lane >> 4;
+  bf16x8_v* const qf = (bf16x8_v*)lds;                          // [steps][HT][64]
+  float* const merged = (float*)lds;                            // [4][H][v], at the end
+  const int body = max(steps * HT * 1024, 16 * a.H * v);
+  float* const pw = (float*)(lds + body) + wid * (DEC_ROWS + 1) * p_row;
+  float* const al = pw + DEC_ROWS * p_row;                      // rescaling
+  float2* const ml = (float2*)((float*)(lds + body) + 4 * (DEC_ROWS + 1) * p_row);  // [4][H]
+
+  const int seq = blockIdx.x, pos = a.seq_lens[seq] - 1;
+  const int64_t row0 = (int64_t)seq * a.H;
+  const int lo = first_key(a, pos), n_keys = pos + 1 - lo;
+  // whole blocks of 32 keys per split
+  const int blocks = (n_keys + 31) / 32;
+  const int per_split = (blocks + a.n_split - 1) / a.n_split * 32;
+  const int x0 = lo + min(n_keys, (int)blockIdx.y * per_split);
+  const int x1 = min(pos + 1, x0 + per_split);
+  if (x0 >= x1) {
+    for (int h = threadIdx.x; h < a.H; h += 256)
+      a.part_ml[(int64_t)blockIdx.y * a.rows + row0 + h] = float2{NEG, -1.f};
+    return;
+  }
+
+  {  // long queries, as fragments: step u / 4, lane (u % 4) * 16 + h % 16
+    const bf16_t* q = (const bf16_t*)a.q + seq * a.q_stride;
+    const int row_units = DK / 8;
+    for (int i = threadIdx.x; i < 16 * HT * row_units; i += 256) {
+      const int u = i % row_units, h = i / row_units;
+      const int g0 = u * 8 / d * group, e0 = u * 8 % d;
+      float x[8] = {};
+      if (h < a.H) {
+        for (int g = g0; g < g0 + group; ++g) {
+          const float t = a.talk[h * a.H + g];
+          float y[8];
+          load_f<8>(y, q + (int64_t)g * d + e0);
+#pragma unroll
+          for (int e = 0; e < 8; ++e) x[e] += t * y[e];
+        }
+      }
+      bf16x8_v f;
+#pragma unroll
+      for (int e = 0; e < 8; ++e) f[e] = (__bf16)x[e];
+      qf[((u >> 2) * HT + (h >> 4)) * 64 + (u & 3) * 16 + (h & 15)] = f;
+    }
+  }
+  __syncthreads();
+
+  const int* table = a.tables + (int64_t)seq * a.max_blocks;
+  const bf16_t* kc = (const bf16_t*)a.k_cache + quad * 8;
+  const bf16_t* vc = (const bf16_t*)a.v_cache;
+  const float mul = a.scale * LOG2E;
+  int unit[UL], kvh[UL];
+#pragma unroll
+  for (int j = 0; j < UL; ++j) {
+    unit[j] = min(lane + 64 * j, units - 1);
+    kvh[j] = unit[j] * 8 / v;
+  }
+  int at[HT];  // where this lane's heads are in a row of weights
+#pragma unroll
+  for (int t = 0; t < HT; ++t) {
+    const int h = t * 16 + c;
+    at[t] = h / group * GM + h % group;
+  }
+  float m[HT], l[HT], acc[GM][UL][8];
+#pragma unroll
+  for (int t = 0; t < HT; ++t) m[t] = NEG, l[t] = 0.f;
+#pragma unroll
+  for (int g = 0; g < GM; ++g)
+#pragma unroll
+    for (int j = 0; j < UL; ++j)
+#pragma unroll
+      for (int e = 0; e < 8; ++e) acc[g][j][e] = 0.f;
+
+  for (int x = x0 + wid * 32; x < x1; x += 128) {
+    const int k = min(x + (lane & 31), x1 - 1);
+    const int slot = table[k / a.kv_block] * a.kv_block + k % a.kv_block;
+    const bf16_t* k0 = kc + (int64_t)__shfl(slot, c, 64) * DK;
+    const bf16_t* k1 = kc + (int64_t)__shfl(slot, c + 16, 64) * DK;
+    f32x4_v s[2][HT] = {};
+#pragma unroll 8
+    for (int st = 0; st < steps; ++st) {
+      const bf16x8_v f0 = *(const bf16x8_v*)(k0 + st * 32);
+      const bf16x8_v f1 = *(const bf16x8_v*)(k1 + st * 32);
+#pragma unroll
+      for (int t = 0; t < HT; ++t) {
+        const bf16x8_v b = qf[(st * HT + t) * 64 + lane];
+        s[0][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(f0, b, s[0][t], 0, 0, 0);
+        s[1][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(f1, b, s[1][t], 0, 0, 0);
+      }
+    }
+    // head c + 16 t, keys x + 16 b + 4 quad + r
+    float alpha[HT];
+    bool moved = false;
+#pragma unroll
+    for (int t = 0; t < HT; ++t) {
+      float mt = m[t];
+#pragma unroll
+      for (int b = 0; b < 2; ++b)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          s[b][t][r] = x + 16 * b + 4 * quad + r < x1 ? s[b][t][r] * mul : -INFINITY;
+          mt = fmaxf(mt, s[b][t][r]);
+        }
+      mt = quad_max(mt);
+      alpha[t] = __builtin_amdgcn_exp2f(m[t] - mt);
+      moved |= mt > m[t];
+      m[t] = mt;
+      l[t] *= alpha[t];
+#pragma unroll
+      for (int b = 0; b < 2; ++b)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          s[b][t][r] = __builtin_amdgcn_exp2f(s[b][t][r] - mt);
+          l[t] += s[b][t][r];
+        }
+    }
+    moved = __any(moved);
+    const int n = min(32, x1 - x);
+#pragma unroll
+    for (int b = 0; b < 2; ++b) {
+      if (16 * b >= n) break;
+      wave_sync();
+#pragma unroll
+      for (int t = 0; t < HT; ++t)
+        if (t * 16 + c < a.H) {
+#pragma unroll
+          for (int r = 0; r < 4; ++r) pw[(4 * quad + r) * p_row + at[t]] = s[b][t][r];
+          if (b == 0 && quad == 0) al[at[t]] = alpha[t];
+        }
+      wave_sync();
+      if (b == 0 && moved) {
+#pragma unroll
+        for (int j = 0; j < UL; ++j)
+#pragma unroll
+          for (int g = 0; g < GM; ++g) {
+            const float f = al[kvh[j] * GM + g];
+#pragma unroll
+            for (int e = 0; e < 8; ++e) acc[g][j][e] *= f;
+          }
+      }
+      constexpr int AHEAD = UL <= 2 ? 8 : 4;
+#pragma unroll
+      for (int i0 = 0; i0 < 16; i0 += AHEAD) {
+        Pack<bf16_t, 8> val[AHEAD][UL];
+#pragma unroll
+        for (int i = 0; i < AHEAD; ++i) {  // past the end: the last key again, weight 0
+          const int64_t sl = __builtin_amdgcn_readlane(slot, 16 * b + i0 + i);
+#pragma unroll
+          for (int j = 0; j < UL; ++j)
+            val[i][j] = *(const Pack<bf16_t, 8>*)(vc + (sl * units + unit[j]) * 8);
+        }
+#pragma unroll
+        for (int i = 0; i < AHEAD; ++i)
+#pragma unroll
+          for (int j = 0; j < UL; ++j) {
+            const Pack<float, GM> p = *(const Pack<float, GM>*)(pw + (i0 + i) * p_row + kvh[j] * GM);
+#pragma unroll
+            for (int e = 0; e < 8; ++e) {
+              const float y = to_f(val[i][j].v[e]);
+#pragma unroll
+              for (int g = 0; g < GM; ++g) acc[g][j][e] += p.v[g] * y;
+            }
+          }
+      }
+    }
+  }
+
+  __syncthreads();  // the long queries are read
+#pragma unroll
+  for (int t = 0; t < HT; ++t) {
+    const float sum = quad_sum(l[t]);
+    if (quad == 0 && t * 16 + c < a.H) ml[wid * a.H + t * 16 + c] = float2{m[t], sum};
+  }
+#pragma unroll
+  for (int j = 0; j < UL; ++j) {
+    if (lane + 64 * j >= units) continue;
+    const int e0 = unit[j] * 8 % v;
+#pragma unroll
+    for (int g = 0; g < GM; ++g)
+      if (g < group) {
+        float* o = merged + ((int64_t)wid * a.H + kvh[j] * group + g) * v + e0;
+        *(f32x4_v*)o = f32x4_v{acc[g][j][0], acc[g][j][1], acc[g][j][2], acc[g][j][3]};
+        *(f32x4_v*)(o + 4) = f32x4_v{acc[g][j][4], acc[g][j][5], acc[g][j][6], acc[g][j][7]};
+      }
+  }
+  __syncthreads();
+  for (int i = threadIdx.x; i < a.H * v; i += 256) {
+    const int h = i / v, e = i - h * v;
+    float mx = NEG, sum = 0.f, o = 0.f;
+#pragma unroll
+    for (int w = 0; w < 4; ++w) mx = fmaxf(mx, ml[w * a.H + h].x);
+#pragma unroll
+    for (int w = 0; w < 4; ++w) {
+      const float f = __builtin_amdgcn_exp2f(ml[w * a.H + h].x - mx);
+      sum += f * ml[w * a.H + h].y;
+      o += f * merged[(int64_t)w * a.H * v + i];
+    }
+    if (a.n_split == 1) {
+      ((bf16_t*)a.out)[seq * a.out_stride + i] = from_f<bf16_t>(o / sum);
+    } else {
+      const int64_t r = (int64_t)blockIdx.y * a.rows + row0 + h;
+      a.part[r * v + e] = o;
+      if (e == 0) a.part_ml[r] = float2{mx, sum};
+    }
+  }
+}
+
+static int decode_bytes(const GroupedArgs& a, int d, int v, int ht, int gm) {
+  const int q = a.G * d / 32 * ht * 1024, o = 16 * a.H * v;
+  return (q > o ? q : o) + 16 * (DEC_ROWS + 1) * (a.G * gm + 4) + 32 * a.H;
+}
+
+template <int HT, int GM, int UL>
+static void launch_decode(const GroupedArgs& a, int d, int v, int seqs, hipStream_t stream) {
+  static bool attr_set = false;
+  if (!attr_set) {
+    (void)hipFuncSetAttribute((const void*)talk_decode_kernel<HT, GM, UL>,
+                              hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+    attr_set = true;
+  }
+  talk_decode_kernel<HT, GM, UL>
+      <<<dim3(seqs, a.n_split), 256, decode_bytes(a, d, v, HT, GM), stream>>>(a, d, v);
+}
+
+template <int HT, int GM>
+static void launch_decode_units(const GroupedArgs& a, int d, int v, int seqs,
+                                hipStream_t stream) {
+  const int ul = (a.G * v / 8 + 63) / 64;
+  if (ul <= 1)
+    launch_decode<HT, GM, 1>(a, d, v, seqs, stream);
+  else if (ul <= 2)
+    launch_decode<HT, GM, 2>(a, d, v, seqs, stream);
+  else if constexpr (GM <= 4)
+    launch_decode<HT, GM, 4>(a, d, v, seqs, stream);
+}
+
+template <int HT>
+static void launch_decode_group(const GroupedArgs& a, int d, int v, int gm, int seqs,
+                                hipStream_t stream) {
+  (gm == 1   ? launch_decode_units<HT, 1>
+   : gm == 2 ? launch_decode_units<HT, 2>
+   : gm == 4 ? launch_decode_units<HT, 4>
+             : launch_decode_units<HT, 8>)(a, d, v, seqs, stream);
+}
+
+// ------------------------------------------------------------------ prompts
+
+#define KT 32   // keys of a tile
+#define PARTS 3  // bf16 parts of a score
+
+// Top, middle and low 8 bits of a score's 24, each a bf16.
+DEV void split_score(float s, unsigned* part) {
+  unsigned b = __float_as_uint(s);
+#pragma unroll
+  for (int i = 0; i < PARTS; ++i) {
+    part[i] = b >> 16;
+    s -= __uint_as_float(b & 0xffff0000u);
+    b = __float_as_uint(s);
+  }
+}
+
+struct PromptLds {  // offsets in bytes
+  int pitch, scores, part, weights, values, alpha, stats, total;
+};
+
+static __host__ __device__ inline PromptLds prompt_lds(int H, int G, int tokens, int v) {
+  PromptLds l;
+  l.pitch = (H + 7) / 8 * 16;  // of a (token, key) pair's scores in one part
+  if (l.pitch % 64 == 0) l.pitch += 16;
+  l.scores = 0;
+  l.part = tokens * KT * l.pitch;
+  l.weights = PARTS * l.part;               // [G][32 rows][KT] bf16
+  l.values = l.weights + G * 32 * KT * 2;   // [G][KT][v] bf16, swizzled
+  l.alpha = l.values + G * KT * v * 2;      // [G][32]
+  l.stats = l.alpha + G * 32 * 4;           // [tokens][H] maximum and sum
+  l.total = l.stats + tokens * H * 8;
+  return l;
+}
+
+// G waves, wave g for key/value head g: 32 rows, token * group + head of the group.
+// HT: 16-head tiles of the mix, KH: its inner steps of 32 heads.
+template <int DN, int VN, int HT>
+__global__ __launch_bounds__(512, 2) void talk_prefill_kernel(const GroupedArgs a) {
+  constexpr int D = 64 * DN, V = 64 * VN, STEPS = D / 32, VT = V / 16, VU = V / 8;
+  constexpr int KH = (HT + 1) / 2;
+  extern __shared__ char lds[];
+  const int group = a.H / a.G, TQ = 32 / group;
+  const PromptLds L = prompt_lds(a.H, a.G, TQ, V);
+  const int tile = a.n_tiles - 1 - blockIdx.x;
+  const int seq = a.tile_seq[tile], q0 = a.tile_q0[tile];
+  const int ctx = a.ctx_lens[seq];
+  const int tokens = min(TQ, a.seq_lens[seq] - ctx - q0);
+  const int64_t row0 = a.row_starts[seq] + q0;
+  const int* table = a.tables + (int64_t)seq * a.max_blocks;
+  const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
+  const int c = lane & 15, quad = lane >> 4;
+  const int head_end = (a.H + 7) / 8 * 8;  // scores beyond the heads, up to here, are zero
+
+  for (int i = threadIdx.x; i < L.weights / 16; i += blockDim.x)
+    ((ulonglong2*)lds)[i] = ulonglong2{0, 0};
+  float2* const stats = (float2*)(lds + L.stats);
+  for (int i = threadIdx.x; i < TQ * a.H; i += blockDim.x) stats[i] = float2{NEG, 0.f};
+
+  // this wave's queries; row 16 i + c.  Rows past the end repeat valid ones
+  bf16x8_v qf[2][STEPS];
+#pragma unroll
+  for (int i = 0; i < 2; ++i) {
+    const int r = 16 * i + c, t = min(r / group, tokens - 1);
+    const bf16_t* q = (const bf16_t*)a.q + (row0 + t) * a.q_stride +
+                      (int64_t)(wid * group + r % group) * D + quad * 8;
+#pragma unroll
+    for (int s = 0; s < STEPS; ++s) qf[i][s] = *(const bf16x8_v*)(q + s * 32);
+  }
+  // T, as the fragments of its product: output head 16 t + c, input heads 32 k + 8 quad ..
+  bf16x8_v tf[HT][KH];
+#pragma unroll
+  for (int t = 0; t < HT; ++t)
+#pragma unroll
+    for (int k = 0; k < KH; ++k)
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        const int h = 16 * t + c, g = 32 * k + 8 * quad + e;
+        tf[t][k][e] = (__bf16)(h < a.H && g < a.H ? a.talk[h * a.H + g] : 0.f);
+      }
+
+  const int k_end = ctx + q0 + tokens;
+  const int first = first_key(a, ctx + q0) / KT * KT;
+  const bf16_t* kc = (const bf16_t*)a.k_cache + (int64_t)wid * D + quad * 8;
+  const bf16_t* vc = (const bf16_t*)a.v_cache + (int64_t)wid * V;
+  char* const values = lds + L.values + wid * KT * V * 2;
+  char* const weights = lds + L.weights + wid * 32 * KT * 2;
+  auto find_slot = [&](int key0) {
+    const int k = min(key0 + (lane & 31), k_end - 1);
+    return table[k / a.kv_block] * a.kv_block + k % a.kv_block;
+  };
+  bf16x8_v kf[2][STEPS];
+  auto load_keys = [&](int slot) {
+#pragma unroll
+    for (int b = 0; b < 2; ++b) {
+      const bf16_t* k = kc + (int64_t)__shfl(slot, 16 * b + c, 64) * a.G * D;
+#pragma unroll
+      for (int s = 0; s < STEPS; ++s) kf[b][s] = *(const bf16x8_v*)(k + s * 32);
+    }
+  };
+
+  const float mul = a.scale * LOG2E;
+  f32x4_v o[2][VT] = {};
+  int slot = find_slot(first);
+  load_keys(slot);
+  __syncthreads();
+  for (int key0 = first; key0 < k_end; key0 += KT) {
+    // values of this tile, for this wave alone
+#pragma unroll
+    for (int i = 0; i < VU / 2; ++i) {
+      const int u = i * 64 + lane, key = u / VU;
+      const int unit = (u - key * VU) ^ (((key & 3) << 1) | ((key >> 2) & 1));
+      __builtin_amdgcn_global_load_lds(
+          (glob_char*)(vc + (int64_t)__shfl(slot, key, 64) * a.G * V + unit * 8),
+          (lds_char*)(values + i * 1024), 16, 0, 0);
+    }
+    const bool more = key0 + KT < k_end;
+    if (more) slot = find_slot(key0 + KT);
+
+    // raw scores: key 16 b + c, rows 16 i + 4 quad + r
+#pragma unroll
+    for (int b = 0; b < 2; ++b)
+#pragma unroll
+      for (int i = 0; i < 2; ++i) {
+        f32x4_v s = {};
+#pragma unroll
+        for (int st = 0; st < STEPS; ++st)
+          s = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qf[i][st], kf[b][st], s, 0, 0, 0);
+        unsigned p[4][PARTS];
+#pragma unroll
+        for (int r = 0; r < 4; ++r) split_score(s[r] * mul, p[r]);
+        const int r0 = 16 * i + 4 * quad;
+        char* dst = lds + (16 * b + c) * L.pitch;
+        if (group % 4 == 0) {  // four heads of one token
+          char* at = dst + r0 / group * KT * L.pitch + (wid * group + r0 % group) * 2;
+          if (r0 < TQ * group)
+#pragma unroll
+            for (int n = 0; n < PARTS; ++n)
+              *(uint2*)(at + n * L.part) =
+                  uint2{p[0][n] | p[1][n] << 16, p[2][n] | p[3][n] << 16};
+        } else if (group == 2) {  // two heads of two tokens
+#pragma unroll
+          for (int r = 0; r < 4; r += 2) {
+            char* at = dst + (r0 + r) / 2 * KT * L.pitch + wid * 4;
+#pragma unroll
+            for (int n = 0; n < PARTS; ++n)
+              *(unsigned*)(at + n * L.part) = p[r][n] | p[r + 1][n] << 16;
+          }
+        } else {
+#pragma unroll
+          for (int r = 0; r < 4; ++r) {
+            const int row = r0 + r;
+            char* at = dst + row / group * KT * L.pitch + (wid * group + row % group) * 2;
+            if (row < TQ * group)
+#pragma unroll
+              for (int n = 0; n < PARTS; ++n) *(unsigned short*)(at + n * L.part) = p[r][n];
+          }
+        }
+      }
+    if (more) load_keys(slot);
+    __syncthreads();
+
+    // mix and weigh, a wave per token: head 16 t + c, keys key0 + 16 b + 4 quad + r
+    for (int q = wid; q < tokens; q += a.G) {
+      const int pos = ctx + q0 + q, lo = first_key(a, pos);
+      f32x4_v s[2][HT] = {};
+#pragma unroll
+      for (int b = 0; b < 2; ++b) {
+        const char* src = lds + (q * KT + 16 * b + c) * L.pitch + quad * 16;
+#pragma unroll
+        for (int k = 0; k < KH; ++k)
+#pragma unroll
+          for (int n = 0; n < PARTS; ++n) {
+            bf16x8_v f = {};
+            if (32 * k + 8 * quad < head_end)
+              f = *(const bf16x8_v*)(src + k * 64 + n * L.part);
+#pragma unroll
+            for (int t = 0; t < HT; ++t)
+              s[b][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(f, tf[t][k], s[b][t], 0, 0, 0);
+          }
+      }
+      if (key0 + KT - 1 > pos || key0 < lo) {
+#pragma unroll
+        for (int b = 0; b < 2; ++b)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) {
+            const int key = key0 + 16 * b + 4 * quad + r;
+            if (key > pos || key < lo)
+#pragma unroll
+              for (int t = 0; t < HT; ++t) s[b][t][r] = -INFINITY;
+          }
+      }
+#pragma unroll
+      for (int t = 0; t < HT; ++t) {
+        const int h = 16 * t + c;
+        const bool has = h < a.H;
+        float mt = NEG;
+#pragma unroll
+        for (int b = 0; b < 2; ++b)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) mt = fmaxf(mt, s[b][t][r]);
+        const float2 old = stats[q * a.H + (has ? h : 0)];
+        mt = fmaxf(quad_max(mt), old.x);
+        float sum = 0.f;
+        const int g = h / group, row = q * group + h % group;
+        char* dst = lds + L.weights + (g * 32 + row) * KT * 2 + quad * 8;
+#pragma unroll
+        for (int b = 0; b < 2; ++b) {
+          float p[4];
+#pragma unroll
+          for (int r = 0; r < 4; ++r) {
+            p[r] = __builtin_amdgcn_exp2f(s[b][t][r] - mt);
+            sum += p[r];
+          }
+          if (has) store_f<4>((bf16_t*)(dst + b * 32), p);
+        }
+        sum = quad_sum(sum);
+        if (has && quad == 0) {
+          const float f = __builtin_amdgcn_exp2f(old.x - mt);
+          stats[q * a.H + h] = float2{mt, old.y * f + sum};
+          ((float*)(lds + L.alpha))[g * 32 + row] = f;
+        }
+      }
+    }
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");  // this wave's values have landed
+    __syncthreads();
+
+    // rows 16 i + 4 quad + r, dims 16 n + c
+    f32x4_v f[2];
+#pragma unroll
+    for (int i = 0; i < 2; ++i)
+      f[i] = *(const f32x4_v*)(lds + L.alpha + (wid * 32 + 16 * i + 4 * quad) * 4);
+    bool moved = false;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) moved |= f[0][r] != 1.f || f[1][r] != 1.f;
+    if (__any(moved)) {
+#pragma unroll
+      for (int i = 0; i < 2; ++i)
+#pragma unroll
+        for (int n = 0; n < VT; ++n) o[i][n] *= f[i];
+    }
+    bf16x8_v pf[2];
+#pragma unroll
+    for (int i = 0; i < 2; ++i)
+      pf[i] = *(const bf16x8_v*)(weights + (16 * i + c) * KT * 2 + quad * 16);
+    const int j = c >> 2, sw = j << 1;
+    const char* vrow = values + (quad * 8 + j) * V * 2 + (c & 1) * 8;
+#pragma unroll
+    for (int n = 0; n < VT; ++n) {
+      const int unit = n * 2 + ((c & 3) >> 1);
+      const bf16x4_v a0 = __builtin_amdgcn_ds_read_tr16_b64_v4bf16(
+          (lds_bf16x4*)(vrow + ((unit ^ sw) << 4)));
+      const bf16x4_v a1 = __builtin_amdgcn_ds_read_tr16_b64_v4bf16(
+          (lds_bf16x4*)(vrow + 4 * V * 2 + ((unit ^ (sw | 1)) << 4)));
+      const bf16x8_v vf = __builtin_shufflevector(a0, a1, 0, 1, 2, 3, 4, 5, 6, 7);
+#pragma unroll
+      for (int i = 0; i < 2; ++i)
+        o[i][n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pf[i], vf, o[i][n], 0, 0, 0);
+    }
+    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");  // the values may be overwritten
+  }
+
+#pragma unroll
+  for (int i = 0; i < 2; ++i)
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int row = 16 * i + 4 * quad + r, t = row / group;
+      if (t >= tokens || t >= TQ) continue;
+      const int h = wid * group + row % group;
+      const float inv = 1.f / stats[t * a.H + h].y;
+      bf16_t* dst = (bf16_t*)a.out + (row0 + t) * a.out_stride + (int64_t)h * V + c;
+#pragma unroll
+      for (int n = 0; n < VT; ++n) dst[16 * n] = from_f<bf16_t>(o[i][n][r] * inv);
+    }
+}
+
+template <int DN, int VN, int HT>
+static bool launch_prefill(const GroupedArgs& a, hipStream_t stream) {
+  const int bytes = prompt_lds(a.H, a.G, 32 / (a.H / a.G), 64 * VN).total;
+  if (bytes > 160 * 1024) return false;
+  static bool attr_set = false;
+  if (!attr_set) {
+    (void)hipFuncSetAttribute((const void*)talk_prefill_kernel<DN, VN, HT>,
+                              hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+    attr_set = true;
+  }
+  talk_prefill_kernel<DN, VN, HT><<<a.n_tiles, 64 * a.G, bytes, stream>>>(a);
+  return true;
+}
+
+template <int DN, int VN>
+static bool launch_prefill_heads(const GroupedArgs& a, hipStream_t stream) {
+  return a.H <= 16   ? launch_prefill<DN, VN, 1>(a, stream)
+         : a.H <= 32 ? launch_prefill<DN, VN, 2>(a, stream)
+                     : launch_prefill<DN, VN, 4>(a, stream);
+}
+
+static bool mixes(const GroupedArgs& a) {
+  return a.talk && !a.sink && !a.bias && !a.gate && !a.sigmoid && a.cap == 0.f && a.keep == 0;
+}
+
+extern "C" {
+
+// Tokens per workgroup of the prompt kernel for these sizes; 0: the plain kernel.
+int talk_prefill_tokens(int H, int G, int d, int v) {
+  const int group = H / G;
+  if ((d != 64 && d != 128) || (v != 64 && v != 128) || G > 8 || H > 64 || group > 32) return 0;
+  return prompt_lds(H, G, 32 / group, v).total <= 160 * 1024 ? 32 / group : 0;
+}
+
+bool launch_talk_prefill(const GroupedArgs* a, int d, int v, hipStream_t stream) {
+  if (!mixes(*a) || !talk_prefill_tokens(a->H, a->G, d, v)) return false;
+  if (d == 64)
+    return v == 64 ? launch_prefill_heads<1, 1>(*a, stream) : launch_prefill_heads<1, 2>(*a, stream);
+  return v == 64 ? launch_prefill_heads<2, 1>(*a, stream) : launch_prefill_heads<2, 2>(*a, stream);
+}
+
+static int group_width(int group) { return group <= 1 ? 1 : group <= 2 ? 2 : group <= 4 ? 4 : 8; }
+
+// Does the decode kernel take these sizes?
+bool talk_decode_fits(int H, int G, int d, int v) {
+  GroupedArgs a{};
+  a.H = H;
+  a.G = G;
+  const int gm = group_width(H / G), ul = (G * v / 8 + 63) / 64;
+  return d % 64 == 0 && v % 64 == 0 && H <= 64 && H / G <= 8 && ul <= (gm == 8 ? 2 : 4) &&
+         decode_bytes(a, d, v, H <= 16 ? 1 : H <= 32 ? 2 : 4, gm) <= 160 * 1024;
+}
+
+bool launch_talk_decode(const GroupedArgs* a, int d, int v, int seqs, hipStream_t stream) {
+  if (!mixes(*a) || !talk_decode_fits(a->H, a->G, d, v)) return false;
+  const int gm = group_width(a->H / a->G);
+  (a->H <= 16   ? launch_decode_group<1>
+   : a->H <= 32 ? launch_decode_group<2>
+                : launch_decode_group<4>)(*a, d, v, gm, seqs, stream);
+  if (a->n_split > 1) {
+    const SplitOut out = {a->out, a->gate, a->out_stride, a->gate_stride, a->H, a->sigmoid};
+    launch_split_combine(&out, a->part, a->part_ml, a->rows, v, a->n_split, stream);
+  }
+  return true;
+}
+
+}  // extern "C"

@@ -261,6 +261,8 @@ def test_cache_keys_values(device, dtype):
 class DeltaCase:
     """Inputs of several sequences and a step function over portions of them."""
 
+    options = {}  # of the op
+
     def __init__(self, H, G, D, V, taps, lens, dtype, device, seed=0, slots=None):
         self.shape = H, G, D, V, taps
         self.dtype, self.device, self.lens = dtype, device, lens
@@ -317,6 +319,7 @@ class DeltaCase:
             wide[:, : self.C], self.conv.to(self.device), wide[:, pad : pad + H], dev(self.z),
             self.A_log.to(self.device), self.dt_bias.to(self.device), dev(self.gate),
             self.norm.to(self.device), self.eps, self.unit_eps, G, self.state, self.ring, batch,
+            **self.options,
         ).cpu()
         at, got = 0, {}
         for s, n in chunks + single:
