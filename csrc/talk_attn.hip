@@ -25,7 +25,6 @@ typedef __bf16 bf16x4_v __attribute__((ext_vector_type(4)));
 typedef float f32x4_v __attribute__((ext_vector_type(4)));
 typedef __attribute__((address_space(3))) char lds_char;
 typedef __attribute__((address_space(3))) bf16x4_v lds_bf16x4;
-typedef __attribute__((address_space(1))) const char glob_char;
 
 #define NEG -1e30f
 #define LOG2E 1.44269504088896f
@@ -37,13 +36,21 @@ DEV void wave_sync() {
   __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
 }
 
-DEV float quad_max(float v) {  // over the lanes with this lane & 15
-  v = fmaxf(v, __shfl_xor(v, 16, 64));
-  return fmaxf(v, __shfl_xor(v, 32, 64));
+// Over the lanes with this lane & 15.  Swapping rows of 16 (halves) of a register with
+// itself leaves both members of every pair side by side.
+DEV float quad_max(float v) {
+  const unsigned b = __float_as_uint(v);
+  auto p = __builtin_amdgcn_permlane16_swap(b, b, false, false);
+  const unsigned m = __float_as_uint(fmaxf(__uint_as_float(p[0]), __uint_as_float(p[1])));
+  p = __builtin_amdgcn_permlane32_swap(m, m, false, false);
+  return fmaxf(__uint_as_float(p[0]), __uint_as_float(p[1]));
 }
 DEV float quad_sum(float v) {
-  v += __shfl_xor(v, 16, 64);
-  return v + __shfl_xor(v, 32, 64);
+  const unsigned b = __float_as_uint(v);
+  auto p = __builtin_amdgcn_permlane16_swap(b, b, false, false);
+  const unsigned m = __float_as_uint(__uint_as_float(p[0]) + __uint_as_float(p[1]));
+  p = __builtin_amdgcn_permlane32_swap(m, m, false, false);
+  return __uint_as_float(p[0]) + __uint_as_float(p[1]);
 }
 
 // ------------------------------------------------------------------ decode
@@ -308,38 +315,56 @@ static void launch_decode_group(const GroupedArgs& a, int d, int v, int gm, int 
 #define KT 32   // keys of a tile
 #define PARTS 3  // bf16 parts of a score
 
-// Top, middle and low 8 bits of a score's 24, each a bf16.
-DEV void split_score(float s, unsigned* part) {
-  unsigned b = __float_as_uint(s);
+// Eight scores as fragments of the mix: top, middle and low 8 bits of their 24.
+DEV void split_scores(const float* x, bf16x8_v* part) {
+  unsigned w[PARTS][4];
 #pragma unroll
-  for (int i = 0; i < PARTS; ++i) {
-    part[i] = b >> 16;
-    s -= __uint_as_float(b & 0xffff0000u);
-    b = __float_as_uint(s);
+  for (int e = 0; e < 8; e += 2) {
+    float lo = x[e], hi = x[e + 1];
+#pragma unroll
+    for (int n = 0; n < PARTS; ++n) {
+      const unsigned l = __float_as_uint(lo), h = __float_as_uint(hi);
+      w[n][e / 2] = __builtin_amdgcn_perm(h, l, 0x07060302);  // upper halves
+      lo -= __uint_as_float(l & 0xffff0000u);
+      hi -= __uint_as_float(h & 0xffff0000u);
+    }
   }
+#pragma unroll
+  for (int n = 0; n < PARTS; ++n) part[n] = __builtin_bit_cast(bf16x8_v, w[n]);
+}
+
+// 16 bytes a lane straight to LDS, lanes side by side.  As assembly, since the compiler
+// would wait for the builtin's loads ahead of every LDS access; the caller waits, once.
+DEV void load_to_lds(char* dst, const void* src) {
+  const unsigned at =
+      __builtin_amdgcn_readfirstlane((unsigned)(uintptr_t)(lds_char*)dst);
+  asm volatile("s_mov_b32 m0, %0\n\ts_nop 0\n\tglobal_load_lds_dwordx4 %1, off"
+               :: "s"(at), "v"(src) : "memory", "m0");
 }
 
 struct PromptLds {  // offsets in bytes
-  int pitch, scores, part, weights, values, alpha, stats, total;
+  int pitch, weights, values, alpha, stats, total;
 };
 
 static __host__ __device__ inline PromptLds prompt_lds(int H, int G, int tokens, int v) {
   PromptLds l;
-  l.pitch = (H + 7) / 8 * 16;  // of a (token, key) pair's scores in one part
-  if (l.pitch % 64 == 0) l.pitch += 16;
-  l.scores = 0;
-  l.part = tokens * KT * l.pitch;
-  l.weights = PARTS * l.part;               // [G][32 rows][KT] bf16
-  l.values = l.weights + G * 32 * KT * 2;   // [G][KT][v] bf16, swizzled
-  l.alpha = l.values + G * KT * v * 2;      // [G][32]
-  l.stats = l.alpha + G * 32 * 4;           // [tokens][H] maximum and sum
+  // of a (token, key) pair's fp32 scores, an odd number of 16-byte units
+  l.pitch = ((H + 3) / 4 | 1) * 16;
+  l.weights = tokens * KT * l.pitch;            // [2][G][32 rows][KT] bf16
+  l.values = l.weights + 2 * G * 32 * KT * 2;   // [G][KT][v] bf16, swizzled
+  l.alpha = l.values + G * KT * v * 2;          // [2][G][32]
+  l.stats = l.alpha + 2 * G * 32 * 4;           // [tokens][H] maximum and sum
   l.total = l.stats + tokens * H * 8;
   return l;
 }
 
 // G waves, wave g for key/value head g: 32 rows, token * group + head of the group.
-// HT: 16-head tiles of the mix, KH: its inner steps of 32 heads.
-template <int DN, int VN, int HT>
+// HT: 16-head tiles of the mix, KH: its inner steps of 32 heads.  GV: heads of a group that
+// are stored together, 4, 2 or 1.
+//
+// Between two barriers a wave mixes a tile's scores for its tokens, makes the next tile's
+// raw scores and adds the last tile's values; the raw scores then replace the mixed ones.
+template <int DN, int VN, int HT, int GV>
 __global__ __launch_bounds__(512, 2) void talk_prefill_kernel(const GroupedArgs a) {
   constexpr int D = 64 * DN, V = 64 * VN, STEPS = D / 32, VT = V / 16, VU = V / 8;
   constexpr int KH = (HT + 1) / 2;
@@ -354,8 +379,8 @@ __global__ __launch_bounds__(512, 2) void talk_prefill_kernel(const GroupedArgs 
   const int* table = a.tables + (int64_t)seq * a.max_blocks;
   const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
   const int c = lane & 15, quad = lane >> 4;
-  const int head_end = (a.H + 7) / 8 * 8;  // scores beyond the heads, up to here, are zero
 
+  // scores beyond the heads stay zero
   for (int i = threadIdx.x; i < L.weights / 16; i += blockDim.x)
     ((ulonglong2*)lds)[i] = ulonglong2{0, 0};
   float2* const stats = (float2*)(lds + L.stats);
@@ -376,22 +401,26 @@ __global__ __launch_bounds__(512, 2) void talk_prefill_kernel(const GroupedArgs 
 #pragma unroll
   for (int t = 0; t < HT; ++t)
 #pragma unroll
-    for (int k = 0; k < KH; ++k)
+    for (int k = 0; k < KH; ++k) {
+      float x[8];
 #pragma unroll
-      for (int e = 0; e < 8; ++e) {
-        const int h = 16 * t + c, g = 32 * k + 8 * quad + e;
-        tf[t][k][e] = (__bf16)(h < a.H && g < a.H ? a.talk[h * a.H + g] : 0.f);
-      }
+      for (int e = 0; e < 8; ++e)
+        x[e] = a.talk[min(16 * t + c, a.H - 1) * a.H + min(32 * k + 8 * quad + e, a.H - 1)];
+#pragma unroll
+      for (int e = 0; e < 8; ++e)
+        tf[t][k][e] = (__bf16)(16 * t + c < a.H && 32 * k + 8 * quad + e < a.H ? x[e] : 0.f);
+    }
 
   const int k_end = ctx + q0 + tokens;
   const int first = first_key(a, ctx + q0) / KT * KT;
+  const int n_tiles = (k_end - first + KT - 1) / KT;
   const bf16_t* kc = (const bf16_t*)a.k_cache + (int64_t)wid * D + quad * 8;
   const bf16_t* vc = (const bf16_t*)a.v_cache + (int64_t)wid * V;
   char* const values = lds + L.values + wid * KT * V * 2;
-  char* const weights = lds + L.weights + wid * 32 * KT * 2;
-  auto find_slot = [&](int key0) {
-    const int k = min(key0 + (lane & 31), k_end - 1);
-    return table[k / a.kv_block] * a.kv_block + k % a.kv_block;
+  // this lane's key of tile t: its page's place in the table, its place in the page
+  auto key_of = [&](int t) { return min(first + t * KT + (lane & 31), k_end - 1); };
+  auto slot_of = [&](int t, int page, int block) {
+    return block * a.kv_block + key_of(t) - page * a.kv_block;
   };
   bf16x8_v kf[2][STEPS];
   auto load_keys = [&](int slot) {
@@ -402,138 +431,67 @@ __global__ __launch_bounds__(512, 2) void talk_prefill_kernel(const GroupedArgs 
       for (int s = 0; s < STEPS; ++s) kf[b][s] = *(const bf16x8_v*)(k + s * 32);
     }
   };
-
-  const float mul = a.scale * LOG2E;
-  f32x4_v o[2][VT] = {};
-  int slot = find_slot(first);
-  load_keys(slot);
-  __syncthreads();
-  for (int key0 = first; key0 < k_end; key0 += KT) {
-    // values of this tile, for this wave alone
+  auto load_values = [&](int slot) {  // for this wave alone
 #pragma unroll
     for (int i = 0; i < VU / 2; ++i) {
       const int u = i * 64 + lane, key = u / VU;
       const int unit = (u - key * VU) ^ (((key & 3) << 1) | ((key >> 2) & 1));
-      __builtin_amdgcn_global_load_lds(
-          (glob_char*)(vc + (int64_t)__shfl(slot, key, 64) * a.G * V + unit * 8),
-          (lds_char*)(values + i * 1024), 16, 0, 0);
+      load_to_lds(values + i * 1024, vc + (int64_t)__shfl(slot, key, 64) * a.G * V + unit * 8);
     }
-    const bool more = key0 + KT < k_end;
-    if (more) slot = find_slot(key0 + KT);
+  };
 
-    // raw scores: key 16 b + c, rows 16 i + 4 quad + r
+  const float mul = a.scale * LOG2E;
+  // where this lane's rows 16 i + 4 quad + (0, GV, ..) of raw scores go, or -1
+  int put[2][4 / GV];
+#pragma unroll
+  for (int i = 0; i < 2; ++i)
+#pragma unroll
+    for (int r = 0; r < 4 / GV; ++r) {
+      const int row = 16 * i + 4 * quad + r * GV;
+      put[i][r] = row < TQ * group ? (row / group * KT + c) * L.pitch +
+                                         (wid * group + row % group) * 4 : -1;
+    }
+  f32x4_v raw[2][2];  // key 16 b + c, rows 16 i + 4 quad + r
+  auto score = [&]() {
+#pragma unroll
+    for (int b = 0; b < 2; ++b)
+#pragma unroll
+      for (int i = 0; i < 2; ++i) raw[b][i] = f32x4_v{};
+#pragma unroll
+    for (int st = 0; st < STEPS; ++st)
+#pragma unroll
+      for (int b = 0; b < 2; ++b)
+#pragma unroll
+        for (int i = 0; i < 2; ++i)
+          raw[b][i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qf[i][st], kf[b][st], raw[b][i], 0,
+                                                              0, 0);
+  };
+  auto put_scores = [&]() {
 #pragma unroll
     for (int b = 0; b < 2; ++b)
 #pragma unroll
       for (int i = 0; i < 2; ++i) {
-        f32x4_v s = {};
+        const f32x4_v s = raw[b][i] * mul;
 #pragma unroll
-        for (int st = 0; st < STEPS; ++st)
-          s = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qf[i][st], kf[b][st], s, 0, 0, 0);
-        unsigned p[4][PARTS];
+        for (int r = 0; r < 4 / GV; ++r) {
+          if (put[i][r] < 0) continue;
+          float* at = (float*)(lds + put[i][r] + 16 * b * L.pitch);
+          if constexpr (GV == 4) {
+            *(f32x4_v*)at = s;
+          } else {
 #pragma unroll
-        for (int r = 0; r < 4; ++r) split_score(s[r] * mul, p[r]);
-        const int r0 = 16 * i + 4 * quad;
-        char* dst = lds + (16 * b + c) * L.pitch;
-        if (group % 4 == 0) {  // four heads of one token
-          char* at = dst + r0 / group * KT * L.pitch + (wid * group + r0 % group) * 2;
-          if (r0 < TQ * group)
-#pragma unroll
-            for (int n = 0; n < PARTS; ++n)
-              *(uint2*)(at + n * L.part) =
-                  uint2{p[0][n] | p[1][n] << 16, p[2][n] | p[3][n] << 16};
-        } else if (group == 2) {  // two heads of two tokens
-#pragma unroll
-          for (int r = 0; r < 4; r += 2) {
-            char* at = dst + (r0 + r) / 2 * KT * L.pitch + wid * 4;
-#pragma unroll
-            for (int n = 0; n < PARTS; ++n)
-              *(unsigned*)(at + n * L.part) = p[r][n] | p[r + 1][n] << 16;
-          }
-        } else {
-#pragma unroll
-          for (int r = 0; r < 4; ++r) {
-            const int row = r0 + r;
-            char* at = dst + row / group * KT * L.pitch + (wid * group + row % group) * 2;
-            if (row < TQ * group)
-#pragma unroll
-              for (int n = 0; n < PARTS; ++n) *(unsigned short*)(at + n * L.part) = p[r][n];
+            for (int e = 0; e < GV; ++e) at[e] = s[r * GV + e];
           }
         }
       }
-    if (more) load_keys(slot);
-    __syncthreads();
-
-    // mix and weigh, a wave per token: head 16 t + c, keys key0 + 16 b + 4 quad + r
-    for (int q = wid; q < tokens; q += a.G) {
-      const int pos = ctx + q0 + q, lo = first_key(a, pos);
-      f32x4_v s[2][HT] = {};
-#pragma unroll
-      for (int b = 0; b < 2; ++b) {
-        const char* src = lds + (q * KT + 16 * b + c) * L.pitch + quad * 16;
-#pragma unroll
-        for (int k = 0; k < KH; ++k)
-#pragma unroll
-          for (int n = 0; n < PARTS; ++n) {
-            bf16x8_v f = {};
-            if (32 * k + 8 * quad < head_end)
-              f = *(const bf16x8_v*)(src + k * 64 + n * L.part);
-#pragma unroll
-            for (int t = 0; t < HT; ++t)
-              s[b][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(f, tf[t][k], s[b][t], 0, 0, 0);
-          }
-      }
-      if (key0 + KT - 1 > pos || key0 < lo) {
-#pragma unroll
-        for (int b = 0; b < 2; ++b)
-#pragma unroll
-          for (int r = 0; r < 4; ++r) {
-            const int key = key0 + 16 * b + 4 * quad + r;
-            if (key > pos || key < lo)
-#pragma unroll
-              for (int t = 0; t < HT; ++t) s[b][t][r] = -INFINITY;
-          }
-      }
-#pragma unroll
-      for (int t = 0; t < HT; ++t) {
-        const int h = 16 * t + c;
-        const bool has = h < a.H;
-        float mt = NEG;
-#pragma unroll
-        for (int b = 0; b < 2; ++b)
-#pragma unroll
-          for (int r = 0; r < 4; ++r) mt = fmaxf(mt, s[b][t][r]);
-        const float2 old = stats[q * a.H + (has ? h : 0)];
-        mt = fmaxf(quad_max(mt), old.x);
-        float sum = 0.f;
-        const int g = h / group, row = q * group + h % group;
-        char* dst = lds + L.weights + (g * 32 + row) * KT * 2 + quad * 8;
-#pragma unroll
-        for (int b = 0; b < 2; ++b) {
-          float p[4];
-#pragma unroll
-          for (int r = 0; r < 4; ++r) {
-            p[r] = __builtin_amdgcn_exp2f(s[b][t][r] - mt);
-            sum += p[r];
-          }
-          if (has) store_f<4>((bf16_t*)(dst + b * 32), p);
-        }
-        sum = quad_sum(sum);
-        if (has && quad == 0) {
-          const float f = __builtin_amdgcn_exp2f(old.x - mt);
-          stats[q * a.H + h] = float2{mt, old.y * f + sum};
-          ((float*)(lds + L.alpha))[g * 32 + row] = f;
-        }
-      }
-    }
-    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");  // this wave's values have landed
-    __syncthreads();
-
-    // rows 16 i + 4 quad + r, dims 16 n + c
+  };
+  f32x4_v o[2][VT] = {};  // rows 16 i + 4 quad + r, dims 16 n + c
+  auto add_values = [&](int t) {
+    const char* weights = lds + L.weights + ((t & 1) * a.G + wid) * 32 * KT * 2;
+    const float* alpha = (const float*)(lds + L.alpha) + ((t & 1) * a.G + wid) * 32;
     f32x4_v f[2];
 #pragma unroll
-    for (int i = 0; i < 2; ++i)
-      f[i] = *(const f32x4_v*)(lds + L.alpha + (wid * 32 + 16 * i + 4 * quad) * 4);
+    for (int i = 0; i < 2; ++i) f[i] = *(const f32x4_v*)(alpha + 16 * i + 4 * quad);
     bool moved = false;
 #pragma unroll
     for (int r = 0; r < 4; ++r) moved |= f[0][r] != 1.f || f[1][r] != 1.f;
@@ -561,8 +519,113 @@ __global__ __launch_bounds__(512, 2) void talk_prefill_kernel(const GroupedArgs 
       for (int i = 0; i < 2; ++i)
         o[i][n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pf[i], vf, o[i][n], 0, 0, 0);
     }
-    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");  // the values may be overwritten
+  };
+
+  // slots of the keys of tiles t, t + 1 and t + 2
+  int page = key_of(0) / a.kv_block;
+  int here = slot_of(0, page, table[page]);
+  load_keys(here);
+  page = key_of(1) / a.kv_block;
+  int next = slot_of(1, page, table[page]);
+  page = key_of(2) / a.kv_block;
+  int block = table[page];
+  __syncthreads();
+  score();
+  load_keys(next);
+  put_scores();
+  __syncthreads();
+
+  for (int t = 0; t < n_tiles; ++t) {
+    const int key0 = first + t * KT;
+    // a wave per token: head 16 h + c, keys key0 + 16 b + 4 quad + r
+    for (int q = wid; q < tokens; q += a.G) {
+      const int pos = ctx + q0 + q, lo = first_key(a, pos);
+      f32x4_v s[2][HT] = {};
+#pragma unroll
+      for (int b = 0; b < 2; ++b) {
+        const char* src = lds + (q * KT + 16 * b + c) * L.pitch;
+#pragma unroll
+        for (int k = 0; k < KH; ++k) {
+          float x[8];
+#pragma unroll
+          for (int e = 0; e < 8; e += 4) {
+            const int at = (32 * k + 8 * quad + e) * 4;
+            f32x4_v y = {};
+            if (at < L.pitch) y = *(const f32x4_v*)(src + at);
+#pragma unroll
+            for (int i = 0; i < 4; ++i) x[e + i] = y[i];
+          }
+          bf16x8_v f[PARTS];
+          split_scores(x, f);
+#pragma unroll
+          for (int n = 0; n < PARTS; ++n)
+#pragma unroll
+            for (int h = 0; h < HT; ++h)
+              s[b][h] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(f[n], tf[h][k], s[b][h], 0, 0, 0);
+        }
+      }
+      if (key0 + KT - 1 > pos || key0 < lo) {
+#pragma unroll
+        for (int b = 0; b < 2; ++b)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) {
+            const int key = key0 + 16 * b + 4 * quad + r;
+            const bool seen = key <= pos && key >= lo;
+#pragma unroll
+            for (int h = 0; h < HT; ++h) s[b][h][r] = seen ? s[b][h][r] : -INFINITY;
+          }
+      }
+#pragma unroll
+      for (int n = 0; n < HT; ++n) {
+        const int h = 16 * n + c;
+        const bool has = h < a.H;
+        float mt = NEG;
+#pragma unroll
+        for (int b = 0; b < 2; ++b)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) mt = fmaxf(mt, s[b][n][r]);
+        const float2 old = stats[q * a.H + (has ? h : 0)];
+        mt = fmaxf(quad_max(mt), old.x);
+        float sum = 0.f;
+        const int at = ((t & 1) * a.G + h / group) * 32 + q * group + h % group;
+        char* dst = lds + L.weights + at * KT * 2 + quad * 8;
+#pragma unroll
+        for (int b = 0; b < 2; ++b) {
+          float p[4];
+#pragma unroll
+          for (int r = 0; r < 4; ++r) {
+            p[r] = __builtin_amdgcn_exp2f(s[b][n][r] - mt);
+            sum += p[r];
+          }
+          if (has) store_f<4>((bf16_t*)(dst + b * 32), p);
+        }
+        sum = quad_sum(sum);
+        if (has && quad == 0) {
+          const float f = __builtin_amdgcn_exp2f(old.x - mt);
+          stats[q * a.H + h] = float2{mt, old.y * f + sum};
+          ((float*)(lds + L.alpha))[at] = f;
+        }
+      }
+    }
+    score();  // of tile t + 1
+    if (t > 0) {
+      asm volatile("s_waitcnt vmcnt(0)" ::: "memory");    // the last tile's values are here
+      add_values(t - 1);
+      asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");  // and may be overwritten
+    }
+    const int after = slot_of(t + 2, page, block);
+    load_keys(after);
+    load_values(here);
+    here = next;
+    next = after;
+    page = key_of(t + 3) / a.kv_block;
+    block = table[page];
+    __syncthreads();
+    put_scores();
+    __syncthreads();
   }
+  asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+  add_values(n_tiles - 1);
 
 #pragma unroll
   for (int i = 0; i < 2; ++i)
@@ -578,25 +641,33 @@ __global__ __launch_bounds__(512, 2) void talk_prefill_kernel(const GroupedArgs 
     }
 }
 
-template <int DN, int VN, int HT>
+template <int DN, int VN, int HT, int GV>
 static bool launch_prefill(const GroupedArgs& a, hipStream_t stream) {
   const int bytes = prompt_lds(a.H, a.G, 32 / (a.H / a.G), 64 * VN).total;
   if (bytes > 160 * 1024) return false;
   static bool attr_set = false;
   if (!attr_set) {
-    (void)hipFuncSetAttribute((const void*)talk_prefill_kernel<DN, VN, HT>,
+    (void)hipFuncSetAttribute((const void*)talk_prefill_kernel<DN, VN, HT, GV>,
                               hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
     attr_set = true;
   }
-  talk_prefill_kernel<DN, VN, HT><<<a.n_tiles, 64 * a.G, bytes, stream>>>(a);
+  talk_prefill_kernel<DN, VN, HT, GV><<<a.n_tiles, 64 * a.G, bytes, stream>>>(a);
   return true;
+}
+
+template <int DN, int VN, int HT>
+static bool launch_prefill_group(const GroupedArgs& a, hipStream_t stream) {
+  const int group = a.H / a.G;
+  return group % 4 == 0   ? launch_prefill<DN, VN, HT, 4>(a, stream)
+         : group % 2 == 0 ? launch_prefill<DN, VN, HT, 2>(a, stream)
+                          : launch_prefill<DN, VN, HT, 1>(a, stream);
 }
 
 template <int DN, int VN>
 static bool launch_prefill_heads(const GroupedArgs& a, hipStream_t stream) {
-  return a.H <= 16   ? launch_prefill<DN, VN, 1>(a, stream)
-         : a.H <= 32 ? launch_prefill<DN, VN, 2>(a, stream)
-                     : launch_prefill<DN, VN, 4>(a, stream);
+  return a.H <= 16   ? launch_prefill_group<DN, VN, 1>(a, stream)
+         : a.H <= 32 ? launch_prefill_group<DN, VN, 2>(a, stream)
+                     : launch_prefill_group<DN, VN, 4>(a, stream);
 }
 
 static bool mixes(const GroupedArgs& a) {
