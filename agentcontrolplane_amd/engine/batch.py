@@ -181,11 +181,12 @@ class PrefillMeta:
     def build(prefills: List[SeqMeta], device, tile_q: int = 64,
               stager=None, rows_per_token: int = 1,
               only: Optional[Sequence[int]] = None, row_base: int = 0,
-              window: Optional[int] = None) -> "PrefillMeta":
+              window: Optional[int] = None, chunk: Optional[int] = None) -> "PrefillMeta":
         """Tiles of ``tile_q`` query rows; a token is ``rows_per_token`` rows
         (its heads, for kernels that tile over both).  ``only`` picks chunks;
         rows count from ``row_base``.  ``window`` lays out the keys the chunks
-        see one after the other."""
+        see one after the other.  ``chunk`` orders the tiles by the keys they see, the
+        fewest first, where a query sees those of its own chunk of positions."""
         picked = [
             (i, m) for i, m in enumerate(prefills) if only is None or i in set(only)
         ]
@@ -210,8 +211,16 @@ class PrefillMeta:
                 key_starts.append(num_keys)
                 num_keys += m.seq_len - key_first[-1]
                 max_keys = max(max_keys, m.seq_len - key_first[-1])
+        if chunk is not None:
+            def keys(tile):
+                m, q0 = picked[tile[0]][1], tile[1] // rows_per_token
+                start = (m.ctx_len + q0) // chunk * chunk
+                return m.ctx_len + min(q0 + tile_q // rows_per_token, m.query_len) - start
+
+            tiles = sorted(zip(tile_seq, tile_q0), key=keys)
+            tile_seq, tile_q0 = [s for s, _ in tiles], [q for _, q in tiles]
         if stager is not None:
-            tag = f"pm{tile_q}x{rows_per_token}o{only}b{row_base}w{window}"
+            tag = f"pm{tile_q}x{rows_per_token}o{only}b{row_base}w{window}c{chunk}"
             t = lambda n, x: stager.tensor(f"{tag}_{n}", x, "int32")  # noqa: E731
         else:
             t = lambda n, x: torch.tensor(x, device=device, dtype=torch.int32)  # noqa: E731

@@ -357,7 +357,7 @@ def grouped_attention(q, k_cache, v_cache, batch, scale: float, cap, window, kee
     else:
         tiled = bf16 and not (sigmoid or cap or keep_first) and all(
             t is None for t in (sink, bias, gate))
-        tile = _C.talk_prefill_tokens(H, G, d, v) if tiled else 0
+        tile = _C.talk_prefill_tokens(H, G, d, v, k_cache.shape[1]) if tiled else 0
         tiled = tiled and _C.talk_decode_fits(H, G, d, v)
         kinds = (_TALK_DECODE if tiled else _PLAIN, _TALK_PREFILL if tile else _PLAIN)
     P = batch.num_prefill_tokens
@@ -366,7 +366,10 @@ def grouped_attention(q, k_cache, v_cache, batch, scale: float, cap, window, kee
         return None if gate is None else gate[r]
 
     if batch.prefills:
-        meta = batch.prefill_meta(tile if kinds[1] != _PLAIN else 1)
+        if kinds[1] == _TALK_PREFILL:
+            meta = batch.prefill_meta(tile, chunk=chunk or _NO_WINDOW)
+        else:
+            meta = batch.prefill_meta(1 if kinds[1] == _PLAIN else tile)
         _C.grouped_attn(
             out[:P], q[:P], k_cache, v_cache, meta.block_tables, meta.seq_lens, meta.ctx_lens,
             meta.row_starts, meta.tile_seq, meta.tile_q0, sink, bias, gates(slice(0, P)), talk,

@@ -57,7 +57,7 @@ void launch_softcap(bool, float*, const void*, float, int64_t, hipStream_t);
 bool launch_grouped_decode(const GroupedArgs*, int, int, int, int, hipStream_t);
 bool launch_grouped_plain(bool, const GroupedArgs*, int, int, int, hipStream_t);
 bool launch_grouped_prefill(const GroupedArgs*, int, int, hipStream_t);
-int talk_prefill_tokens(int, int, int, int);
+int talk_prefill_tokens(int, int, int, int, int);
 bool talk_decode_fits(int, int, int, int);
 bool launch_talk_prefill(const GroupedArgs*, int, int, hipStream_t);
 bool launch_talk_decode(const GroupedArgs*, int, int, int, hipStream_t);

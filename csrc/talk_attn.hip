@@ -90,24 +90,30 @@ __global__ __launch_bounds__(256, 2) void talk_decode_kernel(const GroupedArgs a
 
   {  // long queries, as fragments: step u / 4, lane (u % 4) * 16 + h % 16
     const bf16_t* q = (const bf16_t*)a.q + seq * a.q_stride;
-    const int row_units = DK / 8;
-    for (int i = threadIdx.x; i < 16 * HT * row_units; i += 256) {
-      const int u = i % row_units, h = i / row_units;
+    // a thread has one unit of 8 dims at a time, for every ``turns``-th head
+    const int row_units = DK / 8, turns = max(1, 256 / row_units);
+    const int turn = row_units < 256 ? threadIdx.x / row_units : 0;
+    for (int u = threadIdx.x - turn * row_units; u < row_units && turn < turns; u += 256) {
       const int g0 = u * 8 / d * group, e0 = u * 8 % d;
-      float x[8] = {};
-      if (h < a.H) {
-        for (int g = g0; g < g0 + group; ++g) {
-          const float t = a.talk[h * a.H + g];
-          float y[8];
-          load_f<8>(y, q + (int64_t)g * d + e0);
+      float y[GM][8];
 #pragma unroll
-          for (int e = 0; e < 8; ++e) x[e] += t * y[e];
+      for (int g = 0; g < GM; ++g)
+        load_f<8>(y[g], q + (int64_t)(g0 + min(g, group - 1)) * d + e0);
+#pragma unroll 4
+      for (int h = turn; h < 16 * HT; h += turns) {
+        float x[8] = {};
+#pragma unroll
+        for (int g = 0; g < GM; ++g) {
+          const float t = a.talk[min(h, a.H - 1) * a.H + g0 + min(g, group - 1)];
+          const float f = h < a.H && g < group ? t : 0.f;
+#pragma unroll
+          for (int e = 0; e < 8; ++e) x[e] += f * y[g][e];
         }
-      }
-      bf16x8_v f;
+        bf16x8_v f;
 #pragma unroll
-      for (int e = 0; e < 8; ++e) f[e] = (__bf16)x[e];
-      qf[((u >> 2) * HT + (h >> 4)) * 64 + (u & 3) * 16 + (h & 15)] = f;
+        for (int e = 0; e < 8; ++e) f[e] = (__bf16)x[e];
+        qf[((u >> 2) * HT + (h >> 4)) * 64 + (u & 3) * 16 + (h & 15)] = f;
+      }
     }
   }
   __syncthreads();
@@ -333,28 +339,42 @@ DEV void split_scores(const float* x, bf16x8_v* part) {
   for (int n = 0; n < PARTS; ++n) part[n] = __builtin_bit_cast(bf16x8_v, w[n]);
 }
 
-// 16 bytes a lane straight to LDS, lanes side by side.  As assembly, since the compiler
-// would wait for the builtin's loads ahead of every LDS access; the caller waits, once.
-DEV void load_to_lds(char* dst, const void* src) {
-  const unsigned at =
-      __builtin_amdgcn_readfirstlane((unsigned)(uintptr_t)(lds_char*)dst);
-  asm volatile("s_mov_b32 m0, %0\n\ts_nop 0\n\tglobal_load_lds_dwordx4 %1, off"
-               :: "s"(at), "v"(src) : "memory", "m0");
+// 16 bytes a lane, from src (the same in all lanes) + offset straight to LDS, lanes side by
+// side.  As assembly, since the compiler would wait for the builtin's loads ahead of every
+// LDS access; the caller waits, once.
+DEV void load_to_lds(unsigned dst, const char* src, unsigned offset) {
+  const uint64_t p = (uint64_t)src;
+  const uint64_t at = (uint64_t)__builtin_amdgcn_readfirstlane((unsigned)(p >> 32)) << 32 |
+                      (unsigned)__builtin_amdgcn_readfirstlane((unsigned)p);
+  asm volatile("s_mov_b32 m0, %0\n\ts_nop 0\n\tglobal_load_lds_dwordx4 %1, %2"
+               :: "s"(dst), "v"(offset), "s"(at) : "memory", "m0");
+}
+
+// unit of a key's values in LDS: the keys that one transposing read takes are spread over
+// the banks
+template <int VU>
+DEV int swizzled(int unit, int key) {
+  return unit ^ (((key & 3) << 1 | (key >> 2 & 1) | (key & 8)) & (VU - 1));
 }
 
 struct PromptLds {  // offsets in bytes
-  int pitch, weights, values, alpha, stats, total;
+  int pitch, weights, values, alpha, stats, lows, total;
 };
+
+// weights of one key/value head: 32 rows of KT bf16, and an offset between heads that
+// spreads them over the banks
+#define W_HEAD (32 * KT * 2 + 32)
 
 static __host__ __device__ inline PromptLds prompt_lds(int H, int G, int tokens, int v) {
   PromptLds l;
   // of a (token, key) pair's fp32 scores, an odd number of 16-byte units
   l.pitch = ((H + 3) / 4 | 1) * 16;
-  l.weights = tokens * KT * l.pitch;            // [2][G][32 rows][KT] bf16
-  l.values = l.weights + 2 * G * 32 * KT * 2;   // [G][KT][v] bf16, swizzled
+  l.weights = tokens * KT * l.pitch;            // [2][G] W_HEAD
+  l.values = l.weights + 2 * G * W_HEAD;        // [G][KT][v] bf16, swizzled
   l.alpha = l.values + G * KT * v * 2;          // [2][G][32]
   l.stats = l.alpha + 2 * G * 32 * 4;           // [tokens][H] maximum and sum
-  l.total = l.stats + tokens * H * 8;
+  l.lows = l.stats + tokens * H * 8;            // [tokens] first visible key
+  l.total = l.lows + tokens * 4;
   return l;
 }
 
@@ -385,6 +405,8 @@ __global__ __launch_bounds__(512, 2) void talk_prefill_kernel(const GroupedArgs 
     ((ulonglong2*)lds)[i] = ulonglong2{0, 0};
   float2* const stats = (float2*)(lds + L.stats);
   for (int i = threadIdx.x; i < TQ * a.H; i += blockDim.x) stats[i] = float2{NEG, 0.f};
+  int* const lows = (int*)(lds + L.lows);
+  if ((int)threadIdx.x < tokens) lows[threadIdx.x] = first_key(a, ctx + q0 + threadIdx.x);
 
   // this wave's queries; row 16 i + c.  Rows past the end repeat valid ones
   bf16x8_v qf[2][STEPS];
@@ -414,30 +436,66 @@ __global__ __launch_bounds__(512, 2) void talk_prefill_kernel(const GroupedArgs 
   const int k_end = ctx + q0 + tokens;
   const int first = first_key(a, ctx + q0) / KT * KT;
   const int n_tiles = (k_end - first + KT - 1) / KT;
-  const bf16_t* kc = (const bf16_t*)a.k_cache + (int64_t)wid * D + quad * 8;
-  const bf16_t* vc = (const bf16_t*)a.v_cache + (int64_t)wid * V;
+  const int k_row = a.G * D * 2, v_row = a.G * V * 2;  // bytes of a cached key and value
+  const int me = __builtin_amdgcn_readfirstlane(wid);
+  const char* const kc = (const char*)a.k_cache + me * D * 2;
+  const char* const vc = (const char*)a.v_cache + me * V * 2;
   char* const values = lds + L.values + wid * KT * V * 2;
-  // this lane's key of tile t: its page's place in the table, its place in the page
-  auto key_of = [&](int t) { return min(first + t * KT + (lane & 31), k_end - 1); };
-  auto slot_of = [&](int t, int page, int block) {
-    return block * a.kv_block + key_of(t) - page * a.kv_block;
+  // 16 keys lie in one page: everything about them but a lane's constant offset is scalar
+  struct Half {
+    int page, in;  // place in the table, first key within the page
   };
-  bf16x8_v kf[2][STEPS];
-  auto load_keys = [&](int slot) {
+  Half ahead = {first / a.kv_block, first % a.kv_block};
+  const int last_page = (k_end - 1) / a.kv_block;
+  int blocks[2], ins[2];  // of the tile after those whose slots are known
+  auto look_up = [&]() {
 #pragma unroll
     for (int b = 0; b < 2; ++b) {
-      const bf16_t* k = kc + (int64_t)__shfl(slot, 16 * b + c, 64) * a.G * D;
-#pragma unroll
-      for (int s = 0; s < STEPS; ++s) kf[b][s] = *(const bf16x8_v*)(k + s * 32);
+      blocks[b] = table[min(ahead.page, last_page)];
+      ins[b] = ahead.in;
+      ahead.in += 16;
+      if (ahead.in == a.kv_block) ahead = {ahead.page + 1, 0};
     }
   };
-  auto load_values = [&](int slot) {  // for this wave alone
+  struct Slots {
+    int64_t of[2];
+  };
+  auto found = [&]() {
+    Slots s;
 #pragma unroll
-    for (int i = 0; i < VU / 2; ++i) {
-      const int u = i * 64 + lane, key = u / VU;
-      const int unit = (u - key * VU) ^ (((key & 3) << 1) | ((key >> 2) & 1));
-      load_to_lds(values + i * 1024, vc + (int64_t)__shfl(slot, key, 64) * a.G * V + unit * 8);
+    for (int b = 0; b < 2; ++b)
+      s.of[b] = (int64_t)__builtin_amdgcn_readfirstlane(blocks[b]) * a.kv_block + ins[b];
+    return s;
+  };
+  bf16x8_v kf[2][STEPS];
+  const unsigned k_lane = c * k_row + quad * 16;
+  auto load_keys = [&](const Slots& s) {
+#pragma unroll
+    for (int b = 0; b < 2; ++b) {
+      const char* k = kc + s.of[b] * k_row;
+#pragma unroll
+      for (int st = 0; st < STEPS; ++st)
+        kf[b][st] = *(const bf16x8_v*)(k + (k_lane + st * 64));
     }
+  };
+  constexpr int KEYS = 64 / VU;  // of a load; a lane's place in one repeats every 16 keys
+  unsigned v_lane[16 / KEYS];
+#pragma unroll
+  for (int i = 0; i < 16 / KEYS; ++i) {
+    const int key = i * KEYS + lane / VU;
+    v_lane[i] = key * v_row + swizzled<VU>(lane % VU, key) * 16;
+  }
+  const unsigned v_dst =
+      __builtin_amdgcn_readfirstlane((unsigned)(uintptr_t)(lds_char*)values);
+  auto load_values = [&](const Slots& s) {  // for this wave alone
+#pragma unroll
+    for (int i = 0; i < KT / KEYS; ++i)
+      load_to_lds(v_dst + i * 1024, vc + s.of[i * KEYS / 16] * v_row, v_lane[i % (16 / KEYS)]);
+  };
+  // keys past the end have weight zero, but what lies there need not be a number
+  auto clear_values = [&](int from) {
+    for (int i = from * VU + lane; i < KT * VU; i += 64)
+      ((ulonglong2*)values)[i] = ulonglong2{0, 0};
   };
 
   const float mul = a.scale * LOG2E;
@@ -487,7 +545,7 @@ __global__ __launch_bounds__(512, 2) void talk_prefill_kernel(const GroupedArgs 
   };
   f32x4_v o[2][VT] = {};  // rows 16 i + 4 quad + r, dims 16 n + c
   auto add_values = [&](int t) {
-    const char* weights = lds + L.weights + ((t & 1) * a.G + wid) * 32 * KT * 2;
+    const char* weights = lds + L.weights + ((t & 1) * a.G + wid) * W_HEAD;
     const float* alpha = (const float*)(lds + L.alpha) + ((t & 1) * a.G + wid) * 32;
     f32x4_v f[2];
 #pragma unroll
@@ -505,15 +563,15 @@ __global__ __launch_bounds__(512, 2) void talk_prefill_kernel(const GroupedArgs 
 #pragma unroll
     for (int i = 0; i < 2; ++i)
       pf[i] = *(const bf16x8_v*)(weights + (16 * i + c) * KT * 2 + quad * 16);
-    const int j = c >> 2, sw = j << 1;
-    const char* vrow = values + (quad * 8 + j) * V * 2 + (c & 1) * 8;
+    const int key = quad * 8 + (c >> 2);
+    const char* vrow = values + key * V * 2 + (c & 1) * 8;
 #pragma unroll
     for (int n = 0; n < VT; ++n) {
       const int unit = n * 2 + ((c & 3) >> 1);
       const bf16x4_v a0 = __builtin_amdgcn_ds_read_tr16_b64_v4bf16(
-          (lds_bf16x4*)(vrow + ((unit ^ sw) << 4)));
+          (lds_bf16x4*)(vrow + (swizzled<VU>(unit, key) << 4)));
       const bf16x4_v a1 = __builtin_amdgcn_ds_read_tr16_b64_v4bf16(
-          (lds_bf16x4*)(vrow + 4 * V * 2 + ((unit ^ (sw | 1)) << 4)));
+          (lds_bf16x4*)(vrow + 4 * V * 2 + (swizzled<VU>(unit, key + 4) << 4)));
       const bf16x8_v vf = __builtin_shufflevector(a0, a1, 0, 1, 2, 3, 4, 5, 6, 7);
 #pragma unroll
       for (int i = 0; i < 2; ++i)
@@ -521,14 +579,13 @@ __global__ __launch_bounds__(512, 2) void talk_prefill_kernel(const GroupedArgs 
     }
   };
 
-  // slots of the keys of tiles t, t + 1 and t + 2
-  int page = key_of(0) / a.kv_block;
-  int here = slot_of(0, page, table[page]);
+  // slots of tiles t and t + 1, pages of tile t + 2
+  look_up();
+  Slots here = found();
   load_keys(here);
-  page = key_of(1) / a.kv_block;
-  int next = slot_of(1, page, table[page]);
-  page = key_of(2) / a.kv_block;
-  int block = table[page];
+  look_up();
+  Slots next = found();
+  look_up();
   __syncthreads();
   score();
   load_keys(next);
@@ -539,7 +596,7 @@ __global__ __launch_bounds__(512, 2) void talk_prefill_kernel(const GroupedArgs 
     const int key0 = first + t * KT;
     // a wave per token: head 16 h + c, keys key0 + 16 b + 4 quad + r
     for (int q = wid; q < tokens; q += a.G) {
-      const int pos = ctx + q0 + q, lo = first_key(a, pos);
+      const int pos = ctx + q0 + q, lo = lows[q];
       f32x4_v s[2][HT] = {};
 #pragma unroll
       for (int b = 0; b < 2; ++b) {
@@ -587,8 +644,8 @@ __global__ __launch_bounds__(512, 2) void talk_prefill_kernel(const GroupedArgs 
         const float2 old = stats[q * a.H + (has ? h : 0)];
         mt = fmaxf(quad_max(mt), old.x);
         float sum = 0.f;
-        const int at = ((t & 1) * a.G + h / group) * 32 + q * group + h % group;
-        char* dst = lds + L.weights + at * KT * 2 + quad * 8;
+        const int g = (t & 1) * a.G + h / group, row = q * group + h % group;
+        char* dst = lds + L.weights + g * W_HEAD + row * KT * 2 + quad * 8;
 #pragma unroll
         for (int b = 0; b < 2; ++b) {
           float p[4];
@@ -603,28 +660,29 @@ __global__ __launch_bounds__(512, 2) void talk_prefill_kernel(const GroupedArgs 
         if (has && quad == 0) {
           const float f = __builtin_amdgcn_exp2f(old.x - mt);
           stats[q * a.H + h] = float2{mt, old.y * f + sum};
-          ((float*)(lds + L.alpha))[at] = f;
+          ((float*)(lds + L.alpha))[g * 32 + row] = f;
         }
       }
     }
     score();  // of tile t + 1
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");      // the last tile's values are here
+    const Slots after = found();
+    load_keys(after);
     if (t > 0) {
-      asm volatile("s_waitcnt vmcnt(0)" ::: "memory");    // the last tile's values are here
       add_values(t - 1);
       asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");  // and may be overwritten
     }
-    const int after = slot_of(t + 2, page, block);
-    load_keys(after);
     load_values(here);
     here = next;
     next = after;
-    page = key_of(t + 3) / a.kv_block;
-    block = table[page];
+    look_up();
     __syncthreads();
     put_scores();
     __syncthreads();
   }
   asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+  clear_values(k_end - (first + (n_tiles - 1) * KT));
+  wave_sync();
   add_values(n_tiles - 1);
 
 #pragma unroll
@@ -677,14 +735,15 @@ static bool mixes(const GroupedArgs& a) {
 extern "C" {
 
 // Tokens per workgroup of the prompt kernel for these sizes; 0: the plain kernel.
-int talk_prefill_tokens(int H, int G, int d, int v) {
+int talk_prefill_tokens(int H, int G, int d, int v, int kv_block) {
+  if (kv_block % 16) return 0;
   const int group = H / G;
   if ((d != 64 && d != 128) || (v != 64 && v != 128) || G > 8 || H > 64 || group > 32) return 0;
   return prompt_lds(H, G, 32 / group, v).total <= 160 * 1024 ? 32 / group : 0;
 }
 
 bool launch_talk_prefill(const GroupedArgs* a, int d, int v, hipStream_t stream) {
-  if (!mixes(*a) || !talk_prefill_tokens(a->H, a->G, d, v)) return false;
+  if (!mixes(*a) || !talk_prefill_tokens(a->H, a->G, d, v, a->kv_block)) return false;
   if (d == 64)
     return v == 64 ? launch_prefill_heads<1, 1>(*a, stream) : launch_prefill_heads<1, 2>(*a, stream);
   return v == 64 ? launch_prefill_heads<2, 1>(*a, stream) : launch_prefill_heads<2, 2>(*a, stream);
