@@ -167,6 +167,20 @@ def test_mixed_scores_in_chunks(device, dtype, H, G, d, e, chunk, talk, block, c
         at += new
 
 
+def test_prompt_tiles_are_ordered_by_their_keys():
+    batch, chunks, _, _ = make_batch([(0, 70), (25, 30), (7, 1), (100, 9)], 16, "cpu")
+    meta = batch.prefill_meta(8, chunk=30)
+    tiles = list(zip(meta.tile_seq.tolist(), meta.tile_q0.tolist()))
+    plain = batch.prefill_meta(8)
+    assert sorted(tiles) == sorted(zip(plain.tile_seq.tolist(), plain.tile_q0.tolist()))
+
+    def keys(s, q0):
+        ctx, new = chunks[s]
+        return ctx + min(q0 + 8, new) - (ctx + q0) // 30 * 30
+
+    assert [keys(*t) for t in tiles] == sorted(keys(*t) for t in tiles)
+
+
 @pytest.mark.parametrize("H,G", [(6, 3), (8, 2), (32, 8)])
 @pytest.mark.parametrize("portion", [1, 3, 100], ids=["decode", "portion", "prompt"])
 def test_every_head_hears_the_right_one(device, dtype, portion, H, G):
