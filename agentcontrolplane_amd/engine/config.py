@@ -416,7 +416,7 @@ def _lobuvik(name: str, *, width: int, layers: int, heads: int, kv_heads: int, d
 def _noganex(name: str, *, width: int, layers: int, heads: int, kv_heads: int, dim: int,
              vdim: int, chunk: int, rotary: RotarySpec, d_heads: int, d_kv_heads: int,
              d_dim: int, d_vdim: int, ff: int, experts: ExpertsSpec, vocab: int, conv: int = 4,
-             logit_scale: float = 0.5, **kw) -> ModelConfig:
+             logit_scale: float = 0.25, **kw) -> ModelConfig:
     """Chunked attention with a dense feed-forward and delta layers with experts in turn;
     every second delta layer uses the one before's weights."""
     attention = LayerSpec(GroupedAttentionSpec(

@@ -285,8 +285,9 @@ def grouped_attention(q, k_cache, v_cache, batch, scale: float, cap, window, kee
                       sink, out, bias=None, sigmoid: bool = False, gate=None, chunk=None,
                       talk=None):
     """Attention of a FlatBatch's rows over the paged cache; query head n uses
-    key/value head n // (H / G).  ``talk`` [H, H] (fp32) mixes the scores over the heads:
-    head h's are sum_g talk[h, g] * head g's.  Scores are capped if ``cap``; a query sees
+    key/value head n // (H / G).  ``talk`` [H, H] (fp32, of values that the
+    model's dtype holds) mixes the scores over the heads: head h's are
+    sum_g talk[h, g] * head g's.  Scores are capped if ``cap``; a query sees
     itself and the ``window`` - 1 tokens before it (None = all) and the ``keep_first``
     first tokens, with ``chunk`` (no keep_first) only those of its own chunk, position
     // chunk; ``sink`` [H] (fp32) or None joins the softmax denominator.

@@ -181,7 +181,7 @@ def test_prompt_tiles_are_ordered_by_their_keys():
     assert [keys(*t) for t in tiles] == sorted(keys(*t) for t in tiles)
 
 
-@pytest.mark.parametrize("H,G", [(6, 3), (8, 2), (32, 8)])
+@pytest.mark.parametrize("H,G", [(9, 3), (8, 2), (32, 8)])
 @pytest.mark.parametrize("portion", [1, 3, 100], ids=["decode", "portion", "prompt"])
 def test_every_head_hears_the_right_one(device, dtype, portion, H, G):
     """Talk weights that permute the heads: a head attends by another one's scores, to its
